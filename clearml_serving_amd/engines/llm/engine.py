@@ -19,6 +19,10 @@ Engine step (continuous batching):
 
 Model families: llama / qwen2 (models/llama.py) and gpt2 (models/gpt2.py)
 share one forward interface, so every scheduler feature serves both.
+Token-batch families (models/bimipel.py) take steps 2 and 3 as ONE forward
+over a flat batch of prompt portions and single tokens (token_batch.py); next
+to pages they hold one state slot per running sequence for their recurrent
+layers, and a step of single tokens only is hipGraph-replayed as above.
 Opt-in subsystems, each exact by test: fp8 weights (fused activation
 quant), fp8 KV cache, ngram speculation, automatic prefix caching
 (content-addressed blocks, prompt + generated), TP over RCCL/xGMI with
@@ -43,7 +47,9 @@ from typing import Any, AsyncGenerator, Dict, List, Optional
 import torch
 
 from ... import ops
+from ...models import arch_of_config, token_batch_builder
 from ...models.llama import PRESETS, LlamaConfig, LlamaForCausalLM
+from .token_batch import TokenBatch
 
 
 # --------------------------------------------------------------------- #
@@ -261,6 +267,8 @@ class LlmEngineConfig:
     weights: Optional[str] = None
     tokenizer_path: Optional[str] = None
     device: Optional[str] = None
+    model_config: Optional[Dict[str, Any]] = None  # a model folder's
+                                # config.json (families that read one)
     # speculative decoding (vLLM parity): {"method": "ngram",
     # "num_spec_tokens": K, "ngram": N}. Prompt-lookup proposals verified
     # in ONE multi-token forward; EXACT under greedy sampling (accepted
@@ -290,6 +298,13 @@ class LlmEngineConfig:
                 w = os.path.join(model_path, "model.safetensors")
                 if os.path.exists(w):
                     cfg.weights = w
+                hf = os.path.join(model_path, "config.json")
+                if os.path.exists(hf):
+                    with open(hf) as f:
+                        raw = json.load(f)
+                    arch = arch_of_config(raw)
+                    if arch is not None:
+                        cfg.arch, cfg.model_config = arch, raw
             elif model_path.endswith(".json"):
                 with open(model_path) as f:
                     card = json.load(f)
@@ -430,6 +445,26 @@ class PrefixCacheAllocator(BlockAllocator):
         return len(self._free) + len(self._lru)
 
 
+class StateSlots:
+    """Recurrent-state slots, one per running sequence. A slot is never
+    cleared: kernels start a sequence's first token from zero state."""
+
+    def __init__(self, num_slots: int):
+        self._free = list(range(num_slots - 1, -1, -1))
+
+    def alloc(self) -> int:
+        if not self._free:
+            raise RuntimeError("no recurrent-state slot free")
+        return self._free.pop()
+
+    def free(self, slot: int) -> None:
+        self._free.append(slot)
+
+    @property
+    def available(self) -> int:
+        return len(self._free)
+
+
 class Sequence:
     def __init__(self, req_id: str, prompt_ids: List[int],
                  params: SamplingParams):
@@ -440,6 +475,7 @@ class Sequence:
         self.prefilled = 0  # prompt tokens already in the KV cache
         self.params = params
         self.blocks: List[int] = []
+        self.state_slot = -1  # recurrent-state slot (token-batch families)
         self.stream: "asyncio.Queue" = asyncio.Queue()
         self.finished = False
         self.finish_reason: Optional[str] = None
@@ -473,6 +509,8 @@ class LlmEngine:
         self.model: Optional[LlamaForCausalLM] = None
         self.kv_caches: List = []
         self.allocator: Optional[BlockAllocator] = None
+        self.state_slots: Optional[StateSlots] = None
+        self.token_batch = False  # set by start(): the family's batch form
         self.tokenizer = None
         self.waiting: List[Sequence] = []
         self.running: List[Sequence] = []
@@ -516,9 +554,21 @@ class LlmEngine:
         self.tp_size = tp_mod.world_size()
         self.tp_rank = tp_mod.rank()
         torch.manual_seed(1234)  # identical replicated params across ranks
-        gpt2 = (str(cfg.arch).lower() == "gpt2"
+        builder = token_batch_builder(cfg.arch)
+        gpt2 = builder is None and (str(cfg.arch).lower() == "gpt2"
                 or str(cfg.preset).startswith("gpt2"))
-        if gpt2:
+        if builder is not None:
+            self._check_token_batch_config()
+            model = builder(cfg.model_config, cfg.preset, cfg.overrides)
+            mcfg = self.model_config = model.cfg
+            self.token_batch = True
+            if str(cfg.dtype) == "float32":
+                # exact runs: no reduced-precision matrix mode either
+                torch.set_float32_matmul_precision("highest")
+                self.dtype = torch.float32
+            if not cfg.weights:
+                model.init_random()
+        elif gpt2:
             # GPT-2 family: same engine-facing forward interface as llama
             # (paged kv_caches + attn_ctx modes), so scheduling, chunked
             # prefill, decode graphs and speculation serve it unchanged
@@ -565,6 +615,8 @@ class LlmEngine:
 
                 load_weights(model, cfg.weights)
         self.model = model.eval().to(self.device).to(self.dtype)
+        if self.token_batch:
+            self.model.finalize()
         if cfg.quantization == "fp8":
             if self.device.type != "cuda":
                 raise ValueError("fp8 quantization needs a GPU (hipBLASLt)")
@@ -582,6 +634,10 @@ class LlmEngine:
 
         # KV cache sizing from free HBM (heads sharded under TP)
         bs = cfg.block_size
+        if self.token_batch:
+            self._start_token_batch_caches()
+            self._started = True
+            return
         kv_heads = mcfg.kv_heads // self.tp_size
         fp8_kv = str(cfg.kv_dtype).lower() in ("fp8", "float8", "e4m3")
         kv_itemsize = 1 if fp8_kv else self.dtype.itemsize
@@ -636,6 +692,81 @@ class LlmEngine:
 
             self._plan_codec = PlanCodec(cfg, self.device)
         self._started = True
+
+    # ------------------------------------------------------------------ #
+    # token-batch families: caches
+    # ------------------------------------------------------------------ #
+    def _check_token_batch_config(self) -> None:
+        """Refuse options whose mechanism does not exist for these models,
+        rather than serve without them."""
+        cfg = self.cfg
+        bad = []
+        if self.tp_size > 1:
+            bad.append("tensor parallelism")
+        if cfg.quantization:
+            bad.append("quantization")
+        if str(cfg.kv_dtype).lower() in ("fp8", "float8", "e4m3"):
+            bad.append("fp8 KV cache")
+        if cfg.enable_prefix_caching:
+            # a shared prefix would need the recurrent state at its end
+            bad.append("prefix caching")
+        if cfg.speculative:
+            # a rejected token cannot be taken out of the recurrent state
+            bad.append("speculative decoding")
+        if bad:
+            raise ValueError("arch '{}' does not support {}".format(
+                cfg.arch, ", ".join(bad)))
+
+    def _new_layer_caches(self, num_blocks: int, num_slots: int) -> List:
+        """Per layer: page tensor [blocks, block_size, row], (state float
+        [slots, channels], ring [slots, taps, channels]), or the tensor of
+        the layer it shares with."""
+        caches: List = []
+        for kind, *dims in self.model.cache_layout():
+            if kind == "paged":
+                caches.append(torch.zeros(
+                    num_blocks, self.cfg.block_size, dims[0],
+                    dtype=self.dtype, device=self.device))
+            elif kind == "state":
+                channels, taps = dims
+                caches.append((
+                    torch.zeros(num_slots, channels, dtype=torch.float32,
+                                device=self.device),
+                    torch.zeros(num_slots, taps, channels, dtype=self.dtype,
+                                device=self.device)))
+            else:  # shared
+                caches.append(caches[dims[0]])
+        return caches
+
+    def _start_token_batch_caches(self) -> None:
+        cfg = self.cfg
+        rows = [d[0] for kind, *d in self.model.cache_layout()
+                if kind == "paged"]
+        per_block = max(sum(rows), 1) * cfg.block_size * self.dtype.itemsize
+        if cfg.num_kv_blocks:
+            num_blocks = int(cfg.num_kv_blocks)
+        elif self.device.type == "cuda":
+            free, _ = torch.cuda.mem_get_info(self.device)
+            # no more than every slot can fill
+            most = cfg.max_num_seqs * (-(-cfg.max_model_len // cfg.block_size)
+                                       + 1)
+            num_blocks = max(min(int(free * cfg.gpu_memory_fraction)
+                                 // per_block, most), 64)
+        else:
+            num_blocks = 512
+        self.allocator = BlockAllocator(num_blocks)
+        self.state_slots = StateSlots(cfg.max_num_seqs)
+        self.kv_caches = self._new_layer_caches(num_blocks, cfg.max_num_seqs)
+        self._batch_params = self.model.batch_params(self.dtype)
+
+    def _release(self, seq: "Sequence") -> None:
+        """give back what a sequence holds"""
+        if seq.blocks:
+            self.allocator.free(seq.blocks)
+            seq.blocks = []
+        if seq.state_slot >= 0:
+            self.state_slots.free(seq.state_slot)
+            seq.state_slot = -1
 
     # ------------------------------------------------------------------ #
     # request API
@@ -768,9 +899,7 @@ class LlmEngine:
                 for seq in self.waiting + self.running:
                     seq.stream.put_nowait(
                         {"error": str(ex), "finished": True, "token_ids": []})
-                    if seq.blocks:
-                        self.allocator.free(seq.blocks)
-                        seq.blocks = []
+                    self._release(seq)
                 self.waiting.clear()
                 self.running.clear()
                 raise
@@ -789,6 +918,10 @@ class LlmEngine:
         self.stats["steps"] += 1
         self._drain_aborts()
         self._admit()
+        if self.token_batch:
+            self._step_token_batch()
+            self._retire_finished()
+            return
         budget = self.cfg.prefill_chunk
         pending = [s for s in self.running
                    if s.prefilled < len(s.prompt_ids)]
@@ -828,12 +961,14 @@ class LlmEngine:
                 self._decode_spec(spec, spec_k)
             if rest:
                 self._decode(rest)
+        self._retire_finished()
+
+    def _retire_finished(self) -> None:
         for s in list(self.running):
             self._register_prefix(s)  # publish newly-FILLED blocks
             if s.finished:
                 self.running.remove(s)
-                self.allocator.free(s.blocks)
-                s.blocks = []
+                self._release(s)
 
     def _drain_aborts(self) -> None:
         """Apply aborts queued by abort() -- all scheduler-state mutation
@@ -847,9 +982,7 @@ class LlmEngine:
                 self.waiting.remove(seq)
             if seq in self.running:
                 self.running.remove(seq)
-            if seq.blocks:
-                self.allocator.free(seq.blocks)
-                seq.blocks = []
+            self._release(seq)
 
     def _admit(self) -> List[Sequence]:
         admitted: List[Sequence] = []
@@ -880,6 +1013,8 @@ class LlmEngine:
                     self.allocator.free(cached)
                 break
             seq.blocks = cached + self.allocator.alloc(need_blocks)
+            if self.state_slots is not None:
+                seq.state_slot = self.state_slots.alloc()
             seq.prefilled = ncached  # cached prefix skips its prefill
             # registration chain restarts at the match point (also resets
             # stale state on preemption re-admission)
@@ -948,15 +1083,10 @@ class LlmEngine:
         self.stats["prompt_tokens"] += sum(len(p) for p in plan["prompts"])
         self._sample_and_emit(seqs, logits, sample=plan["sample"])
 
-    def _prefill_chunk(self, seqs: List["Sequence"], budget: int) -> None:
-        """Advance several sequences' prefill by up to ``budget`` tokens
-        total in ONE batched paged-attention forward; samples first tokens
-        for the sequences whose chunk completes the prompt.
-
-        Fair-share: the budget splits evenly across chunking prompts (then
-        leftovers go FCFS), so a newly arrived long prompt advances every
-        step instead of starving behind an earlier prompt's remaining
-        chunks (round-1 packed strictly FCFS)."""
+    @staticmethod
+    def _share_budget(seqs: List["Sequence"], budget: int) -> List[tuple]:
+        """-> [(sequence, prompt tokens to take)], at most ``budget`` in all;
+        evenly first, then leftovers in order of arrival."""
         batch = []
         if len(seqs) > 1:
             share = max(budget // len(seqs), 1)
@@ -985,6 +1115,18 @@ class LlmEngine:
                 chunk = min(budget, len(s.prompt_ids) - s.prefilled)
                 batch.append((s, chunk))
                 budget -= chunk
+        return batch
+
+    def _prefill_chunk(self, seqs: List["Sequence"], budget: int) -> None:
+        """Advance several sequences' prefill by up to ``budget`` tokens
+        total in ONE batched paged-attention forward; samples first tokens
+        for the sequences whose chunk completes the prompt.
+
+        Fair-share: the budget splits evenly across chunking prompts (then
+        leftovers go FCFS), so a newly arrived long prompt advances every
+        step instead of starving behind an earlier prompt's remaining
+        chunks (round-1 packed strictly FCFS)."""
+        batch = self._share_budget(seqs, budget)
         if not batch:
             return
         self.stats["prefill_batches"] += 1
@@ -1095,6 +1237,12 @@ class LlmEngine:
         lens = [len(p) for p in prompts]
         smax = max(lens)
         dev = self.device
+        if self.token_batch:
+            flat = self._embed_token_batch(prompts).float()
+            pooled = torch.stack([p.mean(0) for p in flat.split(lens)])
+            if plan.get("normalize", True):
+                pooled = torch.nn.functional.normalize(pooled, dim=-1)
+            return pooled
         tokens = torch.zeros(b, smax, dtype=torch.long)
         positions = torch.zeros(b, smax, dtype=torch.int32)
         for i in range(b):
@@ -1143,16 +1291,16 @@ class LlmEngine:
             return False
         victim = max(candidates, key=lambda s: s.created)
         self.running.remove(victim)
-        self.allocator.free(victim.blocks)
-        victim.blocks = []
+        self._release(victim)
         victim.prompt_ids = victim.prompt_ids + victim.output_ids
         victim.output_ids = []
         self.waiting.insert(0, victim)
         self.stats["preemptions"] = self.stats.get("preemptions", 0) + 1
         return True
 
-    def _decode(self, seqs: List[Sequence]) -> None:
-        self.stats["decode_batches"] += 1
+    def _grow_for_decode(self, seqs: List[Sequence]) -> None:
+        """a page for each sequence's newest token; preempted sequences
+        leave ``seqs``"""
         bs_cfg = self.cfg.block_size
         # grow block tables for the token being generated; under KV pressure
         # preempt the newest sequences instead of failing the whole engine
@@ -1175,6 +1323,10 @@ class LlmEngine:
         # above and out of the batch -- make that invariant explicit so the
         # plan below can never index a freed block list
         seqs[:] = [s for s in seqs if s in self.running]
+
+    def _decode(self, seqs: List[Sequence]) -> None:
+        self.stats["decode_batches"] += 1
+        self._grow_for_decode(seqs)
         if not seqs:
             return
         plan = {
@@ -1261,6 +1413,120 @@ class LlmEngine:
             }
             parts.append((tokens, positions, attn_ctx))
         return self.model.forward_pipelined(parts, self.kv_caches)
+
+    # -------------------- token-batch families ------------------------ #
+    def _step_token_batch(self) -> None:
+        """One forward for everything that runs: the newest token of each
+        decoding sequence beside up to ``prefill_chunk`` prompt tokens."""
+        decoding = [s for s in self.running if not s.finished
+                    and s.prefilled >= len(s.prompt_ids) and s.output_ids]
+        self._grow_for_decode(decoding)
+        pending = [s for s in self.running
+                   if not s.finished and s.prefilled < len(s.prompt_ids)]
+        portions = self._share_budget(pending, self.cfg.prefill_chunk)
+        items = [(s, [s.output_ids[-1]], len(s) - 1, [0]) for s in decoding]
+        done = list(decoding)
+        for s, n in portions:
+            complete = s.prefilled + n >= len(s.prompt_ids)
+            items.append((s, s.prompt_ids[s.prefilled:s.prefilled + n],
+                          s.prefilled, [n - 1] if complete else []))
+            if complete:
+                done.append(s)
+        if not items:
+            return
+        self.stats["decode_batches"] += bool(decoding)
+        self.stats["prefill_batches"] += bool(portions)
+        logits = self._exec_batch(self._batch_plan(items))
+        for s, n in portions:
+            s.prefilled += n
+            self.stats["prompt_tokens"] += n
+        if done:
+            self._sample_and_emit(done, logits)
+
+    @staticmethod
+    def _batch_plan(items: List[tuple]) -> Dict[str, Any]:
+        """items: (sequence, tokens, first position, places among the tokens
+        whose logits are wanted)"""
+        return {
+            "mode": "batch",
+            "tokens": [t for _, t, _, _ in items],
+            "starts": [p for _, _, p, _ in items],
+            "blocks": [s.blocks for s, _, _, _ in items],
+            "state_slots": [s.state_slot for s, _, _, _ in items],
+            "want": [w for _, _, _, w in items],
+        }
+
+    @torch.inference_mode()
+    def _exec_batch(self, plan: Dict[str, Any]) -> torch.Tensor:
+        """-> logits of the wanted places [rows, vocab], in plan order"""
+        if (all(len(t) == 1 for t in plan["tokens"])
+                and len(plan["tokens"]) <= self.cfg.max_num_seqs
+                and self._use_decode_graphs()):
+            bs = self.cfg.block_size
+            starts = plan["starts"]
+            logits = self._exec_decode_graph({
+                "tokens": [t[0] for t in plan["tokens"]],
+                "positions": starts,
+                "slots": [b[p // bs] * bs + p % bs
+                          for b, p in zip(plan["blocks"], starts)],
+                "seq_lens": [p + 1 for p in starts],
+                "blocks": plan["blocks"],
+                "state_slots": plan["state_slots"],
+            })
+            rows = [i for i, w in enumerate(plan["want"]) for _ in w]
+            return logits if rows == list(range(len(starts))) \
+                else logits[rows]
+        tokens, batch, rows = TokenBatch.build(
+            plan, self.cfg.block_size, self.device, **self._batch_params)
+        return self.model(tokens, batch.positions, kv_caches=self.kv_caches,
+                          attn_ctx=batch, last_token_idx=rows)
+
+    def open_sequence(self, seq: Sequence) -> None:
+        """Take a state slot for a sequence that the caller feeds itself
+        (``feed``) instead of queueing it for generation."""
+        with self._exec_lock:
+            seq.state_slot = self.state_slots.alloc()
+
+    def close_sequence(self, seq: Sequence) -> None:
+        with self._exec_lock:
+            self._release(seq)
+
+    def feed(self, entries: List[tuple]) -> torch.Tensor:
+        """Run given next tokens of several open sequences as one batch:
+        entries (sequence, tokens, wanted places) -> their logits. What the
+        scheduler does in a step, with the caller choosing the tokens."""
+        bs = self.cfg.block_size
+        with self._exec_lock:
+            items = []
+            for s, tokens, want in entries:
+                end = s.prefilled + len(tokens)
+                need = -(-end // bs) - len(s.blocks)
+                if need > 0:
+                    s.blocks.extend(self.allocator.alloc(need))
+                items.append((s, tokens, s.prefilled, want))
+            logits = self._exec_batch(self._batch_plan(items))
+            for s, tokens, _ in entries:
+                s.prefilled += len(tokens)
+            return logits
+
+    def _embed_token_batch(self, prompts: List[List[int]]) -> torch.Tensor:
+        """final hidden states of every token, on caches of their own:
+        running sequences keep theirs"""
+        bs = self.cfg.block_size
+        plan = {"tokens": prompts, "starts": [0] * len(prompts), "blocks": [],
+                "state_slots": list(range(len(prompts))),
+                "want": [range(len(p)) for p in prompts]}
+        used = 0
+        for p in prompts:
+            n = -(-len(p) // bs)
+            plan["blocks"].append(list(range(used, used + n)))
+            used += n
+        tokens, batch, rows = TokenBatch.build(
+            plan, bs, self.device, **self._batch_params)
+        return self.model(
+            tokens, batch.positions, attn_ctx=batch, last_token_idx=rows,
+            kv_caches=self._new_layer_caches(used, len(prompts)),
+            return_hidden=True)
 
     # -------------------- speculative decoding (ngram) ---------------- #
     # Prompt-lookup speculation (vLLM's "ngram" method): propose the K
@@ -1463,6 +1729,14 @@ class LlmEngine:
         attn_ctx = {"mode": "decode", "seq_lens": static["seq_lens"],
                     "block_table": static["block_table"],
                     "slot_mapping": static["slots"]}
+        if self.token_batch:
+            static["state_slots"] = torch.full_like(static["slots"], -1)
+            attn_ctx = TokenBatch.of_single_tokens(
+                static["positions"], static["slots"],
+                torch.arange(bucket, dtype=torch.int32, device=dev),
+                static["block_table"], static["state_slots"],
+                tile=self._batch_params["tile"],
+                max_keys=self.cfg.max_model_len)
 
         def fwd():
             return self.model(static["tokens"], static["positions"],
@@ -1511,6 +1785,9 @@ class LlmEngine:
                 "block_table": torch.zeros(bucket, mb, dtype=torch.int32,
                                            pin_memory=True),
             }
+            if self.token_batch:
+                pin["state_slots"] = torch.full(
+                    (bucket,), -1, dtype=torch.int32, pin_memory=True)
             self._decode_pin[bucket] = pin
         pin["tokens"][:b] = torch.tensor(plan["tokens"], dtype=torch.long)
         pin["tokens"][b:] = 0
@@ -1526,7 +1803,11 @@ class LlmEngine:
         bt.zero_()
         for i, bl in enumerate(plan["blocks"]):
             bt[i, :len(bl)] = torch.tensor(bl, dtype=torch.int32)
-        for k in ("tokens", "positions", "slots", "seq_lens", "block_table"):
+        if self.token_batch:
+            pin["state_slots"][:b] = torch.tensor(plan["state_slots"],
+                                                  dtype=torch.int32)
+            pin["state_slots"][b:] = -1
+        for k in pin:
             entry[k].copy_(pin[k], non_blocking=True)
         entry["graph"].replay()
         self.stats["graph_replays"] += 1

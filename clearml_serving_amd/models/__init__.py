@@ -30,6 +30,28 @@ def register_arch(name: str):
     return deco
 
 
+# LLM families that run on flat token batches (engines/llm/token_batch.py):
+# arch -> builder(config, preset, overrides); and the "architecture" that a
+# model folder's config.json names -> arch
+_TOKEN_BATCH = {}
+_ARCHITECTURES = {}
+
+
+def register_token_batch_arch(arch: str, builder, architecture: str) -> None:
+    _TOKEN_BATCH[arch] = builder
+    _ARCHITECTURES[architecture] = arch
+
+
+def token_batch_builder(arch: str):
+    """the family's builder, or None for other families"""
+    return _TOKEN_BATCH.get(str(arch).lower())
+
+
+def arch_of_config(config: dict) -> Optional[str]:
+    """arch for a config.json, None if it names no family of this library"""
+    return _ARCHITECTURES.get(config.get("architecture"))
+
+
 def list_archs():
     return sorted(_BUILDERS.keys())
 
@@ -65,6 +87,9 @@ def load_weights(model: torch.nn.Module, path: str) -> None:
         state = load_file(path)
     else:
         state = torch.load(path, map_location="cpu", weights_only=True)
+    if hasattr(model, "load_checkpoint"):  # packs its own checkpoint layout
+        model.load_checkpoint(state)
+        return
     # raw HuggingFace checkpoints convert on the fly (key-layout
     # detection; native layouts pass through) -- a hub download drops in
     # without a manual conversion step
@@ -73,4 +98,4 @@ def load_weights(model: torch.nn.Module, path: str) -> None:
     model.load_state_dict(convert_hf_auto(state))
 
 
-from . import bert, gpt2, llama, resnet  # noqa: E402,F401  (register architectures)
+from . import bert, bimipel, gpt2, llama, resnet  # noqa: E402,F401  (register architectures)

@@ -1,0 +1,286 @@
+"""Bimipel: a decoder of sliding-window latent attention and gated linear
+recurrence layers, normalised on the sublayers' outputs.
+
+    x = embed[token]
+    x <- x + norm1(mixer(x));  x <- x + norm2(ff(x))   (ff where it has one)
+    logits = logit_scale * embed @ norm(x)
+
+The residual stream is float and is what the sublayers read; the norms'
+weights are stored around zero. Layers are listed one by one in the
+configuration, so order, sizes and windows are per layer. An attention layer
+may use an earlier layer's cached latent instead of its own (``kv_from``).
+
+Runs on flat token batches (engines/llm/token_batch.py): prompt portions and
+single tokens of different sequences in one forward.
+"""
+
+import copy
+from typing import Any, Dict, List, Optional
+
+import torch
+import torch.nn as nn
+
+from ..ops import lm
+from ..ops.lm import pad32
+from . import register_arch, register_token_batch_arch
+from .mixers import GatedMlp, LatentAttention, RgLru, _fill, _param, linear
+
+
+class BimipelConfig:
+    """``layers``: list of {"type", "mixer", "mlp"} as in config.json."""
+
+    def __init__(self, raw: Dict[str, Any]):
+        self.raw = copy.deepcopy(raw)
+        self.vocab_size = int(raw["vocab"])
+        self.hidden = int(raw["width"])
+        self.eps = float(raw["norm"]["eps"])
+        self.logit_scale = float(raw["logit_scale"])
+        self.layers = self.raw["layers"]
+        for n, layer in enumerate(self.layers):
+            src = layer["mixer"].get("kv_from")
+            if src is None:
+                continue
+            other = self.layers[src] if 0 <= src < n else None
+            if (other is None or other["type"] != "latent_attention"
+                    or other["mixer"].get("kv_from") is not None):
+                raise ValueError(
+                    "layer {}: kv_from {} is not an earlier attention layer "
+                    "with a latent of its own".format(n, src))
+            for key in ("kv_rank", "rot_dim", "rot"):
+                if layer["mixer"][key] != other["mixer"][key]:
+                    raise ValueError(
+                        "layer {}: {} differs from layer {}, whose latent it "
+                        "uses".format(n, key, src))
+
+
+class BimipelLayer(nn.Module):
+    def __init__(self, cfg: BimipelConfig, index: int):
+        super().__init__()
+        spec = cfg.layers[index]
+        m = spec["mixer"]
+        self.width, self.eps = cfg.hidden, cfg.eps
+        if spec["type"] == "latent_attention":
+            self.kv_from = m.get("kv_from")
+            self.mix = LatentAttention(
+                cfg.hidden, int(m["heads"]), int(m["dim"]),
+                int(m["rot_dim"]), int(m["vdim"]), int(m["kv_rank"]),
+                float(m["scale"]), int(m["mask"]["size"]),
+                float(m["rot"]["base"]), int(m["rot"]["dims"]), cfg.eps,
+                owns_kv=self.kv_from is None)
+        elif spec["type"] == "rglru":
+            self.kv_from = None
+            self.mix = RgLru(cfg.hidden, int(m["width"]), int(m["blocks"]),
+                             int(m["conv"]))
+        else:
+            raise ValueError("layer {}: unknown mixer '{}'".format(
+                index, spec["type"]))
+        wp = pad32(cfg.hidden)
+        self.norm1 = _param(wp)
+        self.mlp: Optional[GatedMlp] = None
+        mlp = spec.get("mlp")
+        if mlp is not None:
+            if mlp["kind"] != "dense":
+                raise ValueError("layer {}: unknown mlp kind '{}'".format(
+                    index, mlp["kind"]))
+            self.mlp = GatedMlp(cfg.hidden, int(mlp["ff"]))
+            self.norm2 = _param(wp)
+
+    def parts(self):
+        """(prefix, module) of what a checkpoint holds for this layer"""
+        yield "mix.", self.mix
+        if self.mlp is not None:
+            yield "mlp.", self.mlp
+
+    def forward(self, x, h, batch, cache):
+        h = lm.post_norm_add(self.mix(h, batch, cache), None, self.norm1, x,
+                             self.width, self.eps)
+        if self.mlp is not None:
+            h = lm.post_norm_add(self.mlp(h), self.mlp.down_b, self.norm2, x,
+                                 self.width, self.eps)
+        return h
+
+
+class BimipelForCausalLM(nn.Module):
+    # one forward for prompt portions and single tokens together
+    token_batch = True
+    supports_float32 = True
+    tp_size = 1
+
+    def __init__(self, cfg: BimipelConfig):
+        super().__init__()
+        self.cfg = cfg
+        wp = pad32(cfg.hidden)
+        self.embed = _param(pad32(cfg.vocab_size), wp)
+        self.layers = nn.ModuleList(
+            [BimipelLayer(cfg, i) for i in range(len(cfg.layers))])
+        self.final_norm = _param(wp)
+
+    # ---- weights ---------------------------------------------------- #
+    def checkpoint_shapes(self) -> Dict[str, tuple]:
+        c = self.cfg
+        out = {"embed": (c.vocab_size, c.hidden), "final.norm": (c.hidden,)}
+        for i, layer in enumerate(self.layers):
+            p = "l{}.".format(i)
+            out[p + "norm1"] = (c.hidden,)
+            if layer.mlp is not None:
+                out[p + "norm2"] = (c.hidden,)
+            for q, mod in layer.parts():
+                for k, s in mod.shapes().items():
+                    out[p + q + k] = s
+        return out
+
+    def load_checkpoint(self, state: Dict[str, torch.Tensor]) -> None:
+        want = self.checkpoint_shapes()
+        missing = sorted(set(want) - set(state))
+        extra = sorted(set(state) - set(want))
+        if missing or extra:
+            raise ValueError("checkpoint does not fit the configuration: "
+                             "missing {}, unexpected {}".format(
+                                 missing[:8], extra[:8]))
+        for k, s in want.items():
+            if tuple(state[k].shape) != tuple(s):
+                raise ValueError("checkpoint tensor '{}' is {}, expected {}"
+                                 .format(k, tuple(state[k].shape), s))
+        _fill(self.embed.data, state["embed"])
+        _fill(self.final_norm.data, state["final.norm"])
+        for i, layer in enumerate(self.layers):
+            p = "l{}.".format(i)
+            _fill(layer.norm1.data, state[p + "norm1"])
+            if layer.mlp is not None:
+                _fill(layer.norm2.data, state[p + "norm2"])
+            for q, mod in layer.parts():
+                mod.pack(lambda name, q=p + q: state[q + name])
+
+    def init_random(self, seed: int = 1234) -> None:
+        self.load_checkpoint(random_checkpoint(self, seed))
+
+    def finalize(self) -> None:
+        """call once weights, device and type are settled"""
+        for layer in self.layers:
+            layer.mix.finalize()
+
+    # ---- what the engine needs to know ------------------------------ #
+    def cache_layout(self) -> List[tuple]:
+        """per layer: ("paged", elements per token), ("state", channels,
+        taps) or ("shared", layer)"""
+        out: List[tuple] = []
+        for layer in self.layers:
+            if isinstance(layer.mix, RgLru):
+                out.append(("state", layer.mix.wp, layer.mix.taps))
+            elif layer.kv_from is not None:
+                out.append(("shared", layer.kv_from))
+            else:
+                out.append(("paged", layer.mix.row))
+        return out
+
+    def batch_params(self, dtype: torch.dtype) -> Dict[str, Any]:
+        """how a TokenBatch for this model is to be cut"""
+        attn = [m.mix for m in self.layers
+                if isinstance(m.mix, LatentAttention)]
+        rec = [m.mix for m in self.layers if isinstance(m.mix, RgLru)]
+        # the recurrence's tile of one block's channels must fit LDS
+        wide = max([m.bp for m in rec], default=32)
+        tile = 64 if 64 * (wide + 8) * dtype.itemsize <= 160 * 1024 else 16
+        return {"tile": tile, "absorb_max": None,
+                "windows": sorted({m.window for m in attn})}
+
+    # ---- forward ---------------------------------------------------- #
+    def forward(self, tokens, positions, kv_caches, attn_ctx,
+                last_token_idx=None, return_hidden=False,
+                gather_logits=True):
+        """attn_ctx: TokenBatch; logits [rows, vocab] at last_token_idx
+        (int32; None: every token)"""
+        x, h = lm.embed_stream(tokens, self.embed)
+        for layer, cache in zip(self.layers, kv_caches):
+            h = layer(x, h, attn_ctx, cache)
+        c = self.cfg
+        out = lm.output_norm(x, last_token_idx, self.final_norm, c.hidden,
+                             c.eps, 1.0 if return_hidden else c.logit_scale)
+        if return_hidden:
+            return out[:, :c.hidden]
+        logits = linear(out, self.embed)
+        if logits.shape[1] != c.vocab_size:
+            logits = logits[:, :c.vocab_size].contiguous()
+        return logits
+
+
+def random_checkpoint(model: BimipelForCausalLM, seed: int
+                      ) -> Dict[str, torch.Tensor]:
+    """seeded weights in checkpoint layout, scaled like a fresh model's"""
+    gen = torch.Generator().manual_seed(seed)
+    out = {}
+    for name, shape in model.checkpoint_shapes().items():
+        w = torch.empty(shape, dtype=torch.float32)
+        if name.endswith("lam"):
+            w.uniform_(-4.0, 1.0, generator=gen)
+        elif name.endswith("dkv.norm"):
+            w.fill_(1.0)
+        elif len(shape) == 1:
+            w.normal_(std=0.02, generator=gen)
+        else:
+            w.normal_(std=shape[-1] ** -0.5, generator=gen)
+        out[name] = w.to(torch.bfloat16)
+    return out
+
+
+def _attn(heads, dim, rot, vdim, rank, window, base=10000.0, kv_from=None):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim,
+         "kv_rank": rank, "scale": (dim + rot) ** -0.5,
+         "mask": {"size": window}, "rot": {"base": base, "dims": rot}}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return m
+
+
+def _stack(vocab, width, ff, mixers) -> Dict[str, Any]:
+    return {"architecture": "Bimipel", "vocab": vocab, "width": width,
+            "norm": {"eps": 1e-6}, "logit_scale": 1.0,
+            "layers": [{"type": t, "mixer": m,
+                        "mlp": None if t == "rglru" and not f else
+                        {"kind": "dense", "ff": ff}}
+                       for t, m, f in mixers]}
+
+
+def _griffin_like(vocab, width, ff, heads, dim, rot, rank, channels, blocks,
+                  window, periods) -> Dict[str, Any]:
+    rec = {"width": channels, "blocks": blocks, "conv": 4}
+    mixers: List[tuple] = []
+    for p in range(periods):
+        src = len(mixers) - 3 if p % 2 else None  # every other pair shares
+        mixers.append(("latent_attention",
+                       _attn(heads, dim, rot, dim, rank, window,
+                             kv_from=src), True))
+        mixers.append(("rglru", dict(rec), True))
+        mixers.append(("rglru", dict(rec), True))
+    return _stack(vocab, width, ff, mixers)
+
+
+PRESETS = {
+    "bimipel-tiny": _stack(512, 96, 160, [
+        ("latent_attention", _attn(3, 32, 16, 24, 40, 24), True),
+        ("rglru", {"width": 144, "blocks": 3, "conv": 3}, False),
+        ("latent_attention", _attn(2, 24, 16, 40, 40, 9, kv_from=0), True),
+    ]),
+    # llama-3-1b's width, depth class and vocabulary
+    "bimipel-1b": _griffin_like(128256, 2048, 6144, 16, 96, 32, 384, 2560,
+                                20, 1024, 6),
+    "bimipel-300m": _griffin_like(32000, 1024, 3072, 8, 96, 32, 256, 1280,
+                                  10, 512, 4),
+}
+
+
+def _build(config: Optional[Dict[str, Any]] = None,
+           preset: str = "bimipel-tiny",
+           overrides: Optional[Dict[str, Any]] = None) -> BimipelForCausalLM:
+    raw = dict(config if config is not None else PRESETS[preset])
+    raw.update(overrides or {})
+    return BimipelForCausalLM(BimipelConfig(raw))
+
+
+register_token_batch_arch("bimipel", _build, architecture="Bimipel")
+
+
+@register_arch("bimipel")
+def bimipel(preset: str = "bimipel-tiny", config=None,
+            **overrides) -> BimipelForCausalLM:
+    return _build(config, preset, overrides)

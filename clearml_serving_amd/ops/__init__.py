@@ -3,7 +3,8 @@
 The compute tier the reference outsources to Triton/vLLM
 lives here as hand-written gfx950 kernels (``csrc/*.hip``), compiled in-tree
 to ``_hip_ops.so`` by ``__graft_entry__.build()`` (hipcc --offload-arch=gfx950
-via torch.utils.cpp_extension).
+via torch.utils.cpp_extension). The kernels of token-batch models (``ops.lm``,
+``csrc/lm``) are a library of their own, ``_hip_lm.so``.
 
 Dispatch policy:
 - tensor on GPU  -> the HIP extension is REQUIRED; a missing .so raises
@@ -26,25 +27,39 @@ import torch
 
 _ext = None
 _ext_error: Optional[str] = None
+_lm_ext = None
+_lm_ext_error: Optional[str] = None
 _FORCE_EAGER = os.environ.get("CLEARML_SERVING_AMD_FORCE_EAGER") == "1"
 
 
-def _try_load_ext() -> None:
-    global _ext, _ext_error
-    if _ext is not None or _ext_error is not None:
-        return
-    so_path = os.path.join(os.path.dirname(__file__), "_hip_ops.so")
+def _load_so(name: str):
+    """-> (module, None) or (None, reason)"""
+    so_path = os.path.join(os.path.dirname(__file__), name + ".so")
     if not os.path.exists(so_path):
-        _ext_error = "extension not built ({} missing)".format(so_path)
-        return
+        return None, "extension not built ({} missing)".format(so_path)
     try:
-        loader = importlib.machinery.ExtensionFileLoader("_hip_ops", so_path)
-        spec = importlib.util.spec_from_loader("_hip_ops", loader)
+        loader = importlib.machinery.ExtensionFileLoader(name, so_path)
+        spec = importlib.util.spec_from_loader(name, loader)
         mod = importlib.util.module_from_spec(spec)
         loader.exec_module(mod)
-        _ext = mod
+        return mod, None
     except Exception as ex:  # loud, but deferred to first GPU use
-        _ext_error = "failed loading {}: {}".format(so_path, ex)
+        return None, "failed loading {}: {}".format(so_path, ex)
+
+
+def _try_load_ext() -> None:
+    global _ext, _ext_error, _lm_ext, _lm_ext_error
+    if _ext is None and _ext_error is None:
+        _ext, _ext_error = _load_so("_hip_ops")
+    if _lm_ext is None and _lm_ext_error is None:
+        _lm_ext, _lm_ext_error = _load_so("_hip_lm")
+
+
+def reload_extensions() -> None:
+    """Look again for libraries that were built after the first import."""
+    global _ext_error, _lm_ext_error
+    _ext_error = _lm_ext_error = None
+    _try_load_ext()
 
 
 _try_load_ext()
@@ -54,16 +69,32 @@ def has_extension() -> bool:
     return _ext is not None
 
 
+def has_lm_extension() -> bool:
+    return _lm_ext is not None
+
+
 def _require_ext(opname: str):
     if _FORCE_EAGER:
         return None
     if _ext is None:
+        if hasattr(_lm_ext, opname):  # ops that both libraries carry
+            return _lm_ext
         raise RuntimeError(
             "clearml_serving_amd HIP extension required for GPU op '{}' but "
             "not loaded: {}. Build it with __graft_entry__.build() "
             "(hipcc --offload-arch=gfx950).".format(opname, _ext_error)
         )
     return _ext
+
+
+def require_lm_ext(opname: str):
+    """The token-batch kernel library; there is no eager path on the GPU."""
+    if _lm_ext is None:
+        raise RuntimeError(
+            "clearml_serving_amd token-batch HIP library required for GPU op "
+            "'{}' but not loaded: {}. Build it with __graft_entry__.build() "
+            "(hipcc --offload-arch=gfx950).".format(opname, _lm_ext_error))
+    return _lm_ext
 
 
 def extension_or_none():

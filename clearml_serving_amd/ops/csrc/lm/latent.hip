@@ -1,0 +1,491 @@
+// Latent attention: one cached latent c (plus one rotated key part) per
+// token, shared by all heads.
+//
+// Cache row = [c, padded to CP | rotated key part, padded to RP], in pages of
+// block_size rows. Two ways to attend to it:
+//
+// - absorbed (few queries per sequence): q' = [W_uk^T q | q_rot] per head, so
+//   every head scores against the cache row itself and sums rows of c; W_uv
+//   follows. Reads each cached row once for all heads of a workgroup.
+// - expanded (prompts): keys and values are rebuilt per head from the rows a
+//   portion can see, then ordinary flash attention runs on them; several
+//   times fewer multiply-adds when kv_rank exceeds the head size.
+//
+// Both take a sliding window and a per-head sink (a term exp(sink) in the
+// softmax denominator that has no key).
+#include "lm_common.h"
+
+namespace {
+
+constexpr float LOG2E = 1.4426950408889634f;
+
+// ------------------------------------------------------------------- //
+// prepare: rotate q, normalise the latent, rotate the shared key part,
+// write the cache row
+// ------------------------------------------------------------------- //
+// u at an even index, v behind it: (u cos - v sin, v cos + u sin)
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(
+    T* __restrict__ qkv, int ld, const int* __restrict__ positions,
+    const int* __restrict__ slots, const float* __restrict__ inv_freq,
+    int n_rot, int heads, int DP, int RP, int CP, int kv_rank, float eps,
+    const T* __restrict__ kv_norm,  // null: the layer owns no latent
+    T* __restrict__ cache, long n_slots, T* __restrict__ q_abs, int n_abs) {
+  __shared__ float cs[256], sn[256];
+  __shared__ float tmp[16];
+  const int t = blockIdx.x;
+  const int tid = threadIdx.x;
+  const int pairs = n_rot / 2;
+  const float pos = (float)positions[t];
+  for (int i = tid; i < pairs; i += 256) {
+    float s, c;
+    sincosf(pos * inv_freq[i], &s, &c);
+    cs[i] = c;
+    sn[i] = s;
+  }
+  __syncthreads();
+  T* row = qkv + (long)t * ld;
+  const int hp = RP / 2;
+  const bool absorbed = t < n_abs;
+  const int q_pairs = absorbed ? hp : pairs;  // the rest passes unchanged
+  for (int i = tid; i < heads * q_pairs; i += 256) {
+    const int hd = i / q_pairs, p = i % q_pairs;
+    T* src = row + hd * (DP + RP) + DP + 2 * p;
+    float u = to_f32(src[0]), v = to_f32(src[1]);
+    if (p < pairs) {
+      const float a = u * cs[p] - v * sn[p];
+      v = v * cs[p] + u * sn[p];
+      u = a;
+    }
+    T* dst = absorbed
+                 ? q_abs + ((long)t * heads + hd) * (CP + RP) + CP + 2 * p
+                 : src;
+    dst[0] = from_f32<T>(u);
+    dst[1] = from_f32<T>(v);
+  }
+  if (!kv_norm) return;
+  const T* lat = row + heads * (DP + RP);
+  float ss = 0.f;
+  for (int c = tid * 8; c < CP; c += 256 * 8) {
+    float f[8];
+    load8<T>(lat + c, f);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
+  }
+  ss = block_reduce(ss, tmp, SumOp{}, 0.f);
+  const long slot = slots[t];
+  if (slot < 0 || slot >= n_slots) return;
+  const float inv = 1.f / sqrtf(ss / (float)kv_rank + eps);
+  T* dst = cache + slot * (CP + RP);
+  for (int c = tid * 8; c < CP; c += 256 * 8) {
+    float f[8], g[8];
+    load8<T>(lat + c, f);
+    load8<T>(kv_norm + c, g);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] = f[e] * inv * g[e];
+    store8(dst + c, f);
+  }
+  for (int p = tid; p < hp; p += 256) {
+    float u = to_f32(lat[CP + 2 * p]), v = to_f32(lat[CP + 2 * p + 1]);
+    if (p < pairs) {
+      const float a = u * cs[p] - v * sn[p];
+      v = v * cs[p] + u * sn[p];
+      u = a;
+    }
+    dst[CP + 2 * p] = from_f32<T>(u);
+    dst[CP + 2 * p + 1] = from_f32<T>(v);
+  }
+}
+
+// ------------------------------------------------------------------- //
+// per-head product: out[t, h, :N] = a[t, h, :K] @ w[h]^T   (w [H, N, K])
+// one wave per 16 x 16 output tile; operands straight from L2/HBM
+// ------------------------------------------------------------------- //
+template <typename T>
+__global__ __launch_bounds__(256) void head_gemm_kernel(
+    const T* __restrict__ a, long a_t, long a_h, const T* __restrict__ w,
+    T* __restrict__ out, long o_t, long o_h, int M, int N, int K) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int n0 = (blockIdx.x * 4 + wave) * 16;
+  const int h = blockIdx.y;
+  const int m0 = blockIdx.z * 16;
+  if (n0 >= N) return;
+  const int r16 = lane & 15, ko = (lane >> 4) * 8;
+  const T* wr = w + ((long)h * N + n0 + r16) * K + ko;
+  const T* ar = a + (long)min(m0 + r16, M - 1) * a_t + (long)h * a_h + ko;
+  lm_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k = 0; k < K; k += 32)
+    acc = mma32(load_frag(wr + k), load_frag(ar + k), acc);
+  // C: row (n) = 4 * (lane >> 4) + r, column (token) = lane & 15
+  const int m = m0 + r16;
+  if (m < M) {
+    const float f[4] = {acc[0], acc[1], acc[2], acc[3]};
+    store4(out + (long)m * o_t + (long)h * o_h + n0 + 4 * (lane >> 4), f);
+  }
+}
+
+// ------------------------------------------------------------------- //
+// absorbed attention: one token x 16 heads x one key range per workgroup
+// ------------------------------------------------------------------- //
+// Four waves share a tile of KT cached rows in LDS: they split the keys for
+// the scores and the latent columns for the weighted sum. NT: 16-column
+// tiles of the latent per wave (4 * NT * 16 columns per workgroup).
+template <typename T, int KT, int NT>
+__global__ __launch_bounds__(256) void latent_attn_kernel(
+    const T* __restrict__ q_abs,  // [n, H, CP+RP]
+    const T* __restrict__ cache, const int* __restrict__ block_table,
+    const int* __restrict__ tok_seq, const int* __restrict__ positions,
+    const T* __restrict__ sink, T* __restrict__ out,  // [n, H, CP]
+    float* __restrict__ part_o, float* __restrict__ part_ml, int splits,
+    int col_groups, int H, int CP, int RP, int block_size, int max_blocks,
+    int n_blocks, int window, float scale) {
+  constexpr int SUB = KT / 16;             // 16-key subtiles
+  constexpr int SPW = (SUB + 3) / 4;       // subtiles per wave
+  constexpr int PP = KT + 8;               // pitch of the weights
+  const int ROW = CP + RP, PITCH = ROW + 8;
+  extern __shared__ __align__(16) char smem[];
+  T* tile = (T*)smem;                      // [KT][PITCH]
+  T* qs = tile + KT * PITCH;               // [16][PITCH]
+  T* ps = qs + 16 * PITCH;                 // [16][PP]
+  float* wred = (float*)(ps + 16 * PP);    // [4][16]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int r16 = lane & 15, g = lane >> 4, ko = g * 8;
+  const int t = blockIdx.x;
+  const int h0 = blockIdx.y * 16;
+  const int split = blockIdx.z / col_groups;
+  const int c_base = (blockIdx.z % col_groups) * (NT * 64);
+  const float scale2 = scale * LOG2E;
+
+  const int pos = positions[t];
+  const int* btab = block_table + (long)tok_seq[t] * max_blocks;
+  const int lo_all = window > 0 ? max(0, pos - window + 1) : 0;
+  const int n_keys = pos + 1 - lo_all;
+  const int chunk = ((n_keys + splits - 1) / splits + KT - 1) / KT * KT;
+  const int lo = lo_all + split * chunk;
+  const int hi = min(pos + 1, lo + chunk);
+
+  const int row8 = ROW / 8;
+  for (int i = tid; i < 16 * row8; i += 256) {
+    const int r = i / row8, c = (i % row8) * 8;
+    if (h0 + r < H) copy8(qs + r * PITCH + c,
+                          q_abs + ((long)t * H + h0 + r) * ROW + c);
+    else zero8(qs + r * PITCH + c);
+  }
+
+  float m_run = -INFINITY, l_run = 0.f;  // head r16; l over this wave's keys
+  lm_f32x4 acc[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) acc[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
+
+  for (int n0 = lo; n0 < hi; n0 += KT) {
+    __syncthreads();  // the tile and the weights are free again
+    for (int i = tid; i < KT * row8; i += 256) {
+      const int r = i / row8, c = (i % row8) * 8;
+      const int key = n0 + r;
+      if (key < hi) {
+        const int blk = min(max(btab[key / block_size], 0), n_blocks - 1);
+        copy8(tile + r * PITCH + c,
+              cache + ((long)blk * block_size + key % block_size) * ROW + c);
+      } else {
+        zero8(tile + r * PITCH + c);
+      }
+    }
+    __syncthreads();
+    // scores^T: rows = keys, column = head
+    lm_f32x4 s[SPW];
+    float mx = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < SPW; ++i) {
+      s[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
+      const int sub = wave + 4 * i;
+      if (sub < SUB) {
+#pragma unroll 4
+        for (int k = 0; k < ROW; k += 32)
+          s[i] = mma32(load_frag(tile + (sub * 16 + r16) * PITCH + k + ko),
+                       load_frag(qs + r16 * PITCH + k + ko), s[i]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int key = n0 + sub * 16 + 4 * g + r;
+          s[i][r] = key < hi ? s[i][r] * scale2 : -INFINITY;
+          mx = fmaxf(mx, s[i][r]);
+        }
+      }
+    }
+    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    if (g == 0) wred[wave * 16 + r16] = mx;
+    __syncthreads();
+    float m_new = m_run;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) m_new = fmaxf(m_new, wred[w * 16 + r16]);
+    const float alpha = exp2f(m_run - m_new);  // m_new is finite: hi > n0
+    m_run = m_new;
+    l_run *= alpha;
+#pragma unroll
+    for (int i = 0; i < SPW; ++i) {
+      const int sub = wave + 4 * i;
+      if (sub < SUB) {
+        float p[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          p[r] = exp2f(s[i][r] - m_new);
+          l_run += p[r];
+        }
+        store4(ps + r16 * PP + sub * 16 + 4 * g, p);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < NT; ++i) acc[i] *= alpha;
+    __syncthreads();
+    // o^T[c][head] += c^T p^T
+#pragma unroll
+    for (int kc = 0; kc < KT; kc += 32) {
+      const Frag<T> pf = load_frag(ps + r16 * PP + kc + ko);
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        const int c0 = c_base + (wave * NT + i) * 16;
+        if (c0 < CP)
+          acc[i] = mma32(load_frag_col(tile + (kc + ko) * PITCH + c0 + r16,
+                                       PITCH), pf, acc[i]);
+      }
+    }
+  }
+  // denominator over the four waves
+  l_run += __shfl_xor(l_run, 16, 64);
+  l_run += __shfl_xor(l_run, 32, 64);
+  __syncthreads();
+  if (g == 0) wred[wave * 16 + r16] = l_run;
+  __syncthreads();
+  float l = 0.f;
+#pragma unroll
+  for (int w = 0; w < 4; ++w) l += wred[w * 16 + r16];
+  const int h = h0 + r16;
+  if (h >= H) return;
+  if (splits > 1) {
+    const long pi = ((long)t * H + h) * splits + split;
+    if (wave == 0 && g == 0 && c_base == 0) {
+      part_ml[2 * pi] = m_run;
+      part_ml[2 * pi + 1] = l;
+    }
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const int c0 = c_base + (wave * NT + i) * 16;
+      const float f[4] = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+      if (c0 < CP) store4(part_o + pi * CP + c0 + 4 * g, f);
+    }
+    return;
+  }
+  const float sk = to_f32(sink[h]) * LOG2E;
+  const float m_f = fmaxf(m_run, sk);
+  const float e = exp2f(m_run - m_f);
+  const float inv = e / (l * e + exp2f(sk - m_f));
+#pragma unroll
+  for (int i = 0; i < NT; ++i) {
+    const int c0 = c_base + (wave * NT + i) * 16;
+    const float f[4] = {acc[i][0] * inv, acc[i][1] * inv, acc[i][2] * inv,
+                        acc[i][3] * inv};
+    if (c0 < CP) store4(out + ((long)t * H + h) * CP + c0 + 4 * g, f);
+  }
+}
+
+// merge key ranges; a range without keys has m = -inf
+template <typename T>
+__global__ __launch_bounds__(64) void latent_combine_kernel(
+    const float* __restrict__ part_o, const float* __restrict__ part_ml,
+    const T* __restrict__ sink, T* __restrict__ out, int splits, int H,
+    int CP) {
+  const long th = blockIdx.x;
+  const float sk = to_f32(sink[th % H]) * LOG2E;
+  float m = sk;
+  for (int s = 0; s < splits; ++s)
+    m = fmaxf(m, part_ml[(th * splits + s) * 2]);
+  float l = exp2f(sk - m);
+  for (int s = 0; s < splits; ++s)
+    l += part_ml[(th * splits + s) * 2 + 1] *
+         exp2f(part_ml[(th * splits + s) * 2] - m);
+  const float inv = 1.f / l;
+  for (int c = threadIdx.x * 4; c < CP; c += 64 * 4) {
+    float f[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < splits; ++s) {
+      const float ms = part_ml[(th * splits + s) * 2];
+      if (ms == -INFINITY) continue;
+      const float e = exp2f(ms - m) * inv;
+      const lm_f32x4 o = *reinterpret_cast<const lm_f32x4*>(
+          part_o + (th * splits + s) * CP + c);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) f[r] += o[r] * e;
+    }
+    store4(out + th * CP + c, f);
+  }
+}
+
+}  // namespace
+
+void lm_latent_prep(torch::Tensor qkv, torch::Tensor positions,
+                    torch::Tensor slots, torch::Tensor inv_freq, long heads,
+                    long DP, long RP, long CP, long kv_rank, double eps,
+                    c10::optional<torch::Tensor> kv_norm,
+                    c10::optional<torch::Tensor> cache,
+                    c10::optional<torch::Tensor> q_abs, long n_abs) {
+  LM_CHECK_CONTIG(qkv);
+  LM_CHECK_I32(positions);
+  LM_CHECK_I32(slots);
+  LM_CHECK_CONTIG(inv_freq);
+  TORCH_CHECK(inv_freq.scalar_type() == at::kFloat);
+  const int T = qkv.size(0), ld = qkv.size(1);
+  const int pairs = inv_freq.numel();
+  const bool own = kv_norm.has_value();
+  TORCH_CHECK(DP % 32 == 0 && RP % 32 == 0 && CP % 32 == 0);
+  TORCH_CHECK(2 * pairs <= RP && pairs <= 256, "rotated size too large");
+  TORCH_CHECK(ld == heads * (DP + RP) + (own ? CP + RP : 0));
+  TORCH_CHECK(positions.numel() == T && slots.numel() == T);
+  TORCH_CHECK(n_abs >= 0 && n_abs <= T);
+  if (n_abs > 0) {
+    TORCH_CHECK(q_abs.has_value());
+    LM_CHECK_CONTIG(*q_abs);
+    TORCH_CHECK(q_abs->numel() == n_abs * heads * (CP + RP) &&
+                q_abs->scalar_type() == qkv.scalar_type());
+  }
+  long n_slots = 0;
+  if (own) {
+    TORCH_CHECK(cache.has_value());
+    LM_CHECK_CONTIG(*cache);
+    TORCH_CHECK(cache->dim() == 3 && cache->size(2) == CP + RP &&
+                cache->scalar_type() == qkv.scalar_type());
+    TORCH_CHECK(kv_norm->is_contiguous() && kv_norm->numel() == CP &&
+                kv_norm->scalar_type() == qkv.scalar_type());
+    n_slots = (long)cache->size(0) * cache->size(1);
+  }
+  if (T == 0) return;
+  LM_DISPATCH(qkv, "lm_latent_prep", [&] {
+    hipLaunchKernelGGL(
+        (latent_prep_kernel<scalar_t>), dim3(T), dim3(256), 0,
+        cmls::current_stream(), (scalar_t*)qkv.data_ptr(), ld,
+        positions.data_ptr<int>(), slots.data_ptr<int>(),
+        inv_freq.data_ptr<float>(), 2 * pairs, (int)heads, (int)DP, (int)RP,
+        (int)CP, (int)kv_rank, (float)eps,
+        own ? (const scalar_t*)kv_norm->data_ptr() : nullptr,
+        own ? (scalar_t*)cache->data_ptr() : nullptr, n_slots,
+        n_abs > 0 ? (scalar_t*)q_abs->data_ptr() : nullptr, (int)n_abs);
+  });
+  LM_LAUNCHED();
+}
+
+void lm_head_gemm(torch::Tensor a, torch::Tensor w, torch::Tensor out) {
+  LM_CHECK_CUDA(a);
+  LM_CHECK_CUDA(out);
+  LM_CHECK_CONTIG(w);
+  TORCH_CHECK(a.dim() == 3 && w.dim() == 3 && out.dim() == 3);
+  const int M = a.size(0), H = a.size(1), K = a.size(2), N = w.size(1);
+  TORCH_CHECK(w.size(0) == H && w.size(2) == K);
+  TORCH_CHECK(out.size(0) == M && out.size(1) == H && out.size(2) == N);
+  TORCH_CHECK(a.stride(2) == 1 && out.stride(2) == 1);
+  TORCH_CHECK(K % 32 == 0 && N % 16 == 0, "lm_head_gemm: K % 32, N % 16");
+  TORCH_CHECK(a.stride(0) % 8 == 0 && a.stride(1) % 8 == 0 &&
+              out.stride(0) % 4 == 0 && out.stride(1) % 4 == 0 &&
+              a.storage_offset() % 8 == 0 && out.storage_offset() % 4 == 0);
+  TORCH_CHECK(a.scalar_type() == w.scalar_type() &&
+              out.scalar_type() == w.scalar_type());
+  if (M == 0) return;
+  TORCH_CHECK((M + 15) / 16 <= 65535 && H <= 65535);
+  LM_DISPATCH(w, "lm_head_gemm", [&] {
+    hipLaunchKernelGGL((head_gemm_kernel<scalar_t>),
+                       dim3((N + 63) / 64, H, (M + 15) / 16), dim3(256), 0,
+                       cmls::current_stream(),
+                       (const scalar_t*)a.data_ptr(), a.stride(0),
+                       a.stride(1), (const scalar_t*)w.data_ptr(),
+                       (scalar_t*)out.data_ptr(), out.stride(0),
+                       out.stride(1), M, N, K);
+  });
+  LM_LAUNCHED();
+}
+
+torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
+                                  torch::Tensor block_table,
+                                  torch::Tensor tok_seq,
+                                  torch::Tensor positions,
+                                  torch::Tensor sink, double scale,
+                                  long window, long CP, long max_keys) {
+  LM_CHECK_CONTIG(q_abs);
+  LM_CHECK_CONTIG(cache);
+  LM_CHECK_I32(block_table);
+  LM_CHECK_I32(tok_seq);
+  LM_CHECK_I32(positions);
+  LM_CHECK_CONTIG(sink);
+  TORCH_CHECK(q_abs.dim() == 3 && cache.dim() == 3 && block_table.dim() == 2);
+  const int n = q_abs.size(0), H = q_abs.size(1), ROW = q_abs.size(2);
+  TORCH_CHECK(cache.size(2) == ROW && CP % 32 == 0 && ROW % 32 == 0 &&
+              CP > 0 && CP < ROW);
+  TORCH_CHECK(tok_seq.numel() >= n && positions.numel() >= n);
+  TORCH_CHECK(sink.numel() == H && sink.scalar_type() == q_abs.scalar_type()
+              && cache.scalar_type() == q_abs.scalar_type());
+  auto out = torch::empty({n, H, CP}, q_abs.options());
+  if (n == 0) return out;
+  const int hg = (H + 15) / 16;
+  const int tiles = (int)((CP + 63) / 64);      // 16-column tiles per wave
+  const int nt = tiles <= 1 ? 1 : tiles <= 2 ? 2 : tiles <= 4 ? 4 : 8;
+  const int cgroups = (tiles + nt - 1) / nt;
+  const int isz = q_abs.element_size();
+  auto lds = [&](int kt) {
+    return (long)((kt + 16) * (ROW + 8) + 16 * (kt + 8)) * isz + 256;
+  };
+  const bool big = isz == 2 && lds(64) <= 80 * 1024;
+  const int kt = big ? 64 : 32;
+  TORCH_CHECK(lds(kt) <= 160 * 1024, "lm_latent_attention: kv_rank + rot_dim ",
+              ROW, " does not fit LDS");
+  // enough workgroups for 256 CUs, at least two key tiles each
+  const long keys = window > 0 ? std::min(window, max_keys) : max_keys;
+  long splits = 512 / std::max<long>(1, (long)n * hg * cgroups);
+  splits = std::max<long>(1, std::min(splits, (keys + 2 * kt - 1) / (2 * kt)));
+  TORCH_CHECK(hg <= 65535 && splits * cgroups <= 65535);
+  torch::Tensor po, pml;
+  if (splits > 1) {
+    auto f32 = q_abs.options().dtype(at::kFloat);
+    po = torch::empty({n, H, splits, CP}, f32);
+    pml = torch::empty({n, H, splits, 2}, f32);
+  }
+  hipStream_t st = cmls::current_stream();
+#define LM_LA(KT, NT)                                                        \
+  do {                                                                       \
+    const int bytes = (int)lds(KT);                                          \
+    auto* fn = &latent_attn_kernel<scalar_t, KT, NT>;                        \
+    if (bytes > 64 * 1024)                                                   \
+      HIP_CHECK(hipFuncSetAttribute(                                         \
+          reinterpret_cast<const void*>(fn),                                 \
+          hipFuncAttributeMaxDynamicSharedMemorySize, bytes));               \
+    hipLaunchKernelGGL(fn, dim3(n, hg, splits * cgroups), dim3(256), bytes,  \
+                       st, (const scalar_t*)q_abs.data_ptr(),                \
+                       (const scalar_t*)cache.data_ptr(),                    \
+                       block_table.data_ptr<int>(), tok_seq.data_ptr<int>(), \
+                       positions.data_ptr<int>(),                            \
+                       (const scalar_t*)sink.data_ptr(),                     \
+                       (scalar_t*)out.data_ptr(),                            \
+                       splits > 1 ? po.data_ptr<float>() : nullptr,          \
+                       splits > 1 ? pml.data_ptr<float>() : nullptr,         \
+                       (int)splits, cgroups, H, (int)CP, (int)(ROW - CP),    \
+                       (int)cache.size(1), (int)block_table.size(1),         \
+                       (int)cache.size(0), (int)window, (float)scale);       \
+  } while (0)
+#define LM_LA_NT(KT)                                                         \
+  do {                                                                       \
+    if (nt == 1) LM_LA(KT, 1);                                               \
+    else if (nt == 2) LM_LA(KT, 2);                                          \
+    else if (nt == 4) LM_LA(KT, 4);                                          \
+    else LM_LA(KT, 8);                                                       \
+  } while (0)
+  LM_DISPATCH(q_abs, "lm_latent_attention", [&] {
+    if (kt == 64) LM_LA_NT(64);
+    else LM_LA_NT(32);
+    if (splits > 1)
+      hipLaunchKernelGGL((latent_combine_kernel<scalar_t>), dim3(n * H),
+                         dim3(64), 0, st, po.data_ptr<float>(),
+                         pml.data_ptr<float>(),
+                         (const scalar_t*)sink.data_ptr(),
+                         (scalar_t*)out.data_ptr(), (int)splits, H, (int)CP);
+  });
+#undef LM_LA_NT
+#undef LM_LA
+  LM_LAUNCHED();
+  return out;
+}
