@@ -1731,10 +1731,13 @@ class LlmEngine:
                     "slot_mapping": static["slots"]}
         if self.token_batch:
             static["state_slots"] = torch.full_like(static["slots"], -1)
+            # every tensor the graph reads must outlive it: kept in the entry
+            static["tok_seq"] = torch.arange(bucket, dtype=torch.int32,
+                                             device=dev)
             attn_ctx = TokenBatch.of_single_tokens(
                 static["positions"], static["slots"],
-                torch.arange(bucket, dtype=torch.int32, device=dev),
-                static["block_table"], static["state_slots"],
+                static["tok_seq"], static["block_table"],
+                static["state_slots"],
                 tile=self._batch_params["tile"],
                 max_keys=self.cfg.max_model_len)
 

@@ -139,7 +139,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
     const T* __restrict__ sink, T* __restrict__ out,  // [n, H, CP]
     float* __restrict__ part_o, float* __restrict__ part_ml, int splits,
     int col_groups, int H, int CP, int RP, int block_size, int max_blocks,
-    int n_blocks, int window, float scale) {
+    int n_blocks, int n_seqs, int window, float scale) {
   constexpr int SUB = KT / 16;             // 16-key subtiles
   constexpr int SPW = (SUB + 3) / 4;       // subtiles per wave
   constexpr int PP = KT + 8;               // pitch of the weights
@@ -157,8 +157,9 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
   const int c_base = (blockIdx.z % col_groups) * (NT * 64);
   const float scale2 = scale * LOG2E;
 
-  const int pos = positions[t];
-  const int* btab = block_table + (long)tok_seq[t] * max_blocks;
+  const int pos = min(max(positions[t], 0), max_blocks * block_size - 1);
+  const int* btab = block_table +
+                    (long)min(max(tok_seq[t], 0), n_seqs - 1) * max_blocks;
   const int lo_all = window > 0 ? max(0, pos - window + 1) : 0;
   const int n_keys = pos + 1 - lo_all;
   const int chunk = ((n_keys + splits - 1) / splits + KT - 1) / KT * KT;
@@ -418,6 +419,7 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
   TORCH_CHECK(cache.size(2) == ROW && CP % 32 == 0 && ROW % 32 == 0 &&
               CP > 0 && CP < ROW);
   TORCH_CHECK(tok_seq.numel() >= n && positions.numel() >= n);
+  TORCH_CHECK(n == 0 || block_table.numel() > 0);
   TORCH_CHECK(sink.numel() == H && sink.scalar_type() == q_abs.scalar_type()
               && cache.scalar_type() == q_abs.scalar_type());
   auto out = torch::empty({n, H, CP}, q_abs.options());
@@ -465,7 +467,8 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
                        splits > 1 ? pml.data_ptr<float>() : nullptr,         \
                        (int)splits, cgroups, H, (int)CP, (int)(ROW - CP),    \
                        (int)cache.size(1), (int)block_table.size(1),         \
-                       (int)cache.size(0), (int)window, (float)scale);       \
+                       (int)cache.size(0), (int)block_table.size(0),         \
+                       (int)window, (float)scale);                           \
   } while (0)
 #define LM_LA_NT(KT)                                                         \
   do {                                                                       \
