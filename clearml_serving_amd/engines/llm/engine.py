@@ -530,6 +530,7 @@ class LlmEngine:
         # decode hipGraphs: one per batch bucket, shared memory pool
         self._decode_graphs: Dict[int, Dict[str, Any]] = {}
         self._decode_pin: Dict[int, Dict[str, Any]] = {}
+        self._decode_pin_read: Dict[int, Any] = {}  # event: copies done
         self._graph_pool = None
         self._decode_buckets = [n for n in
                                 (1, 2, 4, 8, 16, 24, 32, 48, 64, 96, 128,
@@ -882,6 +883,7 @@ class LlmEngine:
         self.tp_shutdown()
         self._decode_graphs.clear()
         self._decode_pin.clear()
+        self._decode_pin_read.clear()
         self._graph_pool = None
         self.kv_caches = []
         self.model = None
@@ -1792,6 +1794,10 @@ class LlmEngine:
                 pin["state_slots"] = torch.full(
                     (bucket,), -1, dtype=torch.int32, pin_memory=True)
             self._decode_pin[bucket] = pin
+            self._decode_pin_read[bucket] = torch.cuda.Event()
+        # the previous step's copies read these buffers; a step whose logits
+        # nobody fetched has not been waited for
+        self._decode_pin_read[bucket].synchronize()
         pin["tokens"][:b] = torch.tensor(plan["tokens"], dtype=torch.long)
         pin["tokens"][b:] = 0
         pin["positions"][:b] = torch.tensor(plan["positions"],
@@ -1812,6 +1818,7 @@ class LlmEngine:
             pin["state_slots"][b:] = -1
         for k in pin:
             entry[k].copy_(pin[k], non_blocking=True)
+        self._decode_pin_read[bucket].record()
         entry["graph"].replay()
         self.stats["graph_replays"] += 1
         return entry["logits"][:b]

@@ -659,7 +659,7 @@ def skinny_linear(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
         m, k = x.shape
         n = weight.shape[0]
         if ((1 <= m <= 16 and n <= 8192 and k <= 8192)
-                or (m <= 2 and n <= 8192)):
+                or (1 <= m <= 2 and n <= 8192)):
             ext = _require_ext("skinny_gemm")
             if ext is not None:
                 return ext.skinny_gemm(x.contiguous(), weight, 1)
