@@ -12,6 +12,9 @@ requests through the full serving path (ModelRequestProcessor dispatch ->
 dynamic batcher -> hipGraph replay on the GPU) and awaits all responses.
 
   python bench.py --gpus N --steps K --warmup W
+
+``--workload lm`` measures another thing: prefill and decode of the Bimipel
+family beside llama at equal size (benchmarks/lm_bench.py).
 """
 
 import argparse
@@ -115,7 +118,24 @@ def main():
     ap.add_argument("--steps", type=int, default=1600)
     ap.add_argument("--warmup", type=int, default=50)
     ap.add_argument("--no-graphs", action="store_true")
+    ap.add_argument("--workload", default="serving",
+                    choices=("serving", "lm"),
+                    help="serving: the headline benchmark; lm: prefill and "
+                         "decode of the Bimipel family beside llama")
+    ap.add_argument("--lm-size", default="300m,1b,4k")
+    ap.add_argument("--lm-model", default="bimipel,llama")
+    ap.add_argument("--lm-prompt", type=int, default=2048)
+    ap.add_argument("--lm-batch", default="1,16,64")
+    ap.add_argument("--lm-phase", default="prefill,decode")
+    ap.add_argument("--lm-iters", type=int, default=20)
     args = ap.parse_args()
+    if args.workload == "lm":
+        from benchmarks.lm_bench import run
+
+        run(args.lm_size.split(","), args.lm_model.split(","),
+            args.lm_prompt, [int(b) for b in args.lm_batch.split(",")],
+            args.lm_iters, args.lm_phase.split(","))
+        return
 
     rank = int(os.environ.get("RANK", 0))
     world = int(os.environ.get("WORLD_SIZE", 1))

@@ -11,6 +11,8 @@ from typing import Any, Dict, List, Optional, Sequence as Seq
 import numpy as np
 import torch
 
+from ...ops.lm import PROMPT_TILE
+
 
 class TokenBatch:
     """Device-side description of a flat token batch.
@@ -21,7 +23,9 @@ class TokenBatch:
     n_single: leading entries of one token (token i is entry i);
     n_abs: leading tokens whose attention runs in absorbed form;
     tiles [n, 5], seqs [m, 6]: recurrence tiles of the other entries (see
-    ops.lm.rglru_prefill); max_keys: bound on position + 1 in the first n_abs
+    ops.lm.rglru_prefill); prompts: window -> (cache rows that the entries
+    behind the first n_abs tokens can see, query tiles into them; see
+    ops.lm.latent_prompt); max_keys: bound on position + 1 in the first n_abs
     tokens."""
 
     mode = "token_batch"
@@ -43,6 +47,9 @@ class TokenBatch:
         tiles: List[List[int]] = []
         seqs: List[List[int]] = []
         n_single = n_abs = max_keys = at = 0
+        gathered = {w: [] for w in windows}
+        qtiles: Dict[int, List[List[int]]] = {w: [] for w in windows}
+        n_rows = dict.fromkeys(windows, 0)
         mb = max(len(b) for b in plan["blocks"])
         btab = np.zeros((n, mb), dtype=np.int32)
         for row, i in enumerate(order):
@@ -68,6 +75,16 @@ class TokenBatch:
             if absorb_max is None or ln <= absorb_max:
                 n_abs = at
                 max_keys = max(max_keys, start + ln)
+                continue
+            for w in windows:
+                lo = max(0, start - w + 1) if w else 0
+                p = np.arange(lo, start + ln, dtype=np.int32)
+                gathered[w].append(blocks[p // block_size] * block_size
+                                   + p % block_size)
+                for j in range(0, ln, PROMPT_TILE):
+                    qtiles[w].append([first[i] + j, min(PROMPT_TILE, ln - j),
+                                      start + j, n_rows[w], lo, len(p)])
+                n_rows[w] += len(p)
         want = [first[i] + w for i in range(n) for w in plan["want"][i]]
         parts = {
             "positions": np.concatenate(pos),
@@ -80,11 +97,19 @@ class TokenBatch:
             "seqs": np.asarray(seqs, dtype=np.int32).reshape(-1, 6),
             "want": np.asarray(want, dtype=np.int32),
         }
+        for w in windows:
+            if qtiles[w]:
+                parts["rows", w] = np.concatenate(gathered[w])
+                # long-sighted tiles first
+                parts["qtiles", w] = np.asarray(
+                    sorted(qtiles[w], key=lambda q: -q[2]), dtype=np.int32)
         dev = to_device(parts, device)
         rows = dev.pop("want")
+        prompts = {w: (dev.pop(("rows", w)), dev.pop(("qtiles", w)))
+                   for w in windows if qtiles[w]}
         tokens = torch.from_numpy(np.concatenate(toks)).to(device)
         return tokens, cls(n_single=n_single, n_abs=n_abs, tile=tile,
-                           max_keys=max_keys, **dev), rows
+                           max_keys=max_keys, prompts=prompts, **dev), rows
 
     @classmethod
     def of_single_tokens(cls, positions, slot_mapping, tok_seq, block_table,
@@ -96,7 +121,7 @@ class TokenBatch:
                    tok_seq=tok_seq, block_table=block_table,
                    state_slots=state_slots, tiles=empty.view(0, 5),
                    seqs=empty.view(0, 6), n_single=n, n_abs=n, tile=tile,
-                   max_keys=max_keys)
+                   max_keys=max_keys, prompts={})
 
 
 def to_device(parts: Dict[str, np.ndarray], device) -> Dict[str, torch.Tensor]:

@@ -181,7 +181,10 @@ class BimipelForCausalLM(nn.Module):
         # the recurrence's tile of one block's channels must fit LDS
         wide = max([m.bp for m in rec], default=32)
         tile = 64 if 64 * (wide + 8) * dtype.itemsize <= 160 * 1024 else 16
-        return {"tile": tile, "absorb_max": None,
+        # few queries per sequence: absorbed attention; prompts: rebuilt keys
+        expand = (dtype == torch.bfloat16
+                  and all(m.can_expand() for m in attn))
+        return {"tile": tile, "absorb_max": 8 if expand else None,
                 "windows": sorted({m.window for m in attn})}
 
     # ---- forward ---------------------------------------------------- #

@@ -104,6 +104,15 @@ class LatentAttention(nn.Module):
         i = torch.arange(self.rot_dims // 2, dtype=torch.float64)
         self.inv_freq = (float(self.rot_base) ** (
             -2.0 * i / self.rot_dims)).to(torch.float32).to(dev)
+        # prompts rebuild keys and values: [H*dp | H*vp] rows
+        self.kv_up = torch.cat([
+            self.uk_t.data.transpose(1, 2).reshape(-1, self.cp),
+            self.uv.data.reshape(-1, self.cp)])
+
+    def can_expand(self) -> bool:
+        """whether ops.lm.latent_prompt takes this head size"""
+        return (self.dp + self.rp <= lm.PROMPT_MAX_HEAD
+                and self.vp <= lm.PROMPT_MAX_HEAD)
 
     def forward(self, h, batch, cache):
         t = h.shape[0]
@@ -123,6 +132,13 @@ class LatentAttention(nn.Module):
                 batch.positions, self.sink, self.scale, self.window, self.cp,
                 batch.max_keys)
             lm.head_gemm(lat, self.uv, ctx[:n])
+        if n < t:
+            kv_rows, qtiles = batch.prompts[self.window]
+            rows = lm.gather_rows(cache, kv_rows)
+            kv = linear(rows[:, :self.cp], self.kv_up)
+            lm.latent_prompt(qkv, kv, rows, self.sink, qtiles, ctx,
+                             self.heads, self.dp, self.rp, self.cp, self.vp,
+                             self.window, self.scale)
         return linear(ctx.view(t, -1), self.o)
 
 

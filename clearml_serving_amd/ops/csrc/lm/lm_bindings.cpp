@@ -19,6 +19,9 @@ void lm_head_gemm(Tensor a, Tensor w, Tensor out);
 Tensor lm_latent_attention(Tensor q_abs, Tensor cache, Tensor block_table,
                            Tensor tok_seq, Tensor positions, Tensor sink,
                            double scale, long window, long CP, long max_keys);
+void lm_latent_prompt(Tensor q, Tensor kv, Tensor lat, Tensor sink,
+                      Tensor qtiles, Tensor out, long H, long DP, long RP,
+                      long CP, long VP, long window, double scale);
 void lm_rglru_prefill(Tensor yx, Tensor byx, Tensor cw, Tensor cb, Tensor ra,
                       Tensor ba, Tensor ri, Tensor bi, Tensor lam,
                       Tensor state, Tensor ring, Tensor tiles, Tensor seqs,
@@ -39,6 +42,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("lm_latent_prep", &lm_latent_prep);
   m.def("lm_head_gemm", &lm_head_gemm);
   m.def("lm_latent_attention", &lm_latent_attention);
+  m.def("lm_latent_prompt", &lm_latent_prompt);
   m.def("lm_rglru_prefill", &lm_rglru_prefill);
   m.def("lm_rglru_step", &lm_rglru_step);
   m.def("skinny_gemm", &skinny_gemm, py::arg("a"), py::arg("w"),

@@ -177,6 +177,38 @@ def latent_attention(q_abs: torch.Tensor, cache: torch.Tensor,
     return out
 
 
+PROMPT_TILE = 128     # queries per workgroup of latent_prompt
+PROMPT_MAX_HEAD = 256  # largest padded key and value size it takes
+
+
+def latent_prompt(q: torch.Tensor, kv: torch.Tensor, lat: torch.Tensor,
+                  sink: torch.Tensor, qtiles: torch.Tensor,
+                  out: torch.Tensor, heads: int, dp: int, rp: int, cp: int,
+                  vp: int, window: int, scale: float) -> None:
+    """Expanded form, for prompt portions. q [T, heads * (dp + rp)]; kv
+    [rows, heads * dp | heads * vp] keys and values of the gathered cache
+    rows lat [rows, cp + rp]; qtiles [n, 6]: first token, tokens, first
+    position, first gathered row, its position, gathered rows of the
+    sequence. Writes out [T, heads, vp] at the tiles' tokens."""
+    if q.is_cuda:
+        require_lm_ext("latent_prompt").lm_latent_prompt(
+            q, kv, lat, sink, qtiles, out, heads, dp, rp, cp, vp, window,
+            scale)
+        return
+    for t0, n, p0, r0, k_lo, nk in qtiles.tolist():
+        qq = q[t0:t0 + n, :heads * (dp + rp)].float().view(n, heads, -1)
+        rows = kv[r0:r0 + nk].float()
+        k = rows[:, :heads * dp].view(nk, heads, dp)
+        v = rows[:, heads * dp:].view(nk, heads, vp)
+        s = torch.einsum("nhd,khd->hnk", qq[..., :dp], k) + torch.einsum(
+            "nhd,kd->hnk", qq[..., dp:], lat[r0:r0 + nk, cp:].float())
+        dist = (p0 + torch.arange(n))[:, None] - (k_lo + torch.arange(nk))
+        ok = (dist >= 0) & ((dist < window) if window else True)
+        w = _sink_softmax((s * scale).masked_fill(~ok, float("-inf")),
+                          sink.float()[:, None, None])
+        out[t0:t0 + n] = torch.einsum("hnk,khd->nhd", w, v).to(out.dtype)
+
+
 # --------------------------------------------------------------------- #
 # gated linear recurrence
 # --------------------------------------------------------------------- #
