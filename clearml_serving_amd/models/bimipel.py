@@ -178,9 +178,9 @@ class BimipelForCausalLM(nn.Module):
         attn = [m.mix for m in self.layers
                 if isinstance(m.mix, LatentAttention)]
         rec = [m.mix for m in self.layers if isinstance(m.mix, RgLru)]
-        # the recurrence's tile of one block's channels must fit LDS
+        # the recurrence holds two tiles of one block's channels in LDS
         wide = max([m.bp for m in rec], default=32)
-        tile = 64 if 64 * (wide + 8) * dtype.itemsize <= 160 * 1024 else 16
+        tile = 64 if 128 * (wide + 8) * dtype.itemsize <= 160 * 1024 else 16
         # few queries per sequence: absorbed attention; prompts: rebuilt keys
         expand = (dtype == torch.bfloat16
                   and all(m.can_expand() for m in attn))

@@ -128,11 +128,13 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(
 // ------------------------------------------------------------------- //
 // absorbed attention: one token x 16 heads x one key range per workgroup
 // ------------------------------------------------------------------- //
-// Four waves share a tile of KT cached rows in LDS: they split the keys for
-// the scores and the latent columns for the weighted sum. NT: 16-column
-// tiles of the latent per wave (4 * NT * 16 columns per workgroup).
-template <typename T, int KT, int NT>
-__global__ __launch_bounds__(256) void latent_attn_kernel(
+// Each wave walks 32-key tiles of its own: rows go through registers into a
+// wave-private LDS tile (the next tile's loads are in flight while this one
+// is multiplied), S^T = K Q^T stays in registers and is directly the second
+// product's operand, o^T[c][head] += c^T p^T. No barrier until the waves'
+// partial sums meet at the end. NT: 16-column latent tiles per workgroup.
+template <typename T, int NT>
+__global__ __launch_bounds__(256, 1) void latent_attn_kernel(
     const T* __restrict__ q_abs,  // [n, H, CP+RP]
     const T* __restrict__ cache, const int* __restrict__ block_table,
     const int* __restrict__ tok_seq, const int* __restrict__ positions,
@@ -140,159 +142,200 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
     float* __restrict__ part_o, float* __restrict__ part_ml, int splits,
     int col_groups, int H, int CP, int RP, int block_size, int max_blocks,
     int n_blocks, int n_seqs, int window, float scale) {
-  constexpr int SUB = KT / 16;             // 16-key subtiles
-  constexpr int SPW = (SUB + 3) / 4;       // subtiles per wave
-  constexpr int PP = KT + 8;               // pitch of the weights
+  // prefetched 8-element pieces per lane; 32-bit tiles load late instead
+  constexpr int PF = sizeof(T) == 2 ? NT + 4 : 0;
   const int ROW = CP + RP, PITCH = ROW + 8;
+  const int nw = blockDim.x >> 6;
   extern __shared__ __align__(16) char smem[];
-  T* tile = (T*)smem;                      // [KT][PITCH]
-  T* qs = tile + KT * PITCH;               // [16][PITCH]
-  T* ps = qs + 16 * PITCH;                 // [16][PP]
-  float* wred = (float*)(ps + 16 * PP);    // [4][16]
+  __shared__ float stat[4][16][2];
+  T* qs = (T*)smem;                        // [16][PITCH]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  T* tile = qs + 16 * PITCH + wave * 32 * PITCH;  // [32][PITCH]
   const int r16 = lane & 15, g = lane >> 4, ko = g * 8;
   const int t = blockIdx.x;
   const int h0 = blockIdx.y * 16;
   const int split = blockIdx.z / col_groups;
-  const int c_base = (blockIdx.z % col_groups) * (NT * 64);
+  const int c_base = (blockIdx.z % col_groups) * (NT * 16);
   const float scale2 = scale * LOG2E;
 
   const int pos = min(max(positions[t], 0), max_blocks * block_size - 1);
   const int* btab = block_table +
                     (long)min(max(tok_seq[t], 0), n_seqs - 1) * max_blocks;
-  const int lo_all = window > 0 ? max(0, pos - window + 1) : 0;
-  const int n_keys = pos + 1 - lo_all;
-  const int chunk = ((n_keys + splits - 1) / splits + KT - 1) / KT * KT;
-  const int lo = lo_all + split * chunk;
-  const int hi = min(pos + 1, lo + chunk);
+  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  const int n_tiles = (pos + 1 - lo + 31) / 32;
+  const int stride = splits * nw;
+  int j = split * nw + wave;
 
   const int row8 = ROW / 8;
-  for (int i = tid; i < 16 * row8; i += 256) {
+  // cached row of key `lane & 31` of a tile; behind the last key, that key's
+  auto row_of = [&](int jt) {
+    const int key = min(lo + jt * 32 + (lane & 31), pos);
+    const int blk = min(max(btab[key / block_size], 0), n_blocks - 1);
+    return blk * block_size + key % block_size;
+  };
+  // pieces lane, lane + 64, ...: (key, column) advance without divisions
+  const int key0 = lane / row8, col0 = lane % row8;
+  const int dk = 64 / row8, dc = 64 % row8;
+  const int pieces = row8 / 2;  // 32 rows over 64 lanes
+  uint32x4 pre[PF > 0 ? PF : 1];
+  auto load = [&](int rows) {
+    int k = key0, c = col0;
+#pragma unroll
+    for (int i = 0; i < PF; ++i) {
+      if (i < pieces) {
+        const long r = __shfl(rows, k, 64);
+        pre[i] = *reinterpret_cast<const uint32x4*>(cache + r * ROW + c * 8);
+        k += dk;
+        c += dc;
+        if (c >= row8) { c -= row8; ++k; }
+      }
+    }
+  };
+  auto store = [&](int rows) {
+    int k = key0, c = col0;
+#pragma unroll
+    for (int i = 0; i < PF; ++i) {
+      if (i < pieces) {
+        *reinterpret_cast<uint32x4*>(tile + k * PITCH + c * 8) = pre[i];
+        k += dk;
+        c += dc;
+        if (c >= row8) { c -= row8; ++k; }
+      }
+    }
+#pragma unroll 4
+    for (int i = PF; i < pieces; ++i) {
+      const long r = __shfl(rows, k, 64);
+      copy8(tile + k * PITCH + c * 8, cache + r * ROW + c * 8);
+      k += dk;
+      c += dc;
+      if (c >= row8) { c -= row8; ++k; }
+    }
+  };
+
+  int rows = row_of(j), rows_n = row_of(j + stride);
+  if (j < n_tiles) load(rows);
+  for (int i = tid; i < 16 * row8; i += blockDim.x) {
     const int r = i / row8, c = (i % row8) * 8;
     if (h0 + r < H) copy8(qs + r * PITCH + c,
                           q_abs + ((long)t * H + h0 + r) * ROW + c);
     else zero8(qs + r * PITCH + c);
   }
+  __syncthreads();
 
-  float m_run = -INFINITY, l_run = 0.f;  // head r16; l over this wave's keys
+  float m_run = -INFINITY, l_run = 0.f;  // head r16, this lane group's keys
   lm_f32x4 acc[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) acc[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
 
-  for (int n0 = lo; n0 < hi; n0 += KT) {
-    __syncthreads();  // the tile and the weights are free again
-    for (int i = tid; i < KT * row8; i += 256) {
-      const int r = i / row8, c = (i % row8) * 8;
-      const int key = n0 + r;
-      if (key < hi) {
-        const int blk = min(max(btab[key / block_size], 0), n_blocks - 1);
-        copy8(tile + r * PITCH + c,
-              cache + ((long)blk * block_size + key % block_size) * ROW + c);
-      } else {
-        zero8(tile + r * PITCH + c);
-      }
+  for (; j < n_tiles; j += stride) {
+    wave_lds_fence();  // the previous tile has been read
+    store(rows);
+    rows = rows_n;
+    if (j + stride < n_tiles) load(rows);
+    rows_n = row_of(j + 2 * stride);
+    wave_lds_fence();
+    lm_f32x4 s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll 4
+    for (int k = 0; k < ROW; k += 32) {
+      const Frag<T> qf = load_frag(qs + r16 * PITCH + k + ko);
+      s[0] = mma32(load_frag(tile + r16 * PITCH + k + ko), qf, s[0]);
+      s[1] = mma32(load_frag(tile + (16 + r16) * PITCH + k + ko), qf, s[1]);
     }
-    __syncthreads();
-    // scores^T: rows = keys, column = head
-    lm_f32x4 s[SPW];
     float mx = -INFINITY;
 #pragma unroll
-    for (int i = 0; i < SPW; ++i) {
-      s[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
-      const int sub = wave + 4 * i;
-      if (sub < SUB) {
-#pragma unroll 4
-        for (int k = 0; k < ROW; k += 32)
-          s[i] = mma32(load_frag(tile + (sub * 16 + r16) * PITCH + k + ko),
-                       load_frag(qs + r16 * PITCH + k + ko), s[i]);
+    for (int i = 0; i < 2; ++i) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int key = n0 + sub * 16 + 4 * g + r;
-          s[i][r] = key < hi ? s[i][r] * scale2 : -INFINITY;
-          mx = fmaxf(mx, s[i][r]);
-        }
+      for (int r = 0; r < 4; ++r) {
+        const int key = lo + j * 32 + i * 16 + 4 * g + r;
+        s[i][r] = key <= pos ? s[i][r] * scale2 : -INFINITY;
+        mx = fmaxf(mx, s[i][r]);
       }
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-    if (g == 0) wred[wave * 16 + r16] = mx;
-    __syncthreads();
-    float m_new = m_run;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) m_new = fmaxf(m_new, wred[w * 16 + r16]);
-    const float alpha = exp2f(m_run - m_new);  // m_new is finite: hi > n0
+    const float m_new = fmaxf(m_run, mx);  // finite: a tile has a key
+    const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
     m_run = m_new;
     l_run *= alpha;
 #pragma unroll
-    for (int i = 0; i < SPW; ++i) {
-      const int sub = wave + 4 * i;
-      if (sub < SUB) {
-        float p[4];
+    for (int i = 0; i < 2; ++i) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          p[r] = exp2f(s[i][r] - m_new);
-          l_run += p[r];
-        }
-        store4(ps + r16 * PP + sub * 16 + 4 * g, p);
+      for (int r = 0; r < 4; ++r) {
+        s[i][r] = __builtin_amdgcn_exp2f(s[i][r] - m_new);
+        l_run += s[i][r];
       }
     }
-#pragma unroll
-    for (int i = 0; i < NT; ++i) acc[i] *= alpha;
-    __syncthreads();
-    // o^T[c][head] += c^T p^T
-#pragma unroll
-    for (int kc = 0; kc < KT; kc += 32) {
-      const Frag<T> pf = load_frag(ps + r16 * PP + kc + ko);
-#pragma unroll
-      for (int i = 0; i < NT; ++i) {
-        const int c0 = c_base + (wave * NT + i) * 16;
-        if (c0 < CP)
-          acc[i] = mma32(load_frag_col(tile + (kc + ko) * PITCH + c0 + r16,
-                                       PITCH), pf, acc[i]);
-      }
-    }
-  }
-  // denominator over the four waves
-  l_run += __shfl_xor(l_run, 16, 64);
-  l_run += __shfl_xor(l_run, 32, 64);
-  __syncthreads();
-  if (g == 0) wred[wave * 16 + r16] = l_run;
-  __syncthreads();
-  float l = 0.f;
-#pragma unroll
-  for (int w = 0; w < 4; ++w) l += wred[w * 16 + r16];
-  const int h = h0 + r16;
-  if (h >= H) return;
-  if (splits > 1) {
-    const long pi = ((long)t * H + h) * splits + split;
-    if (wave == 0 && g == 0 && c_base == 0) {
-      part_ml[2 * pi] = m_run;
-      part_ml[2 * pi + 1] = l;
-    }
+    const Frag<T> pf = frag_of<T>(s[0], s[1]);
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
-      const int c0 = c_base + (wave * NT + i) * 16;
-      const float f[4] = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
-      if (c0 < CP) store4(part_o + pi * CP + c0 + 4 * g, f);
+      const int c0 = c_base + i * 16;
+      if (c0 < CP) {
+        acc[i] *= alpha;
+        acc[i] = mma32(load_frag_rows(tile + c0, PITCH), pf, acc[i]);
+      }
     }
-    return;
   }
-  const float sk = to_f32(sink[h]) * LOG2E;
-  const float m_f = fmaxf(m_run, sk);
-  const float e = exp2f(m_run - m_f);
-  const float inv = e / (l * e + exp2f(sk - m_f));
+
+  // meet: scale to the common maximum, sum over the waves through LDS
+  l_run += __shfl_xor(l_run, 16, 64);
+  l_run += __shfl_xor(l_run, 32, 64);
+  if (g == 0) {
+    stat[wave][r16][0] = m_run;
+    stat[wave][r16][1] = l_run;
+  }
+  __syncthreads();
+  float m_f = -INFINITY;
+  for (int w = 0; w < nw; ++w) m_f = fmaxf(m_f, stat[w][r16][0]);
+  const float f = m_run == -INFINITY ? 0.f
+                                     : __builtin_amdgcn_exp2f(m_run - m_f);
+  const int cols = min(NT * 16, CP - c_base), OP = cols + 4;
+  // 16 * OP floats of the wave's own tile region
+  float* ow = (float*)(qs + 16 * PITCH + wave * 32 * PITCH);
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
-    const int c0 = c_base + (wave * NT + i) * 16;
-    const float f[4] = {acc[i][0] * inv, acc[i][1] * inv, acc[i][2] * inv,
-                        acc[i][3] * inv};
-    if (c0 < CP) store4(out + ((long)t * H + h) * CP + c0 + 4 * g, f);
+    if (i * 16 < cols) {
+      const float v[4] = {acc[i][0] * f, acc[i][1] * f, acc[i][2] * f,
+                          acc[i][3] * f};
+      store4(ow + r16 * OP + i * 16 + 4 * g, v);
+    }
+  }
+  __syncthreads();
+  const float* o0 = (const float*)(qs + 16 * PITCH);
+  const int wstep = 32 * PITCH * (int)sizeof(T) / 4;
+  const int c4 = cols / 4;
+  for (int i = tid; i < 16 * c4; i += blockDim.x) {
+    const int r = i / c4, c = (i % c4) * 4, h = h0 + r;
+    if (h >= H) break;
+    float m = -INFINITY, l = 0.f;
+    for (int w = 0; w < nw; ++w) m = fmaxf(m, stat[w][r][0]);
+    for (int w = 0; w < nw; ++w)
+      if (stat[w][r][0] != -INFINITY)
+        l += stat[w][r][1] * __builtin_amdgcn_exp2f(stat[w][r][0] - m);
+    lm_f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    for (int w = 0; w < nw; ++w)
+      o += *reinterpret_cast<const lm_f32x4*>(o0 + w * wstep + r * OP + c);
+    if (splits > 1) {
+      const long pi = ((long)t * H + h) * splits + split;
+      const float v[4] = {o[0], o[1], o[2], o[3]};
+      store4(part_o + pi * CP + c_base + c, v);
+      if (c == 0 && c_base == 0) {
+        part_ml[2 * pi] = m;
+        part_ml[2 * pi + 1] = l;
+      }
+    } else {
+      const float sk = to_f32(sink[h]) * LOG2E;
+      const float m_s = fmaxf(m, sk);
+      const float e = __builtin_amdgcn_exp2f(m - m_s);
+      const float inv = e / (l * e + __builtin_amdgcn_exp2f(sk - m_s));
+      const float v[4] = {o[0] * inv, o[1] * inv, o[2] * inv, o[3] * inv};
+      store4(out + ((long)t * H + h) * CP + c_base + c, v);
+    }
   }
 }
 
 // merge key ranges; a range without keys has m = -inf
 template <typename T>
-__global__ __launch_bounds__(64) void latent_combine_kernel(
+__global__ __launch_bounds__(128) void latent_combine_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     const T* __restrict__ sink, T* __restrict__ out, int splits, int H,
     int CP) {
@@ -306,12 +349,12 @@ __global__ __launch_bounds__(64) void latent_combine_kernel(
     l += part_ml[(th * splits + s) * 2 + 1] *
          exp2f(part_ml[(th * splits + s) * 2] - m);
   const float inv = 1.f / l;
-  for (int c = threadIdx.x * 4; c < CP; c += 64 * 4) {
+  for (int c = threadIdx.x * 4; c < CP; c += 128 * 4) {
     float f[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
     for (int s = 0; s < splits; ++s) {
-      const float ms = part_ml[(th * splits + s) * 2];
-      if (ms == -INFINITY) continue;
-      const float e = exp2f(ms - m) * inv;
+      // an empty range wrote zeros and weighs exp2(-inf) = 0
+      const float e = exp2f(part_ml[(th * splits + s) * 2] - m) * inv;
       const lm_f32x4 o = *reinterpret_cast<const lm_f32x4*>(
           part_o + (th * splits + s) * CP + c);
 #pragma unroll
@@ -425,21 +468,23 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
   auto out = torch::empty({n, H, CP}, q_abs.options());
   if (n == 0) return out;
   const int hg = (H + 15) / 16;
-  const int tiles = (int)((CP + 63) / 64);      // 16-column tiles per wave
-  const int nt = tiles <= 1 ? 1 : tiles <= 2 ? 2 : tiles <= 4 ? 4 : 8;
+  const int tiles = (int)(CP / 16);
+  const int nt = tiles <= 2 ? 2 : tiles <= 4 ? 4 : tiles <= 6 ? 6
+               : tiles <= 8 ? 8 : tiles <= 12 ? 12 : tiles <= 16 ? 16
+               : tiles <= 24 ? 24 : 32;
   const int cgroups = (tiles + nt - 1) / nt;
   const int isz = q_abs.element_size();
-  auto lds = [&](int kt) {
-    return (long)((kt + 16) * (ROW + 8) + 16 * (kt + 8)) * isz + 256;
-  };
-  const bool big = isz == 2 && lds(64) <= 80 * 1024;
-  const int kt = big ? 64 : 32;
-  TORCH_CHECK(lds(kt) <= 160 * 1024, "lm_latent_attention: kv_rank + rot_dim ",
+  auto lds = [&](int nw) { return (long)(16 + 32 * nw) * (ROW + 8) * isz; };
+  int nw = 4;
+  while (nw > 1 && lds(nw) > 156 * 1024) nw /= 2;
+  TORCH_CHECK(lds(nw) <= 156 * 1024, "lm_latent_attention: kv_rank + rot_dim ",
               ROW, " does not fit LDS");
-  // enough workgroups for 256 CUs, at least two key tiles each
+  // fill 256 CUs as far as there are 32-key tiles for every wave
   const long keys = window > 0 ? std::min(window, max_keys) : max_keys;
-  long splits = 512 / std::max<long>(1, (long)n * hg * cgroups);
-  splits = std::max<long>(1, std::min(splits, (keys + 2 * kt - 1) / (2 * kt)));
+  const long per_cu = std::min<long>(2, 156 * 1024 / lds(nw));
+  long splits = 256 * per_cu / std::max<long>(1, (long)n * hg * cgroups);
+  splits = std::max<long>(1, std::min(splits,
+                                      (keys + 32 * nw - 1) / (32 * nw)));
   TORCH_CHECK(hg <= 65535 && splits * cgroups <= 65535);
   torch::Tensor po, pml;
   if (splits > 1) {
@@ -448,16 +493,15 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
     pml = torch::empty({n, H, splits, 2}, f32);
   }
   hipStream_t st = cmls::current_stream();
-#define LM_LA(KT, NT)                                                        \
+#define LM_LA(NT)                                                            \
   do {                                                                       \
-    const int bytes = (int)lds(KT);                                          \
-    auto* fn = &latent_attn_kernel<scalar_t, KT, NT>;                        \
-    if (bytes > 64 * 1024)                                                   \
-      HIP_CHECK(hipFuncSetAttribute(                                         \
-          reinterpret_cast<const void*>(fn),                                 \
-          hipFuncAttributeMaxDynamicSharedMemorySize, bytes));               \
-    hipLaunchKernelGGL(fn, dim3(n, hg, splits * cgroups), dim3(256), bytes,  \
-                       st, (const scalar_t*)q_abs.data_ptr(),                \
+    const int bytes = (int)lds(nw);                                          \
+    auto* fn = &latent_attn_kernel<scalar_t, NT>;                            \
+    HIP_CHECK(hipFuncSetAttribute(                                           \
+        reinterpret_cast<const void*>(fn),                                   \
+        hipFuncAttributeMaxDynamicSharedMemorySize, bytes));                 \
+    hipLaunchKernelGGL(fn, dim3(n, hg, splits * cgroups), dim3(64 * nw),     \
+                       bytes, st, (const scalar_t*)q_abs.data_ptr(),         \
                        (const scalar_t*)cache.data_ptr(),                    \
                        block_table.data_ptr<int>(), tok_seq.data_ptr<int>(), \
                        positions.data_ptr<int>(),                            \
@@ -470,24 +514,24 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
                        (int)cache.size(0), (int)block_table.size(0),         \
                        (int)window, (float)scale);                           \
   } while (0)
-#define LM_LA_NT(KT)                                                         \
-  do {                                                                       \
-    if (nt == 1) LM_LA(KT, 1);                                               \
-    else if (nt == 2) LM_LA(KT, 2);                                          \
-    else if (nt == 4) LM_LA(KT, 4);                                          \
-    else LM_LA(KT, 8);                                                       \
-  } while (0)
   LM_DISPATCH(q_abs, "lm_latent_attention", [&] {
-    if (kt == 64) LM_LA_NT(64);
-    else LM_LA_NT(32);
+    switch (nt) {
+      case 2: LM_LA(2); break;
+      case 4: LM_LA(4); break;
+      case 6: LM_LA(6); break;
+      case 8: LM_LA(8); break;
+      case 12: LM_LA(12); break;
+      case 16: LM_LA(16); break;
+      case 24: LM_LA(24); break;
+      default: LM_LA(32); break;
+    }
     if (splits > 1)
       hipLaunchKernelGGL((latent_combine_kernel<scalar_t>), dim3(n * H),
-                         dim3(64), 0, st, po.data_ptr<float>(),
+                         dim3(128), 0, st, po.data_ptr<float>(),
                          pml.data_ptr<float>(),
                          (const scalar_t*)sink.data_ptr(),
                          (scalar_t*)out.data_ptr(), (int)splits, H, (int)CP);
   });
-#undef LM_LA_NT
 #undef LM_LA
   LM_LAUNCHED();
   return out;

@@ -6,11 +6,9 @@
 // queries of one head (8 waves x 16) and walks the 64-key tiles that any of
 // them can see. S^T = K Q^T leaves each lane with keys of ONE query, so max,
 // sum and the running state are lane-local up to two shuffles; and because
-// the k order of an MFMA is free, V^T is stored in LDS in the key order that
-// the S^T registers already have -- the weights go from registers straight
-// into the second product:
-//   lane group g holds keys 16 t + 4 g + r of a 64-key tile; slot g*8 + 4*hi
-//   + r of its 32-key half is key 16*hi + 4*g + r.
+// the k order of an MFMA is free, V is read (transposing LDS reads) in the key
+// order that the S^T registers already have -- the weights go from registers
+// straight into the second product.
 #include "lm_common.h"
 
 namespace {
@@ -28,9 +26,9 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
     const int* __restrict__ qtiles, bf16* __restrict__ out, int H, int DP,
     int RP, int VP, int window, float scale) {
   constexpr int KP = QS * 32 + 8;   // LDS pitches
-  constexpr int VPP = BN + 8;
+  constexpr int VPP = VT * 16 + 8;
   __shared__ __align__(16) short lk[2][BN * KP];
-  __shared__ __align__(16) short lv[2][VT * 16 * VPP];
+  __shared__ __align__(16) bf16 lv[2][BN * VPP];
   const int QD = DP + RP;
   const int h = blockIdx.x;
   const int* td = qtiles + (long)blockIdx.y * 6;
@@ -93,15 +91,8 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
     for (int i = 0; i < VPC; ++i) {
       const int p = tid + i * NW * 64;
       const int key = p / v8, d = (p % v8) * 8;
-      if (key < BN) {
-        // key order of the S^T registers; the 8-slot group is swizzled by
-        // the column so that the transposing writes spread over the banks
-        const int slot = (key & 32) + ((key >> 2) & 3) * 8 +
-                         ((key >> 4) & 1) * 4 + (key & 3);
-        const int sw = slot ^ (((d >> 3) & 7) << 3);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) lv[buf][(d + e) * VPP + sw] = vreg[i][e];
-      }
+      if (key < BN)
+        *reinterpret_cast<lm_s16x8*>(&lv[buf][key * VPP + d]) = vreg[i];
     }
   };
 
@@ -167,22 +158,13 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
     for (int i = 0; i < VT; ++i) acc[i] *= alpha;
 #pragma unroll
     for (int kc = 0; kc < BN / 32; ++kc) {
-      union { lm_s16x8 v; bf16 b[8]; } pf;
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        pf.b[r] = __float2bfloat16(s[2 * kc][r]);
-        pf.b[4 + r] = __float2bfloat16(s[2 * kc + 1][r]);
-      }
+      const Frag<bf16> pf = frag_of<bf16>(s[2 * kc], s[2 * kc + 1]);
 #pragma unroll
       for (int i = 0; i < VT; ++i) {
-        if (i * 16 < VP) {
-          const int row = i * 16 + r16;
-          const lm_s16x8 vf = *reinterpret_cast<const lm_s16x8*>(
-              &lv[buf][row * VPP +
-                       ((kc * 32 + ko) ^ (((row >> 3) & 7) << 3))]);
-          acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf.v, acc[i],
-                                                           0, 0, 0);
-        }
+        if (i * 16 < VP)
+          acc[i] = mma32(
+              load_frag_rows(&lv[buf][kc * 32 * VPP + i * 16], VPP), pf,
+              acc[i]);
       }
     }
   };

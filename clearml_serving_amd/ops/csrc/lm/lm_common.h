@@ -32,21 +32,67 @@ __device__ __forceinline__ Frag<float> load_frag(const float* p) {
   for (int e = 0; e < 4; ++e) { f.v[e] = lo[e]; f.v[4 + e] = hi[e]; }
   return f;
 }
-// the same eight elements, one k step apart by `stride` elements
-__device__ __forceinline__ Frag<bf16> load_frag_col(const bf16* p,
-                                                    int stride) {
+// Operands whose k runs down the rows of an LDS tile. k order of the eight
+// slots of lane group g: rows 4g..4g+3, then 16+4g..16+4g+3 -- the order in
+// which a 16x16 result holds its rows, so a result register file is directly
+// the other operand. Column = lane & 15.
+typedef __attribute__((address_space(3))) lm_s16x4 lm_lds_s16x4;
+__device__ __forceinline__ Frag<bf16> load_frag_rows(const bf16* tile,
+                                                     int pitch) {
+  // ds_read_b64_tr_b16: a 16-lane group reads 4 rows x 16 columns, lane i
+  // supplying row i/4, columns 4*(i%4)..+3, and receives column i
+  const int lane = threadIdx.x & 63, i = lane & 15;
+  const bf16* p = tile + (4 * (lane >> 4) + (i >> 2)) * pitch + (i & 3) * 4;
+  const lm_s16x4 lo =
+      __builtin_amdgcn_ds_read_tr16_b64_v4i16((lm_lds_s16x4*)p);
+  const lm_s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+      (lm_lds_s16x4*)(p + 16 * pitch));
   Frag<bf16> f;
-#pragma unroll
-  for (int e = 0; e < 8; ++e)
-    f.v[e] = *reinterpret_cast<const short*>(p + e * stride);
+  f.v = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
   return f;
 }
-__device__ __forceinline__ Frag<float> load_frag_col(const float* p,
-                                                     int stride) {
+__device__ __forceinline__ Frag<float> load_frag_rows(const float* tile,
+                                                      int pitch) {
+  const int lane = threadIdx.x & 63;
+  const float* p = tile + 4 * (lane >> 4) * pitch + (lane & 15);
   Frag<float> f;
 #pragma unroll
-  for (int e = 0; e < 8; ++e) f.v[e] = p[e * stride];
+  for (int e = 0; e < 4; ++e) {
+    f.v[e] = p[e * pitch];
+    f.v[4 + e] = p[(16 + e) * pitch];
+  }
   return f;
+}
+// the operand made of two such results (rows 0..15 and 16..31)
+template <typename T>
+__device__ __forceinline__ Frag<T> frag_of(const lm_f32x4& lo,
+                                           const lm_f32x4& hi);
+template <>
+__device__ __forceinline__ Frag<bf16> frag_of<bf16>(const lm_f32x4& lo,
+                                                    const lm_f32x4& hi) {
+  union { lm_s16x8 v; bf16 b[8]; } u;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    u.b[e] = __float2bfloat16(lo[e]);
+    u.b[4 + e] = __float2bfloat16(hi[e]);
+  }
+  Frag<bf16> f;
+  f.v = u.v;
+  return f;
+}
+template <>
+__device__ __forceinline__ Frag<float> frag_of<float>(const lm_f32x4& lo,
+                                                      const lm_f32x4& hi) {
+  Frag<float> f;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) { f.v[e] = lo[e]; f.v[4 + e] = hi[e]; }
+  return f;
+}
+// LDS traffic between the lanes of one wave: order it without a barrier
+__device__ __forceinline__ void wave_lds_fence() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 template <typename T> __device__ __forceinline__ Frag<T> zero_frag();
 template <> __device__ __forceinline__ Frag<bf16> zero_frag<bf16>() {
@@ -128,13 +174,27 @@ __device__ __forceinline__ void zero8(float* d) {
   reinterpret_cast<uint32x4*>(d)[1] = uint32x4{0u, 0u, 0u, 0u};
 }
 
+// v_exp_f32 and v_rcp_f32: full float, within about 1 ulp
+__device__ __forceinline__ float exp_f(float z) {
+  return __builtin_amdgcn_exp2f(z * 1.4426950408889634f);
+}
 __device__ __forceinline__ float sigmoid_f(float z) {
-  return 1.f / (1.f + expf(-z));
+  return __builtin_amdgcn_rcpf(1.f + exp_f(-z));
 }
 // tanh form: 0.5 z (1 + tanh k) = z * sigmoid(2 k)
 __device__ __forceinline__ float gelu_tanh_f(float z) {
   const float k = 0.7978845608028654f * (z + 0.044715f * z * z * z);
   return z * sigmoid_f(2.f * k);
+}
+// 1 - exp(v) for v <= 0: the power series where the difference would cancel
+__device__ __forceinline__ float one_minus_exp_f(float v) {
+  const float p =
+      1.f + v * (1.f / 2) *
+                (1.f + v * (1.f / 3) *
+                           (1.f + v * (1.f / 4) *
+                                      (1.f + v * (1.f / 5) *
+                                                 (1.f + v * (1.f / 6)))));
+  return v > -0.25f ? -v * p : 1.f - exp_f(v);
 }
 __device__ __forceinline__ float softplus_f(float z) {
   return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));

@@ -28,8 +28,8 @@ constexpr int NWV = 4;
 __device__ __forceinline__ void decay_and_input(float zr, float zi, float sp,
                                                 float u, float* a, float* b) {
   const float la = -8.f * sigmoid_f(zr) * sp;
-  *a = expf(la);
-  *b = sqrtf(-expm1f(2.f * la)) * sigmoid_f(zi) * u;
+  *a = exp_f(la);
+  *b = __builtin_amdgcn_sqrtf(one_minus_exp_f(2.f * la)) * sigmoid_f(zi) * u;
 }
 
 // pre-activations of 16 channels x MT*16 tokens:
@@ -48,7 +48,7 @@ __device__ __forceinline__ void gate_products(const T* us, int pitch,
     zr[m] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
     zi[m] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
   }
-#pragma unroll 2
+#pragma unroll 4
   for (int k = 0; k < BP; k += 32) {
     const Frag<T> wr = load_frag(pr + k), wi = load_frag(pi + k);
 #pragma unroll
@@ -214,6 +214,7 @@ __global__ __launch_bounds__(256) void rglru_out_kernel(
   extern __shared__ __align__(16) char smem[];
   T* us = (T*)smem;
   const int pitch = BP + 8;
+  T* ys = us + TT * pitch;  // y, then the result
   const int tile = blockIdx.x, ch0 = blockIdx.y * BP;
   const int* td = tiles + tile * 5;
   const int t0 = td[0], len = td[1];
@@ -221,9 +222,13 @@ __global__ __launch_bounds__(256) void rglru_out_kernel(
   const int bp8 = BP / 8;
   for (int i = tid; i < TT * bp8; i += 256) {
     const int tt = i / bp8, c = (i % bp8) * 8;
-    if (tt < len) copy8(us + tt * pitch + c,
-                        u_in + (long)(t0 + tt) * W + ch0 + c);
-    else zero8(us + tt * pitch + c);
+    if (tt < len) {
+      copy8(us + tt * pitch + c, u_in + (long)(t0 + tt) * W + ch0 + c);
+      copy8(ys + tt * pitch + c, yx + (long)(t0 + tt) * ld + ch0 + c);
+    } else {
+      zero8(us + tt * pitch + c);
+      zero8(ys + tt * pitch + c);
+    }
   }
   __syncthreads();
   const long wofs = (long)blockIdx.y * BP * BP;
@@ -261,14 +266,17 @@ __global__ __launch_bounds__(256) void rglru_out_kernel(
       for (int r = 0; r < 4; ++r) {
         const int tt = m * 16 + 4 * g + r;
         s = a[r] * s + b[r];
-        if (tt < len) {
-          const float y = to_f32(yx[(long)(t0 + tt) * ld + ch]) + by;
-          out[(long)(t0 + tt) * W + ch] = from_f32<T>(s * gelu_tanh_f(y));
-        }
+        T* yp = ys + tt * pitch + c;  // read and written by this lane only
+        *yp = from_f32<T>(s * gelu_tanh_f(to_f32(*yp) + by));
       }
       S = __shfl(a4, 48 + (lane & 15), 64) * S +
           __shfl(b4, 48 + (lane & 15), 64);
     }
+  }
+  __syncthreads();
+  for (int i = tid; i < len * bp8; i += 256) {
+    const int tt = i / bp8, c = (i % bp8) * 8;
+    copy8(out + (long)(t0 + tt) * W + ch0 + c, ys + tt * pitch + c);
   }
 }
 
@@ -306,7 +314,8 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(
     const T* cur = yx + (long)t * ld + W + ch;
     conv_tap<T>(cur, bx, cw + (long)(taps - 1) * W + ch, u);
     if (has_state) {
-      for (int d = 1; d < taps && d <= pos; ++d)
+#pragma unroll 4
+      for (int d = 1; d < min(taps, pos + 1); ++d)
         conv_tap<T>(ring + ((long)slot * taps + (pos - d) % taps) * W + ch,
                     bx, cw + (long)(taps - 1 - d) * W + ch, u);
       // this slice's part of the ring; nobody reads this entry at this step
@@ -415,7 +424,7 @@ void lm_rglru_prefill(torch::Tensor yx, torch::Tensor byx, torch::Tensor cw,
   if (nt == 0) return;
   TORCH_CHECK(ns <= 65535);
   const int bytes = (int)(tile * (d.BP + 8) * yx.element_size());
-  TORCH_CHECK(bytes <= 160 * 1024, "rglru: block of ", d.BP,
+  TORCH_CHECK(2 * bytes <= 160 * 1024, "rglru: block of ", d.BP,
               " channels does not fit LDS");
   auto u = torch::empty({d.T, d.W}, yx.options());
   auto comp = torch::empty({nt, 2, d.W}, yx.options().dtype(at::kFloat));
@@ -424,7 +433,7 @@ void lm_rglru_prefill(torch::Tensor yx, torch::Tensor byx, torch::Tensor cw,
 #define LM_RG(TT)                                                            \
   do {                                                                       \
     allow_lds(&rglru_tile_kernel<scalar_t, TT>, bytes);                      \
-    allow_lds(&rglru_out_kernel<scalar_t, TT>, bytes);                       \
+    allow_lds(&rglru_out_kernel<scalar_t, TT>, 2 * bytes);                   \
     hipLaunchKernelGGL((rglru_tile_kernel<scalar_t, TT>), dim3(nt, d.blocks),\
                        dim3(256), bytes, st, P(yx), d.ld, P(byx), P(cw),     \
                        P(cb), P(ra), P(ba), P(ri), P(bi), P(lam), P(ring),   \
@@ -437,7 +446,7 @@ void lm_rglru_prefill(torch::Tensor yx, torch::Tensor byx, torch::Tensor cw,
                        state.data_ptr<float>(), (scalar_t*)ring.data_ptr(),  \
                        P(yx), d.ld, d.W, d.taps, d.n_state);                 \
     hipLaunchKernelGGL((rglru_out_kernel<scalar_t, TT>), dim3(nt, d.blocks), \
-                       dim3(256), bytes, st, P(yx), d.ld, P(byx), P(u),      \
+                       dim3(256), 2 * bytes, st, P(yx), d.ld, P(byx), P(u),  \
                        P(ra), P(ba), P(ri), P(bi), P(lam),                   \
                        tiles.data_ptr<int>(), comp.data_ptr<float>(),        \
                        (scalar_t*)out.data_ptr(), d.W, d.BP);                \
