@@ -142,8 +142,9 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
     float* __restrict__ part_o, float* __restrict__ part_ml, int splits,
     int col_groups, int H, int CP, int RP, int block_size, int max_blocks,
     int n_blocks, int n_seqs, int window, float scale) {
-  // prefetched 8-element pieces per lane; 32-bit tiles load late instead
-  constexpr int PF = sizeof(T) == 2 ? NT + 4 : 0;
+  // bf16: the next tile's rows wait in registers, one 16-byte piece of every
+  // row per lane; 32-bit tiles (exact runs) load when they are stored
+  constexpr bool PRE = sizeof(T) == 2;
   const int ROW = CP + RP, PITCH = ROW + 8;
   const int nw = blockDim.x >> 6;
   extern __shared__ __align__(16) char smem[];
@@ -173,42 +174,32 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
     const int blk = min(max(btab[key / block_size], 0), n_blocks - 1);
     return blk * block_size + key % block_size;
   };
-  // pieces lane, lane + 64, ...: (key, column) advance without divisions
-  const int key0 = lane / row8, col0 = lane % row8;
-  const int dk = 64 / row8, dc = 64 % row8;
-  const int pieces = row8 / 2;  // 32 rows over 64 lanes
-  uint32x4 pre[PF > 0 ? PF : 1];
+  // Lane l moves columns 8l..8l+7 of each row, so that a row's address is
+  // uniform; columns behind the 64th piece (rows of more than 512) go late.
+  uint32x4 pre[PRE ? 32 : 1];
+  const bool has_piece = lane < row8;
   auto load = [&](int rows) {
-    int k = key0, c = col0;
+    if (PRE && has_piece) {
 #pragma unroll
-    for (int i = 0; i < PF; ++i) {
-      if (i < pieces) {
-        const long r = __shfl(rows, k, 64);
-        pre[i] = *reinterpret_cast<const uint32x4*>(cache + r * ROW + c * 8);
-        k += dk;
-        c += dc;
-        if (c >= row8) { c -= row8; ++k; }
+      for (int k = 0; k < 32; ++k) {
+        const long r = __builtin_amdgcn_readlane(rows, k);
+        pre[PRE ? k : 0] = *reinterpret_cast<const uint32x4*>(
+            cache + r * ROW + lane * 8);
       }
     }
   };
   auto store = [&](int rows) {
-    int k = key0, c = col0;
+    if (PRE && has_piece) {
 #pragma unroll
-    for (int i = 0; i < PF; ++i) {
-      if (i < pieces) {
-        *reinterpret_cast<uint32x4*>(tile + k * PITCH + c * 8) = pre[i];
-        k += dk;
-        c += dc;
-        if (c >= row8) { c -= row8; ++k; }
-      }
+      for (int k = 0; k < 32; ++k)
+        *reinterpret_cast<uint32x4*>(tile + k * PITCH + lane * 8) =
+            pre[PRE ? k : 0];
     }
-#pragma unroll 4
-    for (int i = PF; i < pieces; ++i) {
+    const int c0 = PRE ? 64 : 0, rest = row8 - c0;
+    for (int p = lane; p < 32 * rest; p += 64) {
+      const int k = p / rest, c = (c0 + p % rest) * 8;
       const long r = __shfl(rows, k, 64);
-      copy8(tile + k * PITCH + c * 8, cache + r * ROW + c * 8);
-      k += dk;
-      c += dc;
-      if (c >= row8) { c -= row8; ++k; }
+      copy8(tile + k * PITCH + c, cache + r * ROW + c);
     }
   };
 
@@ -266,14 +257,14 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
       }
     }
     const Frag<T> pf = frag_of<T>(s[0], s[1]);
+    // columns behind CP (NT is rounded up) sum what lies there in LDS and
+    // are dropped at the end
 #pragma unroll
-    for (int i = 0; i < NT; ++i) {
-      const int c0 = c_base + i * 16;
-      if (c0 < CP) {
-        acc[i] *= alpha;
-        acc[i] = mma32(load_frag_rows(tile + c0, PITCH), pf, acc[i]);
-      }
-    }
+    for (int i = 0; i < NT; ++i) acc[i] *= alpha;
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+      acc[i] = mma32(load_frag_rows(tile + c_base + i * 16, PITCH), pf,
+                     acc[i]);
   }
 
   // meet: scale to the common maximum, sum over the waves through LDS
@@ -474,9 +465,13 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
                : tiles <= 24 ? 24 : 32;
   const int cgroups = (tiles + nt - 1) / nt;
   const int isz = q_abs.element_size();
-  auto lds = [&](int nw) { return (long)(16 + 32 * nw) * (ROW + 8) * isz; };
+  // the slack holds reads of rounded-up columns behind the last row
+  const long slack = (long)std::max<long>(0, (long)cgroups * nt * 16 - ROW);
+  auto lds = [&](int nw) {
+    return ((long)(16 + 32 * nw) * (ROW + 8) + slack) * isz;
+  };
   int nw = 4;
-  while (nw > 1 && lds(nw) > 156 * 1024) nw /= 2;
+  while (nw > 1 && lds(nw) > 156 * 1024) --nw;
   TORCH_CHECK(lds(nw) <= 156 * 1024, "lm_latent_attention: kv_rank + rot_dim ",
               ROW, " does not fit LDS");
   // fill 256 CUs as far as there are 32-key tiles for every wave

@@ -28,8 +28,9 @@ constexpr int NWV = 4;
 __device__ __forceinline__ void decay_and_input(float zr, float zi, float sp,
                                                 float u, float* a, float* b) {
   const float la = -8.f * sigmoid_f(zr) * sp;
-  *a = exp_f(la);
-  *b = __builtin_amdgcn_sqrtf(one_minus_exp_f(2.f * la)) * sigmoid_f(zi) * u;
+  const float d = one_minus_exp_f(la);  // 1 - a, exact also for a near 1
+  *a = 1.f - d;
+  *b = __builtin_amdgcn_sqrtf(d * (2.f - d)) * sigmoid_f(zi) * u;
 }
 
 // pre-activations of 16 channels x MT*16 tokens:
