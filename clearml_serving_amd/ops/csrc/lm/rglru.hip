@@ -300,6 +300,41 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(
   const int s0 = blockIdx.z * 64;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int bp8 = BP / 8;
+  // what the second half needs and the first does not change is loaded
+  // ahead of it: gate weights, state, gated branch
+  const int n0 = s0 + wave * 16;
+  const bool active = n0 < BP;
+  const int r16 = lane & 15, ko = (lane >> 4) * 8;
+  const int c0 = n0 + r16, cch = ch0 + c0;
+  constexpr int PK = 4;  // k steps of weights in registers
+  Frag<T> wr[PK], wi[PK];
+  float s_old[4], y_in[4];
+  int slot4[4];
+  const T* pr = ra + (long)blockIdx.y * BP * BP + (long)c0 * BP + ko;
+  const T* pi = ri + (long)blockIdx.y * BP * BP + (long)c0 * BP + ko;
+  if (active) {
+#pragma unroll
+    for (int k = 0; k < PK; ++k) {
+      if (k * 32 < BP) {
+        wr[k] = load_frag(pr + k * 32);
+        wi[k] = load_frag(pi + k * 32);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = row0 + 4 * (lane >> 4) + r;
+      slot4[r] = -1;
+      s_old[r] = y_in[r] = 0.f;
+      if (t < n) {
+        const int slot = slots[t];
+        y_in[r] = to_f32(yx[(long)t * ld + cch]);
+        if (slot >= 0 && slot < n_state) {
+          slot4[r] = slot;
+          if (positions[t] > 0) s_old[r] = state[(long)slot * W + cch];
+        }
+      }
+    }
+  }
   for (int i = tid; i < 16 * bp8; i += 256) {
     const int rr = i / bp8, c = (i % bp8) * 8, ch = ch0 + c;
     const int t = row0 + rr;
@@ -326,32 +361,35 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(
     store8(us + rr * pitch + c, u);
   }
   __syncthreads();
-  const int n0 = s0 + wave * 16;
-  if (n0 >= BP) return;
-  const long wofs = (long)blockIdx.y * BP * BP;
-  lm_f32x4 zr[1], zi[1];
-  gate_products<T, 1>(us, pitch, ra + wofs, ri + wofs, n0, BP, zr, zi);
-  const int c = n0 + (lane & 15), ch = ch0 + c;
-  const float vr = to_f32(ba[ch]), vi = to_f32(bi[ch]);
-  const float sp = softplus_f(to_f32(lam[ch]));
-  const float by = to_f32(byx[ch]);
+  if (!active) return;
+  lm_f32x4 zr = {0.f, 0.f, 0.f, 0.f}, zi = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int k = 0; k < PK; ++k) {
+    if (k * 32 < BP) {
+      const Frag<T> uf = load_frag(us + r16 * pitch + k * 32 + ko);
+      zr = mma32(uf, wr[k], zr);
+      zi = mma32(uf, wi[k], zi);
+    }
+  }
+#pragma unroll 4
+  for (int k = PK * 32; k < BP; k += 32) {
+    const Frag<T> uf = load_frag(us + r16 * pitch + k + ko);
+    zr = mma32(uf, load_frag(pr + k), zr);
+    zi = mma32(uf, load_frag(pi + k), zi);
+  }
+  const float vr = to_f32(ba[cch]), vi = to_f32(bi[cch]);
+  const float sp = softplus_f(to_f32(lam[cch]));
+  const float by = to_f32(byx[cch]);
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int rr = 4 * (lane >> 4) + r, t = row0 + rr;
     if (t >= n) continue;
-    const int pos = positions[t], slot = slots[t];
-    const bool has_state = slot >= 0 && slot < n_state;
     float a, b;
-    decay_and_input(zr[0][r] + vr, zi[0][r] + vi, sp,
-                    to_f32(us[rr * pitch + c]), &a, &b);
-    float S = b;
-    if (has_state) {
-      float* sp_ = state + (long)slot * W + ch;
-      if (pos > 0) S = a * *sp_ + b;
-      *sp_ = S;
-    }
-    const float y = to_f32(yx[(long)t * ld + ch]) + by;
-    out[(long)t * W + ch] = from_f32<T>(S * gelu_tanh_f(y));
+    decay_and_input(zr[r] + vr, zi[r] + vi, sp, to_f32(us[rr * pitch + c0]),
+                    &a, &b);
+    const float S = a * s_old[r] + b;  // s_old: 0 at position 0
+    if (slot4[r] >= 0) state[(long)slot4[r] * W + cch] = S;
+    out[(long)t * W + cch] = from_f32<T>(S * gelu_tanh_f(y_in[r] + by));
   }
 }
 
