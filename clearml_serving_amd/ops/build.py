@@ -5,8 +5,8 @@ Two libraries, each a torch extension next to this file:
 - ``_hip_ops.so``: every kernel in ``csrc/*.hip`` (vision, encoder and
   llama/gpt2 serving)
 - ``_hip_lm.so``: the token-batch kernels in ``csrc/lm/*.hip`` (latent
-  attention, gated linear recurrence, sandwich-free norms) plus the decode
-  GEMM they share with ``_hip_ops``. It is a library of its own so that a
+  attention, gated linear recurrence, norms and the residual stream) plus
+  the decode GEMM they share with ``_hip_ops``. It is a library of its own so that a
   fresh checkout can serve a model of that kind after compiling only this.
 """
 

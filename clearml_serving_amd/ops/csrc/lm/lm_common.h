@@ -189,11 +189,8 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
 // 1 - exp(v) for v <= 0: the power series where the difference would cancel
 __device__ __forceinline__ float one_minus_exp_f(float v) {
   const float p =
-      1.f + v * (1.f / 2) *
-                (1.f + v * (1.f / 3) *
-                           (1.f + v * (1.f / 4) *
-                                      (1.f + v * (1.f / 5) *
-                                                 (1.f + v * (1.f / 6)))));
+      1.f + v * (1.f / 2 + v * (1.f / 6 + v * (1.f / 24 +
+            v * (1.f / 120 + v * (1.f / 720)))));
   return v > -0.25f ? -v * p : 1.f - exp_f(v);
 }
 __device__ __forceinline__ float softplus_f(float z) {
