@@ -15,7 +15,7 @@ import time
 import torch
 
 SIZES = {
-    # size -> (bimipel preset or stack, llama preset, llama overrides)
+    # size -> (bimipel preset, llama preset, llama overrides)
     "300m": ("bimipel-300m", "llama-3-8b", dict(
         vocab_size=32000, hidden=1024, layers=12, heads=16, kv_heads=4,
         intermediate=3584)),
@@ -24,15 +24,6 @@ SIZES = {
     "4k": ("bimipel-4k", "llama-3-8b", dict(vocab_size=32000, layers=6,
                                             intermediate=12288)),
 }
-
-
-def _presets():
-    from clearml_serving_amd.models import bimipel
-
-    if "bimipel-4k" not in bimipel.PRESETS:
-        bimipel.PRESETS["bimipel-4k"] = bimipel._griffin_like(
-            32000, 4096, 12288, 32, 96, 32, 512, 4096, 16, 2048, 2)
-    return bimipel.PRESETS
 
 
 def _params(model):
@@ -47,7 +38,6 @@ def _engine(kind, size, batch, max_len):
                                                         LlmEngineConfig)
 
     bim, preset, over = SIZES[size]
-    _presets()
     blocks = max(batch, 1) * (-(-max_len // 16) + 1)
     cfg = LlmEngineConfig(
         arch="bimipel" if kind == "bimipel" else "llama",

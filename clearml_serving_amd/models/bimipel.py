@@ -269,6 +269,9 @@ PRESETS = {
                                 20, 1024, 6),
     "bimipel-300m": _griffin_like(32000, 1024, 3072, 8, 96, 32, 256, 1280,
                                   10, 512, 4),
+    # six layers as wide as an 8B model's
+    "bimipel-4k": _griffin_like(32000, 4096, 12288, 32, 96, 32, 512, 4096,
+                                16, 2048, 2),
 }
 
 
