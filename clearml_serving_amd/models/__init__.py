@@ -98,4 +98,5 @@ def load_weights(model: torch.nn.Module, path: str) -> None:
     model.load_state_dict(convert_hf_auto(state))
 
 
-from . import bert, bimipel, gpt2, llama, resnet  # noqa: E402,F401  (register architectures)
+from . import (bert, bimipel, gpt2, kakipel, llama,  # noqa: E402,F401
+               resnet)  # (register architectures)

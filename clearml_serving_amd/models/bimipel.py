@@ -23,7 +23,8 @@ import torch.nn as nn
 from ..ops import lm
 from ..ops.lm import pad32
 from . import register_arch, register_token_batch_arch
-from .mixers import GatedMlp, LatentAttention, RgLru, _fill, _param, linear
+from .mixers import GatedMlp, LatentAttention, RgLru, _param, linear
+from .token_lm import TokenBatchForCausalLM, TokenBatchLayer, held
 
 
 class BimipelConfig:
@@ -53,7 +54,7 @@ class BimipelConfig:
                         "uses".format(n, key, src))
 
 
-class BimipelLayer(nn.Module):
+class BimipelLayer(TokenBatchLayer):
     def __init__(self, cfg: BimipelConfig, index: int):
         super().__init__()
         spec = cfg.layers[index]
@@ -85,11 +86,11 @@ class BimipelLayer(nn.Module):
             self.mlp = GatedMlp(cfg.hidden, int(mlp["ff"]))
             self.norm2 = _param(wp)
 
-    def parts(self):
-        """(prefix, module) of what a checkpoint holds for this layer"""
-        yield "mix.", self.mix
+    def held(self):
+        out = {"norm1": held(self.norm1, self.width)}
         if self.mlp is not None:
-            yield "mlp.", self.mlp
+            out["norm2"] = held(self.norm2, self.width)
+        return out
 
     def forward(self, x, h, batch, cache):
         h = lm.post_norm_add(self.mix(h, batch, cache), None, self.norm1, x,
@@ -100,12 +101,7 @@ class BimipelLayer(nn.Module):
         return h
 
 
-class BimipelForCausalLM(nn.Module):
-    # one forward for prompt portions and single tokens together
-    token_batch = True
-    supports_float32 = True
-    tp_size = 1
-
+class BimipelForCausalLM(TokenBatchForCausalLM):
     def __init__(self, cfg: BimipelConfig):
         super().__init__()
         self.cfg = cfg
@@ -115,54 +111,22 @@ class BimipelForCausalLM(nn.Module):
             [BimipelLayer(cfg, i) for i in range(len(cfg.layers))])
         self.final_norm = _param(wp)
 
-    # ---- weights ---------------------------------------------------- #
-    def checkpoint_shapes(self) -> Dict[str, tuple]:
+    def held(self):
         c = self.cfg
-        out = {"embed": (c.vocab_size, c.hidden), "final.norm": (c.hidden,)}
-        for i, layer in enumerate(self.layers):
-            p = "l{}.".format(i)
-            out[p + "norm1"] = (c.hidden,)
-            if layer.mlp is not None:
-                out[p + "norm2"] = (c.hidden,)
-            for q, mod in layer.parts():
-                for k, s in mod.shapes().items():
-                    out[p + q + k] = s
-        return out
+        return {"embed": held(self.embed, c.vocab_size, c.hidden),
+                "final.norm": held(self.final_norm, c.hidden)}
 
-    def load_checkpoint(self, state: Dict[str, torch.Tensor]) -> None:
-        want = self.checkpoint_shapes()
-        missing = sorted(set(want) - set(state))
-        extra = sorted(set(state) - set(want))
-        if missing or extra:
-            raise ValueError("checkpoint does not fit the configuration: "
-                             "missing {}, unexpected {}".format(
-                                 missing[:8], extra[:8]))
-        for k, s in want.items():
-            if tuple(state[k].shape) != tuple(s):
-                raise ValueError("checkpoint tensor '{}' is {}, expected {}"
-                                 .format(k, tuple(state[k].shape), s))
-        _fill(self.embed.data, state["embed"])
-        _fill(self.final_norm.data, state["final.norm"])
-        for i, layer in enumerate(self.layers):
-            p = "l{}.".format(i)
-            _fill(layer.norm1.data, state[p + "norm1"])
-            if layer.mlp is not None:
-                _fill(layer.norm2.data, state[p + "norm2"])
-            for q, mod in layer.parts():
-                mod.pack(lambda name, q=p + q: state[q + name])
+    def random_tensor(self, name, shape, gen):
+        w = torch.empty(shape, dtype=torch.float32)
+        if name.endswith("lam"):
+            return w.uniform_(-4.0, 1.0, generator=gen)
+        if name.endswith("dkv.norm"):
+            return w.fill_(1.0)
+        if len(shape) == 1:
+            return w.normal_(std=0.02, generator=gen)
+        return w.normal_(std=shape[-1] ** -0.5, generator=gen)
 
-    def init_random(self, seed: int = 1234) -> None:
-        self.load_checkpoint(random_checkpoint(self, seed))
-
-    def finalize(self) -> None:
-        """call once weights, device and type are settled"""
-        for layer in self.layers:
-            layer.mix.finalize()
-
-    # ---- what the engine needs to know ------------------------------ #
     def cache_layout(self) -> List[tuple]:
-        """per layer: ("paged", elements per token), ("state", channels,
-        taps) or ("shared", layer)"""
         out: List[tuple] = []
         for layer in self.layers:
             if isinstance(layer.mix, RgLru):
@@ -172,20 +136,6 @@ class BimipelForCausalLM(nn.Module):
             else:
                 out.append(("paged", layer.mix.row))
         return out
-
-    def batch_params(self, dtype: torch.dtype) -> Dict[str, Any]:
-        """how a TokenBatch for this model is to be cut"""
-        attn = [m.mix for m in self.layers
-                if isinstance(m.mix, LatentAttention)]
-        rec = [m.mix for m in self.layers if isinstance(m.mix, RgLru)]
-        # the recurrence holds two tiles of one block's channels in LDS
-        wide = max([m.bp for m in rec], default=32)
-        tile = 64 if 128 * (wide + 8) * dtype.itemsize <= 160 * 1024 else 16
-        # few queries per sequence: absorbed attention; prompts: rebuilt keys
-        expand = (dtype == torch.bfloat16
-                  and all(m.can_expand() for m in attn))
-        return {"tile": tile, "absorb_max": 8 if expand else None,
-                "windows": sorted({m.window for m in attn})}
 
     # ---- forward ---------------------------------------------------- #
     def forward(self, tokens, positions, kv_caches, attn_ctx,
@@ -205,25 +155,6 @@ class BimipelForCausalLM(nn.Module):
         if logits.shape[1] != c.vocab_size:
             logits = logits[:, :c.vocab_size].contiguous()
         return logits
-
-
-def random_checkpoint(model: BimipelForCausalLM, seed: int
-                      ) -> Dict[str, torch.Tensor]:
-    """seeded weights in checkpoint layout, scaled like a fresh model's"""
-    gen = torch.Generator().manual_seed(seed)
-    out = {}
-    for name, shape in model.checkpoint_shapes().items():
-        w = torch.empty(shape, dtype=torch.float32)
-        if name.endswith("lam"):
-            w.uniform_(-4.0, 1.0, generator=gen)
-        elif name.endswith("dkv.norm"):
-            w.fill_(1.0)
-        elif len(shape) == 1:
-            w.normal_(std=0.02, generator=gen)
-        else:
-            w.normal_(std=shape[-1] ** -0.5, generator=gen)
-        out[name] = w.to(torch.bfloat16)
-    return out
 
 
 def _attn(heads, dim, rot, vdim, rank, window, base=10000.0, kv_from=None):

@@ -11,8 +11,9 @@
 //   portion can see, then ordinary flash attention runs on them; several
 //   times fewer multiply-adds when kv_rank exceeds the head size.
 //
-// Both take a sliding window and a per-head sink (a term exp(sink) in the
-// softmax denominator that has no key).
+// Both take a sliding window, a per-head sink (a term exp(sink) in the softmax
+// denominator that has no key) and a gate on the heads' outputs, each of them
+// optional. Queries may come from a normed latent of their own.
 #include "lm_common.h"
 
 namespace {
@@ -20,80 +21,138 @@ namespace {
 constexpr float LOG2E = 1.4426950408889634f;
 
 // ------------------------------------------------------------------- //
-// prepare: rotate q, normalise the latent, rotate the shared key part,
-// write the cache row
+// rotary positions
 // ------------------------------------------------------------------- //
-// u at an even index, v behind it: (u cos - v sin, v cos + u sin)
+// Pair p of a rotated part is (2p, 2p+1) or, with `half`, (p, p + pairs):
+// (u, v) -> gain * (u cos - v sin, v cos + u sin). Elements behind the pairs
+// pass unchanged.
+struct Rot {
+  const float* inv_freq;
+  int pairs, half;
+  float gain;
+};
+
+__device__ __forceinline__ void rot_places(const Rot& r, int p, int* u,
+                                           int* v) {
+  const bool h = r.half && p < r.pairs;
+  *u = h ? p : 2 * p;
+  *v = h ? p + r.pairs : 2 * p + 1;
+}
+
+// ------------------------------------------------------------------- //
+// prepare: rotate q; normalise the query latent and the cached latent, rotate
+// the shared key part, write the cache row. Each part is optional.
+// ------------------------------------------------------------------- //
 template <typename T>
-__global__ __launch_bounds__(256) void latent_prep_kernel(
-    T* __restrict__ qkv, int ld, const int* __restrict__ positions,
-    const int* __restrict__ slots, const float* __restrict__ inv_freq,
-    int n_rot, int heads, int DP, int RP, int CP, int kv_rank, float eps,
-    const T* __restrict__ kv_norm,  // null: the layer owns no latent
-    T* __restrict__ cache, long n_slots, T* __restrict__ q_abs, int n_abs) {
-  __shared__ float cs[256], sn[256];
-  __shared__ float tmp[16];
-  const int t = blockIdx.x;
-  const int tid = threadIdx.x;
-  const int pairs = n_rot / 2;
-  const float pos = (float)positions[t];
-  for (int i = tid; i < pairs; i += 256) {
-    float s, c;
-    sincosf(pos * inv_freq[i], &s, &c);
-    cs[i] = c;
-    sn[i] = s;
-  }
-  __syncthreads();
-  T* row = qkv + (long)t * ld;
-  const int hp = RP / 2;
-  const bool absorbed = t < n_abs;
-  const int q_pairs = absorbed ? hp : pairs;  // the rest passes unchanged
-  for (int i = tid; i < heads * q_pairs; i += 256) {
-    const int hd = i / q_pairs, p = i % q_pairs;
-    T* src = row + hd * (DP + RP) + DP + 2 * p;
-    float u = to_f32(src[0]), v = to_f32(src[1]);
-    if (p < pairs) {
-      const float a = u * cs[p] - v * sn[p];
-      v = v * cs[p] + u * sn[p];
-      u = a;
-    }
-    T* dst = absorbed
-                 ? q_abs + ((long)t * heads + hd) * (CP + RP) + CP + 2 * p
-                 : src;
-    dst[0] = from_f32<T>(u);
-    dst[1] = from_f32<T>(v);
-  }
-  if (!kv_norm) return;
-  const T* lat = row + heads * (DP + RP);
+struct PrepArgs {
+  T* q;            // [t, heads * (DP + RP)], rows of ldq; null: no q here
+  long ldq;
+  int heads, DP;
+  T* q_abs;        // rotated part of the first n_abs tokens goes here
+  int n_abs;
+  const T* lat;    // [t, CP + RP], rows of ld_lat; null: no latent here
+  long ld_lat;
+  const T* kv_norm;
+  int kv_rank;
+  T* cache;
+  long n_slots;
+  const T* cq;     // [t, QP], rows of ld_lat; null: no query latent
+  const T* q_norm;
+  T* cq_out;
+  int QP, q_rank;
+};
+
+template <typename T>
+__device__ __forceinline__ float sum_squares(const T* v, int n) {
   float ss = 0.f;
-  for (int c = tid * 8; c < CP; c += 256 * 8) {
+  for (int c = threadIdx.x * 8; c < n; c += 256 * 8) {
     float f[8];
-    load8<T>(lat + c, f);
+    load8<T>(v + c, f);
 #pragma unroll
     for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
   }
-  ss = block_reduce(ss, tmp, SumOp{}, 0.f);
-  const long slot = slots[t];
-  if (slot < 0 || slot >= n_slots) return;
-  const float inv = 1.f / sqrtf(ss / (float)kv_rank + eps);
-  T* dst = cache + slot * (CP + RP);
-  for (int c = tid * 8; c < CP; c += 256 * 8) {
+  return ss;
+}
+
+template <typename T>
+__device__ __forceinline__ void scale_row(T* dst, const T* v, const T* w,
+                                          float inv, int n) {
+  for (int c = threadIdx.x * 8; c < n; c += 256 * 8) {
     float f[8], g[8];
-    load8<T>(lat + c, f);
-    load8<T>(kv_norm + c, g);
+    load8<T>(v + c, f);
+    load8<T>(w + c, g);
 #pragma unroll
     for (int e = 0; e < 8; ++e) f[e] = f[e] * inv * g[e];
     store8(dst + c, f);
   }
-  for (int p = tid; p < hp; p += 256) {
-    float u = to_f32(lat[CP + 2 * p]), v = to_f32(lat[CP + 2 * p + 1]);
-    if (p < pairs) {
-      const float a = u * cs[p] - v * sn[p];
-      v = v * cs[p] + u * sn[p];
-      u = a;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(
+    PrepArgs<T> a, const int* __restrict__ positions,
+    const int* __restrict__ slots, Rot rot, int RP, int CP, float eps) {
+  __shared__ float cs[256], sn[256];
+  __shared__ float tmp[16], tmp2[16];
+  const int t = blockIdx.x;
+  const int tid = threadIdx.x;
+  const int pairs = rot.pairs;
+  const float pos = (float)positions[t];
+  for (int i = tid; i < pairs; i += 256) {
+    float s, c;
+    sincosf(pos * rot.inv_freq[i], &s, &c);
+    cs[i] = rot.gain * c;
+    sn[i] = rot.gain * s;
+  }
+  __syncthreads();
+  const int hp = RP / 2;
+  if (a.q) {
+    T* row = a.q + (long)t * a.ldq;
+    const bool absorbed = t < a.n_abs;
+    const int q_pairs = absorbed ? hp : pairs;  // the rest passes unchanged
+    for (int i = tid; i < a.heads * q_pairs; i += 256) {
+      const int hd = i / q_pairs, p = i % q_pairs;
+      int ui, vi;
+      rot_places(rot, p, &ui, &vi);
+      T* src = row + hd * (a.DP + RP) + a.DP;
+      float u = to_f32(src[ui]), v = to_f32(src[vi]);
+      if (p < pairs) {
+        const float z = u * cs[p] - v * sn[p];
+        v = v * cs[p] + u * sn[p];
+        u = z;
+      }
+      T* dst = absorbed
+                   ? a.q_abs + ((long)t * a.heads + hd) * (CP + RP) + CP
+                   : src;
+      dst[ui] = from_f32<T>(u);
+      dst[vi] = from_f32<T>(v);
     }
-    dst[CP + 2 * p] = from_f32<T>(u);
-    dst[CP + 2 * p + 1] = from_f32<T>(v);
+  }
+  if (a.cq) {
+    const T* src = a.cq + (long)t * a.ld_lat;
+    const float ss =
+        block_reduce(sum_squares(src, a.QP), tmp2, SumOp{}, 0.f);
+    scale_row(a.cq_out + (long)t * a.QP, src, a.q_norm,
+              1.f / sqrtf(ss / (float)a.q_rank + eps), a.QP);
+  }
+  if (!a.lat) return;
+  const T* lat = a.lat + (long)t * a.ld_lat;
+  const float ss = block_reduce(sum_squares(lat, CP), tmp, SumOp{}, 0.f);
+  const long slot = slots[t];
+  if (slot < 0 || slot >= a.n_slots) return;
+  T* dst = a.cache + slot * (CP + RP);
+  scale_row(dst, lat, a.kv_norm, 1.f / sqrtf(ss / (float)a.kv_rank + eps),
+            CP);
+  for (int p = tid; p < hp; p += 256) {
+    int ui, vi;
+    rot_places(rot, p, &ui, &vi);
+    float u = to_f32(lat[CP + ui]), v = to_f32(lat[CP + vi]);
+    if (p < pairs) {
+      const float z = u * cs[p] - v * sn[p];
+      v = v * cs[p] + u * sn[p];
+      u = z;
+    }
+    dst[CP + ui] = from_f32<T>(u);
+    dst[CP + vi] = from_f32<T>(v);
   }
 }
 
@@ -101,14 +160,42 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
 // per-head product: out[t, h, :N] = a[t, h, :K] @ w[h]^T   (w [H, N, K])
 // one wave per 16 x 16 output tile; operands straight from L2/HBM
 // ------------------------------------------------------------------- //
+// gate: out *= sigmoid(gate[t, h * N + n]). rot: the last workgroup of a row
+// also turns a's RP elements behind K and puts them behind out's N.
 template <typename T>
 __global__ __launch_bounds__(256) void head_gemm_kernel(
     const T* __restrict__ a, long a_t, long a_h, const T* __restrict__ w,
-    T* __restrict__ out, long o_t, long o_h, int M, int N, int K) {
+    T* __restrict__ out, long o_t, long o_h, int M, int N, int K,
+    const T* __restrict__ gate, long g_t, Rot rot, int RP,
+    const int* __restrict__ positions) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int n0 = (blockIdx.x * 4 + wave) * 16;
   const int h = blockIdx.y;
   const int m0 = blockIdx.z * 16;
+  if (RP > 0 && blockIdx.x == gridDim.x - 1) {
+    const int hp = RP / 2;
+    for (int i = threadIdx.x; i < 16 * hp; i += 256) {
+      const int t = m0 + i / hp, p = i % hp;
+      if (t >= M) break;
+      int ui, vi;
+      rot_places(rot, p, &ui, &vi);
+      const T* src = a + (long)t * a_t + (long)h * a_h + K;
+      T* dst = out + (long)t * o_t + (long)h * o_h + N;
+      float u = to_f32(src[ui]), v = to_f32(src[vi]);
+      if (p < rot.pairs) {
+        float s, c;
+        sincosf((float)positions[t] * rot.inv_freq[p], &s, &c);
+        c *= rot.gain;
+        s *= rot.gain;
+        const float z = u * c - v * s;
+        v = v * c + u * s;
+        u = z;
+      }
+      dst[ui] = from_f32<T>(u);
+      dst[vi] = from_f32<T>(v);
+    }
+    return;
+  }
+  const int n0 = (blockIdx.x * 4 + wave) * 16;
   if (n0 >= N) return;
   const int r16 = lane & 15, ko = (lane >> 4) * 8;
   const T* wr = w + ((long)h * N + n0 + r16) * K + ko;
@@ -118,10 +205,15 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(
   for (int k = 0; k < K; k += 32)
     acc = mma32(load_frag(wr + k), load_frag(ar + k), acc);
   // C: row (n) = 4 * (lane >> 4) + r, column (token) = lane & 15
-  const int m = m0 + r16;
+  const int m = m0 + r16, n = n0 + 4 * (lane >> 4);
   if (m < M) {
-    const float f[4] = {acc[0], acc[1], acc[2], acc[3]};
-    store4(out + (long)m * o_t + (long)h * o_h + n0 + 4 * (lane >> 4), f);
+    float f[4] = {acc[0], acc[1], acc[2], acc[3]};
+    if (gate) {
+      const T* g = gate + (long)m * g_t + (long)h * N + n;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) f[r] *= sigmoid_f(to_f32(g[r]));
+    }
+    store4(out + (long)m * o_t + (long)h * o_h + n, f);
   }
 }
 
@@ -314,7 +406,8 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
         part_ml[2 * pi + 1] = l;
       }
     } else {
-      const float sk = to_f32(sink[h]) * LOG2E;
+      // without a sink: exp2(-inf) = 0
+      const float sk = sink ? to_f32(sink[h]) * LOG2E : -INFINITY;
       const float m_s = fmaxf(m, sk);
       const float e = __builtin_amdgcn_exp2f(m - m_s);
       const float inv = e / (l * e + __builtin_amdgcn_exp2f(sk - m_s));
@@ -331,8 +424,8 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(
     const T* __restrict__ sink, T* __restrict__ out, int splits, int H,
     int CP) {
   const long th = blockIdx.x;
-  const float sk = to_f32(sink[th % H]) * LOG2E;
-  float m = sk;
+  const float sk = sink ? to_f32(sink[th % H]) * LOG2E : -INFINITY;
+  float m = sk;  // some range has a key: m ends finite
   for (int s = 0; s < splits; ++s)
     m = fmaxf(m, part_ml[(th * splits + s) * 2]);
   float l = exp2f(sk - m);
@@ -357,64 +450,125 @@ __global__ __launch_bounds__(128) void latent_combine_kernel(
 
 }  // namespace
 
-void lm_latent_prep(torch::Tensor qkv, torch::Tensor positions,
-                    torch::Tensor slots, torch::Tensor inv_freq, long heads,
-                    long DP, long RP, long CP, long kv_rank, double eps,
-                    c10::optional<torch::Tensor> kv_norm,
-                    c10::optional<torch::Tensor> cache,
-                    c10::optional<torch::Tensor> q_abs, long n_abs) {
-  LM_CHECK_CONTIG(qkv);
-  LM_CHECK_I32(positions);
-  LM_CHECK_I32(slots);
+static Rot make_rot(const torch::Tensor& inv_freq, double gain, bool half,
+                    long RP) {
   LM_CHECK_CONTIG(inv_freq);
   TORCH_CHECK(inv_freq.scalar_type() == at::kFloat);
-  const int T = qkv.size(0), ld = qkv.size(1);
-  const int pairs = inv_freq.numel();
-  const bool own = kv_norm.has_value();
-  TORCH_CHECK(DP % 32 == 0 && RP % 32 == 0 && CP % 32 == 0);
+  const long pairs = inv_freq.numel();
   TORCH_CHECK(2 * pairs <= RP && pairs <= 256, "rotated size too large");
-  TORCH_CHECK(ld == heads * (DP + RP) + (own ? CP + RP : 0));
-  TORCH_CHECK(positions.numel() == T && slots.numel() == T);
-  TORCH_CHECK(n_abs >= 0 && n_abs <= T);
-  if (n_abs > 0) {
-    TORCH_CHECK(q_abs.has_value());
-    LM_CHECK_CONTIG(*q_abs);
-    TORCH_CHECK(q_abs->numel() == n_abs * heads * (CP + RP) &&
-                q_abs->scalar_type() == qkv.scalar_type());
-  }
-  long n_slots = 0;
-  if (own) {
-    TORCH_CHECK(cache.has_value());
-    LM_CHECK_CONTIG(*cache);
-    TORCH_CHECK(cache->dim() == 3 && cache->size(2) == CP + RP &&
-                cache->scalar_type() == qkv.scalar_type());
-    TORCH_CHECK(kv_norm->is_contiguous() && kv_norm->numel() == CP &&
-                kv_norm->scalar_type() == qkv.scalar_type());
-    n_slots = (long)cache->size(0) * cache->size(1);
-  }
-  if (T == 0) return;
-  LM_DISPATCH(qkv, "lm_latent_prep", [&] {
-    hipLaunchKernelGGL(
-        (latent_prep_kernel<scalar_t>), dim3(T), dim3(256), 0,
-        cmls::current_stream(), (scalar_t*)qkv.data_ptr(), ld,
-        positions.data_ptr<int>(), slots.data_ptr<int>(),
-        inv_freq.data_ptr<float>(), 2 * pairs, (int)heads, (int)DP, (int)RP,
-        (int)CP, (int)kv_rank, (float)eps,
-        own ? (const scalar_t*)kv_norm->data_ptr() : nullptr,
-        own ? (scalar_t*)cache->data_ptr() : nullptr, n_slots,
-        n_abs > 0 ? (scalar_t*)q_abs->data_ptr() : nullptr, (int)n_abs);
-  });
-  LM_LAUNCHED();
+  return Rot{inv_freq.data_ptr<float>(), (int)pairs, half ? 1 : 0,
+             (float)gain};
 }
 
-void lm_head_gemm(torch::Tensor a, torch::Tensor w, torch::Tensor out) {
+// [T, cols] view with 16-byte aligned rows
+static void check_rows(const torch::Tensor& v, long T, long cols,
+                       at::ScalarType type) {
+  TORCH_CHECK(v.is_cuda() && v.dim() == 2 && v.size(0) == T &&
+                  v.size(1) == cols && v.stride(1) == 1 &&
+                  v.stride(0) % 8 == 0 && v.storage_offset() % 8 == 0 &&
+                  v.scalar_type() == type,
+              "lm: operand rows do not fit");
+}
+
+// q [T, heads * (DP + RP)]; lat [T, CP + RP] with kv_norm and cache; cq
+// [T, QP] (same row stride as lat) with q_norm -> returned normed rows
+c10::optional<torch::Tensor> lm_latent_prep(
+    c10::optional<torch::Tensor> q, c10::optional<torch::Tensor> lat,
+    c10::optional<torch::Tensor> cq, torch::Tensor positions,
+    torch::Tensor slots, torch::Tensor inv_freq, double gain, bool half,
+    long heads, long DP, long RP, long CP, long kv_rank, double eps,
+    c10::optional<torch::Tensor> kv_norm, c10::optional<torch::Tensor> cache,
+    c10::optional<torch::Tensor> q_abs, long n_abs,
+    c10::optional<torch::Tensor> q_norm, long q_rank) {
+  LM_CHECK_I32(positions);
+  LM_CHECK_I32(slots);
+  const long T = positions.numel();
+  TORCH_CHECK(q.has_value() || lat.has_value());
+  const auto& any = q ? *q : *lat;
+  const auto type = any.scalar_type();
+  TORCH_CHECK(DP % 32 == 0 && RP % 32 == 0 && CP % 32 == 0);
+  const Rot rot = make_rot(inv_freq, gain, half, RP);
+  TORCH_CHECK(slots.numel() == T);
+  TORCH_CHECK(n_abs >= 0 && n_abs <= T);
+  if (q) check_rows(*q, T, heads * (DP + RP), type);
+  if (n_abs > 0) {
+    TORCH_CHECK(q.has_value() && q_abs.has_value());
+    LM_CHECK_CONTIG(*q_abs);
+    TORCH_CHECK(q_abs->numel() == n_abs * heads * (CP + RP) &&
+                q_abs->scalar_type() == type);
+  }
+  long n_slots = 0;
+  if (lat) {
+    check_rows(*lat, T, CP + RP, type);
+    TORCH_CHECK(cache.has_value() && kv_norm.has_value());
+    LM_CHECK_CONTIG(*cache);
+    TORCH_CHECK(cache->dim() == 3 && cache->size(2) == CP + RP &&
+                cache->scalar_type() == type);
+    TORCH_CHECK(kv_norm->is_contiguous() && kv_norm->numel() == CP &&
+                kv_norm->scalar_type() == type && kv_rank >= 1);
+    n_slots = (long)cache->size(0) * cache->size(1);
+  }
+  c10::optional<torch::Tensor> out;
+  long QP = 0;
+  if (cq) {
+    QP = cq->size(1);
+    TORCH_CHECK(lat.has_value() && QP % 8 == 0 && q_rank >= 1);
+    check_rows(*cq, T, QP, type);
+    TORCH_CHECK(T <= 1 || cq->stride(0) == lat->stride(0));
+    TORCH_CHECK(q_norm.has_value() && q_norm->is_contiguous() &&
+                q_norm->numel() == QP && q_norm->scalar_type() == type);
+    out = torch::empty({T, QP}, any.options());
+  }
+  if (T == 0) return out;
+  LM_DISPATCH(any, "lm_latent_prep", [&] {
+    PrepArgs<scalar_t> a{};
+    if (q) {
+      a.q = (scalar_t*)q->data_ptr();
+      a.ldq = q->stride(0);
+      a.heads = (int)heads;
+      a.DP = (int)DP;
+      a.q_abs = n_abs > 0 ? (scalar_t*)q_abs->data_ptr() : nullptr;
+      a.n_abs = (int)n_abs;
+    }
+    if (lat) {
+      a.lat = (const scalar_t*)lat->data_ptr();
+      a.ld_lat = lat->stride(0);
+      a.kv_norm = (const scalar_t*)kv_norm->data_ptr();
+      a.kv_rank = (int)kv_rank;
+      a.cache = (scalar_t*)cache->data_ptr();
+      a.n_slots = n_slots;
+    }
+    if (cq) {
+      a.cq = (const scalar_t*)cq->data_ptr();
+      a.q_norm = (const scalar_t*)q_norm->data_ptr();
+      a.cq_out = (scalar_t*)out->data_ptr();
+      a.QP = (int)QP;
+      a.q_rank = (int)q_rank;
+    }
+    hipLaunchKernelGGL((latent_prep_kernel<scalar_t>), dim3(T), dim3(256), 0,
+                       cmls::current_stream(), a, positions.data_ptr<int>(),
+                       slots.data_ptr<int>(), rot, (int)RP, (int)CP,
+                       (float)eps);
+  });
+  LM_LAUNCHED();
+  return out;
+}
+
+// with positions and inv_freq: a is [M, H, K + RP] and out [M, H, N + RP],
+// whose last RP elements are a's, turned
+void lm_head_gemm(torch::Tensor a, torch::Tensor w, torch::Tensor out,
+                  c10::optional<torch::Tensor> gate,
+                  c10::optional<torch::Tensor> positions,
+                  c10::optional<torch::Tensor> inv_freq, double gain,
+                  bool half, long RP) {
   LM_CHECK_CUDA(a);
   LM_CHECK_CUDA(out);
   LM_CHECK_CONTIG(w);
   TORCH_CHECK(a.dim() == 3 && w.dim() == 3 && out.dim() == 3);
-  const int M = a.size(0), H = a.size(1), K = a.size(2), N = w.size(1);
-  TORCH_CHECK(w.size(0) == H && w.size(2) == K);
-  TORCH_CHECK(out.size(0) == M && out.size(1) == H && out.size(2) == N);
+  const int M = a.size(0), H = a.size(1), K = w.size(2), N = w.size(1);
+  TORCH_CHECK(RP >= 0 && RP % 2 == 0);
+  TORCH_CHECK(w.size(0) == H && a.size(2) == K + RP);
+  TORCH_CHECK(out.size(0) == M && out.size(1) == H && out.size(2) == N + RP);
   TORCH_CHECK(a.stride(2) == 1 && out.stride(2) == 1);
   TORCH_CHECK(K % 32 == 0 && N % 16 == 0, "lm_head_gemm: K % 32, N % 16");
   TORCH_CHECK(a.stride(0) % 8 == 0 && a.stride(1) % 8 == 0 &&
@@ -422,16 +576,26 @@ void lm_head_gemm(torch::Tensor a, torch::Tensor w, torch::Tensor out) {
               a.storage_offset() % 8 == 0 && out.storage_offset() % 4 == 0);
   TORCH_CHECK(a.scalar_type() == w.scalar_type() &&
               out.scalar_type() == w.scalar_type());
+  Rot rot{nullptr, 0, 0, 1.f};
+  if (RP > 0) {
+    TORCH_CHECK(positions.has_value() && inv_freq.has_value());
+    LM_CHECK_I32(*positions);
+    TORCH_CHECK(positions->numel() >= M);
+    rot = make_rot(*inv_freq, gain, half, RP);
+  }
+  if (gate) check_rows(*gate, M, (long)H * N, w.scalar_type());
   if (M == 0) return;
   TORCH_CHECK((M + 15) / 16 <= 65535 && H <= 65535);
   LM_DISPATCH(w, "lm_head_gemm", [&] {
-    hipLaunchKernelGGL((head_gemm_kernel<scalar_t>),
-                       dim3((N + 63) / 64, H, (M + 15) / 16), dim3(256), 0,
-                       cmls::current_stream(),
-                       (const scalar_t*)a.data_ptr(), a.stride(0),
-                       a.stride(1), (const scalar_t*)w.data_ptr(),
-                       (scalar_t*)out.data_ptr(), out.stride(0),
-                       out.stride(1), M, N, K);
+    hipLaunchKernelGGL(
+        (head_gemm_kernel<scalar_t>),
+        dim3((N + 63) / 64 + (RP > 0 ? 1 : 0), H, (M + 15) / 16), dim3(256),
+        0, cmls::current_stream(), (const scalar_t*)a.data_ptr(), a.stride(0),
+        a.stride(1), (const scalar_t*)w.data_ptr(), (scalar_t*)out.data_ptr(),
+        out.stride(0), out.stride(1), M, N, K,
+        gate ? (const scalar_t*)gate->data_ptr() : nullptr,
+        gate ? gate->stride(0) : 0L, rot, (int)RP,
+        RP > 0 ? positions->data_ptr<int>() : nullptr);
   });
   LM_LAUNCHED();
 }
@@ -440,22 +604,26 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
                                   torch::Tensor block_table,
                                   torch::Tensor tok_seq,
                                   torch::Tensor positions,
-                                  torch::Tensor sink, double scale,
-                                  long window, long CP, long max_keys) {
+                                  c10::optional<torch::Tensor> sink,
+                                  double scale, long window, long CP,
+                                  long max_keys) {
   LM_CHECK_CONTIG(q_abs);
   LM_CHECK_CONTIG(cache);
   LM_CHECK_I32(block_table);
   LM_CHECK_I32(tok_seq);
   LM_CHECK_I32(positions);
-  LM_CHECK_CONTIG(sink);
   TORCH_CHECK(q_abs.dim() == 3 && cache.dim() == 3 && block_table.dim() == 2);
   const int n = q_abs.size(0), H = q_abs.size(1), ROW = q_abs.size(2);
   TORCH_CHECK(cache.size(2) == ROW && CP % 32 == 0 && ROW % 32 == 0 &&
               CP > 0 && CP < ROW);
   TORCH_CHECK(tok_seq.numel() >= n && positions.numel() >= n);
   TORCH_CHECK(n == 0 || block_table.numel() > 0);
-  TORCH_CHECK(sink.numel() == H && sink.scalar_type() == q_abs.scalar_type()
-              && cache.scalar_type() == q_abs.scalar_type());
+  TORCH_CHECK(cache.scalar_type() == q_abs.scalar_type());
+  if (sink) {
+    LM_CHECK_CONTIG(*sink);
+    TORCH_CHECK(sink->numel() == H &&
+                sink->scalar_type() == q_abs.scalar_type());
+  }
   auto out = torch::empty({n, H, CP}, q_abs.options());
   if (n == 0) return out;
   const int hg = (H + 15) / 16;
@@ -500,7 +668,7 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
                        (const scalar_t*)cache.data_ptr(),                    \
                        block_table.data_ptr<int>(), tok_seq.data_ptr<int>(), \
                        positions.data_ptr<int>(),                            \
-                       (const scalar_t*)sink.data_ptr(),                     \
+                       sink ? (const scalar_t*)sink->data_ptr() : nullptr,   \
                        (scalar_t*)out.data_ptr(),                            \
                        splits > 1 ? po.data_ptr<float>() : nullptr,          \
                        splits > 1 ? pml.data_ptr<float>() : nullptr,         \
@@ -524,7 +692,7 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
       hipLaunchKernelGGL((latent_combine_kernel<scalar_t>), dim3(n * H),
                          dim3(128), 0, st, po.data_ptr<float>(),
                          pml.data_ptr<float>(),
-                         (const scalar_t*)sink.data_ptr(),
+                         sink ? (const scalar_t*)sink->data_ptr() : nullptr,
                          (scalar_t*)out.data_ptr(), (int)splits, H, (int)CP);
   });
 #undef LM_LA

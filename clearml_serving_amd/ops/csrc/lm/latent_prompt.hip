@@ -23,6 +23,7 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
     const bf16* __restrict__ q, long q_t,   // q[t * q_t + h * QD]
     const bf16* __restrict__ kv, int ldkv,  // [rows, H*DP + H*VP]
     const bf16* __restrict__ rot, int ld_rot, const bf16* __restrict__ sink,
+    const bf16* __restrict__ gate, long ld_gate,  // [t, H*VP], null: none
     const int* __restrict__ qtiles, bf16* __restrict__ out, int H, int DP,
     int RP, int VP, int window, float scale) {
   constexpr int KP = QS * 32 + 8;   // LDS pitches
@@ -189,7 +190,7 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
   l_run += __shfl_xor(l_run, 16, 64);
   l_run += __shfl_xor(l_run, 32, 64);
   if (qrow < len) {
-    const float sk = __bfloat162float(sink[h]) * LOG2E;
+    const float sk = sink ? __bfloat162float(sink[h]) * LOG2E : -INFINITY;
     const float m_f = fmaxf(m_run, sk);
     const float e = exp2f(m_run - m_f);
     const float inv = e / (l_run * e + exp2f(sk - m_f));
@@ -197,8 +198,16 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
 #pragma unroll
     for (int i = 0; i < VT; ++i) {
       if (i * 16 < VP) {
-        const float f[4] = {acc[i][0] * inv, acc[i][1] * inv,
-                            acc[i][2] * inv, acc[i][3] * inv};
+        float f[4] = {acc[i][0] * inv, acc[i][1] * inv, acc[i][2] * inv,
+                      acc[i][3] * inv};
+        if (gate) {
+          union { uint2 u; bf16 b[4]; } gt;
+          gt.u = *reinterpret_cast<const uint2*>(
+              gate + (long)(t0 + qrow) * ld_gate + h * VP + i * 16 + 4 * g);
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            f[r] *= sigmoid_f(__bfloat162float(gt.b[r]));
+        }
         store4(dst + i * 16 + 4 * g, f);
       }
     }
@@ -208,18 +217,19 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
 }  // namespace
 
 // q [T, heads * (DP + RP)] (row stride free); kv [rows, H*(DP + VP)] =
-// [keys | values]; lat [rows, CP + RP]; out [T, H, VP]: rows of the tiles
+// [keys | values]; lat [rows, CP + RP]; gate [T, H * VP] (row stride free);
+// out [T, H, VP]: rows of the tiles
 void lm_latent_prompt(torch::Tensor q, torch::Tensor kv, torch::Tensor lat,
-                      torch::Tensor sink, torch::Tensor qtiles,
+                      c10::optional<torch::Tensor> sink, torch::Tensor qtiles,
                       torch::Tensor out, long H, long DP, long RP, long CP,
-                      long VP, long window, double scale) {
+                      long VP, long window, double scale,
+                      c10::optional<torch::Tensor> gate) {
   LM_CHECK_CUDA(q);
   LM_CHECK_CONTIG(kv);
   LM_CHECK_CONTIG(lat);
-  LM_CHECK_CONTIG(sink);
   LM_CHECK_CONTIG(out);
   LM_CHECK_I32(qtiles);
-  for (const auto* p : {&q, &kv, &lat, &sink, &out})
+  for (const auto* p : {&q, &kv, &lat, &out})
     TORCH_CHECK(p->scalar_type() == at::kBFloat16,
                 "lm_latent_prompt: bf16 only");
   const int QD = DP + RP;
@@ -229,7 +239,15 @@ void lm_latent_prompt(torch::Tensor q, torch::Tensor kv, torch::Tensor lat,
   TORCH_CHECK(kv.dim() == 2 && kv.size(1) == H * (DP + VP));
   TORCH_CHECK(lat.dim() == 2 && lat.size(1) == CP + RP &&
               lat.size(0) == kv.size(0));
-  TORCH_CHECK(sink.numel() == H);
+  if (sink) {
+    LM_CHECK_CONTIG(*sink);
+    TORCH_CHECK(sink->numel() == H && sink->scalar_type() == at::kBFloat16);
+  }
+  if (gate)
+    TORCH_CHECK(gate->is_cuda() && gate->scalar_type() == at::kBFloat16 &&
+                gate->dim() == 2 && gate->size(0) == q.size(0) &&
+                gate->size(1) == H * VP && gate->stride(1) == 1 &&
+                gate->stride(0) % 8 == 0 && gate->storage_offset() % 8 == 0);
   TORCH_CHECK(out.size(0) == q.size(0) && out.numel() == q.size(0) * H * VP);
   TORCH_CHECK(qtiles.dim() == 2 && qtiles.size(1) == 6);
   TORCH_CHECK(QD <= 256 && VP <= 256, "lm_latent_prompt: head too large");
@@ -242,7 +260,10 @@ void lm_latent_prompt(torch::Tensor q, torch::Tensor kv, torch::Tensor lat,
                      dim3(NW * 64), 0, st, (const bf16*)q.data_ptr(),        \
                      q.stride(0), (const bf16*)kv.data_ptr(),                \
                      (int)kv.size(1), (const bf16*)lat.data_ptr() + CP,      \
-                     (int)lat.size(1), (const bf16*)sink.data_ptr(),         \
+                     (int)lat.size(1),                                       \
+                     sink ? (const bf16*)sink->data_ptr() : nullptr,         \
+                     gate ? (const bf16*)gate->data_ptr() : nullptr,         \
+                     gate ? gate->stride(0) : 0L,                            \
                      qtiles.data_ptr<int>(), (bf16*)out.data_ptr(), (int)H,  \
                      (int)DP, (int)RP, (int)VP, (int)window, (float)scale)
 #define LM_LP_V(QS)                                                          \

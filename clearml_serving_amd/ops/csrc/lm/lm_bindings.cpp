@@ -4,24 +4,35 @@
 using Opt = c10::optional<torch::Tensor>;
 using torch::Tensor;
 
-std::vector<Tensor> lm_embed(Tensor tokens, Tensor table);
+std::vector<Tensor> lm_embed(Tensor tokens, Tensor table, Opt next_w,
+                             double off, long n, double eps, Opt out,
+                             Opt copy);
 Tensor lm_post_norm_add(Tensor o, Opt bias, Tensor w, Tensor x, long n,
-                        double eps);
+                        double eps, double off, Opt next_w, Opt out, Opt pos,
+                        Opt share);
+Tensor lm_add_norm(Tensor x, Tensor add, Opt next_w, double off, long n,
+                   double eps);
 Tensor lm_output_norm(Tensor x, Opt rows, Tensor w, long n, double eps,
-                      double scale);
-Tensor lm_gelu_mul(Tensor gu, Opt bias);
+                      double scale, double off);
+Tensor lm_gated_mul(Tensor gu, Opt bias, long act);
 Tensor lm_gather_rows(Tensor src, Tensor idx);
-void lm_latent_prep(Tensor qkv, Tensor positions, Tensor slots,
-                    Tensor inv_freq, long heads, long DP, long RP, long CP,
-                    long kv_rank, double eps, Opt kv_norm, Opt cache,
-                    Opt q_abs, long n_abs);
-void lm_head_gemm(Tensor a, Tensor w, Tensor out);
+Opt lm_latent_prep(Opt q, Opt lat, Opt cq, Tensor positions, Tensor slots,
+                   Tensor inv_freq, double gain, bool half, long heads,
+                   long DP, long RP, long CP, long kv_rank, double eps,
+                   Opt kv_norm, Opt cache, Opt q_abs, long n_abs, Opt q_norm,
+                   long q_rank);
+void lm_head_gemm(Tensor a, Tensor w, Tensor out, Opt gate, Opt positions,
+                  Opt inv_freq, double gain, bool half, long RP);
 Tensor lm_latent_attention(Tensor q_abs, Tensor cache, Tensor block_table,
-                           Tensor tok_seq, Tensor positions, Tensor sink,
+                           Tensor tok_seq, Tensor positions, Opt sink,
                            double scale, long window, long CP, long max_keys);
-void lm_latent_prompt(Tensor q, Tensor kv, Tensor lat, Tensor sink,
+void lm_latent_prompt(Tensor q, Tensor kv, Tensor lat, Opt sink,
                       Tensor qtiles, Tensor out, long H, long DP, long RP,
-                      long CP, long VP, long window, double scale);
+                      long CP, long VP, long window, double scale, Opt gate);
+std::vector<Tensor> lm_moe_route(Tensor h, Tensor router, long top,
+                                 long rows);
+Tensor lm_moe_gemm(Tensor a, Opt tok, Tensor w, Tensor plan, long n_rows,
+                   long rows, long act);
 void lm_rglru_prefill(Tensor yx, Tensor byx, Tensor cw, Tensor cb, Tensor ra,
                       Tensor ba, Tensor ri, Tensor bi, Tensor lam,
                       Tensor state, Tensor ring, Tensor tiles, Tensor seqs,
@@ -37,12 +48,15 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("lm_embed", &lm_embed);
   m.def("lm_post_norm_add", &lm_post_norm_add);
   m.def("lm_output_norm", &lm_output_norm);
-  m.def("lm_gelu_mul", &lm_gelu_mul);
+  m.def("lm_add_norm", &lm_add_norm);
+  m.def("lm_gated_mul", &lm_gated_mul);
   m.def("lm_gather_rows", &lm_gather_rows);
   m.def("lm_latent_prep", &lm_latent_prep);
   m.def("lm_head_gemm", &lm_head_gemm);
   m.def("lm_latent_attention", &lm_latent_attention);
   m.def("lm_latent_prompt", &lm_latent_prompt);
+  m.def("lm_moe_route", &lm_moe_route);
+  m.def("lm_moe_gemm", &lm_moe_gemm);
   m.def("lm_rglru_prefill", &lm_rglru_prefill);
   m.def("lm_rglru_step", &lm_rglru_step);
   m.def("skinny_gemm", &skinny_gemm, py::arg("a"), py::arg("w"),

@@ -186,6 +186,14 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
   const float k = 0.7978845608028654f * (z + 0.044715f * z * z * z);
   return z * sigmoid_f(2.f * k);
 }
+// activations that kernels take as a template argument
+enum { LM_GELU_TANH = 0, LM_SILU = 1, LM_RELU2 = 2, LM_NO_ACT = 3 };
+template <int ACT> __device__ __forceinline__ float act_f(float z) {
+  if (ACT == LM_GELU_TANH) return gelu_tanh_f(z);
+  if (ACT == LM_SILU) return z * sigmoid_f(z);
+  if (ACT == LM_RELU2) return z > 0.f ? z * z : 0.f;
+  return z;
+}
 // 1 - exp(v) for v <= 0: the power series where the difference would cancel
 __device__ __forceinline__ float one_minus_exp_f(float v) {
   const float p =

@@ -1,45 +1,117 @@
-// Residual-stream kernels: embedding, norm-on-output with residual add,
-// output norm, gated GELU.
+// Residual-stream kernels: embedding, norm-on-output with residual add, the
+// norm in front of the next sublayer, output norm, gated activation.
 //
-// The residual x is float; each step that changes it also writes the copy in
-// the matrix-product type that the next projection reads, so x makes one
-// round trip to HBM per sublayer.
+// The residual x is float; each step that changes it also writes what the
+// next projection reads (a copy of x, or its norm) in the matrix-product type,
+// so x makes one round trip to HBM per sublayer.
+//
+// Rows are `width` (padded) elements of which `n` count; the pad is zero.
+// Norm weights are stored around `off` = 0 or, with off = 1, around zero.
+// NV: 8-element vectors of a row that a thread keeps in registers.
 #include "lm_common.h"
 
 namespace {
 
-template <typename T>
-__global__ __launch_bounds__(256) void embed_kernel(
-    const long* __restrict__ tokens, const T* __restrict__ table,
-    float* __restrict__ x, T* __restrict__ h, int width, long vocab) {
-  const long t = blockIdx.x;
-  long id = tokens[t];
-  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
-  for (int c = threadIdx.x * 8; c < width; c += 256 * 8) {
-    float f[8];
-    load8<T>(table + id * width + c, f);
-    store8(x + t * width + c, f);
-    if (h) store8(h + t * width + c, f);
-  }
-}
-
-// x += (o + bias) / rms(o + bias) * (1 + w); h = x. Rows of `width`
-// (padded) elements of which `n` count; the pad is zero in o, bias and w.
-// NV: 8-element vectors a thread keeps in registers.
+// h = x, or with a weight x / rms(x) * (off + w), for a row in registers
 template <typename T, int NV>
-__global__ __launch_bounds__(256) void post_norm_add_kernel(
-    const T* __restrict__ o, const T* __restrict__ bias,
-    const T* __restrict__ w, float* __restrict__ x, T* __restrict__ h,
-    int width, int n, float eps) {
-  __shared__ float tmp[16];
-  const long row = (long)blockIdx.x * width;
-  float v[NV][8];
-  float ss = 0.f;
+__device__ __forceinline__ void write_next(const float (&r)[NV][8],
+                                           const T* __restrict__ w, float off,
+                                           T* __restrict__ h, int width,
+                                           int n, float eps, float* tmp) {
+  float inv = 1.f;
+  if (w) {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      if ((i * 256 + (int)threadIdx.x) * 8 < width) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += r[i][e] * r[i][e];
+      }
+    }
+    ss = block_reduce(ss, tmp, SumOp{}, 0.f);
+    inv = 1.f / sqrtf(ss / (float)n + eps);
+  }
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int c = (i * 256 + threadIdx.x) * 8;
     if (c < width) {
-      load8<T>(o + row + c, v[i]);
+      float f[8];
+      if (w) {
+        load8<T>(w + c, f);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) f[e] = r[i][e] * inv * (off + f[e]);
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) f[e] = r[i][e];
+      }
+      store8(h + c, f);
+    }
+  }
+}
+
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void embed_kernel(
+    const long* __restrict__ tokens, const T* __restrict__ table,
+    float* __restrict__ x, T* __restrict__ h, long ld_h,
+    T* __restrict__ copy, long ld_copy, const T* __restrict__ next_w,
+    float off, int width, int n, float eps, long vocab) {
+  __shared__ float tmp[16];
+  const long t = blockIdx.x;
+  long id = tokens[t];
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  float v[NV][8];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 8;
+    if (c < width) {
+      load8<T>(table + id * width + c, v[i]);
+      store8(x + t * width + c, v[i]);
+      if (copy) store8(copy + t * ld_copy + c, v[i]);
+    }
+  }
+  if (h)
+    write_next<T, NV>(v, next_w, off, h + t * ld_h, width, n, eps, tmp);
+}
+
+// x += v / rms(v) * (off + w), h from the new x; v = o + bias or, MIX, the
+// sum over a token's `top` slots of share * o[pos]
+template <typename T, int NV, bool MIX>
+__global__ __launch_bounds__(256) void post_norm_add_kernel(
+    const T* __restrict__ o, const T* __restrict__ bias,
+    const int* __restrict__ pos, const float* __restrict__ share, int top,
+    int n_rows, const T* __restrict__ w, float off, float* __restrict__ x,
+    const T* __restrict__ next_w, T* __restrict__ h, long ld_h, int width,
+    int n, float eps) {
+  __shared__ float tmp[16];
+  __shared__ float tmp2[16];
+  const long t = blockIdx.x, row = t * width;
+  float v[NV][8];
+  float ss = 0.f;
+  if (MIX) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[i][e] = 0.f;
+    for (int k = 0; k < top; ++k) {
+      const long p = min(max(pos[t * top + k], 0), n_rows - 1);
+      const float s = share[t * top + k];
+#pragma unroll
+      for (int i = 0; i < NV; ++i) {
+        const int c = (i * 256 + threadIdx.x) * 8;
+        if (c < width) {
+          float f[8];
+          load8<T>(o + p * width + c, f);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) v[i][e] += s * f[e];
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 8;
+    if (c < width) {
+      if (!MIX) load8<T>(o + row + c, v[i]);
       if (bias) {
         float b[8];
         load8<T>(bias + c, b);
@@ -60,19 +132,44 @@ __global__ __launch_bounds__(256) void post_norm_add_kernel(
       load8<T>(w + c, g);
       load8<float>(x + row + c, r);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) r[e] += v[i][e] * inv * (1.f + g[e]);
-      store8(x + row + c, r);
-      if (h) store8(h + row + c, r);
+      for (int e = 0; e < 8; ++e) v[i][e] = r[e] + v[i][e] * inv * (off + g[e]);
+      store8(x + row + c, v[i]);
     }
   }
+  if (h)
+    write_next<T, NV>(v, next_w, off, h + t * ld_h, width, n, eps, tmp2);
 }
 
-// out[i] = norm(x[rows[i]]) * (1 + w) * scale
+// x += add (one vector for all rows); h from the new x
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void add_norm_kernel(
+    float* __restrict__ x, const T* __restrict__ add,
+    const T* __restrict__ next_w, float off, T* __restrict__ h, int width,
+    int n, float eps) {
+  __shared__ float tmp[16];
+  const long row = (long)blockIdx.x * width;
+  float v[NV][8];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 8;
+    if (c < width) {
+      float a[8];
+      load8<T>(add + c, a);
+      load8<float>(x + row + c, v[i]);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[i][e] += a[e];
+      store8(x + row + c, v[i]);
+    }
+  }
+  write_next<T, NV>(v, next_w, off, h + row, width, n, eps, tmp);
+}
+
+// out[i] = norm(x[rows[i]]) * (off + w) * scale
 template <typename T>
 __global__ __launch_bounds__(256) void output_norm_kernel(
     const float* __restrict__ x, const int* __restrict__ rows,
     const T* __restrict__ w, T* __restrict__ out, int width, int n,
-    int n_tok, float eps, float scale) {
+    int n_tok, float eps, float scale, float off) {
   __shared__ float tmp[16];
   int r = rows ? rows[blockIdx.x] : (int)blockIdx.x;
   r = min(max(r, 0), n_tok - 1);
@@ -91,14 +188,14 @@ __global__ __launch_bounds__(256) void output_norm_kernel(
     load8<float>(src + c, f);
     load8<T>(w + c, g);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) f[e] = f[e] * inv * (1.f + g[e]) * scale;
+    for (int e = 0; e < 8; ++e) f[e] = f[e] * inv * (off + g[e]) * scale;
     store8(out + (long)blockIdx.x * width + c, f);
   }
 }
 
-// gu = [gate | up] rows of 2*ff; out = gelu_tanh(gate + bg) * (up + bu)
-template <typename T>
-__global__ __launch_bounds__(256) void gelu_mul_kernel(
+// gu = [gate | up] rows of 2*ff; out = act(gate + bg) * (up + bu)
+template <typename T, int ACT>
+__global__ __launch_bounds__(256) void gated_mul_kernel(
     const T* __restrict__ gu, const T* __restrict__ bias,
     T* __restrict__ out, int ff) {
   const long t = blockIdx.x;
@@ -115,7 +212,7 @@ __global__ __launch_bounds__(256) void gelu_mul_kernel(
     for (int e = 0; e < 8; ++e) { g[e] += bg[e]; u[e] += bu[e]; }
   }
 #pragma unroll
-  for (int e = 0; e < 8; ++e) g[e] = gelu_tanh_f(g[e]) * u[e];
+  for (int e = 0; e < 8; ++e) g[e] = act_f<ACT>(g[e]) * u[e];
   store8(out + t * ff + c, g);
 }
 
@@ -136,67 +233,150 @@ __global__ __launch_bounds__(256) void gather_rows_kernel(
 
 }  // namespace
 
-std::vector<torch::Tensor> lm_embed(torch::Tensor tokens,
-                                    torch::Tensor table) {
+// rows of 8-element vectors per thread -> template argument NV
+#define LM_NV(WIDTH, CALL)                         \
+  do {                                             \
+    const int nv_ = ((WIDTH) + 2047) / 2048;       \
+    if (nv_ <= 1) { CALL(1); }                     \
+    else if (nv_ <= 2) { CALL(2); }                \
+    else if (nv_ <= 4) { CALL(4); }                \
+    else { CALL(8); }                              \
+  } while (0)
+
+// [T, width] view whose rows are 16-byte aligned; -> row stride
+static long row_view(const torch::Tensor& v, long rows, long width,
+                     at::ScalarType type) {
+  TORCH_CHECK(v.is_cuda() && v.dim() == 2 && v.size(0) == rows &&
+                  v.size(1) == width && v.stride(1) == 1 &&
+                  v.stride(0) % 8 == 0 && v.storage_offset() % 8 == 0 &&
+                  v.scalar_type() == type,
+              "lm: output rows do not fit");
+  return v.stride(0);
+}
+
+static void check_weight(const c10::optional<torch::Tensor>& w, long width,
+                         at::ScalarType type) {
+  if (!w.has_value()) return;
+  LM_CHECK_CONTIG(*w);
+  TORCH_CHECK(w->numel() == width && w->scalar_type() == type);
+}
+
+// -> {x, h}. h: the next projection's input, into `out` if given; `copy`
+// receives the rows as they are.
+std::vector<torch::Tensor> lm_embed(torch::Tensor tokens, torch::Tensor table,
+                                    c10::optional<torch::Tensor> next_w,
+                                    double off, long n, double eps,
+                                    c10::optional<torch::Tensor> out,
+                                    c10::optional<torch::Tensor> copy) {
   LM_CHECK_CONTIG(tokens);
   LM_CHECK_CONTIG(table);
   TORCH_CHECK(tokens.scalar_type() == at::kLong && tokens.dim() == 1);
   const int T = tokens.size(0), width = table.size(1);
-  TORCH_CHECK(width % 8 == 0, "lm_embed: width % 8");
+  TORCH_CHECK(width % 8 == 0 && width <= 16384, "lm_embed: width");
+  TORCH_CHECK(n >= 1 && n <= width);
+  const auto type = table.scalar_type();
+  check_weight(next_w, width, type);
   auto x = torch::empty({T, width}, table.options().dtype(at::kFloat));
-  // in 32-bit runs the stream itself is the projection input
-  auto h = table.scalar_type() == at::kFloat ? x : torch::empty(
-      {T, width}, table.options());
+  // in 32-bit runs the stream itself can be the projection input
+  const bool alias = type == at::kFloat && !next_w && !out;
+  auto h = out ? *out : alias ? x : torch::empty({T, width}, table.options());
+  const long ld_h = row_view(h, T, width, type);
+  const long ld_c = copy ? row_view(*copy, T, width, type) : 0;
   if (T == 0) return {x, h};
-  LM_DISPATCH(table, "lm_embed", [&] {
-    scalar_t* hp = h.data_ptr() == x.data_ptr() ? nullptr
-                                                : (scalar_t*)h.data_ptr();
-    hipLaunchKernelGGL((embed_kernel<scalar_t>), dim3(T), dim3(256), 0,
-                       cmls::current_stream(), tokens.data_ptr<long>(),
-                       (const scalar_t*)table.data_ptr(),
-                       x.data_ptr<float>(), hp, width, (long)table.size(0));
-  });
+#define LM_EMBED(NV)                                                         \
+  hipLaunchKernelGGL((embed_kernel<scalar_t, NV>), dim3(T), dim3(256), 0,    \
+                     cmls::current_stream(), tokens.data_ptr<long>(),        \
+                     (const scalar_t*)table.data_ptr(), x.data_ptr<float>(), \
+                     alias ? nullptr : (scalar_t*)h.data_ptr(), ld_h,        \
+                     copy ? (scalar_t*)copy->data_ptr() : nullptr, ld_c,     \
+                     next_w ? (const scalar_t*)next_w->data_ptr() : nullptr, \
+                     (float)off, width, (int)n, (float)eps,                  \
+                     (long)table.size(0))
+  LM_DISPATCH(table, "lm_embed", [&] { LM_NV(width, LM_EMBED); });
+#undef LM_EMBED
   LM_LAUNCHED();
   return {x, h};
 }
 
+// o: [T, width], or with pos, share [T, top] the rows they pick and weigh
 torch::Tensor lm_post_norm_add(torch::Tensor o,
                                c10::optional<torch::Tensor> bias,
                                torch::Tensor w, torch::Tensor x, long n,
-                               double eps) {
+                               double eps, double off,
+                               c10::optional<torch::Tensor> next_w,
+                               c10::optional<torch::Tensor> out,
+                               c10::optional<torch::Tensor> pos,
+                               c10::optional<torch::Tensor> share) {
   LM_CHECK_CONTIG(o);
   LM_CHECK_CONTIG(w);
   LM_CHECK_CONTIG(x);
-  const int T = o.size(0), width = o.size(1);
-  TORCH_CHECK(x.scalar_type() == at::kFloat && x.sizes() == o.sizes());
-  TORCH_CHECK(w.numel() == width && w.scalar_type() == o.scalar_type());
+  TORCH_CHECK(o.dim() == 2 && x.dim() == 2);
+  const int T = x.size(0), width = x.size(1);
+  const auto type = o.scalar_type();
+  TORCH_CHECK(x.scalar_type() == at::kFloat && o.size(1) == width);
+  TORCH_CHECK(w.numel() == width && w.scalar_type() == type);
   TORCH_CHECK(width % 8 == 0 && n >= 1 && n <= width);
   TORCH_CHECK(width <= 16384, "lm_post_norm_add: width > 16384");
-  if (bias.has_value()) {
-    LM_CHECK_CONTIG(*bias);
-    TORCH_CHECK(bias->numel() == width &&
-                bias->scalar_type() == o.scalar_type());
+  check_weight(bias, width, type);
+  check_weight(next_w, width, type);
+  int top = 0;
+  if (pos) {
+    TORCH_CHECK(share.has_value());
+    LM_CHECK_I32(*pos);
+    LM_CHECK_CONTIG(*share);
+    TORCH_CHECK(pos->dim() == 2 && pos->size(0) == T &&
+                share->sizes() == pos->sizes() &&
+                share->scalar_type() == at::kFloat);
+    TORCH_CHECK(T == 0 || o.size(0) > 0);
+    top = pos->size(1);
+  } else {
+    TORCH_CHECK(o.size(0) == T);
   }
-  const bool own = o.scalar_type() != at::kFloat;
-  auto h = own ? torch::empty_like(o) : x;
+  const bool alias = type == at::kFloat && !next_w && !out;
+  auto h = out ? *out : alias ? x : torch::empty({T, width}, o.options());
+  const long ld_h = row_view(h, T, width, type);
   if (T == 0) return h;
-  const int nv = (width + 2047) / 2048;
-#define LM_PN(NV)                                                           \
-  hipLaunchKernelGGL((post_norm_add_kernel<scalar_t, NV>), dim3(T),         \
+#define LM_PN_(NV, MIX)                                                     \
+  hipLaunchKernelGGL((post_norm_add_kernel<scalar_t, NV, MIX>), dim3(T),    \
                      dim3(256), 0, cmls::current_stream(),                  \
                      (const scalar_t*)o.data_ptr(),                         \
-                     bias.has_value() ? (const scalar_t*)bias->data_ptr()   \
-                                      : nullptr,                            \
-                     (const scalar_t*)w.data_ptr(), x.data_ptr<float>(),    \
-                     own ? (scalar_t*)h.data_ptr() : nullptr, width, (int)n,\
-                     (float)eps)
-  LM_DISPATCH(o, "lm_post_norm_add", [&] {
-    if (nv <= 1) LM_PN(1);
-    else if (nv <= 2) LM_PN(2);
-    else if (nv <= 4) LM_PN(4);
-    else LM_PN(8);
-  });
+                     bias ? (const scalar_t*)bias->data_ptr() : nullptr,    \
+                     pos ? pos->data_ptr<int>() : nullptr,                  \
+                     share ? share->data_ptr<float>() : nullptr, top,       \
+                     (int)o.size(0), (const scalar_t*)w.data_ptr(),         \
+                     (float)off, x.data_ptr<float>(),                       \
+                     next_w ? (const scalar_t*)next_w->data_ptr() : nullptr,\
+                     alias ? nullptr : (scalar_t*)h.data_ptr(), ld_h,       \
+                     width, (int)n, (float)eps)
+#define LM_PN(NV) do { if (pos) LM_PN_(NV, true); else LM_PN_(NV, false); } while (0)
+  LM_DISPATCH(o, "lm_post_norm_add", [&] { LM_NV(width, LM_PN); });
 #undef LM_PN
+#undef LM_PN_
+  LM_LAUNCHED();
+  return h;
+}
+
+torch::Tensor lm_add_norm(torch::Tensor x, torch::Tensor add,
+                          c10::optional<torch::Tensor> next_w, double off,
+                          long n, double eps) {
+  LM_CHECK_CONTIG(x);
+  LM_CHECK_CONTIG(add);
+  TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2);
+  const int T = x.size(0), width = x.size(1);
+  TORCH_CHECK(add.numel() == width && width % 8 == 0 && width <= 16384);
+  TORCH_CHECK(n >= 1 && n <= width);
+  check_weight(next_w, width, add.scalar_type());
+  auto h = torch::empty({T, width}, add.options());
+  if (T == 0) return h;
+#define LM_AN(NV)                                                           \
+  hipLaunchKernelGGL((add_norm_kernel<scalar_t, NV>), dim3(T), dim3(256),   \
+                     0, cmls::current_stream(), x.data_ptr<float>(),        \
+                     (const scalar_t*)add.data_ptr(),                       \
+                     next_w ? (const scalar_t*)next_w->data_ptr() : nullptr,\
+                     (float)off, (scalar_t*)h.data_ptr(), width, (int)n,    \
+                     (float)eps)
+  LM_DISPATCH(add, "lm_add_norm", [&] { LM_NV(width, LM_AN); });
+#undef LM_AN
   LM_LAUNCHED();
   return h;
 }
@@ -204,7 +384,7 @@ torch::Tensor lm_post_norm_add(torch::Tensor o,
 torch::Tensor lm_output_norm(torch::Tensor x,
                              c10::optional<torch::Tensor> rows,
                              torch::Tensor w, long n, double eps,
-                             double scale) {
+                             double scale, double off) {
   LM_CHECK_CONTIG(x);
   LM_CHECK_CONTIG(w);
   TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2);
@@ -223,33 +403,33 @@ torch::Tensor lm_output_norm(torch::Tensor x,
                        rows.has_value() ? rows->data_ptr<int>() : nullptr,
                        (const scalar_t*)w.data_ptr(),
                        (scalar_t*)out.data_ptr(), width, (int)n,
-                       (int)x.size(0), (float)eps, (float)scale);
+                       (int)x.size(0), (float)eps, (float)scale, (float)off);
   });
   LM_LAUNCHED();
   return out;
 }
 
-torch::Tensor lm_gelu_mul(torch::Tensor gu,
-                          c10::optional<torch::Tensor> bias) {
+// act: 0 tanh-form GELU, 1 SiLU
+torch::Tensor lm_gated_mul(torch::Tensor gu, c10::optional<torch::Tensor> bias,
+                           long act) {
   LM_CHECK_CONTIG(gu);
   TORCH_CHECK(gu.dim() == 2 && gu.size(1) % 16 == 0);
+  TORCH_CHECK(act == LM_GELU_TANH || act == LM_SILU);
   const int T = gu.size(0), ff = gu.size(1) / 2;
-  if (bias.has_value()) {
-    LM_CHECK_CONTIG(*bias);
-    TORCH_CHECK(bias->numel() == 2 * ff &&
-                bias->scalar_type() == gu.scalar_type());
-  }
+  check_weight(bias, 2 * ff, gu.scalar_type());
   auto out = torch::empty({T, ff}, gu.options());
   if (T == 0) return out;
-  LM_DISPATCH(gu, "lm_gelu_mul", [&] {
-    hipLaunchKernelGGL((gelu_mul_kernel<scalar_t>),
-                       dim3(T, (ff / 8 + 255) / 256), dim3(256), 0,
-                       cmls::current_stream(),
-                       (const scalar_t*)gu.data_ptr(),
-                       bias.has_value() ? (const scalar_t*)bias->data_ptr()
-                                        : nullptr,
-                       (scalar_t*)out.data_ptr(), ff);
+#define LM_GM(ACT)                                                          \
+  hipLaunchKernelGGL((gated_mul_kernel<scalar_t, ACT>),                     \
+                     dim3(T, (ff / 8 + 255) / 256), dim3(256), 0,           \
+                     cmls::current_stream(), (const scalar_t*)gu.data_ptr(),\
+                     bias ? (const scalar_t*)bias->data_ptr() : nullptr,    \
+                     (scalar_t*)out.data_ptr(), ff)
+  LM_DISPATCH(gu, "lm_gated_mul", [&] {
+    if (act == LM_SILU) LM_GM(LM_SILU);
+    else LM_GM(LM_GELU_TANH);
   });
+#undef LM_GM
   LM_LAUNCHED();
   return out;
 }

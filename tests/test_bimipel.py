@@ -301,8 +301,8 @@ def test_rotation_far_positions(device, dtype, tol):
     slots = torch.tensor([0, 5, 7, -1], dtype=torch.int32)
     q_abs = torch.zeros(2, heads, cp + rp, dtype=dtype).to(device)
     dev = qkv.clone().to(device)
-    lm.latent_prep(dev, pos.to(device), slots.to(device), inv.to(device),
-                   heads, dp, rp, cp, 20, 1e-5,
+    lm.latent_prep(dev, pos.to(device), slots.to(device),
+                   lm.Rotary(inv.to(device)), heads, dp, rp, cp, 20, 1e-5,
                    torch.ones(cp, dtype=dtype).to(device), cache, q_abs)
     t = 1e-3 if dtype == torch.float32 else 2e-2
     q = ref[:, :heads * (dp + rp)].view(4, heads, dp + rp)
