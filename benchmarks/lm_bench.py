@@ -1,5 +1,6 @@
-"""Prefill and decode throughput of the token-batch family (Bimipel) beside
-llama at equal size, random weights, through the LLM engine's own forwards.
+"""Prefill and decode throughput of the token-batch families (Kakipel,
+Bimipel) beside llama at equal size, random weights, through the LLM engine's
+own forwards.
 
     python bench.py --workload lm [--lm-size 300m,1b,4k] [--lm-model ...]
 
@@ -15,14 +16,17 @@ import time
 import torch
 
 SIZES = {
-    # size -> (bimipel preset, llama preset, llama overrides)
-    "300m": ("bimipel-300m", "llama-3-8b", dict(
-        vocab_size=32000, hidden=1024, layers=12, heads=16, kv_heads=4,
-        intermediate=3584)),
-    "1b": ("bimipel-1b", "llama-3-1b", {}),
-    # six layers as wide as an 8B model's
-    "4k": ("bimipel-4k", "llama-3-8b", dict(vocab_size=32000, layers=6,
-                                            intermediate=12288)),
+    # size -> model -> (preset, overrides)
+    "300m": {"kakipel": ("kakipel-300m", {}), "bimipel": ("bimipel-300m", {}),
+             "llama": ("llama-3-8b", dict(
+                 vocab_size=32000, hidden=1024, layers=12, heads=16,
+                 kv_heads=4, intermediate=3584))},
+    "1b": {"kakipel": ("kakipel-1b", {}), "bimipel": ("bimipel-1b", {}),
+           "llama": ("llama-3-1b", {})},
+    # few layers, as wide as an 8B model's
+    "4k": {"kakipel": ("kakipel-4k", {}), "bimipel": ("bimipel-4k", {}),
+           "llama": ("llama-3-8b", dict(vocab_size=32000, layers=6,
+                                        intermediate=12288))},
 }
 
 
@@ -37,12 +41,10 @@ def _engine(kind, size, batch, max_len):
     from clearml_serving_amd.engines.llm.engine import (LlmEngine,
                                                         LlmEngineConfig)
 
-    bim, preset, over = SIZES[size]
+    preset, over = SIZES[size][kind]
     blocks = max(batch, 1) * (-(-max_len // 16) + 1)
     cfg = LlmEngineConfig(
-        arch="bimipel" if kind == "bimipel" else "llama",
-        preset=bim if kind == "bimipel" else preset,
-        overrides={} if kind == "bimipel" else dict(over),
+        arch=kind, preset=preset, overrides=dict(over),
         max_num_seqs=batch, max_model_len=max_len, num_kv_blocks=blocks,
         device="cuda:0" if torch.cuda.is_available() else "cpu")
     eng = LlmEngine(cfg)

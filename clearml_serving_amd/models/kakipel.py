@@ -223,7 +223,7 @@ PRESETS = {
                          6144, 1536, 16, 4, (2, 4, 3)),
     # layers as wide as an 8B model's
     "kakipel-4k": _stack(32000, 4096, _attn(32, 96, 32, 96, 1536, 512), 4,
-                         12288, 3072, 16, 4, (0, 2, 2)),
+                         12288, 2560, 16, 4, (0, 2, 2)),
 }
 
 

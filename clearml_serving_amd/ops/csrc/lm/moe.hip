@@ -12,8 +12,13 @@
 
 namespace {
 
-constexpr int RT = 16;   // tokens per routing workgroup
-constexpr int RW = 8;    // its waves; they split the inner dimension
+// The wave's number, as a scalar. An MFMA ignores the lane mask, so a branch
+// around one has to be a scalar branch.
+__device__ __forceinline__ int uniform_wave() {
+  return __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+}
+
+constexpr int RT = 16;  // tokens per routing workgroup
 constexpr int MAX_TOP = 64;
 
 // Rows and tiles in front of each expert, by a whole workgroup (>= 64
@@ -56,99 +61,121 @@ __device__ void scan_experts(const int* tot, int* off, int E, int rows,
   }
 }
 
+// partial logits of 16 tokens and NE * 16 experts over [k_lo, k_hi); a result
+// row is an expert, a column (lane & 15) a token
+template <typename T, int NE>
+__device__ __forceinline__ void router_tiles(const T* hr, const T* router,
+                                             int e0, int E, int K, int k_lo,
+                                             int k_hi, float* part) {
+  const int lane = threadIdx.x & 63, r16 = lane & 15, g = lane >> 4;
+  lm_f32x4 acc[NE];
+  const T* wr[NE];
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    acc[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
+    wr[i] = router + (long)min(e0 + i * 16 + r16, E - 1) * K;
+  }
+#pragma unroll 4
+  for (int k = k_lo; k < k_hi; k += 32) {
+    const Frag<T> hf = load_frag(hr + k);
+#pragma unroll
+    for (int i = 0; i < NE; ++i)
+      acc[i] = mma32(load_frag(wr[i] + k), hf, acc[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < NE; ++i) {
+    const float f[4] = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
+    store4(part + i * 16 + 4 * g, f);
+  }
+}
+
 // Logits in float, the `top` largest (ties: the lower expert), softmax over
 // them. Counts per expert and each slot's rank in it for the grouping; a
-// single workgroup groups right away.
-template <typename T>
-__global__ __launch_bounds__(RW * 64) void moe_route_kernel(
+// single workgroup groups right away. KW: waves, which split the inner
+// dimension.
+template <typename T, int KW>
+__global__ __launch_bounds__(KW * 64) void moe_route_kernel(
     const T* __restrict__ h, const T* __restrict__ router, int n_tok, int K,
     int E, int top, float* __restrict__ share, int* __restrict__ ids,
     int* __restrict__ rank, int* __restrict__ counts, int* __restrict__ pos,
     int* __restrict__ tok, int rows, int* __restrict__ tiles,
     int* __restrict__ n_tiles) {
-  __shared__ __align__(16) float part[RW][RT][64 + 4];
-  __shared__ int chosen[RT][MAX_TOP];
+  constexpr int NTH = KW * 64;
+  constexpr int PER = RT * MAX_TOP / NTH;  // most slots of a thread
+  __shared__ __align__(16) float part[KW][RT][64 + 4];
   extern __shared__ __align__(16) char smem[];
-  float* logits = (float*)smem;         // [RT][E]
-  int* cnt = (int*)(logits + RT * E);   // [E]
-  int* off = cnt + E;                   // [E]
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int r16 = lane & 15, g = lane >> 4, ko = g * 8;
+  const int EP = (E + 3) & ~3;
+  float* logits = (float*)smem;            // [RT][EP]
+  float* best = logits + RT * EP;          // [RT][top]
+  int* chosen = (int*)(best + RT * top);   // [RT][top]
+  int* cnt = chosen + RT * top;            // [E]
+  int* off = cnt + E;                      // [E]
+  const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave();
+  const int r16 = lane & 15, ko = (lane >> 4) * 8;
   const int t0 = blockIdx.x * RT;
   const int nt = min(RT, n_tok - t0);
-  for (int e = tid; e < E; e += RW * 64) cnt[e] = 0;
+  for (int e = tid; e < E; e += NTH) cnt[e] = 0;
+  // whatever the logits are (nan), every slot has an expert
+  for (int i = tid; i < RT * top; i += NTH) {
+    chosen[i] = i % top;
+    best[i] = 0.f;
+  }
 
   const T* hr = h + (long)min(t0 + r16, n_tok - 1) * K + ko;
-  const int steps = K / 32, per = (steps + RW - 1) / RW;
+  const int steps = K / 32, per = (steps + KW - 1) / KW;
   const int k_lo = wave * per * 32, k_hi = min(K, k_lo + per * 32);
   for (int e0 = 0; e0 < E; e0 += 64) {
-    lm_f32x4 acc[4];
-    const T* wr[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      acc[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
-      wr[i] = router + (long)min(e0 + i * 16 + r16, E - 1) * K + ko;
-    }
-#pragma unroll 4
-    for (int k = k_lo; k < k_hi; k += 32) {
-      const Frag<T> hf = load_frag(hr + k);
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        if (e0 + i * 16 < E) acc[i] = mma32(load_frag(wr[i] + k), hf, acc[i]);
-    }
-    // result rows are experts 4g..4g+3 of a tile, columns tokens
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const float f[4] = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
-      store4(&part[wave][r16][i * 16 + 4 * g], f);
-    }
+    const T* wr = router + ko;
+    if (E - e0 <= 16)
+      router_tiles<T, 1>(hr, wr, e0, E, K, k_lo, k_hi, &part[wave][r16][0]);
+    else if (E - e0 <= 32)
+      router_tiles<T, 2>(hr, wr, e0, E, K, k_lo, k_hi, &part[wave][r16][0]);
+    else
+      router_tiles<T, 4>(hr, wr, e0, E, K, k_lo, k_hi, &part[wave][r16][0]);
     __syncthreads();
-    for (int i = tid; i < RT * 64; i += RW * 64) {
-      const int t = i >> 6, e = i & 63;
+    for (int i = tid; i < RT * 64; i += NTH) {
+      const int t = i >> 6, e = e0 + (i & 63);
       float s = 0.f;
 #pragma unroll
-      for (int w = 0; w < RW; ++w) s += part[w][t][e];
-      if (e0 + e < E) logits[t * E + e0 + e] = s;
+      for (int w = 0; w < KW; ++w) s += part[w][t][i & 63];
+      if (e < EP) logits[t * EP + e] = e < E ? s : -INFINITY;
     }
     __syncthreads();
   }
 
-  for (int t = wave; t < nt; t += RW) {
-    float* z = logits + t * E;
-    float mine = 0.f, first = 0.f;
-    int my_id = 0;
-    for (int k = 0; k < top; ++k) {
-      float best = -INFINITY;
-      int at = E - 1;
-      for (int e = lane; e < E; e += 64)
-        if (z[e] > best) { best = z[e]; at = e; }
+  // an expert's place is the number of experts in front of it
+  for (int t = wave; t < nt; t += KW) {
+    const float* z = logits + t * EP;
+    for (int e = lane; e < E; e += 64) {
+      const float mine = z[e];
+      int place = 0;
+#pragma unroll 4
+      for (int j = 0; j < EP; j += 4) {
+        const lm_f32x4 o = *reinterpret_cast<const lm_f32x4*>(z + j);
 #pragma unroll
-      for (int d = 32; d > 0; d >>= 1) {
-        const float b = __shfl_xor(best, d, 64);
-        const int i = __shfl_xor(at, d, 64);
-        if (b > best || (b == best && i < at)) { best = b; at = i; }
+        for (int r = 0; r < 4; ++r)
+          place += o[r] > mine || (o[r] == mine && j + r < e);
       }
-      if (k == 0) first = best;
-      if (lane == k) { mine = best; my_id = at; }
-      if (lane == 0) z[at] = -INFINITY;
-      wave_lds_fence();
+      if (place < top) {
+        chosen[t * top + place] = e;
+        best[t * top + place] = mine;
+      }
     }
-    const float e = lane < top ? expf(mine - first) : 0.f;
-    const float sum = wave_reduce_sum(e);
-    if (lane < top) {
-      share[(long)(t0 + t) * top + lane] = e / sum;
-      chosen[t][lane] = my_id;
-    }
+    wave_lds_fence();
+    const float v = lane < top ? expf(best[t * top + lane] - best[t * top])
+                               : 0.f;
+    const float sum = wave_reduce_sum(v);
+    if (lane < top) share[(long)(t0 + t) * top + lane] = v / sum;
   }
   __syncthreads();
   const bool alone = gridDim.x == 1;
-  int rk[RT * MAX_TOP / (RW * 64)];
+  int rk[PER];
 #pragma unroll
-  for (int j = 0; j < RT * MAX_TOP / (RW * 64); ++j) {
-    const int s = tid + j * RW * 64;
+  for (int j = 0; j < PER; ++j) {
+    const int s = tid + j * NTH;
     rk[j] = 0;
     if (s < nt * top) {
-      const int e = chosen[s / top][s % top];
+      const int e = chosen[s];
       rk[j] = atomicAdd(&cnt[e], 1);
       if (!alone) {
         ids[(long)t0 * top + s] = e;
@@ -158,16 +185,16 @@ __global__ __launch_bounds__(RW * 64) void moe_route_kernel(
   }
   __syncthreads();
   if (!alone) {
-    for (int e = tid; e < E; e += RW * 64)
+    for (int e = tid; e < E; e += NTH)
       counts[(long)blockIdx.x * E + e] = cnt[e];
     return;
   }
   scan_experts(cnt, off, E, rows, tiles, n_tiles);
 #pragma unroll
-  for (int j = 0; j < RT * MAX_TOP / (RW * 64); ++j) {
-    const int s = tid + j * RW * 64;
+  for (int j = 0; j < PER; ++j) {
+    const int s = tid + j * NTH;
     if (s < nt * top) {
-      const int p = off[chosen[s / top][s % top]] + rk[j];
+      const int p = off[chosen[s]] + rk[j];
       pos[s] = p;
       tok[p] = s / top;
     }
@@ -213,25 +240,29 @@ __global__ __launch_bounds__(256) void moe_place_kernel(
 }
 
 // ------------------------------------------------------------------- //
-// grouped product, few rows per expert: 16 columns and up to 16 * MT rows per
-// workgroup, operands straight from memory, waves split the inner dimension
+// grouped product, few rows per expert: 16 * NT columns and up to 16 * MT rows
+// per workgroup, operands straight from memory, waves split the inner
+// dimension
 // ------------------------------------------------------------------- //
 constexpr int GW = 8;
 
-template <typename T, int MT, int ACT>
+template <typename T, int MT, int NT, int ACT>
 __global__ __launch_bounds__(GW * 64) void moe_rows_kernel(
     const T* __restrict__ a, const int* __restrict__ tok,  // null: row = row
     const T* __restrict__ w, T* __restrict__ out,
     const int* __restrict__ tiles, const int* __restrict__ n_tiles, int N,
     int K, int n_rows, int n_a) {
-  __shared__ __align__(16) float part[GW][MT][16][16 + 4];
+  __shared__ __align__(16) float part[GW][MT * 16][NT * 16 + 4];
   if ((int)blockIdx.y >= n_tiles[0]) return;
   const int* td = tiles + (long)blockIdx.y * 3;
   const int e = td[0], r0 = td[1], cnt = td[2];
-  const int n0 = blockIdx.x * 16;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int n0 = blockIdx.x * (NT * 16);
+  const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave();
   const int r16 = lane & 15, g = lane >> 4, ko = g * 8;
-  const T* wr = w + ((long)e * N + n0 + r16) * K + ko;
+  const T* wr[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i)
+    wr[i] = w + ((long)e * N + n0 + i * 16 + r16) * K + ko;
   const T* ar[MT];
 #pragma unroll
   for (int i = 0; i < MT; ++i) {
@@ -239,31 +270,64 @@ __global__ __launch_bounds__(GW * 64) void moe_rows_kernel(
     const int row = tok ? tok[p] : p;
     ar[i] = a + (long)min(row, n_a - 1) * K + ko;
   }
-  lm_f32x4 acc[MT];
+  lm_f32x4 acc[MT][NT];
 #pragma unroll
-  for (int i = 0; i < MT; ++i) acc[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int i = 0; i < MT; ++i)
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[i][j] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
   const int per = (K / 32 + GW - 1) / GW;
   const int k_lo = wave * per * 32, k_hi = min(K, k_lo + per * 32);
-#pragma unroll 4
-  for (int k = k_lo; k < k_hi; k += 32) {
-    const Frag<T> wf = load_frag(wr + k);
+  // U steps of operands in registers, the next U on their way
+  constexpr int U = 4;
+  Frag<T> wf[2][U][NT], af[2][U][MT];
+  auto load = [&](int b, int k0) {
 #pragma unroll
-    for (int i = 0; i < MT; ++i)
-      acc[i] = mma32(wf, load_frag(ar[i] + k), acc[i]);
+    for (int u = 0; u < U; ++u) {
+      const int k = k0 + u * 32;
+      if (k < k_hi) {
+#pragma unroll
+        for (int j = 0; j < NT; ++j) wf[b][u][j] = load_frag(wr[j] + k);
+#pragma unroll
+        for (int i = 0; i < MT; ++i) af[b][u][i] = load_frag(ar[i] + k);
+      }
+    }
+  };
+  auto multiply = [&](int b, int k0) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (k0 + u * 32 < k_hi) {
+#pragma unroll
+        for (int i = 0; i < MT; ++i)
+#pragma unroll
+          for (int j = 0; j < NT; ++j)
+            acc[i][j] = mma32(wf[b][u][j], af[b][u][i], acc[i][j]);
+      }
+    }
+  };
+  load(0, k_lo);
+  for (int k = k_lo; k < k_hi; k += 2 * U * 32) {
+    load(1, k + U * 32);
+    multiply(0, k);
+    load(0, k + 2 * U * 32);
+    multiply(1, k + U * 32);
   }
 #pragma unroll
   for (int i = 0; i < MT; ++i) {
-    const float f[4] = {acc[i][0], acc[i][1], acc[i][2], acc[i][3]};
-    store4(&part[wave][i][r16][4 * g], f);
+#pragma unroll
+    for (int j = 0; j < NT; ++j) {
+      const float f[4] = {acc[i][j][0], acc[i][j][1], acc[i][j][2],
+                          acc[i][j][3]};
+      store4(&part[wave][i * 16 + r16][j * 16 + 4 * g], f);
+    }
   }
   __syncthreads();
-  for (int i = tid; i < MT * 64; i += GW * 64) {
-    const int m = i >> 2, c = (i & 3) * 4;
+  for (int i = tid; i < MT * NT * 64; i += GW * 64) {
+    const int m = i / (NT * 4), c = (i % (NT * 4)) * 4;
     if (m >= cnt) break;
     lm_f32x4 s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int v = 0; v < GW; ++v)
-      s += *reinterpret_cast<const lm_f32x4*>(&part[v][m >> 4][m & 15][c]);
+      s += *reinterpret_cast<const lm_f32x4*>(&part[v][m][c]);
     const float f[4] = {act_f<ACT>(s[0]), act_f<ACT>(s[1]), act_f<ACT>(s[2]),
                         act_f<ACT>(s[3])};
     store4(out + (long)(r0 + m) * N + n0 + c, f);
@@ -271,18 +335,38 @@ __global__ __launch_bounds__(GW * 64) void moe_rows_kernel(
 }
 
 // ------------------------------------------------------------------- //
-// grouped product, many rows per expert (bf16): BM x BN tiles, inner steps of
-// 64 through two LDS buffers filled by direct-to-LDS loads
+// grouped product on BM x BN tiles (bf16): inner steps of 64 through NS LDS
+// buffers filled by direct-to-LDS loads
 // ------------------------------------------------------------------- //
 // The loads write LDS in lane order, so the 16-byte pieces of a row are
 // permuted by (row & 7) at the source and again at the read: fragment reads
 // touch all banks. The weights are the first MFMA operand: a lane then holds
-// four neighbouring columns of one row of the result.
+// four neighbouring columns of one row of the result. One barrier per step:
+// it says that step i's buffer is full and that everyone is done with step
+// i - 1's, which is filled next.
 constexpr int BK = 64;
 
-template <int BM, int BN, int WM, int WN, int ACT>
+// Direct-to-LDS load of 16 bytes per lane, lane l to lds + 16 l. As assembly:
+// the compiler would wait for all of them in front of every LDS read, since it
+// cannot tell the buffers apart. wait_loads says when a step has landed.
+__device__ __forceinline__ void load_to_lds(const bf16* src, unsigned lds) {
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\t"
+               "global_load_lds_dwordx4 %1, off"
+               ::"s"(lds), "v"(src)
+               : "m0", "memory");
+}
+// until at most N of the wave's loads are in flight
+template <int N> __device__ __forceinline__ void wait_loads() {
+  static_assert(N < 64, "six bits");
+  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
+}
+__device__ __forceinline__ unsigned lds_address(const void* p) {
+  return (unsigned)(size_t)(__attribute__((address_space(3))) const char*)p;
+}
+
+template <int BM, int BN, int WM, int WN, int NS, int ACT>
 __global__ __launch_bounds__(WM * WN * 64,
-                             2 * BK * (BM + BN) * 2 > 80 * 1024
+                             NS * BK * (BM + BN) * 2 > 80 * 1024
                                  ? WM * WN / 4 : WM * WN / 2)
 void moe_tile_kernel(
     const bf16* __restrict__ a, const int* __restrict__ tok,
@@ -292,8 +376,9 @@ void moe_tile_kernel(
   constexpr int NTH = WM * WN * 64;
   constexpr int FM = BM / WM / 16, FN = BN / WN / 16;
   constexpr int IA = BM * 8 / NTH, IB = BN * 8 / NTH;
-  __shared__ __align__(16) short la[2][BM * BK];
-  __shared__ __align__(16) short lb[2][BN * BK];
+  static_assert(IA * NTH == BM * 8 && IB * NTH == BN * 8, "whole pieces");
+  __shared__ __align__(16) short la[NS][BM * BK];
+  __shared__ __align__(16) short lb[NS][BN * BK];
   const int nb = (N + BN - 1) / BN;
   const int nwg = n_tiles[0] * nb;
   if ((int)blockIdx.x >= nwg) return;
@@ -305,7 +390,7 @@ void moe_tile_kernel(
   const int* td = tiles + (long)(bid / nb) * 3;
   const int e = td[0], r0 = td[1], cnt = td[2];
   const int n0 = (bid % nb) * BN;
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave();
   const int r16 = lane & 15, g = lane >> 4;
   const int wm = (wave / WN) * (BM / WM), wn = (wave % WN) * (BN / WN);
 
@@ -325,19 +410,15 @@ void moe_tile_kernel(
     const int n = min(n0 + ((i * NTH + tid) >> 3), N - 1);
     pb[i] = w + ((long)e * N + n) * K + piece;
   }
+  const unsigned a_lds = lds_address(la) + wave * 1024;
+  const unsigned b_lds = lds_address(lb) + wave * 1024;
   auto stage = [&](int buf, int k) {
 #pragma unroll
-    for (int i = 0; i < IA; ++i)
-      __builtin_amdgcn_global_load_lds(
-          reinterpret_cast<const unsigned int*>(pa[i] + k),
-          reinterpret_cast<unsigned int*>(&la[buf][(i * NTH + tid) * 8]), 16,
-          0, 0);
-#pragma unroll
     for (int i = 0; i < IB; ++i)
-      __builtin_amdgcn_global_load_lds(
-          reinterpret_cast<const unsigned int*>(pb[i] + k),
-          reinterpret_cast<unsigned int*>(&lb[buf][(i * NTH + tid) * 8]), 16,
-          0, 0);
+      load_to_lds(pb[i] + k, b_lds + (buf * BN * 8 + i * NTH) * 16);
+#pragma unroll
+    for (int i = 0; i < IA; ++i)
+      load_to_lds(pa[i] + k, a_lds + (buf * BM * 8 + i * NTH) * 16);
   };
 
   lm_f32x4 acc[FN][FM];
@@ -346,12 +427,19 @@ void moe_tile_kernel(
 #pragma unroll
     for (int j = 0; j < FM; ++j) acc[i][j] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
 
-  stage(0, 0);
-  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-  __syncthreads();
+  // Steps behind the last one load the last step's pieces again, into a
+  // buffer that nobody reads any more: the count of loads in flight stays
+  // the same for every step. All have landed before the workgroup ends.
+  const int last = K - BK;
+#pragma unroll
+  for (int i = 0; i < NS - 1; ++i) stage(i, min(i * BK, last));
   int cur = 0;
   for (int k = 0; k < K; k += BK) {
-    if (k + BK < K) stage(cur ^ 1, k + BK);
+    wait_loads<(NS - 2) * (IA + IB)>();
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+    if (NS > 2 || k + BK < K)
+      stage(cur == 0 ? NS - 1 : cur - 1, min(k + (NS - 1) * BK, last));
 #pragma unroll
     for (int kc = 0; kc < 2; ++kc) {
       const int s = ((kc * 4 + g) ^ (r16 & 7)) * 8;
@@ -373,10 +461,9 @@ void moe_tile_kernel(
               fb[i], fa[j], acc[i][j], 0, 0, 0);
       __builtin_amdgcn_s_setprio(0);
     }
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();
-    cur ^= 1;
+    cur = cur == NS - 1 ? 0 : cur + 1;
   }
+  wait_loads<0>();
 
 #pragma unroll
   for (int j = 0; j < FM; ++j) {
@@ -433,29 +520,36 @@ std::vector<torch::Tensor> lm_moe_route(torch::Tensor h, torch::Tensor router,
   }
   int* pp = plan.data_ptr<int>();
   hipStream_t st = cmls::current_stream();
+#define LM_MRT(KW)                                                           \
+  do {                                                                       \
+    const int bytes =                                                        \
+        (RT * (((E + 3) & ~3) + 2 * (int)top) + 2 * E) * 4;                  \
+    auto* fn = &moe_route_kernel<scalar_t, KW>;                              \
+    HIP_CHECK(hipFuncSetAttribute(                                           \
+        reinterpret_cast<const void*>(fn),                                   \
+        hipFuncAttributeMaxDynamicSharedMemorySize, bytes));                 \
+    hipLaunchKernelGGL(fn, dim3(n_wg), dim3(KW * 64), bytes, st,             \
+                       (const scalar_t*)h.data_ptr(),                        \
+                       (const scalar_t*)router.data_ptr(), T, K, E,          \
+                       (int)top, share.data_ptr<float>(),                    \
+                       n_wg > 1 ? ids.data_ptr<int>() : nullptr,             \
+                       n_wg > 1 ? rank.data_ptr<int>() : nullptr,            \
+                       n_wg > 1 ? counts.data_ptr<int>() : nullptr,          \
+                       pos.data_ptr<int>(), tok.data_ptr<int>(), (int)rows,  \
+                       pp + 1, pp);                                          \
+  } while (0)
   LM_DISPATCH(h, "lm_moe_route", [&] {
-    const int bytes = (RT * E + 2 * E) * 4;
-    auto* fn = &moe_route_kernel<scalar_t>;
-    HIP_CHECK(hipFuncSetAttribute(reinterpret_cast<const void*>(fn),
-                                  hipFuncAttributeMaxDynamicSharedMemorySize,
-                                  bytes));
-    hipLaunchKernelGGL(fn, dim3(n_wg), dim3(RW * 64), bytes, st,
-                       (const scalar_t*)h.data_ptr(),
-                       (const scalar_t*)router.data_ptr(), T, K, E, (int)top,
-                       share.data_ptr<float>(),
-                       n_wg > 1 ? ids.data_ptr<int>() : nullptr,
-                       n_wg > 1 ? rank.data_ptr<int>() : nullptr,
-                       n_wg > 1 ? counts.data_ptr<int>() : nullptr,
-                       pos.data_ptr<int>(), tok.data_ptr<int>(), (int)rows,
-                       pp + 1, pp);
+    if (n_wg <= 256) LM_MRT(16);  // few workgroups: short chains of loads
+    else LM_MRT(8);
   });
+#undef LM_MRT
   LM_LAUNCHED();
   if (n_wg > 1) {
-    hipLaunchKernelGGL(moe_place_kernel, dim3(n_wg), dim3(256), 3 * E * 4, st,
-                       ids.data_ptr<int>(), rank.data_ptr<int>(),
-                       counts.data_ptr<int>(), n_wg, T, E, (int)top,
-                       pos.data_ptr<int>(), tok.data_ptr<int>(), (int)rows,
-                       pp + 1, pp);
+    hipLaunchKernelGGL(moe_place_kernel, dim3(n_wg), dim3(256),
+                       3 * E * 4, st, ids.data_ptr<int>(),
+                       rank.data_ptr<int>(), counts.data_ptr<int>(), n_wg, T,
+                       E, (int)top, pos.data_ptr<int>(), tok.data_ptr<int>(),
+                       (int)rows, pp + 1, pp);
     LM_LAUNCHED();
   }
   return {share, pos, tok, plan};
@@ -491,41 +585,42 @@ torch::Tensor lm_moe_gemm(torch::Tensor a, c10::optional<torch::Tensor> tok,
 #define LM_MG_ARGS(TY)                                                      \
   (const TY*)a.data_ptr(), tk, (const TY*)w.data_ptr(), (TY*)out.data_ptr(),\
       pp + 1, pp, N, K, (int)n_rows, (int)a.size(0)
-  if (rows >= 128) {
-    TORCH_CHECK(a.scalar_type() == at::kBFloat16 && K % BK == 0,
-                "lm_moe_gemm: large tiles take bf16 and K % 64 == 0");
-#define LM_MT(BM, BN, WM, WN, ACT)                                          \
+  if (rows != 16 && a.scalar_type() == at::kBFloat16 && K % BK == 0) {
+#define LM_MT(BM, BN, WM, WN, NS, ACT)                                      \
   do {                                                                      \
     const long wgs = nt * ((N + BN - 1) / BN);                              \
     TORCH_CHECK(wgs < (1L << 31));                                          \
-    hipLaunchKernelGGL((moe_tile_kernel<BM, BN, WM, WN, ACT>), dim3(wgs),   \
-                       dim3(WM * WN * 64), 0, st, LM_MG_ARGS(bf16));        \
+    hipLaunchKernelGGL((moe_tile_kernel<BM, BN, WM, WN, NS, ACT>),          \
+                       dim3(wgs), dim3(WM * WN * 64), 0, st,                \
+                       LM_MG_ARGS(bf16));                                   \
   } while (0)
-#define LM_MT_ACT(BM, BN, WM, WN)                                           \
+#define LM_MT_ACT(BM, BN, WM, WN, NS)                                       \
   do {                                                                      \
-    if (act == LM_RELU2) LM_MT(BM, BN, WM, WN, LM_RELU2);                   \
-    else LM_MT(BM, BN, WM, WN, LM_NO_ACT);                                  \
+    if (act == LM_RELU2) LM_MT(BM, BN, WM, WN, NS, LM_RELU2);               \
+    else LM_MT(BM, BN, WM, WN, NS, LM_NO_ACT);                              \
   } while (0)
-    if (rows == 256) LM_MT_ACT(256, 256, 2, 4);
-    else if (rows == 128) LM_MT_ACT(128, 128, 2, 2);
-    else TORCH_CHECK(false, "lm_moe_gemm: 128 or 256 rows");
+    if (rows == 256) LM_MT_ACT(256, 256, 2, 4, 2);
+    else if (rows == 128) LM_MT_ACT(128, 128, 2, 2, 2);
+    else if (rows == 64) LM_MT_ACT(64, 64, 2, 2, 4);
+    else if (rows == 32) LM_MT_ACT(32, 64, 1, 4, 4);
+    else TORCH_CHECK(false, "lm_moe_gemm: rows per tile");
 #undef LM_MT_ACT
 #undef LM_MT
   } else {
     TORCH_CHECK(nt <= 65535);
-#define LM_MR(MT, ACT)                                                      \
-  hipLaunchKernelGGL((moe_rows_kernel<scalar_t, MT, ACT>), dim3(N / 16, nt),\
-                     dim3(GW * 64), 0, st, LM_MG_ARGS(scalar_t))
-#define LM_MR_ACT(MT)                                                       \
+#define LM_MR(MT, NT, ACT)                                                  \
+  hipLaunchKernelGGL((moe_rows_kernel<scalar_t, MT, NT, ACT>),              \
+                     dim3(N / (16 * NT), nt), dim3(GW * 64), 0, st,         \
+                     LM_MG_ARGS(scalar_t))
+#define LM_MR_ACT(MT, NT)                                                   \
   do {                                                                      \
-    if (act == LM_RELU2) LM_MR(MT, LM_RELU2);                               \
-    else LM_MR(MT, LM_NO_ACT);                                              \
+    if (act == LM_RELU2) LM_MR(MT, NT, LM_RELU2);                           \
+    else LM_MR(MT, NT, LM_NO_ACT);                                          \
   } while (0)
     LM_DISPATCH(a, "lm_moe_gemm", [&] {
-      if (rows == 16) LM_MR_ACT(1);
-      else if (rows == 32) LM_MR_ACT(2);
-      else if (rows == 64) LM_MR_ACT(4);
-      else TORCH_CHECK(false, "lm_moe_gemm: 16, 32 or 64 rows");
+      if (rows == 16) LM_MR_ACT(1, 1);
+      else if (rows == 64) LM_MR_ACT(4, 2);
+      else TORCH_CHECK(false, "lm_moe_gemm: rows per tile");
     });
 #undef LM_MR_ACT
 #undef LM_MR

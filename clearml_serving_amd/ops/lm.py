@@ -410,12 +410,13 @@ def expert_tile_rows(n_tok: int, experts: int, top: int, dtype,
                      inner: Tuple[int, ...]) -> int:
     """rows per tile for a batch size; ``inner``: the products' inner sizes"""
     each = n_tok * top / experts
-    if each <= 12:
+    if dtype != torch.bfloat16 or any(k % 64 for k in inner):
+        return 16 if each <= 12 else 64
+    if n_tok * top <= 8:  # few tiles: small column ranges fill the chip
         return 16
-    if each <= 24:
+    if each <= 20:
         return 32
-    if (each <= 48 or dtype != torch.bfloat16
-            or any(k % 64 for k in inner)):
+    if each <= 72:
         return 64
     return 128 if each <= 512 else 256
 
