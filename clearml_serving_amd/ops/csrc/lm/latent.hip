@@ -62,22 +62,20 @@ struct PrepArgs {
   int QP, q_rank;
 };
 
+// dst = v / rms(v) * w by one wave; `count` of the `n` elements are real
 template <typename T>
-__device__ __forceinline__ float sum_squares(const T* v, int n) {
+__device__ __forceinline__ void wave_norm(T* dst, const T* v, const T* w,
+                                          int n, int count, float eps) {
+  const int lane = threadIdx.x & 63;
   float ss = 0.f;
-  for (int c = threadIdx.x * 8; c < n; c += 256 * 8) {
+  for (int c = lane * 8; c < n; c += 64 * 8) {
     float f[8];
     load8<T>(v + c, f);
 #pragma unroll
     for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
   }
-  return ss;
-}
-
-template <typename T>
-__device__ __forceinline__ void scale_row(T* dst, const T* v, const T* w,
-                                          float inv, int n) {
-  for (int c = threadIdx.x * 8; c < n; c += 256 * 8) {
+  const float inv = 1.f / sqrtf(wave_reduce_sum(ss) / (float)count + eps);
+  for (int c = lane * 8; c < n; c += 64 * 8) {
     float f[8], g[8];
     load8<T>(v + c, f);
     load8<T>(w + c, g);
@@ -87,29 +85,35 @@ __device__ __forceinline__ void scale_row(T* dst, const T* v, const T* w,
   }
 }
 
+// one wave per token
+constexpr int PREP_W = 4;
+
 template <typename T>
-__global__ __launch_bounds__(256) void latent_prep_kernel(
+__global__ __launch_bounds__(PREP_W * 64) void latent_prep_kernel(
     PrepArgs<T> a, const int* __restrict__ positions,
-    const int* __restrict__ slots, Rot rot, int RP, int CP, float eps) {
-  __shared__ float cs[256], sn[256];
-  __shared__ float tmp[16], tmp2[16];
-  const int t = blockIdx.x;
-  const int tid = threadIdx.x;
+    const int* __restrict__ slots, Rot rot, int RP, int CP, float eps,
+    int n_tok) {
+  __shared__ float trig[PREP_W][2][256];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int t = blockIdx.x * PREP_W + wave;
+  if (t >= n_tok) return;  // no barrier below
+  float* cs = trig[wave][0];
+  float* sn = trig[wave][1];
   const int pairs = rot.pairs;
   const float pos = (float)positions[t];
-  for (int i = tid; i < pairs; i += 256) {
+  for (int i = lane; i < pairs; i += 64) {
     float s, c;
     sincosf(pos * rot.inv_freq[i], &s, &c);
     cs[i] = rot.gain * c;
     sn[i] = rot.gain * s;
   }
-  __syncthreads();
+  wave_lds_fence();
   const int hp = RP / 2;
   if (a.q) {
     T* row = a.q + (long)t * a.ldq;
     const bool absorbed = t < a.n_abs;
     const int q_pairs = absorbed ? hp : pairs;  // the rest passes unchanged
-    for (int i = tid; i < a.heads * q_pairs; i += 256) {
+    for (int i = lane; i < a.heads * q_pairs; i += 64) {
       const int hd = i / q_pairs, p = i % q_pairs;
       int ui, vi;
       rot_places(rot, p, &ui, &vi);
@@ -127,22 +131,16 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(
       dst[vi] = from_f32<T>(v);
     }
   }
-  if (a.cq) {
-    const T* src = a.cq + (long)t * a.ld_lat;
-    const float ss =
-        block_reduce(sum_squares(src, a.QP), tmp2, SumOp{}, 0.f);
-    scale_row(a.cq_out + (long)t * a.QP, src, a.q_norm,
-              1.f / sqrtf(ss / (float)a.q_rank + eps), a.QP);
-  }
+  if (a.cq)
+    wave_norm(a.cq_out + (long)t * a.QP, a.cq + (long)t * a.ld_lat, a.q_norm,
+              a.QP, a.q_rank, eps);
   if (!a.lat) return;
   const T* lat = a.lat + (long)t * a.ld_lat;
-  const float ss = block_reduce(sum_squares(lat, CP), tmp, SumOp{}, 0.f);
   const long slot = slots[t];
   if (slot < 0 || slot >= a.n_slots) return;
   T* dst = a.cache + slot * (CP + RP);
-  scale_row(dst, lat, a.kv_norm, 1.f / sqrtf(ss / (float)a.kv_rank + eps),
-            CP);
-  for (int p = tid; p < hp; p += 256) {
+  wave_norm(dst, lat, a.kv_norm, CP, a.kv_rank, eps);
+  for (int p = lane; p < hp; p += 64) {
     int ui, vi;
     rot_places(rot, p, &ui, &vi);
     float u = to_f32(lat[CP + ui]), v = to_f32(lat[CP + vi]);
@@ -545,10 +543,11 @@ c10::optional<torch::Tensor> lm_latent_prep(
       a.QP = (int)QP;
       a.q_rank = (int)q_rank;
     }
-    hipLaunchKernelGGL((latent_prep_kernel<scalar_t>), dim3(T), dim3(256), 0,
+    hipLaunchKernelGGL((latent_prep_kernel<scalar_t>),
+                       dim3((T + PREP_W - 1) / PREP_W), dim3(PREP_W * 64), 0,
                        cmls::current_stream(), a, positions.data_ptr<int>(),
                        slots.data_ptr<int>(), rot, (int)RP, (int)CP,
-                       (float)eps);
+                       (float)eps, (int)T);
   });
   LM_LAUNCHED();
   return out;

@@ -1,9 +1,6 @@
-"""Small Bimipel configurations, weights and engines for the tests."""
-
-import os
+"""Small Bimipel configurations and weights for the tests."""
 
 import torch
-from safetensors.torch import save_file
 
 
 def attn(heads=3, dim=12, rot=6, vdim=10, rank=20, window=7, base=500.0,
@@ -123,49 +120,3 @@ def weights(cfg, seed=0, sharp=2.5):
             t = t * s[-1] ** -0.5
         out[name] = t.to(torch.bfloat16)
     return out
-
-
-def engine(cfg, state, tmp_path, dtype="float32", device="cpu", blocks=64,
-           block_size=4, slots=4, **kw):
-    from clearml_serving_amd.engines.llm.engine import (LlmEngine,
-                                                        LlmEngineConfig)
-
-    path = os.path.join(str(tmp_path), "model.safetensors")
-    save_file({k: v.contiguous() for k, v in state.items()}, path)
-    kw.setdefault("max_model_len", blocks * block_size)
-    e = LlmEngine(LlmEngineConfig(
-        arch="bimipel", model_config=cfg, weights=path, dtype=dtype,
-        device=device, num_kv_blocks=blocks, block_size=block_size,
-        max_num_seqs=slots, **kw))
-    e.start()
-    return e
-
-
-def open_sequence(eng, name="s"):
-    from clearml_serving_amd.engines.llm.engine import (SamplingParams,
-                                                        Sequence)
-
-    s = Sequence(name, [], SamplingParams())
-    eng.open_sequence(s)
-    return s
-
-
-def feed_in_portions(eng, tokens, portions):
-    """one sequence, cut as given -> logits of every token (CPU, float64)"""
-    s = open_sequence(eng)
-    out, at = [], 0
-    for n in portions:
-        part = tokens[at:at + n]
-        out.append(eng.feed([(s, part, list(range(len(part))))])
-                   .double().cpu())
-        at += n
-    assert at == len(tokens)
-    eng.close_sequence(s)
-    return torch.cat(out)
-
-
-def error(got, want):
-    """per row: rms difference over the rms of all wanted logits"""
-    d = got.double().cpu() - want
-    d = d - d.mean(-1, keepdim=True)
-    return (d.pow(2).mean(-1).sqrt() / want.pow(2).mean().sqrt()).max().item()

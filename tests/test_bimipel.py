@@ -8,7 +8,6 @@ import asyncio
 import io
 import json
 import os
-import random
 import subprocess
 import sys
 
@@ -20,6 +19,10 @@ sys.path.insert(0, os.path.join(os.path.dirname(__file__), "helpers"))
 
 import bimipel_cases as cases  # noqa: E402
 import bimipel_plain as plain  # noqa: E402
+from lm_cases import (check_trace, engine, error,  # noqa: E402
+                      feed_in_portions, generate, greedy,
+                      mixed_batches_error, name_of, open_sequence, padded,
+                      portions_of, rel, tokens_for, trace_lines, write_model)
 
 from clearml_serving_amd.engines.llm.token_batch import TokenBatch  # noqa: E402
 from clearml_serving_amd.models.mixers import (GatedMlp,  # noqa: E402
@@ -41,32 +44,6 @@ MODEL = pytest.mark.parametrize("device,dtype,tol", [
                  marks=pytest.mark.gpu),
     pytest.param("cuda:0", torch.bfloat16, 8e-2, id="gpu-bf16",
                  marks=pytest.mark.gpu)])
-
-
-def name_of(dtype):
-    return {torch.float32: "float32", torch.bfloat16: "bfloat16"}[dtype]
-
-
-def padded(x, n):
-    out = torch.zeros(*x.shape[:-1], n, dtype=x.dtype)
-    out[..., :x.shape[-1]] = x
-    return out
-
-
-def rel(got, want):
-    d = (got.double().cpu() - want.double()).abs().max()
-    return (d / want.abs().max().clamp(min=1e-6)).item()
-
-
-def portions_of(n, sizes):
-    """cut n into the given sizes, cycled"""
-    out, i = [], 0
-    while n:
-        k = min(sizes[i % len(sizes)], n)
-        out.append(k)
-        n -= k
-        i += 1
-    return out
 
 
 # --------------------------------------------------------------------- #
@@ -399,24 +376,19 @@ def model_weights(cfg, seed, dtype):
     return cases.weights(cfg, seed, 2.5 if dtype == torch.float32 else 0.7)
 
 
-def tokens_for(cfg, n, seed):
-    r = random.Random(seed)
-    return [r.randrange(cfg["vocab"]) for _ in range(n)]
-
-
 @MODEL
 @pytest.mark.parametrize("name", sorted(cases.CONFIGS))
 def test_prompt_against_plain(device, dtype, tol, name, tmp_path):
     cfg = cases.CONFIGS[name]()
     st = model_weights(cfg, 11, dtype)
-    eng = cases.engine(cfg, st, tmp_path, name_of(dtype), device)
+    eng = engine(cfg, st, tmp_path, name_of(dtype), device)
     toks = tokens_for(cfg, 190, 1)
     want = plain.forward(cfg, st, toks)
     for portions in ([190], [1] * 190, portions_of(190, [2]),
                      portions_of(190, [64, 5, 1, 1, 33]),
                      portions_of(190, [9, 7])):
-        got = cases.feed_in_portions(eng, toks, portions)
-        assert cases.error(got, want) < tol, portions[:4]
+        got = feed_in_portions(eng, toks, portions)
+        assert error(got, want) < tol, portions[:4]
     assert eng.allocator.available == 64 and eng.state_slots.available == 4
 
 
@@ -424,14 +396,14 @@ def test_prompt_against_plain(device, dtype, tol, name, tmp_path):
 def test_residual_after_every_layer(device, dtype, tol, tmp_path):
     cfg = cases.CONFIGS["mixed"]()
     st = model_weights(cfg, 2, dtype)
-    eng = cases.engine(cfg, st, tmp_path, name_of(dtype), device)
+    eng = engine(cfg, st, tmp_path, name_of(dtype), device)
     toks = tokens_for(cfg, 40, 3)
     want, got = [], []
     plain.forward(cfg, st, toks, collect=want)
     for lay in eng.model.layers:
         lay.register_forward_hook(
             lambda mod, args, out: got.append(args[0].clone()))
-    cases.feed_in_portions(eng, toks, [40])
+    feed_in_portions(eng, toks, [40])
     for g, w in zip(got, want):
         assert g.dtype == torch.float32
         assert rel(g[:, :cfg["width"]], w) < tol
@@ -445,39 +417,12 @@ def test_mixed_batches_and_reuse(device, dtype, tol, name, tmp_path):
     equals that of the request alone."""
     cfg = cases.CONFIGS[name]()
     st = model_weights(cfg, 5, dtype)
-    eng = cases.engine(cfg, st, tmp_path, name_of(dtype), device, blocks=70)
-    r = random.Random(8)
-    left = []
+    eng = engine(cfg, st, tmp_path, name_of(dtype), device, blocks=70)
+    requests = []
     for i, n in enumerate([97, 3, 41, 66, 1, 58, 30, 2, 75]):
         toks = tokens_for(cfg, n, 100 + i)
-        left.append((toks, plain.forward(cfg, st, toks)))
-    live = []
-    worst = 0.0
-    while left or live:
-        while left and len(live) < 4:
-            toks, want = left.pop(0)
-            live.append([cases.open_sequence(eng), toks, want, 0])
-        todo = [x for x in live if r.random() < 0.8] or live[:1]
-        r.shuffle(todo)
-        entries, spans = [], []
-        for x in todo:
-            n = min(r.choice([1, 1, 1, 2, 3, 13, 40]), len(x[1]) - x[3])
-            want = sorted(r.sample(range(n), r.randint(0, n)))
-            entries.append((x[0], x[1][x[3]:x[3] + n], want))
-            spans.append((x, [x[3] + w for w in want]))
-            x[3] += n
-        logits = eng.feed(entries).cpu()
-        at = 0
-        for x, places in spans:
-            if places:
-                worst = max(worst, cases.error(
-                    logits[at:at + len(places)], x[2][places])
-                    if x[2][places].abs().max() > 0 else 0.0)
-            at += len(places)
-        assert at == len(logits)
-        for x in [x for x in live if x[3] == len(x[1])]:
-            eng.close_sequence(x[0])
-            live.remove(x)
+        requests.append((toks, plain.forward(cfg, st, toks)))
+    worst = mixed_batches_error(eng, requests, seed=8)
     assert worst < 2 * tol
     assert eng.allocator.available == 70 and eng.state_slots.available == 4
 
@@ -486,45 +431,11 @@ def test_mixed_batches_and_reuse(device, dtype, tol, name, tmp_path):
 def test_long_decoding(device, dtype, tol, tmp_path):
     cfg = cases.CONFIGS["mixed"]()
     st = model_weights(cfg, 6, dtype)
-    eng = cases.engine(cfg, st, tmp_path, name_of(dtype), device, blocks=160)
+    eng = engine(cfg, st, tmp_path, name_of(dtype), device, blocks=160)
     toks = tokens_for(cfg, 600, 4)
     want = plain.forward(cfg, st, toks)
-    got = cases.feed_in_portions(eng, toks, [5] + [1] * 595)
-    assert cases.error(got, want) < tol
-
-
-def greedy_plain(cfg, st, prompt, n):
-    """-> tokens, smallest lead of a chosen logit over the runner-up"""
-    ids, lead = list(prompt), float("inf")
-    for _ in range(n):
-        row = plain.forward(cfg, st, ids)[-1]
-        top = row.topk(2)
-        lead = min(lead, (top.values[0] - top.values[1]).item())
-        ids.append(int(top.indices[0]))
-    return ids[len(prompt):], lead
-
-
-def generate(eng, prompts, n):
-    from clearml_serving_amd.engines.llm.engine import SamplingParams
-
-    async def one(ids):
-        seq = await eng.add_request(ids, SamplingParams(
-            temperature=0.0, max_tokens=n, ignore_eos=True))
-        out = []
-        while True:
-            item = await seq.stream.get()
-            assert not item.get("error"), item
-            out.extend(item["token_ids"])
-            if item["finished"]:
-                return out
-
-    async def main():
-        out = await asyncio.gather(*[one(p) for p in prompts])
-        # the step that finished the last request also gives back its pages
-        await asyncio.sleep(0.05)
-        return out
-
-    return asyncio.new_event_loop().run_until_complete(main())
+    got = feed_in_portions(eng, toks, [5] + [1] * 595)
+    assert error(got, want) < tol
 
 
 @pytest.mark.parametrize("device,dtype,tol", [CPU, GPU32])
@@ -535,13 +446,13 @@ def test_greedy_generation(device, dtype, tol, chunk, blocks, tmp_path):
     and when sequences are preempted and start again"""
     cfg = cases.CONFIGS["mixed"]()
     st = model_weights(cfg, 7, dtype)
-    eng = cases.engine(cfg, st, tmp_path, name_of(dtype), device,
+    eng = engine(cfg, st, tmp_path, name_of(dtype), device,
                        blocks=blocks, slots=3, prefill_chunk=chunk,
                        max_model_len=130)
     prompts = [tokens_for(cfg, n, 50 + n) for n in (31, 2, 17, 40, 9)]
     got = generate(eng, prompts, 24)
     for p, g in zip(prompts, got):
-        want, lead = greedy_plain(cfg, st, p, 24)
+        want, lead = greedy(lambda t: plain.forward(cfg, st, t), p, 24)
         assert lead > 1e-4  # rounding cannot change a choice
         assert g == want
     if blocks == 20:
@@ -558,9 +469,9 @@ def test_decode_graph_replays_equal_eager(dtype, tmp_path):
     st = cases.weights(cfg, seed=9)
     runs = []
     for graphs in (True, False):
-        eng = cases.engine(cfg, st, tmp_path, dtype, "cuda:0",
+        eng = engine(cfg, st, tmp_path, dtype, "cuda:0",
                            decode_graphs=graphs)
-        seqs = [cases.open_sequence(eng) for _ in range(3)]
+        seqs = [open_sequence(eng) for _ in range(3)]
         toks = [tokens_for(cfg, 60, 20 + i) for i in range(3)]
         out = [eng.feed([(s, t[:9], [8]) for s, t in zip(seqs, toks)]).cpu()]
         for k in range(9, 60):
@@ -585,10 +496,10 @@ def test_embeddings_leave_running_sequences_alone(device, dtype, tol,
                                                   tmp_path):
     cfg = cases.CONFIGS["mixed"]()
     st = model_weights(cfg, 10, dtype)
-    eng = cases.engine(cfg, st, tmp_path, name_of(dtype), device)
+    eng = engine(cfg, st, tmp_path, name_of(dtype), device)
     toks = tokens_for(cfg, 50, 5)
     want = plain.forward(cfg, st, toks)
-    s = cases.open_sequence(eng)
+    s = open_sequence(eng)
     eng.feed([(s, toks[:30], [])])
     prompts = [tokens_for(cfg, n, n) for n in (12, 1, 20)]
     got = eng._embed_sync({"mode": "embed", "prompts": prompts,
@@ -600,23 +511,12 @@ def test_embeddings_leave_running_sequences_alone(device, dtype, tol,
                                       cfg["norm"]["eps"]).mean(0)
         assert rel(torch.tensor(g), hid) < tol
     got = eng.feed([(s, toks[30:], list(range(20)))])
-    assert cases.error(got, want[30:]) < tol
+    assert error(got, want[30:]) < tol
 
 
 # --------------------------------------------------------------------- #
 # configuration, loading, trace runner
 # --------------------------------------------------------------------- #
-def write_model(cfg, st, folder):
-    from safetensors.torch import save_file
-
-    os.makedirs(folder, exist_ok=True)
-    with open(os.path.join(folder, "config.json"), "w") as f:
-        json.dump(cfg, f)
-    save_file({k: v.contiguous() for k, v in st.items()},
-              os.path.join(folder, "model.safetensors"))
-    return str(folder)
-
-
 def test_model_folder_selects_the_family(tmp_path):
     from clearml_serving_amd.engines.llm.engine import LlmEngineConfig
     from clearml_serving_amd.models import build_model, list_archs
@@ -645,16 +545,16 @@ def test_bad_checkpoints_and_configs_are_refused(tmp_path):
         bad = dict(st)
         change(bad)
         with pytest.raises(ValueError, match="checkpoint"):
-            cases.engine(cfg, bad, tmp_path)
+            engine(cfg, bad, tmp_path)
     for src in (1, 2, 5):
         bad = cases.CONFIGS["mixed"]()
         bad["layers"][2]["mixer"]["kv_from"] = src
         with pytest.raises(ValueError, match="kv_from"):
-            cases.engine(bad, st, tmp_path)
+            engine(bad, st, tmp_path)
     bad = cases.CONFIGS["mixed"]()
     bad["layers"][2]["mixer"]["rot"]["base"] = 9.0
     with pytest.raises(ValueError, match="rot"):
-        cases.engine(bad, st, tmp_path)
+        engine(bad, st, tmp_path)
 
 
 @pytest.mark.parametrize("option", [
@@ -663,31 +563,7 @@ def test_bad_checkpoints_and_configs_are_refused(tmp_path):
 def test_options_without_a_mechanism_are_refused(option, tmp_path):
     cfg = cases.CONFIGS["mixed"]()
     with pytest.raises(ValueError, match="does not support"):
-        cases.engine(cfg, cases.weights(cfg), tmp_path, **option)
-
-
-def trace_lines(toks_a, toks_b):
-    yield {"step": 0, "entries": [
-        {"id": "a", "tokens": toks_a[:20], "want": [0, 19]},
-        {"id": "b", "tokens": toks_b[:2], "want": []}], "end": []}
-    yield {"step": 1, "entries": [
-        {"id": "b", "tokens": toks_b[2:], "want": [0, 4]},
-        {"id": "a", "tokens": toks_a[20:21], "want": [0]}], "end": ["b"]}
-    yield {"step": 2, "entries": [
-        {"id": "a", "tokens": toks_a[21:], "want": []}], "end": ["a"]}
-    yield {"step": 3, "entries": [
-        {"id": "c", "tokens": toks_b[:1], "want": [0]}], "end": ["c"]}
-
-
-def check_trace(out, cfg, st, toks_a, toks_b, tol):
-    wa, wb = (plain.forward(cfg, st, t) for t in (toks_a, toks_b))
-    for step, want in ((0, wa[[0, 19]]),
-                       (1, torch.stack([wb[2], wb[6], wa[20]])),
-                       (3, wb[:1])):
-        got = np.fromfile(os.path.join(out, "{}.f32".format(step)),
-                          dtype="<f4").reshape(-1, cfg["vocab"])
-        assert cases.error(torch.from_numpy(got), want) < tol
-    assert not os.path.exists(os.path.join(out, "2.f32"))
+        engine(cfg, cases.weights(cfg), tmp_path, **option)
 
 
 @MODEL
@@ -706,7 +582,8 @@ def test_trace_runner_in_process(device, dtype, tol, tmp_path):
     lines = io.StringIO("\n".join(json.dumps(x) for x in trace_lines(a, b)))
     trace.run(eng, lines, out, steps.append)
     assert steps == [0, 1, 2, 3]
-    check_trace(out, cfg, st, a, b, tol)
+    check_trace(out, cfg["vocab"], *(plain.forward(cfg, st, t)
+                                      for t in (a, b)), tol)
 
 
 def test_trace_runner_program(tmp_path):
@@ -733,7 +610,8 @@ def test_trace_runner_program(tmp_path):
         assert p.wait(timeout=60) == 0
     finally:
         p.kill()
-    check_trace(str(tmp_path), cfg, st, a, b, 2e-5)
+    check_trace(str(tmp_path), cfg["vocab"],
+                *(plain.forward(cfg, st, t) for t in (a, b)), 2e-5)
 
 
 @pytest.mark.gpu
