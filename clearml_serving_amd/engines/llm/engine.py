@@ -19,7 +19,7 @@ Engine step (continuous batching):
 
 Model families: llama / qwen2 (models/llama.py) and gpt2 (models/gpt2.py)
 share one forward interface, so every scheduler feature serves both.
-Token-batch families (models/bimipel.py) take steps 2 and 3 as ONE forward
+Token-batch families (models/token_lm.py) take steps 2 and 3 as ONE forward
 over a flat batch of prompt portions and single tokens (token_batch.py); next
 to pages they hold one state slot per running sequence for their recurrent
 layers, and a step of single tokens only is hipGraph-replayed as above.
@@ -709,19 +709,19 @@ class LlmEngine:
         if str(cfg.kv_dtype).lower() in ("fp8", "float8", "e4m3"):
             bad.append("fp8 KV cache")
         if cfg.enable_prefix_caching:
-            # a shared prefix would need the recurrent state at its end
+            # a shared prefix would need a recurrent state at its end
             bad.append("prefix caching")
         if cfg.speculative:
-            # a rejected token cannot be taken out of the recurrent state
+            # a rejected token cannot be taken out of a recurrent state
             bad.append("speculative decoding")
         if bad:
             raise ValueError("arch '{}' does not support {}".format(
                 cfg.arch, ", ".join(bad)))
 
     def _new_layer_caches(self, num_blocks: int, num_slots: int) -> List:
-        """Per layer: page tensor [blocks, block_size, row], (state float
+        """Per layer run: page tensor [blocks, block_size, row], (state float
         [slots, channels], ring [slots, taps, channels]), or the tensor of
-        the layer it shares with."""
+        the run it shares with."""
         caches: List = []
         for kind, *dims in self.model.cache_layout():
             if kind == "paged":

@@ -18,8 +18,10 @@ constexpr int BM = 128, BN = 64, NW = 8;
 
 // qtiles: int32 [n, 6] = first token (flat), tokens, first position, first
 // row in the gathered keys, that row's position, gathered rows
+// two workgroups per CU (128 registers) where their LDS fits
 template <int QS, int VT>
-__global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
+__global__ __launch_bounds__(NW * 64, QS * 2 + VT <= 16 ? 4 : 2)
+void latent_prompt_kernel(
     const bf16* __restrict__ q, long q_t,   // q[t * q_t + h * QD]
     const bf16* __restrict__ kv, int ldkv,  // [rows, H*DP + H*VP]
     const bf16* __restrict__ rot, int ld_rot, const bf16* __restrict__ sink,
@@ -35,7 +37,7 @@ __global__ __launch_bounds__(NW * 64, 2) void latent_prompt_kernel(
   const int* td = qtiles + (long)blockIdx.y * 6;
   const int t0 = td[0], len = td[1], p0 = td[2], kv0 = td[3], k_lo = td[4],
             nk = td[5];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave();
   const int r16 = lane & 15, g = lane >> 4, ko = g * 8;
   const int qrow = wave * 16 + r16;
   const float scale2 = scale * LOG2E;

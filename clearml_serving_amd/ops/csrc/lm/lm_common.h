@@ -94,6 +94,11 @@ __device__ __forceinline__ void wave_lds_fence() {
   __builtin_amdgcn_wave_barrier();
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
+// The wave's number, as a scalar. An MFMA ignores the lane mask, so a branch
+// around one has to be a scalar branch.
+__device__ __forceinline__ int uniform_wave() {
+  return __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+}
 template <typename T> __device__ __forceinline__ Frag<T> zero_frag();
 template <> __device__ __forceinline__ Frag<bf16> zero_frag<bf16>() {
   Frag<bf16> f;

@@ -12,12 +12,6 @@
 
 namespace {
 
-// The wave's number, as a scalar. An MFMA ignores the lane mask, so a branch
-// around one has to be a scalar branch.
-__device__ __forceinline__ int uniform_wave() {
-  return __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-}
-
 constexpr int RT = 16;  // tokens per routing workgroup
 constexpr int MAX_TOP = 64;
 
