@@ -719,31 +719,40 @@ class LlmEngine:
                 cfg.arch, ", ".join(bad)))
 
     def _new_layer_caches(self, num_blocks: int, num_slots: int) -> List:
-        """Per layer run: page tensor [blocks, block_size, row], (state float
-        [slots, channels], ring [slots, taps, channels]), or the tensor of
-        the run it shares with."""
-        caches: List = []
-        for kind, *dims in self.model.cache_layout():
+        """Per layer run: page tensor [blocks, block_size, row], tuple (state
+        float [slots, ...], ring [slots, taps, channels] where there is one),
+        the tensor of the run it shares with, or a tuple of two of these."""
+        def zeros(dtype, *shape):
+            return torch.zeros(*shape, dtype=dtype, device=self.device)
+
+        def make(kind, *dims):
             if kind == "paged":
-                caches.append(torch.zeros(
-                    num_blocks, self.cfg.block_size, dims[0],
-                    dtype=self.dtype, device=self.device))
-            elif kind == "state":
-                channels, taps = dims
-                caches.append((
-                    torch.zeros(num_slots, channels, dtype=torch.float32,
-                                device=self.device),
-                    torch.zeros(num_slots, taps, channels, dtype=self.dtype,
-                                device=self.device)))
-            else:  # shared
-                caches.append(caches[dims[0]])
+                return zeros(self.dtype, num_blocks, self.cfg.block_size,
+                             dims[0])
+            if kind == "state":
+                return tuple(zeros(dtype, num_slots, *shape) for shape, dtype
+                             in zip(dims, (torch.float32, self.dtype)))
+            if kind == "both":
+                return tuple(make(*d) for d in dims)
+            return caches[dims[0]]  # shared
+
+        caches: List = []
+        for layout in self.model.cache_layout():
+            caches.append(make(*layout))
         return caches
+
+    @staticmethod
+    def _paged_elements(layout: tuple) -> int:
+        """cached elements per token of a layer run"""
+        kind, *dims = layout
+        if kind == "both":
+            return sum(LlmEngine._paged_elements(d) for d in dims)
+        return dims[0] if kind == "paged" else 0
 
     def _start_token_batch_caches(self) -> None:
         cfg = self.cfg
-        rows = [d[0] for kind, *d in self.model.cache_layout()
-                if kind == "paged"]
-        per_block = max(sum(rows), 1) * cfg.block_size * self.dtype.itemsize
+        row = sum(map(self._paged_elements, self.model.cache_layout()))
+        per_block = max(row, 1) * cfg.block_size * self.dtype.itemsize
         if cfg.num_kv_blocks:
             num_blocks = int(cfg.num_kv_blocks)
         elif self.device.type == "cuda":

@@ -23,9 +23,10 @@ class TokenBatch:
     n_single: leading entries of one token (token i is entry i);
     n_abs: leading tokens whose attention runs in absorbed form;
     tiles [n, 5], seqs [m, 6]: recurrence tiles of the other entries (see
-    ops.lm.rglru_prefill); prompts: window -> (cache rows that the entries
-    behind the first n_abs tokens can see, query tiles into them; see
-    ops.lm.latent_prompt); max_keys: bound on position + 1 in the first n_abs
+    ops.lm.rglru_prefill); prompts: per view -- a window or (window, first
+    tokens that are kept) -- the cache rows that the entries behind the first
+    n_abs tokens can see and query tiles into them (see ops.lm.latent_prompt,
+    ops.grouped.prompt); max_keys: bound on position + 1 in the first n_abs
     tokens."""
 
     mode = "token_batch"
@@ -35,7 +36,7 @@ class TokenBatch:
 
     @classmethod
     def build(cls, plan: Dict[str, Any], block_size: int, device,
-              tile: int, absorb_max: Optional[int], windows: Seq[int]):
+              tile: int, absorb_max: Optional[int], windows: Seq):
         """plan: per entry "tokens", "starts", "blocks", "state_slots",
         "want" (places among its tokens whose logits are asked for).
         -> (tokens [T] int64, batch, wanted rows int32 in plan order)"""
@@ -48,7 +49,7 @@ class TokenBatch:
         seqs: List[List[int]] = []
         n_single = n_abs = max_keys = at = 0
         gathered = {w: [] for w in windows}
-        qtiles: Dict[int, List[List[int]]] = {w: [] for w in windows}
+        qtiles: Dict[Any, List[List[int]]] = {w: [] for w in windows}
         n_rows = dict.fromkeys(windows, 0)
         mb = max(len(b) for b in plan["blocks"])
         btab = np.zeros((n, mb), dtype=np.int32)
@@ -77,13 +78,18 @@ class TokenBatch:
                 max_keys = max(max_keys, start + ln)
                 continue
             for w in windows:
-                lo = max(0, start - w + 1) if w else 0
-                p = np.arange(lo, start + ln, dtype=np.int32)
+                size, keep = w if isinstance(w, tuple) else (w, 0)
+                lo = max(0, start - size + 1) if size else 0
+                keep = min(keep, lo)
+                p = np.concatenate([
+                    np.arange(keep, dtype=np.int32),
+                    np.arange(lo, start + ln, dtype=np.int32)])
                 gathered[w].append(blocks[p // block_size] * block_size
                                    + p % block_size)
                 for j in range(0, ln, PROMPT_TILE):
                     qtiles[w].append([first[i] + j, min(PROMPT_TILE, ln - j),
-                                      start + j, n_rows[w], lo, len(p)])
+                                      start + j, n_rows[w], lo - keep,
+                                      len(p)])
                 n_rows[w] += len(p)
         want = [first[i] + w for i in range(n) for w in plan["want"][i]]
         parts = {

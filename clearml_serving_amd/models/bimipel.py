@@ -130,7 +130,8 @@ class BimipelForCausalLM(TokenBatchForCausalLM):
         out: List[tuple] = []
         for layer in self.layers:
             if isinstance(layer.mix, RgLru):
-                out.append(("state", layer.mix.wp, layer.mix.taps))
+                wp, taps = layer.mix.wp, layer.mix.taps
+                out.append(("state", (wp,), (taps, wp)))
             elif layer.kv_from is not None:
                 out.append(("shared", layer.kv_from))
             else:

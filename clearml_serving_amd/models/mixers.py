@@ -7,20 +7,20 @@ parameters; ``pack`` fills the padded, merged operands from tensors in
 checkpoint layout.
 """
 
-from typing import Callable, Dict, Optional
+from typing import Callable, Dict, Optional, Tuple
 
 import torch
 import torch.nn as nn
 
 from .. import ops
-from ..ops import lm
+from ..ops import delta, grouped, lm
 from ..ops.lm import pad32
 
 Get = Callable[[str], torch.Tensor]
 
 
 def _param(*shape) -> nn.Parameter:
-    return nn.Parameter(torch.zeros(*shape), requires_grad=False)
+    return nn.Parameter(torch.zeros(shape), requires_grad=False)
 
 
 def _fill(dst: torch.Tensor, src: torch.Tensor) -> None:
@@ -154,6 +154,11 @@ class LatentAttention(nn.Module):
             self.uk_t.data.transpose(1, 2).reshape(-1, self.cp),
             self.uv.data.reshape(-1, self.cp)])
 
+    @property
+    def view(self):
+        """what a query sees, as TokenBatch names it"""
+        return self.window
+
     def can_expand(self) -> bool:
         """whether ops.lm.latent_prompt takes this head size"""
         return (self.dp + self.rp <= lm.PROMPT_MAX_HEAD
@@ -210,6 +215,323 @@ class LatentAttention(nn.Module):
                              self.heads, self.dp, self.rp, self.cp, self.vp,
                              self.window, self.scale, gate)
         return linear(ctx.view(t, -1), self.o)
+
+
+class GroupedAttention(nn.Module):
+    """Grouped-query attention (csrc/lm/gqa.hip): ``heads`` query heads on
+    ``kv_heads`` cached key/value heads.
+
+    ``rot``: (base, rotated dimensions, factor that divides the frequencies),
+    pairs (2i, 2i+1), or None. ``window`` 0: all earlier tokens; else the last
+    ``window`` and the first ``keep`` ones. ``cap``: scores become cap *
+    tanh(score / cap). ``qk_norm``: norm per head of queries and keys.
+    ``values_are_keys``: no projection of their own, the keys before norm and
+    rotation. ``sink``: "learned" term per head in the softmax's denominator,
+    "one" (a learned term of 0) or None. ``v_mix``: values mixed with those of
+    the first layer that does."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, scale: float, eps: float = 0.0,
+                 rot: Optional[Tuple[float, int, float]] = None,
+                 window: int = 0, keep: int = 0, cap: float = 0.0,
+                 qk_norm: bool = False, values_are_keys: bool = False,
+                 sink: Optional[str] = None, v_mix: bool = False):
+        super().__init__()
+        if kv_heads < 1 or heads % kv_heads:
+            raise ValueError("{} query heads on {} key/value heads".format(
+                heads, kv_heads))
+        if rot is not None and (rot[1] % 2 or not 0 < rot[1] <= dim):
+            raise ValueError("rotated dimensions {} of {}".format(
+                rot[1], dim))
+        if values_are_keys and (vdim != dim or v_mix or rot is not None):
+            raise ValueError("values that are keys have the keys' size and "
+                             "go with neither mixing nor rotation")
+        if keep and not window:
+            raise ValueError("kept tokens without a window")
+        if sink not in (None, "one", "learned"):
+            raise ValueError("unknown sink '{}'".format(sink))
+        self.width, self.heads, self.kv_heads = width, heads, kv_heads
+        self.dim, self.vdim, self.eps = dim, vdim, eps
+        self.rot_spec, self.v_mix, self.lam = rot, v_mix, 0.0
+        self.kp, self.vp = pad32(dim), pad32(vdim)
+        self.spec = grouped.GroupedSpec(
+            heads, kv_heads, self.kp, self.vp, dim, values_are_keys, window,
+            keep, scale, cap, 1.0)
+        # one product of h: [queries | keys | values]
+        self.k_at = heads * self.kp
+        self.v_at = self.k_at + kv_heads * self.kp
+        self.cols = self.v_at + (0 if values_are_keys else
+                                 kv_heads * self.vp)
+        self.q_norm = _param(self.kp) if qk_norm else None
+        self.k_norm = _param(self.kp) if qk_norm else None
+        self.sink_kind = sink
+        self.sink = None if sink is None else _param(heads)
+        self.vmix = _param() if v_mix else None
+        self.rot: Optional[lm.Rotary] = None
+
+    @property
+    def view(self):
+        """what a query sees, as TokenBatch names it"""
+        s = self.spec
+        return (s.window, s.keep) if s.keep else s.window
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.vp
+
+    def scaled(self, out_scale: float) -> "GroupedAttention":
+        """the result times a constant"""
+        self.spec = self.spec._replace(out_scale=out_scale)
+        return self
+
+    def shapes(self) -> dict:
+        h, g = self.heads, self.kv_heads
+        out = {"q": (h * self.dim, self.width),
+               "k": (g * self.dim, self.width),
+               "o": (self.width, h * self.vdim)}
+        if not self.spec.same:
+            out["v"] = (g * self.vdim, self.width)
+        if self.q_norm is not None:
+            out["q.norm"] = out["k.norm"] = (self.dim,)
+        if self.sink_kind == "learned":
+            out["sink"] = (h,)
+        if self.v_mix:
+            out["vmix"] = ()
+        return out
+
+    def pack_in(self, w: torch.Tensor, get: Get) -> None:
+        """rows of the product of h"""
+        parts = [("q", 0, self.heads, self.kp),
+                 ("k", self.k_at, self.kv_heads, self.kp)]
+        if not self.spec.same:
+            parts.append(("v", self.v_at, self.kv_heads, self.vp))
+        for name, at, n, size in parts:
+            src = get(name)
+            _fill(w[at:at + n * size].view(n, size, -1),
+                  src.view(n, -1, self.width))
+
+    def pack_out(self, w: torch.Tensor, get: Get) -> None:
+        """columns of the product of the heads' results"""
+        _fill(w.view(w.shape[0], self.heads, self.vp),
+              get("o").view(self.width, self.heads, self.vdim))
+
+    def pack_own(self, get: Get) -> None:
+        if self.q_norm is not None:
+            _fill(self.q_norm.data, get("q.norm"))
+            _fill(self.k_norm.data, get("k.norm"))
+        if self.sink_kind == "learned":
+            _fill(self.sink.data, get("sink"))
+        if self.v_mix:
+            _fill(self.vmix.data, get("vmix"))
+
+    def finalize(self, device) -> None:
+        if self.rot_spec is not None:
+            base, dims, factor = self.rot_spec
+            i = torch.arange(dims // 2, dtype=torch.float64)
+            freq = float(base) ** (-2.0 * i / dims) / factor
+            self.rot = lm.Rotary(freq.to(torch.float32).to(device))
+        if self.v_mix:
+            self.lam = float(self.vmix)
+
+    def can_expand(self) -> bool:
+        """whether prompts take tiles of queries (ops.grouped.prompt)"""
+        return max(self.kp, self.vp) <= lm.PROMPT_MAX_HEAD
+
+    def values(self, z) -> torch.Tensor:
+        return z[:, self.v_at:self.cols]
+
+    def attend(self, z, batch, cache, out, first=None):
+        """z [T, >= cols]: the product of h; out [T, out_cols]. ``first``:
+        the values that this layer's are mixed with"""
+        t, n, s = z.shape[0], batch.n_abs, self.spec
+        grouped.prepare(z, self.k_at, self.v_at, batch.positions,
+                        batch.slot_mapping, self.rot, s, self.q_norm,
+                        self.k_norm, self.eps, first, self.lam, cache)
+        q = z[:, :self.k_at]
+        if n:
+            grouped.attention(q, cache, batch.block_table, batch.tok_seq,
+                              batch.positions, self.sink, out, n, s,
+                              batch.max_keys)
+        if n < t:
+            rows, qtiles = batch.prompts[self.view]
+            grouped.prompt(q, lm.gather_rows(cache, rows), self.sink, qtiles,
+                           out, s)
+
+
+class GroupedAttentionMixer(nn.Module):
+    """GroupedAttention as a layer's mixer."""
+
+    def __init__(self, width: int, *args, **kw):
+        super().__init__()
+        self.attn = a = GroupedAttention(width, *args, **kw)
+        wp = pad32(width)
+        self.qkv = _param(a.cols, wp)
+        self.o = _param(wp, a.out_cols)
+
+    def shapes(self) -> dict:
+        return self.attn.shapes()
+
+    def pack(self, get: Get) -> None:
+        self.attn.pack_in(self.qkv.data, get)
+        self.attn.pack_out(self.o.data, get)
+        self.attn.pack_own(get)
+
+    def finalize(self) -> None:
+        self.attn.finalize(self.qkv.device)
+
+    def cache_layout(self) -> tuple:
+        return "paged", self.attn.spec.row
+
+    def forward(self, h, batch, cache, carry):
+        """``carry``: what layers of one forward hand on ("values")"""
+        a, first = self.attn, None
+        z = linear(h, self.qkv)
+        if a.v_mix:
+            first = carry.get("values")
+            if first is None:  # this is the first such layer
+                carry["values"] = a.values(z)
+        ctx = h.new_empty(h.shape[0], a.out_cols)
+        a.attend(z, batch, cache, ctx, first)
+        return linear(ctx, self.o)
+
+
+class DeltaRule(nn.Module):
+    """Generalised delta rule (csrc/lm/delta.hip): a float state per head with
+    decay per key channel, a removal term along the unit key, and outputs that
+    are normed per head and gated. ``rank``: inner size of the decay's
+    projection, which a checkpoint's tensors tell (``fit``)."""
+
+    def __init__(self, width: int, heads: int, dim: int, eps: float,
+                 rank: int = 64):
+        super().__init__()
+        self.width, self.heads, self.dim, self.eps = width, heads, dim, eps
+        self.dp = delta.head_pad(dim)
+        n = heads * self.dp
+        self.ab, self.w0, self.norm = _param(n), _param(n), _param(n)
+        self.out_scale = 1.0
+        self._set_rank(rank)
+
+    def _set_rank(self, rank: int) -> None:
+        self.rank, self.rp = rank, pad32(rank)
+        n = self.heads * self.dp
+        self.w2 = _param(n, self.rp)
+        # one product of h: [r | k | v | g | a | low-rank input of the decay]
+        self.cols = 5 * n + self.rp
+        self._w: Optional[delta.DeltaWeights] = None
+
+    @property
+    def out_cols(self) -> int:
+        return self.heads * self.dp
+
+    def scaled(self, out_scale: float) -> "DeltaRule":
+        """the result times a constant"""
+        self.out_scale = out_scale
+        return self
+
+    def fit(self, get: Get) -> None:
+        rank = get("w1").shape[0]
+        if rank != self.rank:
+            self._set_rank(rank)
+
+    def shapes(self) -> dict:
+        n, w = self.heads * self.dim, self.width
+        out = {k: (n, w) for k in "rkvga"}
+        out.update({"a.b": (n,), "w0": (n,), "norm": (n,),
+                    "w1": (self.rank, w), "w2": (n, self.rank), "o": (w, n)})
+        return out
+
+    def _heads(self, dst: torch.Tensor, src: torch.Tensor) -> None:
+        _fill(dst.view(self.heads, self.dp, -1),
+              src.reshape(self.heads, self.dim, -1))
+
+    def pack_in(self, w: torch.Tensor, get: Get) -> None:
+        n = self.heads * self.dp
+        for i, name in enumerate("rkvga"):
+            self._heads(w[i * n:(i + 1) * n], get(name))
+        _fill(w[5 * n:5 * n + self.rp], get("w1"))
+
+    def pack_out(self, w: torch.Tensor, get: Get) -> None:
+        _fill(w.view(w.shape[0], self.heads, self.dp),
+              get("o").view(self.width, self.heads, self.dim))
+
+    def pack_own(self, get: Get) -> None:
+        self._heads(self.w2.data, get("w2"))
+        for dst, name in ((self.ab, "a.b"), (self.w0, "w0"),
+                          (self.norm, "norm")):
+            self._heads(dst.data, get(name))
+
+    def finalize(self) -> None:
+        self._w = delta.DeltaWeights(self.w2.data, self.w0.data,
+                                     self.ab.data, self.norm.data)
+
+    def state_layout(self) -> tuple:
+        return "state", (self.heads, self.dp, self.dp)
+
+    def scan(self, z, batch, state, out) -> None:
+        """z [T, cols]: the product of h; out [T, out_cols]"""
+        n = self.heads * self.dp
+        delta.delta_rule(z, tuple(i * n for i in range(6)), self._w, state,
+                         batch.positions, batch.state_slots, batch.seqs, out,
+                         batch.n_single, self.dim, self.eps, self.out_scale)
+
+
+class ParallelMixer(nn.Module):
+    """Two mixers that read the same input; the result is their weighted sum.
+    Both inputs are one product, and both outputs another."""
+
+    def __init__(self, width: int, left: GroupedAttention, left_scale: float,
+                 right: DeltaRule, right_scale: float):
+        super().__init__()
+        self.left = left.scaled(left_scale)
+        self.right = right.scaled(right_scale)
+        self.width = width
+        self._alloc()
+
+    def _alloc(self) -> None:
+        wp = pad32(self.width)
+        self.inp = _param(self.left.cols + self.right.cols, wp)
+        self.o = _param(wp, self.left.out_cols + self.right.out_cols)
+
+    def _sides(self):
+        return ("left.", self.left), ("right.", self.right)
+
+    def fit(self, get: Get) -> None:
+        """sizes that only a checkpoint's tensors tell"""
+        self.right.fit(lambda name: get("right." + name))
+        self._alloc()
+
+    def shapes(self) -> dict:
+        return {p + k: s for p, m in self._sides()
+                for k, s in m.shapes().items()}
+
+    def pack(self, get: Get) -> None:
+        row = col = 0
+        for p, m in self._sides():
+            def of(name, p=p):
+                return get(p + name)
+
+            m.pack_in(self.inp.data[row:row + m.cols], of)
+            m.pack_out(self.o.data[:, col:col + m.out_cols], of)
+            m.pack_own(of)
+            row += m.cols
+            col += m.out_cols
+
+    def finalize(self) -> None:
+        self.left.finalize(self.inp.device)
+        self.right.finalize()
+
+    def cache_layout(self) -> tuple:
+        return "both", ("paged", self.left.spec.row), \
+            self.right.state_layout()
+
+    def forward(self, h, batch, cache, carry):
+        pages, (state,) = cache
+        z = linear(h, self.inp)
+        n = self.left.out_cols
+        ctx = h.new_empty(h.shape[0], self.o.shape[1])
+        self.left.attend(z[:, :self.left.cols], batch, pages, ctx[:, :n])
+        self.right.scan(z[:, self.left.cols:], batch, state, ctx[:, n:])
+        return linear(ctx, self.o)
 
 
 class RgLru(nn.Module):
@@ -323,41 +645,117 @@ class GatedMlp(nn.Module):
 
 
 class ExpertMlp(nn.Module):
-    """Of ``experts`` feed-forwards down(act(up h)) each token takes the
-    ``top`` with the largest router logits, weighed by the softmax over
-    those (csrc/lm/moe.hip). The weighted sum is left to the norm that
-    follows: forward -> (rows of all slots, (pos, share))."""
+    """Experts down(act(up h)) or, ``gated``, down(act(gate h) * (up h)),
+    of which each token takes ``top`` (csrc/lm/moe.hip). The weighted sum is
+    left to the kernel that follows: forward -> (rows of all slots,
+    (pos, share)); a slot with pos -1 stands for the input itself.
+
+    Default routing: the largest logits, weighed by the softmax over those.
+    ``correction``: scores are the softmax over all outputs and weigh the
+    chosen experts as they are, the choice adds a learned term; ``groups``
+    (count, keep): only the best groups of outputs are chosen from;
+    ``identity``: so many more outputs stand for the input. ``shared_ff``: an
+    expert of that size for every token, times the sigmoid of a projection;
+    it is held as one or more slices of the experts' size, whose outputs add
+    up."""
 
     def __init__(self, width: int, ff: int, experts: int, top: int,
-                 act: str = "relu2"):
+                 act: str = "relu2", gated: bool = False,
+                 correction: bool = False,
+                 groups: Optional[Tuple[int, int]] = None, identity: int = 0,
+                 shared_ff: Optional[int] = None):
         super().__init__()
-        if not 1 <= top <= experts:
-            raise ValueError("{} of {} experts".format(top, experts))
-        self.width, self.ff, self.act = width, ff, act
-        self.experts, self.top = experts, top
+        outputs = experts + identity
+        if not 1 <= top <= outputs:
+            raise ValueError("{} of {} experts".format(top, outputs))
+        count, keep = groups or (1, 1)
+        if not 1 <= keep <= count or outputs % count:
+            raise ValueError("best {} of {} groups of {} experts".format(
+                keep, count, outputs))
+        if keep * (outputs // count) < top:
+            raise ValueError("{} experts from {} groups of {}".format(
+                top, keep, outputs // count))
+        if gated and act != "silu":
+            raise ValueError("no gated experts with '{}'".format(act))
+        if not correction and (groups or identity):
+            raise ValueError("groups and identity experts go with scores "
+                             "over all outputs")
+        self.width, self.ff, self.shared_ff = width, ff, shared_ff
+        self.act = "swiglu" if gated else act
+        self.experts, self.top, self.identity = experts, top, identity
         w, f = pad32(width), pad32(ff)
-        self.router = _param(experts, w)
-        self.up = _param(experts, f, w)
-        self.down = _param(experts, w, f)
+        self.n_shared = 0 if shared_ff is None else -(-shared_ff // f)
+        self.how = lm.Routing(top, correction, count, keep, identity,
+                              self.n_shared)
+        self.gated = gated
+        self.router = _param(outputs + (1 if self.n_shared else 0), w)
+        self.correction = _param(outputs) if correction else None
+        self._correction = None  # in float, whatever the products' type
+        n = experts + self.n_shared
+        self.up = _param(n, (2 if gated else 1) * f, w)
+        self.down = _param(n, w, f)
+
+    @property
+    def has_skip(self) -> bool:
+        return self.identity > 0
 
     def shapes(self) -> dict:
-        out = {"router": (self.experts, self.width)}
+        out = {"router": (self.experts + self.identity, self.width)}
+        if self.correction is not None:
+            out["correction"] = (self.experts + self.identity,)
+
+        def expert(p, ff):
+            for k in ("gate", "up") if self.gated else ("up",):
+                out[p + k] = (ff, self.width)
+            out[p + "down"] = (self.width, ff)
+
         for e in range(self.experts):
-            out["e{}.up".format(e)] = (self.ff, self.width)
-            out["e{}.down".format(e)] = (self.width, self.ff)
+            expert("e{}.".format(e), self.ff)
+        if self.n_shared:
+            expert("shared.", self.shared_ff)
+            out["shared.sg"] = (1, self.width)
         return out
+
+    def _pack_expert(self, e: int, up, gate, down) -> None:
+        if self.gated:  # rows in pairs
+            pairs = self.up.data[e].view(-1, 2, self.up.shape[2])
+            _fill(pairs[:, 0], gate)
+            _fill(pairs[:, 1], up)
+        else:
+            _fill(self.up.data[e], up)
+        _fill(self.down.data[e], down)
 
     def pack(self, get: Get) -> None:
         _fill(self.router.data, get("router"))
+        if self.correction is not None:
+            _fill(self.correction.data, get("correction"))
+
+        def expert(p):
+            return (get(p + "up"), get(p + "gate") if self.gated else None,
+                    get(p + "down"))
+
         for e in range(self.experts):
-            _fill(self.up.data[e], get("e{}.up".format(e)))
-            _fill(self.down.data[e], get("e{}.down".format(e)))
+            self._pack_expert(e, *expert("e{}.".format(e)))
+        if self.n_shared:
+            _fill(self.router.data[self.experts + self.identity:],
+                  get("shared.sg"))
+            up, gate, down = expert("shared.")
+            f = self.down.shape[2]
+            for i in range(self.n_shared):
+                part = slice(i * f, (i + 1) * f)
+                self._pack_expert(
+                    self.experts + i, up[part],
+                    gate[part] if self.gated else None, down[:, part])
+
+    def finalize(self) -> None:
+        if self.correction is not None:
+            self._correction = self.correction.data.float()
 
     def forward(self, h):
         rows = lm.expert_tile_rows(
             h.shape[0], self.experts, self.top, h.dtype,
             (self.up.shape[2], self.down.shape[2]))
-        plan = lm.moe_route(h, self.router, self.top, rows)
+        plan = lm.moe_route(h, self.router, self.how, rows, self._correction)
         hidden = lm.moe_gemm(h, self.up, plan, self.act, gather=True)
         out = lm.moe_gemm(hidden, self.down, plan, "none", gather=False)
         return out, (plan.pos, plan.share)

@@ -7,7 +7,7 @@ from typing import Any, Dict, Iterator, List, Optional, Tuple
 import torch
 import torch.nn as nn
 
-from .mixers import LatentAttention, RgLru, _fill
+from .mixers import GroupedAttention, LatentAttention, RgLru, _fill
 
 # checkpoint name -> (padded operand, true shape, shape to fill it in)
 Held = Dict[str, Tuple[torch.Tensor, tuple, Optional[tuple]]]
@@ -66,7 +66,19 @@ class TokenBatchForCausalLM(nn.Module):
                     out["l{}.{}{}".format(i, q, k)] = tuple(s)
         return out
 
+    def _fit(self, state: Dict[str, torch.Tensor]) -> None:
+        """sizes that are not in the configuration"""
+        for i, layer in enumerate(self.layers):
+            for q, mod in layer.parts():
+                if hasattr(mod, "fit"):
+                    try:
+                        mod.fit(lambda name, q="l{}.{}".format(i, q):
+                                state[q + name])
+                    except KeyError:
+                        pass  # reported as missing below
+
     def load_checkpoint(self, state: Dict[str, torch.Tensor]) -> None:
+        self._fit(state)
         want = self.checkpoint_shapes()
         missing = sorted(set(want) - set(state))
         extra = sorted(set(state) - set(want) - set(self.ignored()))
@@ -96,18 +108,21 @@ class TokenBatchForCausalLM(nn.Module):
     def finalize(self) -> None:
         """call once weights, device and type are settled"""
         for layer in self.layers:
-            layer.mix.finalize()
+            for _, mod in layer.parts():
+                if hasattr(mod, "finalize"):
+                    mod.finalize()
 
     # ---- what the engine needs to know ------------------------------ #
     def cache_layout(self) -> List[tuple]:
-        """per layer run, in order: ("paged", elements per token),
-        ("state", channels, taps) or ("shared", run)"""
+        """per layer run, in order: ("paged", elements per token), ("state",
+        shape of a slot's float state[, channels and taps of a ring of past
+        inputs]), ("both", layout, layout) or ("shared", run)"""
         raise NotImplementedError
 
     def batch_params(self, dtype: torch.dtype) -> Dict[str, Any]:
         """how a TokenBatch for this model is to be cut"""
-        attn = [m.mix for m in self.layers
-                if isinstance(m.mix, LatentAttention)]
+        attn = [a for m in self.layers for a in m.mix.modules()
+                if isinstance(a, (LatentAttention, GroupedAttention))]
         rec = [m.mix for m in self.layers if isinstance(m.mix, RgLru)]
         # the recurrence holds two tiles of one block's channels in LDS
         wide = max([m.bp for m in rec], default=32)
@@ -116,4 +131,4 @@ class TokenBatchForCausalLM(nn.Module):
         expand = (dtype == torch.bfloat16
                   and all(m.can_expand() for m in attn))
         return {"tile": tile, "absorb_max": 8 if expand else None,
-                "windows": sorted({m.window for m in attn})}
+                "windows": sorted({m.view for m in attn}, key=str)}

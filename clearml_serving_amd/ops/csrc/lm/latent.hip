@@ -14,30 +14,9 @@
 // Both take a sliding window, a per-head sink (a term exp(sink) in the softmax
 // denominator that has no key) and a gate on the heads' outputs, each of them
 // optional. Queries may come from a normed latent of their own.
-#include "lm_common.h"
+#include "lm_attn.h"
 
 namespace {
-
-constexpr float LOG2E = 1.4426950408889634f;
-
-// ------------------------------------------------------------------- //
-// rotary positions
-// ------------------------------------------------------------------- //
-// Pair p of a rotated part is (2p, 2p+1) or, with `half`, (p, p + pairs):
-// (u, v) -> gain * (u cos - v sin, v cos + u sin). Elements behind the pairs
-// pass unchanged.
-struct Rot {
-  const float* inv_freq;
-  int pairs, half;
-  float gain;
-};
-
-__device__ __forceinline__ void rot_places(const Rot& r, int p, int* u,
-                                           int* v) {
-  const bool h = r.half && p < r.pairs;
-  *u = h ? p : 2 * p;
-  *v = h ? p + r.pairs : 2 * p + 1;
-}
 
 // ------------------------------------------------------------------- //
 // prepare: rotate q; normalise the query latent and the cached latent, rotate
@@ -247,7 +226,7 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
   const int h0 = blockIdx.y * 16;
   const int split = blockIdx.z / col_groups;
   const int c_base = (blockIdx.z % col_groups) * (NT * 16);
-  const float scale2 = scale * LOG2E;
+  const float scale2 = scale * LM_LOG2E;
 
   const int pos = min(max(positions[t], 0), max_blocks * block_size - 1);
   const int* btab = block_table +
@@ -357,116 +336,31 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(
                      acc[i]);
   }
 
-  // meet: scale to the common maximum, sum over the waves through LDS
-  l_run += __shfl_xor(l_run, 16, 64);
-  l_run += __shfl_xor(l_run, 32, 64);
-  if (g == 0) {
-    stat[wave][r16][0] = m_run;
-    stat[wave][r16][1] = l_run;
-  }
-  __syncthreads();
-  float m_f = -INFINITY;
-  for (int w = 0; w < nw; ++w) m_f = fmaxf(m_f, stat[w][r16][0]);
-  const float f = m_run == -INFINITY ? 0.f
-                                     : __builtin_amdgcn_exp2f(m_run - m_f);
-  const int cols = min(NT * 16, CP - c_base), OP = cols + 4;
-  // 16 * OP floats of the wave's own tile region
-  float* ow = (float*)(qs + 16 * PITCH + wave * 32 * PITCH);
-#pragma unroll
-  for (int i = 0; i < NT; ++i) {
-    if (i * 16 < cols) {
-      const float v[4] = {acc[i][0] * f, acc[i][1] * f, acc[i][2] * f,
-                          acc[i][3] * f};
-      store4(ow + r16 * OP + i * 16 + 4 * g, v);
-    }
-  }
-  __syncthreads();
-  const float* o0 = (const float*)(qs + 16 * PITCH);
-  const int wstep = 32 * PITCH * (int)sizeof(T) / 4;
-  const int c4 = cols / 4;
-  for (int i = tid; i < 16 * c4; i += blockDim.x) {
-    const int r = i / c4, c = (i % c4) * 4, h = h0 + r;
-    if (h >= H) break;
-    float m = -INFINITY, l = 0.f;
-    for (int w = 0; w < nw; ++w) m = fmaxf(m, stat[w][r][0]);
-    for (int w = 0; w < nw; ++w)
-      if (stat[w][r][0] != -INFINITY)
-        l += stat[w][r][1] * __builtin_amdgcn_exp2f(stat[w][r][0] - m);
-    lm_f32x4 o = {0.f, 0.f, 0.f, 0.f};
-    for (int w = 0; w < nw; ++w)
-      o += *reinterpret_cast<const lm_f32x4*>(o0 + w * wstep + r * OP + c);
-    if (splits > 1) {
-      const long pi = ((long)t * H + h) * splits + split;
-      const float v[4] = {o[0], o[1], o[2], o[3]};
-      store4(part_o + pi * CP + c_base + c, v);
-      if (c == 0 && c_base == 0) {
-        part_ml[2 * pi] = m;
-        part_ml[2 * pi + 1] = l;
-      }
-    } else {
-      // without a sink: exp2(-inf) = 0
-      const float sk = sink ? to_f32(sink[h]) * LOG2E : -INFINITY;
-      const float m_s = fmaxf(m, sk);
-      const float e = __builtin_amdgcn_exp2f(m - m_s);
-      const float inv = e / (l * e + __builtin_amdgcn_exp2f(sk - m_s));
-      const float v[4] = {o[0] * inv, o[1] * inv, o[2] * inv, o[3] * inv};
-      store4(out + ((long)t * H + h) * CP + c_base + c, v);
-    }
-  }
-}
-
-// merge key ranges; a range without keys has m = -inf
-template <typename T>
-__global__ __launch_bounds__(128) void latent_combine_kernel(
-    const float* __restrict__ part_o, const float* __restrict__ part_ml,
-    const T* __restrict__ sink, T* __restrict__ out, int splits, int H,
-    int CP) {
-  const long th = blockIdx.x;
-  const float sk = sink ? to_f32(sink[th % H]) * LOG2E : -INFINITY;
-  float m = sk;  // some range has a key: m ends finite
-  for (int s = 0; s < splits; ++s)
-    m = fmaxf(m, part_ml[(th * splits + s) * 2]);
-  float l = exp2f(sk - m);
-  for (int s = 0; s < splits; ++s)
-    l += part_ml[(th * splits + s) * 2 + 1] *
-         exp2f(part_ml[(th * splits + s) * 2] - m);
-  const float inv = 1.f / l;
-  for (int c = threadIdx.x * 4; c < CP; c += 128 * 4) {
-    float f[4] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int s = 0; s < splits; ++s) {
-      // an empty range wrote zeros and weighs exp2(-inf) = 0
-      const float e = exp2f(part_ml[(th * splits + s) * 2] - m) * inv;
-      const lm_f32x4 o = *reinterpret_cast<const lm_f32x4*>(
-          part_o + (th * splits + s) * CP + c);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) f[r] += o[r] * e;
-    }
-    store4(out + th * CP + c, f);
-  }
+  // the wave's own tile region holds its sums
+  const int cols = min(NT * 16, CP - c_base);
+  meet_waves<NT>(
+      acc, m_run, l_run, cols, min(16, H - h0), stat,
+      (float*)(qs + 16 * PITCH), 32 * PITCH * (int)sizeof(T) / 4,
+      [&](int r, int c, const lm_f32x4& o, float m, float l) {
+        const int h = h0 + r;
+        if (splits > 1) {
+          const long pi = ((long)t * H + h) * splits + split;
+          const float v[4] = {o[0], o[1], o[2], o[3]};
+          store4(part_o + pi * CP + c_base + c, v);
+          if (c == 0 && c_base == 0) {
+            part_ml[2 * pi] = m;
+            part_ml[2 * pi + 1] = l;
+          }
+        } else {
+          const float inv = over_weights(
+              m, l, sink ? to_f32(sink[h]) * LM_LOG2E : -INFINITY);
+          const float v[4] = {o[0] * inv, o[1] * inv, o[2] * inv, o[3] * inv};
+          store4(out + ((long)t * H + h) * CP + c_base + c, v);
+        }
+      });
 }
 
 }  // namespace
-
-static Rot make_rot(const torch::Tensor& inv_freq, double gain, bool half,
-                    long RP) {
-  LM_CHECK_CONTIG(inv_freq);
-  TORCH_CHECK(inv_freq.scalar_type() == at::kFloat);
-  const long pairs = inv_freq.numel();
-  TORCH_CHECK(2 * pairs <= RP && pairs <= 256, "rotated size too large");
-  return Rot{inv_freq.data_ptr<float>(), (int)pairs, half ? 1 : 0,
-             (float)gain};
-}
-
-// [T, cols] view with 16-byte aligned rows
-static void check_rows(const torch::Tensor& v, long T, long cols,
-                       at::ScalarType type) {
-  TORCH_CHECK(v.is_cuda() && v.dim() == 2 && v.size(0) == T &&
-                  v.size(1) == cols && v.stride(1) == 1 &&
-                  v.stride(0) % 8 == 0 && v.storage_offset() % 8 == 0 &&
-                  v.scalar_type() == type,
-              "lm: operand rows do not fit");
-}
 
 // q [T, heads * (DP + RP)]; lat [T, CP + RP] with kv_norm and cache; cq
 // [T, QP] (same row stride as lat) with q_norm -> returned normed rows
@@ -488,7 +382,7 @@ c10::optional<torch::Tensor> lm_latent_prep(
   const Rot rot = make_rot(inv_freq, gain, half, RP);
   TORCH_CHECK(slots.numel() == T);
   TORCH_CHECK(n_abs >= 0 && n_abs <= T);
-  if (q) check_rows(*q, T, heads * (DP + RP), type);
+  if (q) lm_check_rows(*q, T, heads * (DP + RP), type);
   if (n_abs > 0) {
     TORCH_CHECK(q.has_value() && q_abs.has_value());
     LM_CHECK_CONTIG(*q_abs);
@@ -497,7 +391,7 @@ c10::optional<torch::Tensor> lm_latent_prep(
   }
   long n_slots = 0;
   if (lat) {
-    check_rows(*lat, T, CP + RP, type);
+    lm_check_rows(*lat, T, CP + RP, type);
     TORCH_CHECK(cache.has_value() && kv_norm.has_value());
     LM_CHECK_CONTIG(*cache);
     TORCH_CHECK(cache->dim() == 3 && cache->size(2) == CP + RP &&
@@ -511,7 +405,7 @@ c10::optional<torch::Tensor> lm_latent_prep(
   if (cq) {
     QP = cq->size(1);
     TORCH_CHECK(lat.has_value() && QP % 8 == 0 && q_rank >= 1);
-    check_rows(*cq, T, QP, type);
+    lm_check_rows(*cq, T, QP, type);
     TORCH_CHECK(T <= 1 || cq->stride(0) == lat->stride(0));
     TORCH_CHECK(q_norm.has_value() && q_norm->is_contiguous() &&
                 q_norm->numel() == QP && q_norm->scalar_type() == type);
@@ -582,7 +476,7 @@ void lm_head_gemm(torch::Tensor a, torch::Tensor w, torch::Tensor out,
     TORCH_CHECK(positions->numel() >= M);
     rot = make_rot(*inv_freq, gain, half, RP);
   }
-  if (gate) check_rows(*gate, M, (long)H * N, w.scalar_type());
+  if (gate) lm_check_rows(*gate, M, (long)H * N, w.scalar_type());
   if (M == 0) return;
   TORCH_CHECK((M + 15) / 16 <= 65535 && H <= 65535);
   LM_DISPATCH(w, "lm_head_gemm", [&] {
@@ -688,11 +582,12 @@ torch::Tensor lm_latent_attention(torch::Tensor q_abs, torch::Tensor cache,
       default: LM_LA(32); break;
     }
     if (splits > 1)
-      hipLaunchKernelGGL((latent_combine_kernel<scalar_t>), dim3(n * H),
+      hipLaunchKernelGGL((combine_ranges_kernel<scalar_t>), dim3(n * H),
                          dim3(128), 0, st, po.data_ptr<float>(),
                          pml.data_ptr<float>(),
                          sink ? (const scalar_t*)sink->data_ptr() : nullptr,
-                         (scalar_t*)out.data_ptr(), (int)splits, H, (int)CP);
+                         (scalar_t*)out.data_ptr(), H * CP, (int)splits, H,
+                         (int)CP, 1.f);
   });
 #undef LM_LA
   LM_LAUNCHED();

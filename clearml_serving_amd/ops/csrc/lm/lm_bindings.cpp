@@ -29,8 +29,31 @@ Tensor lm_latent_attention(Tensor q_abs, Tensor cache, Tensor block_table,
 void lm_latent_prompt(Tensor q, Tensor kv, Tensor lat, Opt sink,
                       Tensor qtiles, Tensor out, long H, long DP, long RP,
                       long CP, long VP, long window, double scale, Opt gate);
-std::vector<Tensor> lm_moe_route(Tensor h, Tensor router, long top,
-                                 long rows);
+void lm_grouped_prompt(Tensor q, Tensor rows, Opt sink, Tensor qtiles,
+                       Tensor out, long H, long G, long KD, long VD, bool same,
+                       long window, long keep, double scale, double cap,
+                       double out_scale);
+void lm_grouped_prep(Tensor z, long k_at, long v_at, Tensor positions,
+                     Tensor slots, Opt inv_freq, double gain, long H, long G,
+                     long KD, long VD, long dim, Opt q_norm, Opt k_norm,
+                     double eps, Opt first, double lam, Tensor cache);
+void lm_grouped_attention(Tensor q, Tensor cache, Tensor block_table,
+                          Tensor tok_seq, Tensor positions, Opt sink,
+                          Tensor out, long n, long H, long G, long KD, long VD,
+                          bool same, long window, long keep, double scale,
+                          double cap, double out_scale, long max_keys);
+void lm_delta_rule(Tensor z, std::vector<long> at, Tensor w2, Tensor w0,
+                   Tensor ab, Tensor norm, Tensor state, Tensor positions,
+                   Tensor slots, Tensor seqs, Tensor out, long n_single,
+                   long dim, double eps, double out_scale);
+std::vector<Tensor> lm_hyper_embed(Tensor tokens, Tensor table, Tensor coef,
+                                   long S, long n, double eps);
+Tensor lm_hyper_step(Tensor o, Tensor x, Tensor coef, long n, double eps,
+                     bool last, Opt pos, Opt share, Opt skip);
+Tensor lm_soft_cap(Tensor z, long n, double cap);
+std::vector<Tensor> lm_moe_route(Tensor h, Tensor router, long top, long rows,
+                                 bool over_all, Opt correction, long groups,
+                                 long keep, long identity, long shared);
 Tensor lm_moe_gemm(Tensor a, Opt tok, Tensor w, Tensor plan, long n_rows,
                    long rows, long act);
 void lm_rglru_prefill(Tensor yx, Tensor byx, Tensor cw, Tensor cb, Tensor ra,
@@ -55,6 +78,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("lm_head_gemm", &lm_head_gemm);
   m.def("lm_latent_attention", &lm_latent_attention);
   m.def("lm_latent_prompt", &lm_latent_prompt);
+  m.def("lm_grouped_prompt", &lm_grouped_prompt);
+  m.def("lm_grouped_prep", &lm_grouped_prep);
+  m.def("lm_grouped_attention", &lm_grouped_attention);
+  m.def("lm_delta_rule", &lm_delta_rule);
+  m.def("lm_hyper_embed", &lm_hyper_embed);
+  m.def("lm_hyper_step", &lm_hyper_step);
+  m.def("lm_soft_cap", &lm_soft_cap);
   m.def("lm_moe_route", &lm_moe_route);
   m.def("lm_moe_gemm", &lm_moe_gemm);
   m.def("lm_rglru_prefill", &lm_rglru_prefill);

@@ -192,7 +192,10 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
   return z * sigmoid_f(2.f * k);
 }
 // activations that kernels take as a template argument
-enum { LM_GELU_TANH = 0, LM_SILU = 1, LM_RELU2 = 2, LM_NO_ACT = 3 };
+enum {
+  LM_GELU_TANH = 0, LM_SILU = 1, LM_RELU2 = 2, LM_NO_ACT = 3,
+  LM_SWIGLU = 4  // gated products: silu(gate) * up of column pairs
+};
 template <int ACT> __device__ __forceinline__ float act_f(float z) {
   if (ACT == LM_GELU_TANH) return gelu_tanh_f(z);
   if (ACT == LM_SILU) return z * sigmoid_f(z);

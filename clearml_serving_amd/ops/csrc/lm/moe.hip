@@ -5,7 +5,9 @@
 // (pos: slot -> row, tok: row -> token); a tile list cuts each expert's rows
 // into pieces of at most `rows` rows. A grouped product runs one workgroup per
 // (tile, column range) and takes its row count from the list, so nothing is
-// read back to the host. The list's length lies in device memory: a launch
+// read back to the host. Shared experts, which every token takes, are slots
+// behind the `top` chosen ones; identity experts, whose output is the input,
+// have no rows (pos -1). The list's length lies in device memory: a launch
 // covers the most tiles there can be and the surplus workgroups leave at once.
 // A row's result does not depend on where its expert's rows end up.
 #include "lm_common.h"
@@ -83,32 +85,92 @@ __device__ __forceinline__ void router_tiles(const T* hr, const T* router,
   }
 }
 
-// Logits in float, the `top` largest (ties: the lower expert), softmax over
-// them. Counts per expert and each slot's rank in it for the grouping; a
-// single workgroup groups right away. KW: waves, which split the inner
-// dimension.
+// How the chosen experts are found and weighed.
+// over_all: scores are the softmax over all outputs, the choice is by score +
+// correction within the `keep` best of `groups` equal groups (a group's score:
+// its largest choice), weights are the scores. Else by logit, weights are the
+// softmax over the chosen logits.
+struct Routing {
+  const float* correction;  // null: none
+  int E;         // outputs that can be chosen
+  int real;      // experts with weights; those behind are identities
+  int shared;    // slots of shared experts, behind the chosen ones
+  int top, groups, keep;
+  bool over_all;
+  // router row E: gate of the shared experts
+  __host__ __device__ int rows() const { return E + (shared > 0 ? 1 : 0); }
+  __host__ __device__ int slots() const { return top + shared; }
+  __host__ __device__ int plan() const { return real + shared; }
+};
+
+// One token's logits z [E] -> scores s = softmax, choices (in z's place), by
+// one wave. gmax: a float per group.
+__device__ __forceinline__ void choice_scores(float* z, float* s, float* gmax,
+                                              const Routing& how, int EP) {
+  const int lane = threadIdx.x & 63, E = how.E;
+  float mx = -INFINITY;
+  for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[e]);
+  mx = wave_reduce_max(mx);
+  float sum = 0.f;
+  for (int e = lane; e < E; e += 64) {
+    s[e] = expf(z[e] - mx);
+    sum += s[e];
+  }
+  sum = wave_reduce_sum(sum);
+  for (int e = lane; e < E; e += 64) {
+    s[e] /= sum;
+    z[e] = s[e] + (how.correction ? how.correction[e] : 0.f);
+  }
+  wave_lds_fence();
+  if (how.keep >= how.groups) return;
+  const int size = E / how.groups;
+  for (int q = lane; q < how.groups; q += 64) {
+    float m = -INFINITY;
+    for (int e = q * size; e < (q + 1) * size; ++e) m = fmaxf(m, z[e]);
+    gmax[q] = m;
+  }
+  wave_lds_fence();
+  for (int e = lane; e < E; e += 64) {
+    const int q = e / size;
+    const float mine = gmax[q];
+    int place = 0;
+    for (int j = 0; j < how.groups; ++j)
+      place += gmax[j] > mine || (gmax[j] == mine && j < q);
+    if (place >= how.keep) z[e] = -INFINITY;
+  }
+  wave_lds_fence();
+}
+
+// Logits in float, the `top` best (ties: the lower expert), their weights.
+// Counts per expert and each slot's rank in it for the grouping; a single
+// workgroup groups right away. KW: waves, which split the inner dimension.
 template <typename T, int KW>
 __global__ __launch_bounds__(KW * 64) void moe_route_kernel(
     const T* __restrict__ h, const T* __restrict__ router, int n_tok, int K,
-    int E, int top, float* __restrict__ share, int* __restrict__ ids,
+    Routing how, float* __restrict__ share, int* __restrict__ ids,
     int* __restrict__ rank, int* __restrict__ counts, int* __restrict__ pos,
     int* __restrict__ tok, int rows, int* __restrict__ tiles,
     int* __restrict__ n_tiles) {
   constexpr int NTH = KW * 64;
   constexpr int PER = RT * MAX_TOP / NTH;  // most slots of a thread
   __shared__ __align__(16) float part[KW][RT][64 + 4];
+  __shared__ float gate[RT];
   extern __shared__ __align__(16) char smem[];
+  const int E = how.E, top = how.top, NR = how.rows(), PE = how.plan();
+  const int TS = how.slots();
   const int EP = (E + 3) & ~3;
   float* logits = (float*)smem;            // [RT][EP]
   float* best = logits + RT * EP;          // [RT][top]
   int* chosen = (int*)(best + RT * top);   // [RT][top]
-  int* cnt = chosen + RT * top;            // [E]
-  int* off = cnt + E;                      // [E]
+  int* cnt = chosen + RT * top;            // [PE]
+  int* off = cnt + PE;                     // [PE]
+  float* score = (float*)(off + PE);       // [RT][EP] if over_all
+  float* group = score + RT * EP;          // [KW][groups] if over_all
   const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave();
   const int r16 = lane & 15, ko = (lane >> 4) * 8;
   const int t0 = blockIdx.x * RT;
   const int nt = min(RT, n_tok - t0);
-  for (int e = tid; e < E; e += NTH) cnt[e] = 0;
+  for (int e = tid; e < PE; e += NTH) cnt[e] = 0;
   // whatever the logits are (nan), every slot has an expert
   for (int i = tid; i < RT * top; i += NTH) {
     chosen[i] = i % top;
@@ -118,14 +180,14 @@ __global__ __launch_bounds__(KW * 64) void moe_route_kernel(
   const T* hr = h + (long)min(t0 + r16, n_tok - 1) * K + ko;
   const int steps = K / 32, per = (steps + KW - 1) / KW;
   const int k_lo = wave * per * 32, k_hi = min(K, k_lo + per * 32);
-  for (int e0 = 0; e0 < E; e0 += 64) {
+  for (int e0 = 0; e0 < NR; e0 += 64) {
     const T* wr = router + ko;
-    if (E - e0 <= 16)
-      router_tiles<T, 1>(hr, wr, e0, E, K, k_lo, k_hi, &part[wave][r16][0]);
-    else if (E - e0 <= 32)
-      router_tiles<T, 2>(hr, wr, e0, E, K, k_lo, k_hi, &part[wave][r16][0]);
+    if (NR - e0 <= 16)
+      router_tiles<T, 1>(hr, wr, e0, NR, K, k_lo, k_hi, &part[wave][r16][0]);
+    else if (NR - e0 <= 32)
+      router_tiles<T, 2>(hr, wr, e0, NR, K, k_lo, k_hi, &part[wave][r16][0]);
     else
-      router_tiles<T, 4>(hr, wr, e0, E, K, k_lo, k_hi, &part[wave][r16][0]);
+      router_tiles<T, 4>(hr, wr, e0, NR, K, k_lo, k_hi, &part[wave][r16][0]);
     __syncthreads();
     for (int i = tid; i < RT * 64; i += NTH) {
       const int t = i >> 6, e = e0 + (i & 63);
@@ -133,13 +195,16 @@ __global__ __launch_bounds__(KW * 64) void moe_route_kernel(
 #pragma unroll
       for (int w = 0; w < KW; ++w) s += part[w][t][i & 63];
       if (e < EP) logits[t * EP + e] = e < E ? s : -INFINITY;
+      if (e == E && NR > E) gate[t] = 1.f / (1.f + expf(-s));
     }
     __syncthreads();
   }
 
   // an expert's place is the number of experts in front of it
   for (int t = wave; t < nt; t += KW) {
-    const float* z = logits + t * EP;
+    float* z = logits + t * EP;
+    if (how.over_all)
+      choice_scores(z, score + t * EP, group + wave * how.groups, how, EP);
     for (int e = lane; e < E; e += 64) {
       const float mine = z[e];
       int place = 0;
@@ -152,45 +217,56 @@ __global__ __launch_bounds__(KW * 64) void moe_route_kernel(
       }
       if (place < top) {
         chosen[t * top + place] = e;
-        best[t * top + place] = mine;
+        best[t * top + place] = how.over_all ? score[t * EP + e] : mine;
       }
     }
     wave_lds_fence();
-    const float v = lane < top ? expf(best[t * top + lane] - best[t * top])
-                               : 0.f;
-    const float sum = wave_reduce_sum(v);
-    if (lane < top) share[(long)(t0 + t) * top + lane] = v / sum;
+    float v = lane < top ? best[t * top + lane] : 0.f;
+    if (!how.over_all) {
+      v = lane < top ? expf(v - best[t * top]) : 0.f;
+      v /= wave_reduce_sum(v);
+    }
+    if (lane >= top) v = gate[t];
+    if (lane < TS) share[(long)(t0 + t) * TS + lane] = v;
   }
   __syncthreads();
   const bool alone = gridDim.x == 1;
+  // a slot's expert in the plan, -1: an identity
+  auto plan_expert = [&](int s) {
+    const int k = s % TS;
+    if (k >= top) return how.real + k - top;
+    const int e = chosen[s / TS * top + k];
+    return e < how.real ? e : -1;
+  };
   int rk[PER];
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
     const int s = tid + j * NTH;
     rk[j] = 0;
-    if (s < nt * top) {
-      const int e = chosen[s];
-      rk[j] = atomicAdd(&cnt[e], 1);
+    if (s < nt * TS) {
+      const int e = plan_expert(s);
+      if (e >= 0) rk[j] = atomicAdd(&cnt[e], 1);
       if (!alone) {
-        ids[(long)t0 * top + s] = e;
-        rank[(long)t0 * top + s] = rk[j];
+        ids[(long)t0 * TS + s] = e;
+        rank[(long)t0 * TS + s] = rk[j];
       }
     }
   }
   __syncthreads();
   if (!alone) {
-    for (int e = tid; e < E; e += NTH)
-      counts[(long)blockIdx.x * E + e] = cnt[e];
+    for (int e = tid; e < PE; e += NTH)
+      counts[(long)blockIdx.x * PE + e] = cnt[e];
     return;
   }
-  scan_experts(cnt, off, E, rows, tiles, n_tiles);
+  scan_experts(cnt, off, PE, rows, tiles, n_tiles);
 #pragma unroll
   for (int j = 0; j < PER; ++j) {
     const int s = tid + j * NTH;
-    if (s < nt * top) {
-      const int p = off[chosen[s]] + rk[j];
+    if (s < nt * TS) {
+      const int e = plan_expert(s);
+      const int p = e < 0 ? -1 : off[e] + rk[j];
       pos[s] = p;
-      tok[p] = s / top;
+      if (p >= 0) tok[p] = s / TS;
     }
   }
 }
@@ -227,9 +303,34 @@ __global__ __launch_bounds__(256) void moe_place_kernel(
   for (int i = tid; i < n; i += 256) {
     const long s = (long)b * RT * top + i;
     const int e = ids[s];
-    const int p = off[e] + bef[e] + rank[s];
+    const int p = e < 0 ? -1 : off[e] + bef[e] + rank[s];
     pos[s] = p;
-    tok[p] = (int)(s / top);
+    if (p >= 0) tok[p] = (int)(s / top);
+  }
+}
+
+// Four neighbouring columns of a product, behind their activation. A gated one
+// (LM_SWIGLU) takes columns in pairs (gate, up) and makes one of each.
+template <int ACT> __host__ __device__ constexpr long out_cols(long n) {
+  return ACT == LM_SWIGLU ? n / 2 : n;
+}
+__device__ __forceinline__ void store2(bf16* p, float a, float b) {
+  union { unsigned u; bf16 h[2]; } o;
+  o.h[0] = __float2bfloat16(a);
+  o.h[1] = __float2bfloat16(b);
+  *reinterpret_cast<unsigned*>(p) = o.u;
+}
+__device__ __forceinline__ void store2(float* p, float a, float b) {
+  *reinterpret_cast<float2*>(p) = float2{a, b};
+}
+template <typename T, int ACT>
+__device__ __forceinline__ void store_act(T* p, const lm_f32x4& s) {
+  if (ACT == LM_SWIGLU) {
+    store2(p, act_f<LM_SILU>(s[0]) * s[1], act_f<LM_SILU>(s[2]) * s[3]);
+  } else {
+    const float f[4] = {act_f<ACT>(s[0]), act_f<ACT>(s[1]), act_f<ACT>(s[2]),
+                        act_f<ACT>(s[3])};
+    store4(p, f);
   }
 }
 
@@ -322,9 +423,8 @@ __global__ __launch_bounds__(GW * 64) void moe_rows_kernel(
 #pragma unroll
     for (int v = 0; v < GW; ++v)
       s += *reinterpret_cast<const lm_f32x4*>(&part[v][m][c]);
-    const float f[4] = {act_f<ACT>(s[0]), act_f<ACT>(s[1]), act_f<ACT>(s[2]),
-                        act_f<ACT>(s[3])};
-    store4(out + (long)(r0 + m) * N + n0 + c, f);
+    store_act<T, ACT>(out + (long)(r0 + m) * out_cols<ACT>(N) +
+                          out_cols<ACT>(n0 + c), s);
   }
 }
 
@@ -463,15 +563,12 @@ void moe_tile_kernel(
   for (int j = 0; j < FM; ++j) {
     const int m = wm + j * 16 + r16;
     if (m < cnt) {
-      bf16* dst = out + (long)(r0 + m) * N + n0 + wn + 4 * g;
+      bf16* dst = out + (long)(r0 + m) * out_cols<ACT>(N) +
+                  out_cols<ACT>(n0 + wn + 4 * g);
 #pragma unroll
       for (int i = 0; i < FN; ++i) {
-        if (n0 + wn + i * 16 < N) {
-          const float f[4] = {
-              act_f<ACT>(acc[i][j][0]), act_f<ACT>(acc[i][j][1]),
-              act_f<ACT>(acc[i][j][2]), act_f<ACT>(acc[i][j][3])};
-          store4(dst + i * 16, f);
-        }
+        if (n0 + wn + i * 16 < N)
+          store_act<bf16, ACT>(dst + out_cols<ACT>(i * 16), acc[i][j]);
       }
     }
   }
@@ -484,48 +581,77 @@ long max_tiles(long S, long E, long rows) {
 
 }  // namespace
 
-// -> {share float [T, top], pos int [T, top], tok int [T * top],
+// Without `correction` and groups (0): the `top` largest logits, weighed by the
+// softmax over them. router [choices (+ 1 gate row with shared slots), K].
+// -> {share float [T, slots], pos int [T, slots], tok int [T * slots],
 //     plan int [1 + 3 * tiles]: the number of tiles, then (expert, first row,
-//     rows) each}
+//     rows) each}; slots = top + shared
 std::vector<torch::Tensor> lm_moe_route(torch::Tensor h, torch::Tensor router,
-                                        long top, long rows) {
+                                        long top, long rows, bool over_all,
+                                        c10::optional<torch::Tensor> correction,
+                                        long groups, long keep, long identity,
+                                        long shared) {
   LM_CHECK_CONTIG(h);
   LM_CHECK_CONTIG(router);
   TORCH_CHECK(h.dim() == 2 && router.dim() == 2 &&
               h.size(1) == router.size(1) &&
               h.scalar_type() == router.scalar_type());
-  const int T = h.size(0), K = h.size(1), E = router.size(0);
-  TORCH_CHECK(K % 32 == 0 && E >= 1 && E <= 1024, "lm_moe_route: sizes");
-  TORCH_CHECK(top >= 1 && top <= MAX_TOP && top <= E && rows >= 1);
-  TORCH_CHECK((long)T * top < (1L << 30));
+  Routing how{};
+  how.E = (int)router.size(0) - (shared > 0 ? 1 : 0);
+  how.real = how.E - (int)identity;
+  how.shared = (int)shared;
+  how.top = (int)top;
+  how.groups = (int)groups;
+  how.keep = (int)keep;
+  how.over_all = over_all;
+  const int T = h.size(0), K = h.size(1), E = how.E, PE = how.plan();
+  const int slots = how.slots();
+  TORCH_CHECK(K % 32 == 0 && E >= 1 && E <= 1024 && PE <= 1024,
+              "lm_moe_route: sizes");
+  TORCH_CHECK(top >= 1 && slots <= MAX_TOP && top <= E && rows >= 1);
+  TORCH_CHECK(identity >= 0 && shared >= 0 && PE >= 1 && how.real >= 0);
+  TORCH_CHECK(groups >= 1 && keep >= 1 && keep <= groups && E % groups == 0,
+              "lm_moe_route: groups");
+  TORCH_CHECK(over_all || (groups == 1 && !correction));
+  if (correction) {
+    TORCH_CHECK(correction->is_cuda() && correction->is_contiguous() &&
+                correction->numel() == E &&
+                correction->scalar_type() == at::kFloat);
+    how.correction = correction->data_ptr<float>();
+  }
+  TORCH_CHECK((long)T * slots < (1L << 30));
   auto i32 = h.options().dtype(at::kInt);
-  const long S = (long)T * top;
-  auto share = torch::empty({T, top}, h.options().dtype(at::kFloat));
-  auto pos = torch::empty({T, top}, i32);
+  const long S = (long)T * slots;
+  auto share = torch::empty({T, slots}, h.options().dtype(at::kFloat));
+  auto pos = torch::empty({T, slots}, i32);
   auto tok = torch::empty({S}, i32);
-  auto plan = torch::empty({1 + 3 * max_tiles(S, E, rows)}, i32);
+  auto plan = torch::empty({1 + 3 * max_tiles(S, PE, rows)}, i32);
   if (T == 0) return {share, pos, tok, plan};
   const int n_wg = (T + RT - 1) / RT;
   torch::Tensor ids, rank, counts;
   if (n_wg > 1) {
     ids = torch::empty({S}, i32);
     rank = torch::empty({S}, i32);
-    counts = torch::empty({n_wg, E}, i32);
+    counts = torch::empty({n_wg, PE}, i32);
   }
   int* pp = plan.data_ptr<int>();
   hipStream_t st = cmls::current_stream();
 #define LM_MRT(KW)                                                           \
   do {                                                                       \
+    const int ep = (E + 3) & ~3;                                             \
     const int bytes =                                                        \
-        (RT * (((E + 3) & ~3) + 2 * (int)top) + 2 * E) * 4;                  \
+        (RT * (ep + 2 * (int)top) + 2 * PE +                                 \
+         (over_all ? RT * ep + KW * (int)groups : 0)) * 4;                   \
+    TORCH_CHECK(bytes + KW * RT * 68 * 4 + 8192 <= 160 * 1024,               \
+                "lm_moe_route: ", E, " outputs do not fit LDS");             \
     auto* fn = &moe_route_kernel<scalar_t, KW>;                              \
     HIP_CHECK(hipFuncSetAttribute(                                           \
         reinterpret_cast<const void*>(fn),                                   \
         hipFuncAttributeMaxDynamicSharedMemorySize, bytes));                 \
     hipLaunchKernelGGL(fn, dim3(n_wg), dim3(KW * 64), bytes, st,             \
                        (const scalar_t*)h.data_ptr(),                        \
-                       (const scalar_t*)router.data_ptr(), T, K, E,          \
-                       (int)top, share.data_ptr<float>(),                    \
+                       (const scalar_t*)router.data_ptr(), T, K, how,        \
+                       share.data_ptr<float>(),                              \
                        n_wg > 1 ? ids.data_ptr<int>() : nullptr,             \
                        n_wg > 1 ? rank.data_ptr<int>() : nullptr,            \
                        n_wg > 1 ? counts.data_ptr<int>() : nullptr,          \
@@ -540,9 +666,9 @@ std::vector<torch::Tensor> lm_moe_route(torch::Tensor h, torch::Tensor router,
   LM_LAUNCHED();
   if (n_wg > 1) {
     hipLaunchKernelGGL(moe_place_kernel, dim3(n_wg), dim3(256),
-                       3 * E * 4, st, ids.data_ptr<int>(),
+                       3 * PE * 4, st, ids.data_ptr<int>(),
                        rank.data_ptr<int>(), counts.data_ptr<int>(), n_wg, T,
-                       E, (int)top, pos.data_ptr<int>(), tok.data_ptr<int>(),
+                       PE, slots, pos.data_ptr<int>(), tok.data_ptr<int>(),
                        (int)rows, pp + 1, pp);
     LM_LAUNCHED();
   }
@@ -550,6 +676,7 @@ std::vector<torch::Tensor> lm_moe_route(torch::Tensor h, torch::Tensor router,
 }
 
 // out[r] = act(w[expert of r] @ a[tok[r]]); w [E, N, K]; tok absent: a[r].
+// LM_SWIGLU: rows of w in pairs (gate, up), out has N / 2 columns.
 // `rows`: rows per tile that the plan was made for
 torch::Tensor lm_moe_gemm(torch::Tensor a, c10::optional<torch::Tensor> tok,
                           torch::Tensor w, torch::Tensor plan, long n_rows,
@@ -561,7 +688,7 @@ torch::Tensor lm_moe_gemm(torch::Tensor a, c10::optional<torch::Tensor> tok,
               a.scalar_type() == w.scalar_type());
   const int E = w.size(0), N = w.size(1), K = w.size(2);
   TORCH_CHECK(N % 32 == 0 && K % 32 == 0, "lm_moe_gemm: sizes");
-  TORCH_CHECK(act == LM_RELU2 || act == LM_NO_ACT);
+  TORCH_CHECK(act == LM_RELU2 || act == LM_NO_ACT || act == LM_SWIGLU);
   if (tok) {
     LM_CHECK_I32(*tok);
     TORCH_CHECK(tok->numel() == n_rows);
@@ -570,7 +697,8 @@ torch::Tensor lm_moe_gemm(torch::Tensor a, c10::optional<torch::Tensor> tok,
   }
   const long nt = max_tiles(n_rows, E, rows);
   TORCH_CHECK(plan.numel() == 1 + 3 * nt, "lm_moe_gemm: plan for other rows");
-  auto out = torch::empty({n_rows, N}, a.options());
+  auto out = torch::empty({n_rows, act == LM_SWIGLU ? N / 2 : N},
+                          a.options());
   if (n_rows == 0) return out;
   TORCH_CHECK(a.size(0) > 0);
   hipStream_t st = cmls::current_stream();
@@ -591,6 +719,7 @@ torch::Tensor lm_moe_gemm(torch::Tensor a, c10::optional<torch::Tensor> tok,
 #define LM_MT_ACT(BM, BN, WM, WN, NS)                                       \
   do {                                                                      \
     if (act == LM_RELU2) LM_MT(BM, BN, WM, WN, NS, LM_RELU2);               \
+    else if (act == LM_SWIGLU) LM_MT(BM, BN, WM, WN, NS, LM_SWIGLU);        \
     else LM_MT(BM, BN, WM, WN, NS, LM_NO_ACT);                              \
   } while (0)
     if (rows == 256) LM_MT_ACT(256, 256, 2, 4, 2);
@@ -609,6 +738,7 @@ torch::Tensor lm_moe_gemm(torch::Tensor a, c10::optional<torch::Tensor> tok,
 #define LM_MR_ACT(MT, NT)                                                   \
   do {                                                                      \
     if (act == LM_RELU2) LM_MR(MT, NT, LM_RELU2);                           \
+    else if (act == LM_SWIGLU) LM_MR(MT, NT, LM_SWIGLU);                    \
     else LM_MR(MT, NT, LM_NO_ACT);                                          \
   } while (0)
     LM_DISPATCH(a, "lm_moe_gemm", [&] {

@@ -10,7 +10,7 @@ size, which leaves every product and sum of squares unchanged.
 """
 
 import math
-from typing import Optional, Tuple
+from typing import NamedTuple, Optional, Tuple, Union
 
 import torch
 
@@ -126,7 +126,7 @@ def linear_f32(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 
 
 # codes of csrc/lm/lm_common.h
-ACTIVATIONS = {"gelu_tanh": 0, "silu": 1, "relu2": 2, "none": 3}
+ACTIVATIONS = {"gelu_tanh": 0, "silu": 1, "relu2": 2, "none": 3, "swiglu": 4}
 
 
 def activate(z: torch.Tensor, act: str) -> torch.Tensor:
@@ -136,6 +136,8 @@ def activate(z: torch.Tensor, act: str) -> torch.Tensor:
         return torch.nn.functional.silu(z)
     if act == "relu2":
         return torch.relu(z).square()
+    if act == "swiglu":  # columns in pairs (gate, up)
+        return torch.nn.functional.silu(z[..., ::2]) * z[..., 1::2]
     return z
 
 
@@ -395,15 +397,33 @@ def latent_prompt(q: torch.Tensor, kv: torch.Tensor, lat: torch.Tensor,
 # mixture of experts
 # --------------------------------------------------------------------- #
 class ExpertPlan:
-    """Where a batch's T * top slots go: share, pos [T, top] weight and row
-    of each slot; tok [T * top] token of each row (rows in expert order);
-    plan: tiles of up to ``rows`` rows of one expert."""
+    """Where a batch's T * slots slots go: share, pos [T, slots] weight and
+    row of each slot (row -1: an identity expert); tok [T * slots] token of
+    each row (rows in expert order); plan: tiles of up to ``rows`` rows of one
+    expert."""
 
     __slots__ = ("share", "pos", "tok", "plan", "rows")
 
     def __init__(self, share, pos, tok, plan, rows):
         self.share, self.pos, self.tok = share, pos, tok
         self.plan, self.rows = plan, rows
+
+
+class Routing(NamedTuple):
+    """``over_all``: scores are the softmax over all router outputs, the
+    choice is by score + correction (where there is one) among the ``keep``
+    best of ``groups`` equal groups, and the weights are the scores;
+    otherwise the largest logits, weighed by the softmax over them. The last
+    ``identity`` outputs are identity experts. ``shared`` slots behind the
+    chosen ones go to experts that every token takes, weighed by the sigmoid
+    of one more router row."""
+
+    top: int
+    over_all: bool = False
+    groups: int = 1
+    keep: int = 1
+    identity: int = 0
+    shared: int = 0
 
 
 def expert_tile_rows(n_tok: int, experts: int, top: int, dtype,
@@ -421,36 +441,75 @@ def expert_tile_rows(n_tok: int, experts: int, top: int, dtype,
     return 128 if each <= 512 else 256
 
 
-def moe_route(h: torch.Tensor, router: torch.Tensor, top: int,
-              rows: int) -> ExpertPlan:
-    """The ``top`` experts with the largest logits router @ h, weighed by
-    the softmax over those logits; all of it in float."""
+def _choices(z: torch.Tensor, how: Routing,
+             correction: Optional[torch.Tensor]):
+    """-> chosen router outputs [T, top], their weights"""
+    if not how.over_all:
+        z, ids = torch.topk(z, how.top, dim=-1)
+        return ids, torch.softmax(z, -1)
+    s = torch.softmax(z, -1)
+    c = s if correction is None else s + correction
+    if how.keep < how.groups:
+        g = c.view(c.shape[0], how.groups, -1)
+        best = g.max(-1).values.topk(how.keep, dim=-1).indices
+        keep = torch.zeros(g.shape[:2], dtype=torch.bool)
+        keep.scatter_(1, best, True)
+        c = g.masked_fill(~keep[..., None], float("-inf")).view_as(c)
+    ids = torch.topk(c, how.top, dim=-1).indices
+    return ids, s.gather(1, ids)
+
+
+def moe_route(h: torch.Tensor, router: torch.Tensor,
+              how: Union[Routing, int], rows: int,
+              correction: Optional[torch.Tensor] = None) -> ExpertPlan:
+    """Experts of every token and their weights, all of it in float;
+    router [outputs (+ 1 with shared slots), K]. ``how`` can be the number
+    of experts alone."""
+    if isinstance(how, int):
+        how = Routing(how)
     if h.is_cuda:
         return ExpertPlan(*require_lm_ext("moe_route").lm_moe_route(
-            h, router, top, rows), rows)
-    z, ids = torch.topk(h.float() @ router.float().T, top, dim=-1)
+            h, router, how.top, rows, how.over_all, correction, how.groups,
+            how.keep, how.identity, how.shared), rows)
+    z = h.float() @ router.float().T
+    n = router.shape[0] - (1 if how.shared else 0)
+    ids, share = _choices(z[:, :n], how, correction)
+    real = n - how.identity
+    if how.shared:
+        ids = torch.cat([ids, (real + torch.arange(how.shared)).expand(
+            len(ids), -1) + how.identity], 1)
+        share = torch.cat([share, torch.sigmoid(z[:, n:]).expand(
+            -1, how.shared)], 1)
+    # number in the plan: experts, shared ones, identities last
     flat = ids.reshape(-1)
+    own = (flat >= real) & (flat < n)
+    flat = torch.where(flat >= n, flat - how.identity, flat)
+    flat = torch.where(own, real + how.shared, flat)
     order = torch.argsort(flat, stable=True)
     pos = torch.empty_like(order)
     pos[order] = torch.arange(order.numel())
-    return ExpertPlan(torch.softmax(z, -1), pos.view(ids.shape).int(),
-                      (order // top).int(), flat[order], rows)
+    pos[own] = -1
+    return ExpertPlan(share, pos.view(ids.shape).int(),
+                      (order // ids.shape[1]).int(), flat[order], rows)
 
 
 def moe_gemm(a: torch.Tensor, w: torch.Tensor, p: ExpertPlan, act: str,
              gather: bool) -> torch.Tensor:
     """out[r] = act(w[expert of row r] @ a[r]), a of row r's token with
-    ``gather``; w [experts, N, K]"""
+    ``gather``; w [experts, N, K]. ``swiglu``: rows of w in pairs (gate, up),
+    half as many columns."""
     n = p.tok.numel()
     if a.is_cuda:
         return require_lm_ext("moe_gemm").lm_moe_gemm(
             a, p.tok if gather else None, w, p.plan, n, p.rows,
             ACTIVATIONS[act])
     src = a[p.tok.long()] if gather else a
-    out = a.new_empty(n, w.shape[1])
+    out = a.new_zeros(n, w.shape[1] // (2 if act == "swiglu" else 1))
     for e in p.plan.unique().tolist():
-        at = p.plan == e
-        out[at] = activate(src[at].float() @ w[e].float().T, act).to(a.dtype)
+        if e < w.shape[0]:
+            at = p.plan == e
+            out[at] = activate(src[at].float() @ w[e].float().T,
+                               act).to(a.dtype)
     return out
 
 
