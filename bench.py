@@ -13,8 +13,8 @@ dynamic batcher -> hipGraph replay on the GPU) and awaits all responses.
 
   python bench.py --gpus N --steps K --warmup W
 
-``--workload lm`` measures another thing: prefill and decode of the Kakipel
-and Bimipel families beside llama at equal size (benchmarks/lm_bench.py).
+``--workload lm`` measures another thing: prefill and decode of the Pamazen,
+Kakipel and Bimipel families beside llama at equal size (benchmarks/lm_bench.py).
 """
 
 import argparse
@@ -121,9 +121,10 @@ def main():
     ap.add_argument("--workload", default="serving",
                     choices=("serving", "lm"),
                     help="serving: the headline benchmark; lm: prefill and "
-                         "decode of Kakipel and Bimipel beside llama")
+                         "decode of Pamazen, Kakipel and Bimipel beside "
+                         "llama")
     ap.add_argument("--lm-size", default="300m,1b,4k")
-    ap.add_argument("--lm-model", default="kakipel,bimipel,llama")
+    ap.add_argument("--lm-model", default="pamazen,kakipel,bimipel,llama")
     ap.add_argument("--lm-prompt", type=int, default=2048)
     ap.add_argument("--lm-batch", default="1,16,64")
     ap.add_argument("--lm-phase", default="prefill,decode")

@@ -267,7 +267,7 @@ PRESETS = {
     # layers as wide as an 8B model's
     "pamazen-4k": _stack(32000, 4096, 4, _attn_spec(32, 8, 128, 64, 128),
                          _parallel_spec(64, 8, 64, 2048, 16, 64, 64), 3,
-                         _moe(2048, 14, 4, 2, 4, 3, 2048)),
+                         _moe(2048, 12, 4, 4, 4, 3, 2048)),
 }
 
 

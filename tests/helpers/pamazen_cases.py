@@ -50,13 +50,14 @@ CONFIGS = {
         layer(attn(dim=16, rot=2, base=77.0, factor=1.0),
               moe(7, 1, 33, 2, (3, 2), 12))]),
     # one stream, one head, no group is left out, no identity expert, a
-    # window of one token
+    # window of one token (a head of one channel over its root mean square is
+    # near +-1: a large eps keeps it from amplifying)
     "ones": lambda: config([
         layer(parallel(left(1, 1, 40, 1, 1, 30.0), 1, 1, 1)),
         layer(attn(1, 1, 34, 2, 1), moe(3, 3, 1, 0, (1, 1), 1)),
         layer(parallel(left(17, 1, 4, 7, 0), 3, 40, 70), moe(1, 1, 5, 1,
                                                              (2, 2), 9))],
-        vocab=130, width=70, eps=1e-5, streams=1, mult=1.0),
+        vocab=130, width=70, eps=0.05, streams=1, mult=1.0),
     # sizes that the tiled products take; the first layer mixes
     "aligned": lambda: config([
         layer(attn(8, 2, 32, 16, 64, base=1e4), moe(10, 3, 64, 2, (3, 2),
