@@ -472,7 +472,8 @@ class DeltaRule(nn.Module):
         n = self.heads * self.dp
         delta.delta_rule(z, tuple(i * n for i in range(6)), self._w, state,
                          batch.positions, batch.state_slots, batch.seqs, out,
-                         batch.n_single, self.dim, self.eps, self.out_scale)
+                         batch.n_single, self.dim, self.eps, self.out_scale,
+                         batch.tiles.shape[0], batch.tile)
 
 
 class ParallelMixer(nn.Module):

@@ -10,14 +10,21 @@
 // same input; all else is float. The columns of S do not depend on each other,
 // so a workgroup keeps the whole state of one (sequence, head) in registers and
 // walks the sequence's tokens: a wave takes a range of columns, eight lanes
-// share a column's rows, sums over them are DPP adds. The tokens' vectors are
+// share a column's rows, sums over them are DPP adds. k v^T is taken as
+// u (|k| v)^T, so u is read once for both. The tokens' vectors are
 // made in tiles of 16 through LDS -- the low-rank product by MFMA in 32-bit,
 // next tile's projections in flight meanwhile -- and the outputs are normed and
 // gated from there. Single tokens are portions of one: same kernel.
 //
+// Few long portions would leave most CUs idle, so these are cut into chunks. A
+// token's step is S <- A S + k v^T; a chunk's is S <- P S + Q. The same walk
+// makes P, from the identity without values, and Q, from zero; a chain over the
+// chunks gives the state in front of each (delta_chain_kernel), and the chunks
+// are walked again from there, now with outputs.
+//
 // State in memory: [slot][head][value][key]. Slots are never cleared: position
 // 0 starts from zero.
-#include "lm_common.h"
+#include "lm_attn.h"
 
 namespace {
 
@@ -64,10 +71,18 @@ struct DeltaArgs {
   const int *positions, *slots, *seqs;
   int n_single, n_seq, n_state, heads, dim, RP;
   float eps, out_scale;
+  // chunks of `chunk` tiles of `tile` tokens; 0: whole portions
+  int n_chunks, tile, chunk;      // n_chunks: bound on all portions' chunks
+  float *P, *Q;                   // [n_chunks, heads, DP, DP]
 };
 
-// D: 32-channel blocks of a head, NW: waves
-template <typename T, int D, int NW>
+__device__ __forceinline__ int chunks_of(const int* portion, int chunk) {
+  return (portion[1] + chunk - 1) / chunk;
+}
+
+// D: 32-channel blocks of a head, NW: waves. COMPOSE: a chunk's P (grid z 1)
+// or Q (grid z 0) instead of outputs.
+template <typename T, int D, int NW, bool COMPOSE>
 __global__ __launch_bounds__(NW * 64, NW == 4 && D <= 2 ? 2 : 1)
 void delta_rule_kernel(DeltaArgs<T> p) {
   constexpr int DP = D * 32, NTH = NW * 64;
@@ -80,9 +95,8 @@ void delta_rule_kernel(DeltaArgs<T> p) {
   float* su = sm;                // [TT][DP] each
   float* sb = su + TT * DP;
   float* sw = sb + TT * DP;
-  float* sk = sw + TT * DP;
-  float* sr = sk + TT * DP;
-  float* sv = sr + TT * DP;      // values, then outputs
+  float* sr = sw + TT * DP;
+  float* sv = sr + TT * DP;      // values times |k|, then outputs
   float* ssq = sv + TT * DP;     // [NW][TT]
   const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave();
   const int r16 = lane & 15, g = lane >> 4;
@@ -90,12 +104,32 @@ void delta_rule_kernel(DeltaArgs<T> p) {
   const int h = blockIdx.x;
 
   int t0, len, p0, slot;
-  // long sequences first: they are the last of the list
-  if ((int)blockIdx.y < p.n_seq) {
+  const float* start = nullptr;  // state in front of a chunk
+  float* made = nullptr;         // where P or Q goes
+  bool ends = true;              // the portion ends here
+  const int n_work = p.chunk ? p.n_chunks : p.n_seq;
+  if (p.chunk && (int)blockIdx.y < n_work) {
+    int c = blockIdx.y, s = 0;  // chunk c of portion s
+    while (s < p.n_seq && c >= chunks_of(p.seqs + s * 6, p.chunk))
+      c -= chunks_of(p.seqs + s++ * 6, p.chunk);
+    if (s == p.n_seq) return;
+    const int* sd = p.seqs + s * 6;
+    ends = (c + 1) * p.chunk >= sd[1];
+    if (COMPOSE && ends) return;  // nothing follows
+    const int skip = c * p.chunk * p.tile;
+    t0 = sd[2] + skip;
+    len = min(p.chunk * p.tile, sd[3] - skip);
+    p0 = sd[4] + skip;
+    slot = sd[5];
+    const long at = ((long)blockIdx.y * p.heads + h) * DP * DP;
+    start = p.Q + at;
+    made = (blockIdx.z ? p.P : p.Q) + at;
+  } else if ((int)blockIdx.y < n_work) {
+    // long sequences first: they are the last of the list
     const int* sd = p.seqs + (p.n_seq - 1 - (int)blockIdx.y) * 6;
     t0 = sd[2], len = sd[3], p0 = sd[4], slot = sd[5];
   } else {
-    t0 = blockIdx.y - p.n_seq;
+    t0 = blockIdx.y - n_work;
     len = 1;
     p0 = p.positions[t0];
     slot = p.slots[t0];
@@ -110,10 +144,26 @@ void delta_rule_kernel(DeltaArgs<T> p) {
   for (int i = 0; i < CL; ++i)
 #pragma unroll
     for (int j = 0; j < D; ++j)
-      S[i][j] = p0 > 0 && has_state
-                    ? *reinterpret_cast<const lm_f32x4*>(
-                          st + (c0 + i) * DP + j * 32 + kg * 4)
-                    : lm_f32x4{0.f, 0.f, 0.f, 0.f};
+      S[i][j] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
+  if (COMPOSE) {
+    if (blockIdx.z) {
+#pragma unroll
+      for (int i = 0; i < CL; ++i)
+#pragma unroll
+        for (int j = 0; j < D; ++j)
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            S[i][j][e] = j * 32 + kg * 4 + e == c0 + i ? 1.f : 0.f;
+    }
+  } else if (start || (p0 > 0 && has_state)) {
+    const float* from = start ? start : st;
+#pragma unroll
+    for (int i = 0; i < CL; ++i)
+#pragma unroll
+      for (int j = 0; j < D; ++j)
+        S[i][j] = *reinterpret_cast<const lm_f32x4*>(
+            from + (c0 + i) * DP + j * 32 + kg * 4);
+  }
 
   // a lane prepares channels ch[c] + [0, 4) of token r16 of a tile
   bool live[CT];
@@ -154,7 +204,7 @@ void delta_rule_kernel(DeltaArgs<T> p) {
         Frag<float> tf;
         load8<T>(zr + k, tf.v);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) tf.v[e] = tanhf(tf.v[e]);
+        for (int e = 0; e < 8; ++e) tf.v[e] = cap_tanh<T>(tf.v[e]);
 #pragma unroll
         for (int c = 0; c < CT; ++c) {
           if (live[c]) {
@@ -181,7 +231,7 @@ void delta_rule_kernel(DeltaArgs<T> p) {
     sq = 0.f;
 #pragma unroll
     for (int w = 0; w < NW; ++w) sq += ssq[w * TT + r16];
-    const float inv = 1.f / sqrtf(sq + 1e-6f);
+    const float size = sqrtf(sq + 1e-6f), inv = 1.f / size;
 #pragma unroll
     for (int c = 0; c < CT; ++c) {
       if (live[c]) {
@@ -198,16 +248,17 @@ void delta_rule_kernel(DeltaArgs<T> p) {
         *reinterpret_cast<lm_f32x4*>(su + o) = u;
         *reinterpret_cast<lm_f32x4*>(sb + o) = b;
         *reinterpret_cast<lm_f32x4*>(sw + o) = w;
-        *reinterpret_cast<lm_f32x4*>(sk + o) = k;
-        *reinterpret_cast<lm_f32x4*>(sr + o) = floats(fr[c]);
-        *reinterpret_cast<lm_f32x4*>(sv + o) = floats(fv[c]);
+        if (!COMPOSE) *reinterpret_cast<lm_f32x4*>(sr + o) = floats(fr[c]);
+        *reinterpret_cast<lm_f32x4*>(sv + o) =
+            COMPOSE && blockIdx.z ? lm_f32x4{0.f, 0.f, 0.f, 0.f}
+                                  : size * floats(fv[c]);
       }
     }
     __syncthreads();
     if (at + TT < len) load(at + TT);
     Four<T> fg[ON];
 #pragma unroll
-    for (int i = 0; i < ON; ++i) {
+    for (int i = 0; i < (COMPOSE ? 0 : ON); ++i) {
       const int q = tid + i * NTH, tt = min(q / OC, nt - 1);
       fg[i] = load4(p.z + (long)(t0 + at + tt) * p.ld + p.g + h * DP +
                     q % OC * 4);
@@ -215,37 +266,32 @@ void delta_rule_kernel(DeltaArgs<T> p) {
 
     for (int t = 0; t < nt; ++t) {
       const int o = t * DP + kg * 4;
-      lm_f32x4 u[D], b[D], w[D], k[D], r[D];
+      lm_f32x4 u[D], b[D], w[D], r[D];
 #pragma unroll
       for (int j = 0; j < D; ++j) {
         u[j] = *reinterpret_cast<const lm_f32x4*>(su + o + j * 32);
         b[j] = *reinterpret_cast<const lm_f32x4*>(sb + o + j * 32);
         w[j] = *reinterpret_cast<const lm_f32x4*>(sw + o + j * 32);
-        k[j] = *reinterpret_cast<const lm_f32x4*>(sk + o + j * 32);
-        r[j] = *reinterpret_cast<const lm_f32x4*>(sr + o + j * 32);
+        if (!COMPOSE) r[j] = *reinterpret_cast<const lm_f32x4*>(sr + o + j * 32);
       }
       float y[CL];
 #pragma unroll
       for (int i = 0; i < CL; ++i) {
         const float v = sv[t * DP + c0 + i];
-        float x = 0.f;
+        lm_f32x4 a4 = u[0] * S[i][0];
 #pragma unroll
-        for (int j = 0; j < D; ++j)
-#pragma unroll
-          for (int e = 0; e < 4; ++e) x += u[j][e] * S[i][j][e];
-        x = sum8(x);
-        y[i] = 0.f;
+        for (int j = 1; j < D; ++j) a4 += u[j] * S[i][j];
+        const float x = sum8((a4[0] + a4[1]) + (a4[2] + a4[3]));
+        lm_f32x4 y4 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int j = 0; j < D; ++j) {
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            S[i][j][e] = w[j][e] * S[i][j][e] + (k[j][e] * v - b[j][e] * x);
-            y[i] += r[j][e] * S[i][j][e];
-          }
+          S[i][j] = w[j] * S[i][j] + (u[j] * v - b[j] * x);
+          if (!COMPOSE) y4 += r[j] * S[i][j];
         }
+        y[i] = (y4[0] + y4[1]) + (y4[2] + y4[3]);
       }
 #pragma unroll
-      for (int i = 0; i < CL; ++i) {
+      for (int i = 0; i < (COMPOSE ? 0 : CL); ++i) {
         y[i] = sum8(y[i]);
         // this column's value has been read by these eight lanes only
         if (kg == 0) sv[t * DP + c0 + i] = y[i];
@@ -255,7 +301,7 @@ void delta_rule_kernel(DeltaArgs<T> p) {
 
     // norm over the head, weight, gate
 #pragma unroll
-    for (int i = 0; i < ON; ++i) {
+    for (int i = 0; i < (COMPOSE ? 0 : ON); ++i) {
       const int q = tid + i * NTH, tt = q / OC, c = q % OC * 4;
       lm_f32x4 o = {0.f, 0.f, 0.f, 0.f};
       if (tt < nt) o = *reinterpret_cast<const lm_f32x4*>(sv + tt * DP + c);
@@ -282,25 +328,87 @@ void delta_rule_kernel(DeltaArgs<T> p) {
     }
   }
 
-  if (!has_state) return;
+  if (!COMPOSE && !(has_state && ends)) return;
+  float* to = COMPOSE ? made : st;
 #pragma unroll
   for (int i = 0; i < CL; ++i)
 #pragma unroll
     for (int j = 0; j < D; ++j)
-      *reinterpret_cast<lm_f32x4*>(st + (c0 + i) * DP + j * 32 + kg * 4) =
+      *reinterpret_cast<lm_f32x4*>(to + (c0 + i) * DP + j * 32 + kg * 4) =
           S[i][j];
+}
+
+// The state in front of every chunk of a portion, in Q's place: one workgroup
+// per head, portion and 16 columns of the state.
+constexpr int CHAIN_COLS = 16;
+template <int D>
+__global__ __launch_bounds__(256) void delta_chain_kernel(
+    const int* __restrict__ seqs, const float* __restrict__ state,
+    int n_state, int heads, int chunk, const float* __restrict__ P,
+    float* __restrict__ Q) {
+  constexpr int DP = D * 32, C4 = DP / 4;
+  constexpr int N = CHAIN_COLS * C4, PER = (N + 255) / 256;
+  __shared__ __align__(16) float s[CHAIN_COLS][DP];
+  const int h = blockIdx.x, v0 = blockIdx.z * CHAIN_COLS;
+  const int* sd = seqs + blockIdx.y * 6;
+  const int n = chunks_of(sd, chunk), p0 = sd[4], slot = sd[5];
+  int first = 0;  // chunks of the portions in front
+  for (int b = 0; b < (int)blockIdx.y; ++b)
+    first += chunks_of(seqs + b * 6, chunk);
+  const bool has = p0 > 0 && slot >= 0 && slot < n_state;
+  const float* st =
+      state + (((long)(has ? slot : 0) * heads + h) * DP + v0) * DP;
+  for (int g = threadIdx.x; g < N; g += 256)
+    *reinterpret_cast<lm_f32x4*>(&s[g / C4][g % C4 * 4]) =
+        has ? *reinterpret_cast<const lm_f32x4*>(st + g * 4)
+            : lm_f32x4{0.f, 0.f, 0.f, 0.f};
+  __syncthreads();
+  for (int k = 0; k < n; ++k) {
+    const long at = ((long)(first + k) * heads + h) * DP * DP;
+    const float* pc = P + at;
+    float* qc = Q + at + v0 * DP;
+    const bool more = k + 1 < n;  // else Q and P were not made
+    lm_f32x4 acc[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int g = threadIdx.x + i * 256;
+      if (g >= N) continue;
+      const int row = g / C4, c = g % C4 * 4;
+      lm_f32x4* q = reinterpret_cast<lm_f32x4*>(qc + g * 4);
+      if (more) {
+        lm_f32x4 a = *q;
+#pragma unroll 16
+        for (int j = 0; j < DP; ++j)
+          a += s[row][j] * *reinterpret_cast<const lm_f32x4*>(pc + j * DP + c);
+        acc[i] = a;
+      }
+      *q = *reinterpret_cast<const lm_f32x4*>(&s[row][c]);
+    }
+    if (!more) break;
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int g = threadIdx.x + i * 256;
+      if (g < N)
+        *reinterpret_cast<lm_f32x4*>(&s[g / C4][g % C4 * 4]) = acc[i];
+    }
+    __syncthreads();
+  }
 }
 
 }  // namespace
 
 // z [T, cols]: columns at[] = r, k, v, g, a (heads * DP each), w1 (RP); w2
 // [heads * DP, RP]; seqs [m, 6] as in rglru; the first n_single tokens are
-// sequences of their own. out [T, heads * DP], row stride free.
+// sequences of their own. out [T, heads * DP], row stride free. Portions are
+// cut into chunks of `chunk` tiles of `tile` tokens, 0: not at all; n_tiles:
+// tiles of all portions.
 void lm_delta_rule(torch::Tensor z, std::vector<long> at, torch::Tensor w2,
                    torch::Tensor w0, torch::Tensor ab, torch::Tensor norm,
                    torch::Tensor state, torch::Tensor positions,
                    torch::Tensor slots, torch::Tensor seqs, torch::Tensor out,
-                   long n_single, long dim, double eps, double out_scale) {
+                   long n_single, long dim, double eps, double out_scale,
+                   long n_tiles, long tile, long chunk) {
   LM_CHECK_I32(positions);
   LM_CHECK_I32(slots);
   LM_CHECK_I32(seqs);
@@ -330,16 +438,37 @@ void lm_delta_rule(torch::Tensor z, std::vector<long> at, torch::Tensor w2,
   TORCH_CHECK(dim >= 1 && dim <= DP);
   const int m = seqs.size(0);
   if (m + n_single == 0) return;
-  TORCH_CHECK(m + n_single <= 65535);
-#define LM_DR(D, NW)                                                         \
+  TORCH_CHECK(chunk >= 0 && tile >= 1 && n_tiles >= m);
+  if (m == 0) chunk = 0;
+  // every portion's last chunk may be short
+  const long n_chunks = chunk ? (n_tiles - m) / chunk + m : 0;
+  const long work = (chunk ? n_chunks : m) + n_single;
+  TORCH_CHECK(work <= 65535);
+  torch::Tensor P, Q;
+  if (chunk) {
+    P = torch::empty({n_chunks, heads, DP, DP}, state.options());
+    Q = torch::empty_like(P);
+  }
+  hipStream_t stream = cmls::current_stream();
+#define LM_DR_(D, NW, COMPOSE, GRID)                                         \
   do {                                                                       \
-    const int bytes = (6 * TT * DP + NW * TT) * 4;                           \
-    auto* fn = &delta_rule_kernel<scalar_t, D, NW>;                          \
+    const int bytes = (5 * TT * DP + NW * TT) * 4;                           \
+    auto* fn = &delta_rule_kernel<scalar_t, D, NW, COMPOSE>;                 \
     HIP_CHECK(hipFuncSetAttribute(                                           \
         reinterpret_cast<const void*>(fn),                                   \
         hipFuncAttributeMaxDynamicSharedMemorySize, bytes));                 \
-    hipLaunchKernelGGL(fn, dim3(heads, m + n_single), dim3(NW * 64), bytes,  \
-                       cmls::current_stream(), a);                           \
+    hipLaunchKernelGGL(fn, GRID, dim3(NW * 64), bytes, stream, a);           \
+  } while (0)
+#define LM_DR(D, NW)                                                         \
+  do {                                                                       \
+    if (chunk) {                                                             \
+      LM_DR_(D, NW, true, dim3(heads, n_chunks, 2));                         \
+      hipLaunchKernelGGL((delta_chain_kernel<D>),                            \
+                         dim3(heads, m, DP / CHAIN_COLS), dim3(256), 0,      \
+                         stream, a.seqs, state.data_ptr<float>(), a.n_state, \
+                         heads, (int)chunk, a.P, a.Q);                       \
+    }                                                                        \
+    LM_DR_(D, NW, false, dim3(heads, work));                                 \
   } while (0)
   LM_DISPATCH(z, "lm_delta_rule", [&] {
     DeltaArgs<scalar_t> a{};
@@ -369,6 +498,13 @@ void lm_delta_rule(torch::Tensor z, std::vector<long> at, torch::Tensor w2,
     a.RP = (int)RP;
     a.eps = (float)eps;
     a.out_scale = (float)out_scale;
+    a.n_chunks = (int)n_chunks;
+    a.tile = (int)tile;
+    a.chunk = (int)chunk;
+    if (chunk) {
+      a.P = P.data_ptr<float>();
+      a.Q = Q.data_ptr<float>();
+    }
     switch (DP) {
       case 32: LM_DR(1, 4); break;
       case 64: LM_DR(2, 4); break;
@@ -380,5 +516,6 @@ void lm_delta_rule(torch::Tensor z, std::vector<long> at, torch::Tensor w2,
     }
   });
 #undef LM_DR
+#undef LM_DR_
   LM_LAUNCHED();
 }

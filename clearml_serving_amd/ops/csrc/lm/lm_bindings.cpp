@@ -45,7 +45,8 @@ void lm_grouped_attention(Tensor q, Tensor cache, Tensor block_table,
 void lm_delta_rule(Tensor z, std::vector<long> at, Tensor w2, Tensor w0,
                    Tensor ab, Tensor norm, Tensor state, Tensor positions,
                    Tensor slots, Tensor seqs, Tensor out, long n_single,
-                   long dim, double eps, double out_scale);
+                   long dim, double eps, double out_scale, long n_tiles,
+                   long tile, long chunk);
 std::vector<Tensor> lm_hyper_embed(Tensor tokens, Tensor table, Tensor coef,
                                    long S, long n, double eps);
 Tensor lm_hyper_step(Tensor o, Tensor x, Tensor coef, long n, double eps,

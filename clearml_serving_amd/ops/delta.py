@@ -19,6 +19,15 @@ def head_pad(dim: int) -> int:
         dim, HEAD_SIZES[-1]))
 
 
+def chunk_tiles(tiles: int, seqs: int, heads: int) -> int:
+    """how many tiles make a chunk of a portion, 0: portions stay whole.
+    Chunks are walked twice, and once more without outputs, so cutting pays
+    where whole portions leave CUs idle."""
+    if seqs == 0 or seqs * heads > 160 or tiles < 6 * seqs:
+        return 0
+    return max(3, -(-tiles * heads // 1024))
+
+
 class DeltaWeights(NamedTuple):
     """w2 [heads * dp, rank] and w0 make the decay, ab the removal rate, norm
     weighs the output; [heads * dp] each."""
@@ -32,17 +41,19 @@ class DeltaWeights(NamedTuple):
 def delta_rule(z: torch.Tensor, at: Tuple[int, ...], w: DeltaWeights,
                state: torch.Tensor, positions: torch.Tensor,
                slots: torch.Tensor, seqs: torch.Tensor, out: torch.Tensor,
-               n_single: int, dim: int, eps: float, out_scale: float) -> None:
+               n_single: int, dim: int, eps: float, out_scale: float,
+               n_tiles: int, tile: int) -> None:
     """z [T, cols]: columns ``at`` of r, k, v, g, a (heads * dp each) and of
     the decay's low-rank input. The first n_single tokens are one token each
     of different sequences (``positions``, state ``slots``), the others
-    portions: seqs [m, 6], of which columns 2 to 5 are first token, tokens,
-    first position, state slot. state float [slots, heads, dp, dp] as
+    portions: seqs [m, 6] as in ops.lm.rglru_prefill, n_tiles tiles of
+    ``tile`` tokens in all. state float [slots, heads, dp, dp] as
     [value][key]; position 0 starts from zero. -> out [T, heads * dp]"""
     if z.is_cuda:
         require_lm_ext("delta_rule").lm_delta_rule(
             z, list(at), w.w2, w.w0, w.ab, w.norm, state, positions, slots,
-            seqs, out, n_single, dim, eps, out_scale)
+            seqs, out, n_single, dim, eps, out_scale, n_tiles, tile,
+            chunk_tiles(n_tiles, seqs.shape[0], state.shape[1]))
         return
     heads, dp = state.shape[1:3]
     f = z.float()

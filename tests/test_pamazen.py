@@ -28,7 +28,7 @@ from clearml_serving_amd.models.mixers import (DeltaRule,  # noqa: E402
                                                ExpertMlp, GroupedAttention,
                                                GroupedAttentionMixer,
                                                ParallelMixer)
-from clearml_serving_amd.ops import hyper, lm  # noqa: E402
+from clearml_serving_amd.ops import delta, hyper, lm  # noqa: E402
 
 REPO = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
@@ -454,6 +454,34 @@ def test_delta_rule(device, dtype, tol, heads, dim, rank):
     for portions in ([n], portions_of(n, [1]),
                      portions_of(n, [17, 2, 1, 16, 3])):
         assert rel(run_mixer(mod, h, portions, device, dtype), want) < tol
+
+
+@ALL
+@pytest.mark.parametrize("heads,dim,chunk", [
+    (2, 24, 1), (1, 64, 2), (2, 96, 1), (1, 128, 3), (1, 150, 1),
+    (1, 256, 2)])
+def test_delta_rule_in_chunks(device, dtype, tol, heads, dim, chunk,
+                              monkeypatch):
+    """long portions are cut, and walked from the states in front of the
+    chunks; portions end inside, at and right behind a chunk's end"""
+    monkeypatch.setattr(delta, "chunk_tiles", lambda *a: chunk)
+    m, n, width = {"heads": heads, "dim": dim}, 600, 36
+    st = random_state(cases.delta_shapes(m, width, 8), dim)
+    h = torch.randn(n, width, generator=torch.Generator().manual_seed(dim)) \
+        .to(torch.bfloat16)
+    want = plain.delta_rule(h.double(), double(st), m, EPS)
+    mod = DeltaOnly(width, heads, dim, EPS, 8)
+    mod.pack(st.__getitem__)
+    for portions in ([n], [128, 2, 192, 65, 1, 212], [5, 64, 531]):
+        assert rel(run_mixer(mod, h, portions, device, dtype), want) < tol
+
+
+def test_which_portions_are_cut():
+    assert delta.chunk_tiles(0, 0, 4) == 0  # none
+    assert delta.chunk_tiles(4, 1, 4) == 0  # short
+    assert delta.chunk_tiles(4000, 64, 16) == 0  # enough of them
+    for tiles, seqs, heads in ((128, 1, 16), (128, 4, 16), (2000, 1, 1)):
+        assert 3 <= delta.chunk_tiles(tiles, seqs, heads) < tiles / seqs
 
 
 def test_delta_oracle_tells_faults_apart():
