@@ -49,6 +49,7 @@ import torch
 from ... import ops
 from ...models import arch_of_config, token_batch_builder
 from ...models.llama import PRESETS, LlamaConfig, LlamaForCausalLM
+from ...ops.grouped import page_rows
 from .token_batch import TokenBatch
 
 
@@ -719,7 +720,8 @@ class LlmEngine:
                 cfg.arch, ", ".join(bad)))
 
     def _new_layer_caches(self, num_blocks: int, num_slots: int) -> List:
-        """Per layer run: page tensor [blocks, block_size, row], tuple (state
+        """Per layer run: page tensor [blocks, block_size, row] (with pooled
+        rows behind the tokens', see ops.grouped), tuple (state
         float [slots, ...], ring [slots, taps, channels] where there is one),
         the tensor of the run it shares with, or a tuple of two of these."""
         def zeros(dtype, *shape):
@@ -727,7 +729,8 @@ class LlmEngine:
 
         def make(kind, *dims):
             if kind == "paged":
-                return zeros(self.dtype, num_blocks, self.cfg.block_size,
+                return zeros(self.dtype, num_blocks,
+                             page_rows(self.cfg.block_size, *dims[1:] or (0,)),
                              dims[0])
             if kind == "state":
                 return tuple(zeros(dtype, num_slots, *shape) for shape, dtype
@@ -741,18 +744,19 @@ class LlmEngine:
             caches.append(make(*layout))
         return caches
 
-    @staticmethod
-    def _paged_elements(layout: tuple) -> int:
-        """cached elements per token of a layer run"""
+    def _page_elements(self, layout: tuple) -> int:
+        """cached elements per page of a layer run"""
         kind, *dims = layout
         if kind == "both":
-            return sum(LlmEngine._paged_elements(d) for d in dims)
-        return dims[0] if kind == "paged" else 0
+            return sum(map(self._page_elements, dims))
+        if kind != "paged":
+            return 0
+        return dims[0] * page_rows(self.cfg.block_size, *dims[1:] or (0,))
 
     def _start_token_batch_caches(self) -> None:
         cfg = self.cfg
-        row = sum(map(self._paged_elements, self.model.cache_layout()))
-        per_block = max(row, 1) * cfg.block_size * self.dtype.itemsize
+        page = sum(map(self._page_elements, self.model.cache_layout()))
+        per_block = max(page, 1) * self.dtype.itemsize
         if cfg.num_kv_blocks:
             num_blocks = int(cfg.num_kv_blocks)
         elif self.device.type == "cuda":

@@ -11,6 +11,7 @@ from typing import Any, Dict, List, Optional, Sequence as Seq
 import numpy as np
 import torch
 
+from ...ops.grouped import pooled_row, token_row
 from ...ops.lm import PROMPT_TILE
 
 
@@ -23,10 +24,10 @@ class TokenBatch:
     n_single: leading entries of one token (token i is entry i);
     n_abs: leading tokens whose attention runs in absorbed form;
     tiles [n, 5], seqs [m, 6]: recurrence tiles of the other entries (see
-    ops.lm.rglru_prefill); prompts: per view -- a window or (window, first
-    tokens that are kept) -- the cache rows that the entries behind the first
-    n_abs tokens can see and query tiles into them (see ops.lm.latent_prompt,
-    ops.grouped.prompt); max_keys: bound on position + 1 in the first n_abs
+    ops.lm.rglru_prefill); prompts: per view -- a window, (window, first
+    tokens that are kept) or (window, 0, tokens of a pooled block) -- the cache
+    rows that the entries behind the first n_abs tokens can see and query tiles
+    into them (see ops.lm.latent_prompt, ops.grouped.prompt); max_keys: bound on position + 1 in the first n_abs
     tokens."""
 
     mode = "token_batch"
@@ -78,19 +79,31 @@ class TokenBatch:
                 max_keys = max(max_keys, start + ln)
                 continue
             for w in windows:
-                size, keep = w if isinstance(w, tuple) else (w, 0)
+                size, keep, pool = (*w, 0)[:3] if isinstance(w, tuple) \
+                    else (w, 0, 0)
                 lo = max(0, start - size + 1) if size else 0
                 keep = min(keep, lo)
                 p = np.concatenate([
                     np.arange(keep, dtype=np.int32),
                     np.arange(lo, start + ln, dtype=np.int32)])
-                gathered[w].append(blocks[p // block_size] * block_size
-                                   + p % block_size)
+                rows = token_row(blocks[p // block_size], p % block_size,
+                                 block_size, pool)
+                n_pooled = []
+                if pool:  # of the blocks that the last token sees
+                    last = np.arange(pool - 1, start + ln - size, pool,
+                                     dtype=np.int32)
+                    rows = np.concatenate([
+                        pooled_row(blocks[last // block_size],
+                                   last % block_size, block_size, pool),
+                        rows])
+                    keep = len(last)
+                    n_pooled = [keep]
+                gathered[w].append(rows)
                 for j in range(0, ln, PROMPT_TILE):
                     qtiles[w].append([first[i] + j, min(PROMPT_TILE, ln - j),
                                       start + j, n_rows[w], lo - keep,
-                                      len(p)])
-                n_rows[w] += len(p)
+                                      len(rows)] + n_pooled)
+                n_rows[w] += len(rows)
         want = [first[i] + w for i in range(n) for w in plan["want"][i]]
         parts = {
             "positions": np.concatenate(pos),

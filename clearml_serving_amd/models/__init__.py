@@ -99,4 +99,4 @@ def load_weights(model: torch.nn.Module, path: str) -> None:
 
 
 from . import (bert, bimipel, gpt2, kakipel, llama,  # noqa: E402,F401
-               pamazen, resnet)  # (register architectures)
+               nelovik, pamazen, resnet)  # (register architectures)

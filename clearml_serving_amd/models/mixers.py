@@ -7,13 +7,13 @@ parameters; ``pack`` fills the padded, merged operands from tensors in
 checkpoint layout.
 """
 
-from typing import Callable, Dict, Optional, Tuple
+from typing import Callable, Dict, List, Optional, Tuple, Union
 
 import torch
 import torch.nn as nn
 
 from .. import ops
-from ..ops import delta, grouped, lm
+from ..ops import delta, grouped, linear_state, lm
 from ..ops.lm import pad32
 
 Get = Callable[[str], torch.Tensor]
@@ -222,9 +222,12 @@ class GroupedAttention(nn.Module):
     ``kv_heads`` cached key/value heads.
 
     ``rot``: (base, rotated dimensions, factor that divides the frequencies),
-    pairs (2i, 2i+1), or None. ``window`` 0: all earlier tokens; else the last
-    ``window`` and the first ``keep`` ones. ``cap``: scores become cap *
-    tanh(score / cap). ``qk_norm``: norm per head of queries and keys.
+    pairs (2i, 2i+1) or, ``rot_half``, (i, i + dimensions/2), or None.
+    ``window`` 0: all earlier tokens; else the last ``window`` and the first
+    ``keep`` ones, or in front of the window the mean key and value of every
+    whole block of ``pool`` tokens. ``cap``: scores become cap * tanh(score /
+    cap). ``qk_norm``: norm of queries and keys, "head" (or True) one by one,
+    "all" over all heads at once. ``bias``: on queries, keys and values.
     ``values_are_keys``: no projection of their own, the keys before norm and
     rotation. ``sink``: "learned" term per head in the softmax's denominator,
     "one" (a learned term of 0) or None. ``v_mix``: values mixed with those of
@@ -234,8 +237,10 @@ class GroupedAttention(nn.Module):
                  vdim: int, scale: float, eps: float = 0.0,
                  rot: Optional[Tuple[float, int, float]] = None,
                  window: int = 0, keep: int = 0, cap: float = 0.0,
-                 qk_norm: bool = False, values_are_keys: bool = False,
-                 sink: Optional[str] = None, v_mix: bool = False):
+                 qk_norm: Union[bool, str] = False,
+                 values_are_keys: bool = False, sink: Optional[str] = None,
+                 v_mix: bool = False, rot_half: bool = False, pool: int = 0,
+                 bias: bool = False):
         super().__init__()
         if kv_heads < 1 or heads % kv_heads:
             raise ValueError("{} query heads on {} key/value heads".format(
@@ -246,8 +251,14 @@ class GroupedAttention(nn.Module):
         if values_are_keys and (vdim != dim or v_mix or rot is not None):
             raise ValueError("values that are keys have the keys' size and "
                              "go with neither mixing nor rotation")
-        if keep and not window:
-            raise ValueError("kept tokens without a window")
+        if (keep or pool) and not window:
+            raise ValueError("kept tokens or pooled blocks without a window")
+        if keep and pool:
+            raise ValueError("kept tokens beside pooled blocks")
+        whole = qk_norm == "all"
+        if values_are_keys and (whole or pool or bias):
+            raise ValueError("values that are keys go with neither pooled "
+                             "blocks, biases nor a norm over all heads")
         if sink not in (None, "one", "learned"):
             raise ValueError("unknown sink '{}'".format(sink))
         self.width, self.heads, self.kv_heads = width, heads, kv_heads
@@ -256,14 +267,24 @@ class GroupedAttention(nn.Module):
         self.kp, self.vp = pad32(dim), pad32(vdim)
         self.spec = grouped.GroupedSpec(
             heads, kv_heads, self.kp, self.vp, dim, values_are_keys, window,
-            keep, scale, cap, 1.0)
+            keep, scale, cap, 1.0, pool, whole)
         # one product of h: [queries | keys | values]
         self.k_at = heads * self.kp
         self.v_at = self.k_at + kv_heads * self.kp
         self.cols = self.v_at + (0 if values_are_keys else
                                  kv_heads * self.vp)
-        self.q_norm = _param(self.kp) if qk_norm else None
-        self.k_norm = _param(self.kp) if qk_norm else None
+        self.q_norm = self.k_norm = None
+        if qk_norm:
+            self.q_norm = _param(self.kp * (heads if whole else 1))
+            self.k_norm = _param(self.kp * (kv_heads if whole else 1))
+        self.bias = _param(self.cols) if bias else None
+        # the kernels rotate neighbours: halves are brought together when
+        # weights are packed (scores do not depend on the channels' order)
+        self.order = None
+        if rot_half and rot is not None:
+            self.order = torch.arange(dim)
+            self.order[:rot[1]] = self.order[:rot[1]].view(2, -1).t() \
+                .reshape(-1)
         self.sink_kind = sink
         self.sink = None if sink is None else _param(heads)
         self.vmix = _param() if v_mix else None
@@ -273,6 +294,8 @@ class GroupedAttention(nn.Module):
     def view(self):
         """what a query sees, as TokenBatch names it"""
         s = self.spec
+        if s.pool:
+            return s.window, 0, s.pool
         return (s.window, s.keep) if s.keep else s.window
 
     @property
@@ -292,23 +315,36 @@ class GroupedAttention(nn.Module):
         if not self.spec.same:
             out["v"] = (g * self.vdim, self.width)
         if self.q_norm is not None:
-            out["q.norm"] = out["k.norm"] = (self.dim,)
+            n = (h, g) if self.spec.whole else (1, 1)
+            out["q.norm"], out["k.norm"] = ((m * self.dim,) for m in n)
+        if self.bias is not None:
+            for name in "qkv":
+                out[name + ".b"] = out[name][:1]
         if self.sink_kind == "learned":
             out["sink"] = (h,)
         if self.v_mix:
             out["vmix"] = ()
         return out
 
-    def pack_in(self, w: torch.Tensor, get: Get) -> None:
-        """rows of the product of h"""
+    def _channels(self, dst: torch.Tensor, src: torch.Tensor, n: int,
+                  name: str) -> None:
+        """n heads' channels, in the kernels' order"""
+        src = src.reshape(n, src.shape[0] // n, -1)
+        if self.order is not None and name != "v":
+            src = src[:, self.order]
+        _fill(dst.view(n, dst.shape[0] // n, -1), src)
+
+    def _parts(self):
         parts = [("q", 0, self.heads, self.kp),
                  ("k", self.k_at, self.kv_heads, self.kp)]
         if not self.spec.same:
             parts.append(("v", self.v_at, self.kv_heads, self.vp))
-        for name, at, n, size in parts:
-            src = get(name)
-            _fill(w[at:at + n * size].view(n, size, -1),
-                  src.view(n, -1, self.width))
+        return parts
+
+    def pack_in(self, w: torch.Tensor, get: Get) -> None:
+        """rows of the product of h"""
+        for name, at, n, size in self._parts():
+            self._channels(w[at:at + n * size], get(name), n, name)
 
     def pack_out(self, w: torch.Tensor, get: Get) -> None:
         """columns of the product of the heads' results"""
@@ -317,8 +353,13 @@ class GroupedAttention(nn.Module):
 
     def pack_own(self, get: Get) -> None:
         if self.q_norm is not None:
-            _fill(self.q_norm.data, get("q.norm"))
-            _fill(self.k_norm.data, get("k.norm"))
+            n = (self.heads, self.kv_heads) if self.spec.whole else (1, 1)
+            self._channels(self.q_norm.data, get("q.norm"), n[0], "q")
+            self._channels(self.k_norm.data, get("k.norm"), n[1], "k")
+        if self.bias is not None:
+            for name, at, n, size in self._parts():
+                self._channels(self.bias.data[at:at + n * size],
+                               get(name + ".b"), n, name)
         if self.sink_kind == "learned":
             _fill(self.sink.data, get("sink"))
         if self.v_mix:
@@ -340,13 +381,21 @@ class GroupedAttention(nn.Module):
     def values(self, z) -> torch.Tensor:
         return z[:, self.v_at:self.cols]
 
+    def page_layout(self) -> tuple:
+        s = self.spec
+        return ("paged", s.row, s.pool) if s.pool else ("paged", s.row)
+
     def attend(self, z, batch, cache, out, first=None):
         """z [T, >= cols]: the product of h; out [T, out_cols]. ``first``:
         the values that this layer's are mixed with"""
         t, n, s = z.shape[0], batch.n_abs, self.spec
         grouped.prepare(z, self.k_at, self.v_at, batch.positions,
                         batch.slot_mapping, self.rot, s, self.q_norm,
-                        self.k_norm, self.eps, first, self.lam, cache)
+                        self.k_norm, self.eps, first, self.lam, cache,
+                        self.bias)
+        if s.pool:
+            grouped.pool_rows(cache, batch.block_table, batch.tok_seq,
+                              batch.positions, s.pool)
         q = z[:, :self.k_at]
         if n:
             grouped.attention(q, cache, batch.block_table, batch.tok_seq,
@@ -380,7 +429,7 @@ class GroupedAttentionMixer(nn.Module):
         self.attn.finalize(self.qkv.device)
 
     def cache_layout(self) -> tuple:
-        return "paged", self.attn.spec.row
+        return self.attn.page_layout()
 
     def forward(self, h, batch, cache, carry):
         """``carry``: what layers of one forward hand on ("values")"""
@@ -467,52 +516,265 @@ class DeltaRule(nn.Module):
     def state_layout(self) -> tuple:
         return "state", (self.heads, self.dp, self.dp)
 
-    def scan(self, z, batch, state, out) -> None:
+    def scan(self, z, batch, cache, out) -> None:
         """z [T, cols]: the product of h; out [T, out_cols]"""
         n = self.heads * self.dp
+        state, = cache
         delta.delta_rule(z, tuple(i * n for i in range(6)), self._w, state,
                          batch.positions, batch.state_slots, batch.seqs, out,
                          batch.n_single, self.dim, self.eps, self.out_scale,
                          batch.tiles.shape[0], batch.tile)
 
 
+class LinearState(nn.Module):
+    """A recurrence with one decay per head behind short convolutions
+    (ops/linear_state.py). Subclasses say how a checkpoint names its parts."""
+
+    def __init__(self, width: int, spec: linear_state.StateSpec, skip: bool,
+                 conv_bias: bool):
+        super().__init__()
+        s = self.spec = spec
+        if s.groups < 1 or s.heads % s.groups:
+            raise ValueError("{} heads on {} groups of keys".format(
+                s.heads, s.groups))
+        if not 1 <= s.taps <= linear_state.MAX_TAPS:
+            raise ValueError("convolution over {} tokens, 1 to {} are "
+                             "possible".format(s.taps, linear_state.MAX_TAPS))
+        if s.parts < 1 or s.heads * s.vdim % s.parts:
+            raise ValueError("norm of {} channels in {} parts".format(
+                s.heads * s.vdim, s.parts))
+        self.width, self.cols = width, s.cols
+        self.out_cols = s.heads * s.vp
+        self.conv = _param(s.taps, s.channels)
+        self.conv_b = _param(s.channels) if conv_bias else None
+        self.a_log, self.dt_bias = _param(s.heads), _param(s.heads)
+        self.skip = _param(s.heads) if skip else None
+        self.norm = _param(self.out_cols)
+        self._w: Optional[linear_state.StateWeights] = None
+
+    # (place, heads, padded and true channels of a head) of q, k, v, gate
+    def _places(self):
+        s = self.spec
+        return {"q": (0, s.groups, s.kp, s.dim),
+                "k": (s.k_at, s.groups, s.kp, s.dim),
+                "v": (s.v_at, s.heads, s.vp, s.vdim),
+                "gate": (s.channels, s.heads, s.vp, s.vdim)}
+
+    def _put(self, dst: torch.Tensor, part: str, src: torch.Tensor) -> None:
+        """src [heads * channels, ...] into the part's padded rows of dst"""
+        at, n, pad, size = self._places()[part]
+        _fill(dst[at:at + n * pad].view(n, pad, -1), src.reshape(n, size, -1))
+
+    def _put_taps(self, part: str, src: torch.Tensor) -> None:
+        at, n, pad, size = self._places()[part]
+        _fill(self.conv.data[:, at:at + n * pad].view(-1, n, pad),
+              src.t().reshape(-1, n, size))
+
+    def pack_out(self, w: torch.Tensor, get: Get) -> None:
+        s = self.spec
+        _fill(w.view(w.shape[0], s.heads, s.vp),
+              get("o").view(self.width, s.heads, s.vdim))
+
+    def finalize(self) -> None:
+        def data(p):
+            return None if p is None else p.data
+
+        self._w = linear_state.StateWeights(
+            self.conv.data, data(self.conv_b), self.a_log.data,
+            self.dt_bias.data, data(self.skip), self.norm.data)
+
+    def state_layout(self) -> tuple:
+        return self.spec.layout()
+
+    def scan(self, z, batch, cache, out) -> None:
+        """z [T, cols]: the product of h; out [T, out_cols]"""
+        state, ring = cache
+        linear_state.linear_state(
+            z, self.spec, self._w, state, ring, batch.positions,
+            batch.state_slots, batch.tiles, batch.seqs, batch.n_single, out)
+
+
+class GatedDelta(LinearState):
+    """Gated delta rule: ``heads`` states of dim x vdim, on ``kv_heads``
+    queries and keys."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, taps: int, eps: float):
+        super().__init__(width, linear_state.StateSpec(
+            True, heads, kv_heads, dim, vdim, taps, heads, eps), False, False)
+
+    def shapes(self) -> dict:
+        s, w = self.spec, self.width
+        qk, v = s.groups * s.dim, s.heads * s.vdim
+        out = {"q": (qk, w), "k": (qk, w), "v": (v, w), "g": (v, w),
+               "a": (s.heads, w), "b": (s.heads, w), "o": (w, v),
+               "A_log": (s.heads,), "dt_bias": (s.heads,),
+               "norm": (s.vdim,)}
+        out.update({k + ".conv": (out[k][0], s.taps) for k in "qkv"})
+        return out
+
+    def pack_in(self, w: torch.Tensor, get: Get) -> None:
+        s = self.spec
+        for part, name in (("q", "q"), ("k", "k"), ("v", "v"), ("gate", "g")):
+            self._put(w, part, get(name))
+        _fill(w[s.a_at:s.a_at + s.sp], get("a"))
+        _fill(w[s.a_at + s.sp:], get("b"))
+
+    def pack_own(self, get: Get) -> None:
+        for part in "qkv":
+            self._put_taps(part, get(part + ".conv"))
+        _fill(self.a_log.data, get("A_log"))
+        _fill(self.dt_bias.data, get("dt_bias"))
+        s = self.spec
+        _fill(self.norm.data.view(s.heads, s.vp),
+              get("norm").expand(s.heads, -1))
+
+
+class StateSpace(LinearState):
+    """State-space recurrence: ``heads`` states of ``state`` x vdim whose
+    inputs and read-outs ``groups`` of heads share; gate before the norm,
+    which runs in ``parts`` equal parts."""
+
+    def __init__(self, width: int, heads: int, vdim: int, state: int,
+                 groups: int, taps: int, parts: int, eps: float):
+        super().__init__(width, linear_state.StateSpec(
+            False, heads, groups, state, vdim, taps, parts, eps), True, True)
+
+    def shapes(self) -> dict:
+        s, w = self.spec, self.width
+        inner, gn = s.heads * s.vdim, s.groups * s.dim
+        return {"in": (2 * inner + 2 * gn + s.heads, w),
+                "conv": (inner + 2 * gn, s.taps),
+                "conv.b": (inner + 2 * gn,), "A_log": (s.heads,),
+                "dt_bias": (s.heads,), "D": (s.heads,), "norm": (inner,),
+                "o": (w, inner)}
+
+    def _split(self, t: torch.Tensor, gate: bool) -> Dict[str, torch.Tensor]:
+        """a checkpoint's rows [gate | v | k | q | rest] by part"""
+        s = self.spec
+        inner, gn = s.heads * s.vdim, s.groups * s.dim
+        sizes = ([inner] if gate else []) + [inner, gn, gn]
+        names = (["gate"] if gate else []) + ["v", "k", "q"]
+        rest = t.shape[0] - sum(sizes)
+        return dict(zip(names + ["rest"], torch.split(t, sizes + [rest])))
+
+    def pack_in(self, w: torch.Tensor, get: Get) -> None:
+        parts = self._split(get("in"), True)
+        _fill(w[self.spec.a_at:], parts.pop("rest"))
+        for part, src in parts.items():
+            self._put(w, part, src)
+
+    def pack_own(self, get: Get) -> None:
+        parts = self._split(get("conv"), False)
+        parts.pop("rest")
+        for part, src in parts.items():
+            self._put_taps(part, src)
+        parts = self._split(get("conv.b"), False)
+        parts.pop("rest")
+        for part, src in parts.items():
+            self._put(self.conv_b.data, part, src)
+        for dst, name in ((self.a_log, "A_log"), (self.dt_bias, "dt_bias"),
+                          (self.skip, "D")):
+            _fill(dst.data, get(name))
+        s = self.spec
+        _fill(self.norm.data.view(s.heads, s.vp),
+              get("norm").view(s.heads, s.vdim))
+
+
+class RecurrentMixer(nn.Module):
+    """A recurrence as a layer's mixer. Its output product is the layer's,
+    which can take the feed-forward's along."""
+
+    def __init__(self, width: int, scan: LinearState):
+        super().__init__()
+        self.rec = scan
+        self.inp = _param(scan.cols, pad32(width))
+
+    @property
+    def out_cols(self) -> int:
+        return self.rec.out_cols
+
+    def shapes(self) -> dict:
+        return self.rec.shapes()
+
+    def pack(self, get: Get) -> None:
+        self.rec.pack_in(self.inp.data, get)
+        self.rec.pack_own(get)
+
+    def pack_out(self, w: torch.Tensor, get: Get) -> None:
+        self.rec.pack_out(w, get)
+
+    def finalize(self) -> None:
+        self.rec.finalize()
+
+    def cache_layout(self) -> tuple:
+        return self.rec.state_layout()
+
+    def context(self, h, batch, cache, out) -> None:
+        """what the output product reads, into out [T, out_cols]"""
+        self.rec.scan(linear(h, self.inp), batch, cache, out)
+
+
 class ParallelMixer(nn.Module):
     """Two mixers that read the same input; the result is their weighted sum.
-    Both inputs are one product, and both outputs another."""
+    Both inputs are one product, and both outputs another. ``norm_outputs``:
+    each output has a product of its own and, before the sum, a norm, which is
+    left to the kernel that adds them up (``branches``)."""
 
     def __init__(self, width: int, left: GroupedAttention, left_scale: float,
-                 right: DeltaRule, right_scale: float):
+                 right: Union[DeltaRule, LinearState], right_scale: float,
+                 norm_outputs: bool = False):
         super().__init__()
-        self.left = left.scaled(left_scale)
-        self.right = right.scaled(right_scale)
-        self.width = width
+        if norm_outputs:  # constants in front of a norm would do nothing
+            if left_scale != right_scale:
+                raise ValueError("normed outputs have one scale")
+            self.scale = left_scale
+            left_scale = right_scale = 1.0
+        self.left, self.right = left, right
+        for side, scale in ((left, left_scale), (right, right_scale)):
+            if scale != 1.0:
+                side.scaled(scale)
+        self.width, self.norm_outputs = width, norm_outputs
         self._alloc()
 
     def _alloc(self) -> None:
         wp = pad32(self.width)
         self.inp = _param(self.left.cols + self.right.cols, wp)
-        self.o = _param(wp, self.left.out_cols + self.right.out_cols)
+        if self.norm_outputs:
+            self.outs = nn.ParameterList(
+                [_param(wp, m.out_cols) for _, m in self._sides()])
+            self.out_norms = nn.ParameterList([_param(wp), _param(wp)])
+        else:
+            self.o = _param(wp, self.left.out_cols + self.right.out_cols)
 
     def _sides(self):
         return ("left.", self.left), ("right.", self.right)
 
     def fit(self, get: Get) -> None:
         """sizes that only a checkpoint's tensors tell"""
-        self.right.fit(lambda name: get("right." + name))
-        self._alloc()
+        if hasattr(self.right, "fit"):
+            self.right.fit(lambda name: get("right." + name))
+            self._alloc()
 
     def shapes(self) -> dict:
-        return {p + k: s for p, m in self._sides()
-                for k, s in m.shapes().items()}
+        out = {p + k: s for p, m in self._sides()
+               for k, s in m.shapes().items()}
+        if self.norm_outputs:
+            out.update({p + "out": (self.width,) for p, _ in self._sides()})
+        return out
 
     def pack(self, get: Get) -> None:
         row = col = 0
-        for p, m in self._sides():
+        for i, (p, m) in enumerate(self._sides()):
             def of(name, p=p):
                 return get(p + name)
 
             m.pack_in(self.inp.data[row:row + m.cols], of)
-            m.pack_out(self.o.data[:, col:col + m.out_cols], of)
+            if self.norm_outputs:
+                m.pack_out(self.outs[i].data, of)
+                _fill(self.out_norms[i].data, of("out"))
+            else:
+                m.pack_out(self.o.data[:, col:col + m.out_cols], of)
             m.pack_own(of)
             row += m.cols
             col += m.out_cols
@@ -522,17 +784,27 @@ class ParallelMixer(nn.Module):
         self.right.finalize()
 
     def cache_layout(self) -> tuple:
-        return "both", ("paged", self.left.spec.row), \
-            self.right.state_layout()
+        return "both", self.left.page_layout(), self.right.state_layout()
+
+    def _contexts(self, h, batch, cache, left, right) -> None:
+        pages, state = cache
+        z = linear(h, self.inp)
+        self.left.attend(z[:, :self.left.cols], batch, pages, left)
+        self.right.scan(z[:, self.left.cols:], batch, state, right)
 
     def forward(self, h, batch, cache, carry):
-        pages, (state,) = cache
-        z = linear(h, self.inp)
         n = self.left.out_cols
         ctx = h.new_empty(h.shape[0], self.o.shape[1])
-        self.left.attend(z[:, :self.left.cols], batch, pages, ctx[:, :n])
-        self.right.scan(z[:, self.left.cols:], batch, state, ctx[:, n:])
+        self._contexts(h, batch, cache, ctx[:, :n], ctx[:, n:])
         return linear(ctx, self.o)
+
+    def branches(self, h, batch, cache
+                 ) -> List[Tuple[torch.Tensor, torch.Tensor]]:
+        """(output, weight of its norm) of both sides"""
+        ctx = [h.new_empty(h.shape[0], m.out_cols) for _, m in self._sides()]
+        self._contexts(h, batch, cache, *ctx)
+        return [(linear(c, w), norm.data) for c, w, norm in
+                zip(ctx, self.outs, self.out_norms)]
 
 
 class RgLru(nn.Module):
@@ -643,6 +915,40 @@ class GatedMlp(nn.Module):
     def forward(self, h):
         return linear(lm.gated_mul(linear(h, self.gate_up), self.gate_up_b,
                                    self.act), self.down)
+
+
+class DenseMlp(nn.Module):
+    """down(xielu(up h)): a z^2 + z / 2 above zero, b (e^z - 1 - z) + z / 2
+    below, a = softplus(p) and b = 1/2 + softplus(q) of two learned numbers.
+    The layer can take the product with ``down`` along with another."""
+
+    def __init__(self, width: int, ff: int):
+        super().__init__()
+        self.width, self.ff = width, ff
+        w, f = pad32(width), pad32(ff)
+        self.out_cols = f
+        self.up = _param(f, w)
+        self.act = _param(2)
+        self._coef: Optional[torch.Tensor] = None  # (a, b) in float
+
+    def shapes(self) -> dict:
+        return {"up": (self.ff, self.width), "down": (self.width, self.ff),
+                "act": (2,)}
+
+    def pack(self, get: Get) -> None:
+        _fill(self.up.data, get("up"))
+        _fill(self.act.data, get("act"))
+
+    def pack_out(self, w: torch.Tensor, get: Get) -> None:
+        _fill(w, get("down"))
+
+    def finalize(self) -> None:
+        a, b = torch.nn.functional.softplus(self.act.data.double())
+        self._coef = torch.stack([a, b + 0.5]).float()
+
+    def context(self, h, out) -> None:
+        """what ``down`` multiplies, into out [T, out_cols]"""
+        lm.xielu(linear(h, self.up), self._coef, out)
 
 
 class ExpertMlp(nn.Module):

@@ -114,7 +114,8 @@ class TokenBatchForCausalLM(nn.Module):
 
     # ---- what the engine needs to know ------------------------------ #
     def cache_layout(self) -> List[tuple]:
-        """per layer run, in order: ("paged", elements per token), ("state",
+        """per layer run, in order: ("paged", elements per token[, tokens per
+        pooled row]), ("state",
         shape of a slot's float state[, channels and taps of a ring of past
         inputs]), ("both", layout, layout) or ("shared", run)"""
         raise NotImplementedError

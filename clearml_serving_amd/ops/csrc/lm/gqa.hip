@@ -9,8 +9,8 @@
 // Preparation of queries and cache rows: norm per head, rotation of
 // neighbouring pairs, mixing of the values with another layer's. Attention for
 // few queries per sequence is here, for prompts in prompt_attn.hip. All takes
-// a sliding window with kept first tokens, a cap on the scores and a sink, each
-// of them optional.
+// a sliding window with kept first tokens or with the means of the blocks in
+// front of it, a cap on the scores and a sink, each of them optional.
 #include "lm_attn.h"
 
 namespace {
@@ -26,12 +26,27 @@ struct GroupedPrep {
   const T* first;    // [t, G * VD], null: no mixing
   long ld_first;
   float lam;
-  const T *qn, *kn;  // norm weights [KD], null: no norm
+  const T *qn, *kn;  // norm weights [KD], whole: [H * KD], [G * KD], or null
+  const T *qb, *kb, *vb;  // biases, laid out as q, k and v, or null
   T* cache;
   long n_slots;
   int H, G, KD, VD, dim, row;
   float eps;
+  bool whole;        // one norm over all heads
+  PageRows page;
 };
+
+template <typename T>
+__device__ __forceinline__ void load_biased(const T* p, const T* bias,
+                                            float* f) {
+  load8<T>(p, f);
+  if (bias) {
+    float b[8];
+    load8<T>(bias, b);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] += b[e];
+  }
+}
 
 // Units of a token are its heads: H queries, G keys, G values. LPH lanes take
 // a unit, 8 elements each.
@@ -51,18 +66,56 @@ __global__ __launch_bounds__(256) void grouped_prep_kernel(
     trig[tt * 2 * pairs + p] = rot.gain * c;
     trig[(tt * 2 + 1) * pairs + p] = rot.gain * s;
   }
-  __syncthreads();
   const bool same = a.v == nullptr;
   const int per_tok = 256 / tokens_per_wg;  // threads
   const int tt = tid / per_tok, lid = tid % per_tok;
   const int t = t0 + tt;
+  float inv_q = 1.f, inv_k = 1.f;  // of a norm over all heads
+  if (a.whole) {
+    __shared__ float sums[4][2];
+    float sq = 0.f, sk = 0.f;
+    if (t < n_tok) {
+      for (int c = lid * 8; c < a.H * a.KD; c += per_tok * 8) {
+        float f[8];
+        load_biased(a.q + t * a.ld + c, a.qb ? a.qb + c : nullptr, f);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sq += f[e] * f[e];
+      }
+      for (int c = lid * 8; c < a.G * a.KD; c += per_tok * 8) {
+        float f[8];
+        load_biased(a.k + t * a.ld + c, a.kb ? a.kb + c : nullptr, f);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) sk += f[e] * f[e];
+      }
+    }
+#pragma unroll
+    for (int d = 1; d < 64; d <<= 1) {
+      sq += __shfl_xor(sq, d, 64);
+      sk += __shfl_xor(sk, d, 64);
+    }
+    if (tokens_per_wg == 1) {  // else a token is a wave's
+      if ((tid & 63) == 0) {
+        sums[tid >> 6][0] = sq;
+        sums[tid >> 6][1] = sk;
+      }
+      __syncthreads();
+      sq = (sums[0][0] + sums[1][0]) + (sums[2][0] + sums[3][0]);
+      sk = (sums[0][1] + sums[1][1]) + (sums[2][1] + sums[3][1]);
+    }
+    inv_q = 1.f / sqrtf(sq / ((float)a.H * a.dim) + a.eps);
+    inv_k = 1.f / sqrtf(sk / ((float)a.G * a.dim) + a.eps);
+  }
+  __syncthreads();
   if (t >= n_tok) return;
   const float* cs = trig + tt * 2 * pairs;
   const float* sn = cs + pairs;
   const int c = lid % LPH * 8;
   const long slot = slots[t];
   const bool has_slot = slot >= 0 && slot < a.n_slots;
-  T* crow = a.cache + (has_slot ? slot : 0) * (long)a.row;
+  const int page = has_slot ? (int)(slot / a.page.tokens) : 0;
+  T* crow = a.cache +
+            (long)a.page.token(page, has_slot ? (int)(slot % a.page.tokens)
+                                              : 0) * a.row;
   const int SL = same ? a.KD : a.KD + a.VD;
   const int units = a.H + a.G + (same ? 0 : a.G);
   // the LPH lanes of a unit stay together
@@ -73,8 +126,11 @@ __global__ __launch_bounds__(256) void grouped_prep_kernel(
     const T* src = is_q ? a.q + t * a.ld + u * a.KD
                  : is_v ? a.v + t * a.ld + (u - a.H - a.G) * a.VD
                         : a.k + t * a.ld + (u - a.H) * a.KD;
+    const T* bias = is_q ? a.qb ? a.qb + u * a.KD : nullptr
+                  : is_v ? a.vb ? a.vb + (u - a.H - a.G) * a.VD : nullptr
+                         : a.kb ? a.kb + (u - a.H) * a.KD : nullptr;
     float f[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-    if (mine) load8<T>(src + c, f);
+    if (mine) load_biased(src + c, bias ? bias + c : nullptr, f);
     if (is_v) {
       if (!mine || !has_slot) continue;
       const int hd = u - a.H - a.G;
@@ -90,7 +146,10 @@ __global__ __launch_bounds__(256) void grouped_prep_kernel(
     }
     float inv = 1.f;
     const T* w = is_q ? a.qn : a.kn;
-    if (w) {
+    if (a.whole) {
+      inv = is_q ? inv_q : inv_k;
+      w += (is_q ? u : u - a.H) * a.KD;
+    } else if (w) {
       float ss = 0.f;
 #pragma unroll
       for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
@@ -138,10 +197,11 @@ __global__ __launch_bounds__(256) void grouped_prep_kernel(
 // key range per workgroup
 // ------------------------------------------------------------------- //
 struct GroupedDims {
-  int H, R, KD, VD, SL, row, tail, block_size, max_blocks, n_blocks, n_seqs, window,
-      keep, splits, col_groups;
+  int H, R, KD, VD, SL, row, tail, max_blocks, n_blocks, n_seqs, window, keep,
+      splits, col_groups;
   bool same;
   float out_scale;
+  PageRows page;
 };
 
 // Each wave walks 32-key tiles of its own: slices go through registers into a
@@ -175,19 +235,22 @@ __global__ __launch_bounds__(256, 2) void grouped_attn_kernel(
   const int c_base = (blockIdx.z % d.col_groups) * (NT * 16);
   const int cols = min(NT * 16, d.VD - c_base);
 
-  const int pos = min(max(positions[t], 0), d.max_blocks * d.block_size - 1);
+  const int bs = d.page.tokens, pool = d.page.pool;
+  const int pos = min(max(positions[t], 0), d.max_blocks * bs - 1);
   const int* btab = block_table +
                     (long)min(max(tok_seq[t], 0), d.n_seqs - 1) * d.max_blocks;
-  const Visible vis = visible_keys(pos, d.window, d.keep);
+  const Visible vis = visible_keys(pos, d.window, d.keep, pool);
   const int n_tiles = (vis.n + 31) / 32;
   const int stride = d.splits * nw;
   int j = split * nw + wave;
 
   // cached row of key `lane & 31` of a tile; behind the last key, that key's
   auto row_of = [&](int jt) {
-    const int key = vis.position(min(jt * 32 + (lane & 31), vis.n - 1));
-    const int blk = min(max(btab[key / d.block_size], 0), d.n_blocks - 1);
-    return blk * d.block_size + key % d.block_size;
+    const int i = min(jt * 32 + (lane & 31), vis.n - 1);
+    const bool mean = pool > 0 && i < vis.kf;
+    const int key = mean ? i * pool + pool - 1 : vis.position(i);
+    const int blk = min(max(btab[key / bs], 0), d.n_blocks - 1);
+    return mean ? d.page.pooled(blk, key % bs) : d.page.token(blk, key % bs);
   };
   // piece p of a tile: row p / row8, columns 8 * (p % row8)
   const int row8 = d.SL / 8, pieces = 32 * row8;
@@ -329,10 +392,47 @@ __global__ __launch_bounds__(256, 2) void grouped_attn_kernel(
       });
 }
 
+// ------------------------------------------------------------------- //
+// means of whole blocks: a workgroup per token, which leaves unless the token
+// ends a block
+// ------------------------------------------------------------------- //
+template <typename T>
+__global__ __launch_bounds__(256) void grouped_pool_kernel(
+    T* cache, const int* __restrict__ block_table,
+    const int* __restrict__ tok_seq, const int* __restrict__ positions,
+    int row, int max_blocks, int n_blocks, int n_seqs, PageRows page) {
+  const int t = blockIdx.x, pos = positions[t];
+  if (pos < 0 || (pos + 1) % page.pool || pos >= max_blocks * page.tokens)
+    return;
+  const int* btab =
+      block_table + (long)min(max(tok_seq[t], 0), n_seqs - 1) * max_blocks;
+  auto page_of = [&](int p) {
+    return min(max(btab[p / page.tokens], 0), n_blocks - 1);
+  };
+  const float inv = 1.f / (float)page.pool;
+  T* dst = cache +
+           (long)page.pooled(page_of(pos), pos % page.tokens) * row;
+  for (int c = threadIdx.x * 8; c < row; c += blockDim.x * 8) {
+    float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int p = pos + 1 - page.pool; p <= pos; ++p) {
+      float f[8];
+      load8<T>(cache + (long)page.token(page_of(p), p % page.tokens) * row + c,
+               f);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) sum[e] += f[e];
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) sum[e] *= inv;
+    store8(dst + c, sum);
+  }
+}
+
 }  // namespace
 
 // z [T, cols] holds q at column 0, k at k_at, v at v_at (-1: values are keys);
-// q is finished in place, keys and values go to the cache rows of `slots`
+// bias [cols] is added; q is finished in place, keys and values go to the
+// cache rows of `slots`
 void lm_grouped_prep(torch::Tensor z, long k_at, long v_at,
                      torch::Tensor positions, torch::Tensor slots,
                      c10::optional<torch::Tensor> inv_freq, double gain,
@@ -340,7 +440,8 @@ void lm_grouped_prep(torch::Tensor z, long k_at, long v_at,
                      c10::optional<torch::Tensor> q_norm,
                      c10::optional<torch::Tensor> k_norm, double eps,
                      c10::optional<torch::Tensor> first, double lam,
-                     torch::Tensor cache) {
+                     torch::Tensor cache, c10::optional<torch::Tensor> bias,
+                     bool whole, long pool) {
   LM_CHECK_I32(positions);
   LM_CHECK_I32(slots);
   LM_CHECK_CONTIG(cache);
@@ -363,7 +464,14 @@ void lm_grouped_prep(torch::Tensor z, long k_at, long v_at,
   for (const auto* w : {&q_norm, &k_norm})
     if (w->has_value())
       TORCH_CHECK((*w)->is_cuda() && (*w)->is_contiguous() &&
-                  (*w)->numel() == KD && (*w)->scalar_type() == type);
+                  (*w)->numel() ==
+                      KD * (!whole ? 1 : w == &q_norm ? H : G) &&
+                  (*w)->scalar_type() == type);
+  TORCH_CHECK(!whole || (q_norm && k_norm && !same));
+  if (bias)
+    TORCH_CHECK(bias->is_cuda() && bias->is_contiguous() && !same &&
+                bias->numel() >= v_at + G * VD &&
+                bias->scalar_type() == type);
   if (first) lm_check_rows(*first, T, G * VD, type);
   Rot rot{nullptr, 0, 0, 1.f};
   if (inv_freq) rot = make_rot(*inv_freq, gain, false, KD);
@@ -385,8 +493,15 @@ void lm_grouped_prep(torch::Tensor z, long k_at, long v_at,
     }
     a.qn = q_norm ? (const scalar_t*)q_norm->data_ptr() : nullptr;
     a.kn = k_norm ? (const scalar_t*)k_norm->data_ptr() : nullptr;
+    if (bias) {
+      a.qb = (const scalar_t*)bias->data_ptr();
+      a.kb = a.qb + k_at;
+      a.vb = a.qb + v_at;
+    }
+    a.whole = whole;
+    a.page = page_rows(cache.size(1), pool);
     a.cache = (scalar_t*)cache.data_ptr();
-    a.n_slots = (long)cache.size(0) * cache.size(1);
+    a.n_slots = (long)cache.size(0) * a.page.tokens;
     a.H = (int)H;
     a.G = (int)G;
     a.KD = (int)KD;
@@ -403,6 +518,32 @@ void lm_grouped_prep(torch::Tensor z, long k_at, long v_at,
   LM_LAUNCHED();
 }
 
+// the means of the blocks that the given tokens end, into their pages
+void lm_grouped_pool(torch::Tensor cache, torch::Tensor block_table,
+                     torch::Tensor tok_seq, torch::Tensor positions,
+                     long pool) {
+  LM_CHECK_CONTIG(cache);
+  LM_CHECK_I32(block_table);
+  LM_CHECK_I32(tok_seq);
+  LM_CHECK_I32(positions);
+  const long T = positions.numel(), row = cache.size(2);
+  TORCH_CHECK(pool >= 1 && cache.dim() == 3 && row % 8 == 0 &&
+              tok_seq.numel() == T && block_table.dim() == 2);
+  if (T == 0) return;
+  TORCH_CHECK(block_table.numel() > 0);
+  const PageRows page = page_rows(cache.size(1), pool);
+  LM_DISPATCH(cache, "lm_grouped_pool", [&] {
+    hipLaunchKernelGGL((grouped_pool_kernel<scalar_t>), dim3(T),
+                       dim3(row <= 512 ? 64 : 256), 0, cmls::current_stream(),
+                       (scalar_t*)cache.data_ptr(),
+                       block_table.data_ptr<int>(), tok_seq.data_ptr<int>(),
+                       positions.data_ptr<int>(), (int)row,
+                       (int)block_table.size(1), (int)cache.size(0),
+                       (int)block_table.size(0), page);
+  });
+  LM_LAUNCHED();
+}
+
 // tokens [0, n) of q [T, H * KD] (row stride free) attend to their sequences'
 // cache rows -> out [T, H * VD] (row stride free), times out_scale
 void lm_grouped_attention(torch::Tensor q, torch::Tensor cache,
@@ -411,8 +552,8 @@ void lm_grouped_attention(torch::Tensor q, torch::Tensor cache,
                           c10::optional<torch::Tensor> sink,
                           torch::Tensor out, long n, long H, long G, long KD,
                           long VD, bool same, long window, long keep,
-                          double scale, double cap, double out_scale,
-                          long max_keys) {
+                          long pool, double scale, double cap,
+                          double out_scale, long max_keys) {
   LM_CHECK_CONTIG(cache);
   LM_CHECK_I32(block_table);
   LM_CHECK_I32(tok_seq);
@@ -430,7 +571,9 @@ void lm_grouped_attention(torch::Tensor q, torch::Tensor cache,
   TORCH_CHECK(!same || cache.size(2) - G * SL >= 2 * G);
   TORCH_CHECK(block_table.dim() == 2 && tok_seq.numel() >= n &&
               positions.numel() >= n);
-  TORCH_CHECK(window >= 0 && keep >= 0 && (keep == 0 || window > 0));
+  TORCH_CHECK(window >= 0 && keep >= 0 &&
+              ((keep == 0 && pool == 0) || window > 0) &&
+              (keep == 0 || pool == 0) && (pool == 0 || !same));
   if (sink) {
     LM_CHECK_CONTIG(*sink);
     TORCH_CHECK(sink->numel() == H && sink->scalar_type() == type);
@@ -450,7 +593,10 @@ void lm_grouped_attention(torch::Tensor q, torch::Tensor cache,
               " elements does not fit LDS");
   const int hg = (int)(G * ((H / G + 15) / 16));
   // fill 256 CUs as far as there are 32-key tiles for every wave
-  const long keys = window > 0 ? std::min(window + keep, max_keys) : max_keys;
+  const long keys =
+      window > 0 ? std::min(window + keep + (pool ? max_keys / pool : 0),
+                            max_keys)
+                 : max_keys;
   const long per_cu = std::min<long>(2, 156 * 1024 / lds(nw));
   long splits = 256 * per_cu / std::max<long>(1, (long)n * hg * cgroups);
   splits = std::max<long>(1, std::min(splits,
@@ -470,7 +616,7 @@ void lm_grouped_attention(torch::Tensor q, torch::Tensor cache,
   d.SL = (int)SL;
   d.row = (int)cache.size(2);
   d.tail = (int)(G * SL);
-  d.block_size = (int)cache.size(1);
+  d.page = page_rows(cache.size(1), pool);
   d.max_blocks = (int)block_table.size(1);
   d.n_blocks = (int)cache.size(0);
   d.n_seqs = (int)block_table.size(0);

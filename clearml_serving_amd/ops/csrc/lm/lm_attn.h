@@ -53,7 +53,8 @@ template <> __device__ __forceinline__ float cap_tanh<bf16>(float z) {
 
 // A query at position `pos` sees the keys up to it, with a window the last
 // `window` of them and the first `keep` of the sequence. Visible key n lies
-// at position n, from number `kf` on at n + skip.
+// at position n, from number `kf` on at n + skip. With `pool` the first kf keys
+// are the means of the whole blocks of so many tokens in front of the window.
 struct Visible {
   int kf, skip, n;
   __device__ __forceinline__ int position(int i) const {
@@ -61,11 +62,11 @@ struct Visible {
   }
 };
 
-__device__ __forceinline__ Visible visible_keys(int pos, int window,
-                                                int keep) {
+__device__ __forceinline__ Visible visible_keys(int pos, int window, int keep,
+                                                int pool) {
   const int lo = window > 0 ? max(0, pos - window + 1) : 0;
   Visible v;
-  v.kf = min(keep, lo);
+  v.kf = pool > 0 ? lo / pool : min(keep, lo);
   v.skip = lo - v.kf;
   v.n = pos + 1 - v.skip;
   return v;
@@ -158,6 +159,31 @@ __global__ __launch_bounds__(128) void combine_ranges_kernel(
     }
     store4(out + (th / H) * ld_out + (th % H) * C + c, f);
   }
+}
+
+// Pages hold the rows of `tokens` tokens and behind them the means of the
+// blocks of `pool` tokens that end in the page.
+struct PageRows {
+  int tokens, rows, pool;
+  __device__ __forceinline__ int token(int page, int offset) const {
+    return page * rows + offset;
+  }
+  __device__ __forceinline__ int pooled(int page, int offset) const {
+    return page * rows + tokens + offset / pool;
+  }
+};
+
+inline PageRows page_rows(long rows, long pool) {
+  TORCH_CHECK(pool >= 0 && pool < (1 << 20), "lm: pooled block size");
+  PageRows p{};
+  p.rows = (int)rows;
+  p.pool = (int)pool;
+  p.tokens = (int)(pool ? rows * pool / (pool + 1) : rows);
+  TORCH_CHECK(p.tokens >= 1 &&
+                  p.rows == p.tokens + (pool ? (p.tokens + pool - 1) / pool
+                                             : 0),
+              "lm: page of ", rows, " rows");
+  return p;
 }
 
 // [T, cols] view with 16-byte aligned rows

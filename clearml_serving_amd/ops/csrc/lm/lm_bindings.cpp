@@ -7,6 +7,12 @@ using torch::Tensor;
 std::vector<Tensor> lm_embed(Tensor tokens, Tensor table, Opt next_w,
                              double off, long n, double eps, Opt out,
                              Opt copy);
+std::vector<Tensor> lm_embed_norms(Tensor tokens, Tensor table, Tensor wa,
+                                   Opt wb, long n, double eps);
+std::vector<Tensor> lm_add_branches(Tensor x, Opt plain, Opt o1, Opt w1,
+                                    Opt o2, Opt w2, double scale, Opt wa,
+                                    Opt wb, long n, double eps);
+void lm_xielu(Tensor z, Tensor coef, Tensor out);
 Tensor lm_post_norm_add(Tensor o, Opt bias, Tensor w, Tensor x, long n,
                         double eps, double off, Opt next_w, Opt out, Opt pos,
                         Opt share);
@@ -31,17 +37,27 @@ void lm_latent_prompt(Tensor q, Tensor kv, Tensor lat, Opt sink,
                       long CP, long VP, long window, double scale, Opt gate);
 void lm_grouped_prompt(Tensor q, Tensor rows, Opt sink, Tensor qtiles,
                        Tensor out, long H, long G, long KD, long VD, bool same,
-                       long window, long keep, double scale, double cap,
-                       double out_scale);
+                       long window, long keep, long pool, double scale,
+                       double cap, double out_scale);
 void lm_grouped_prep(Tensor z, long k_at, long v_at, Tensor positions,
                      Tensor slots, Opt inv_freq, double gain, long H, long G,
                      long KD, long VD, long dim, Opt q_norm, Opt k_norm,
-                     double eps, Opt first, double lam, Tensor cache);
+                     double eps, Opt first, double lam, Tensor cache, Opt bias,
+                     bool whole, long pool);
+void lm_grouped_pool(Tensor cache, Tensor block_table, Tensor tok_seq,
+                     Tensor positions, long pool);
 void lm_grouped_attention(Tensor q, Tensor cache, Tensor block_table,
                           Tensor tok_seq, Tensor positions, Opt sink,
                           Tensor out, long n, long H, long G, long KD, long VD,
-                          bool same, long window, long keep, double scale,
-                          double cap, double out_scale, long max_keys);
+                          bool same, long window, long keep, long pool,
+                          double scale, double cap, double out_scale,
+                          long max_keys);
+void lm_linear_state(Tensor z, bool delta, long heads, long groups, long dim,
+                     long vdim, long parts, double eps, Tensor conv,
+                     Opt conv_b, Tensor a_log, Tensor dt_bias, Opt skip,
+                     Tensor norm, Tensor state, Tensor ring, Tensor positions,
+                     Tensor slots, Tensor tiles, Tensor seqs, long n_single,
+                     Tensor out);
 void lm_delta_rule(Tensor z, std::vector<long> at, Tensor w2, Tensor w0,
                    Tensor ab, Tensor norm, Tensor state, Tensor positions,
                    Tensor slots, Tensor seqs, Tensor out, long n_single,
@@ -82,6 +98,11 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("lm_grouped_prompt", &lm_grouped_prompt);
   m.def("lm_grouped_prep", &lm_grouped_prep);
   m.def("lm_grouped_attention", &lm_grouped_attention);
+  m.def("lm_grouped_pool", &lm_grouped_pool);
+  m.def("lm_linear_state", &lm_linear_state);
+  m.def("lm_embed_norms", &lm_embed_norms);
+  m.def("lm_add_branches", &lm_add_branches);
+  m.def("lm_xielu", &lm_xielu);
   m.def("lm_delta_rule", &lm_delta_rule);
   m.def("lm_hyper_embed", &lm_hyper_embed);
   m.def("lm_hyper_step", &lm_hyper_step);

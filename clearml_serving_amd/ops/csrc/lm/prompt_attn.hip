@@ -40,7 +40,9 @@ struct PromptOut {
 
 // qtiles: int32 [n, 6] = first token (flat), tokens, first position, first
 // row in the gathered keys, what a row's number lacks to its position (rows
-// behind the `keep` first ones), gathered rows.
+// behind the `keep` first ones), gathered rows. With `pool` [n, 7]: in the end
+// the number of pooled rows, which stand first; row n is the mean of block n
+// and is seen from position (n + 1) pool - 1 + window on.
 // Two workgroups per CU (128 registers) where their LDS fits.
 template <int QS, int VT, bool SAME>
 __global__ __launch_bounds__(NW * 64, QS * 2 + VT <= 16 ? 4 : 2)
@@ -48,7 +50,7 @@ void prompt_attn_kernel(
     const bf16* __restrict__ q, long q_t,   // q[t * q_t + h * QD]
     PromptKeys src, const bf16* __restrict__ sink, PromptOut dst_,
     const int* __restrict__ qtiles, int H, int QD, int VP, int window,
-    int keep, Score score) {
+    int keep, int pool, Score score) {
   constexpr int KP = QS * 32 + 8;   // LDS pitches
   constexpr int VPP = VT * 16 + 8;
   __shared__ __align__(16) short lk[2][BN * KP];
@@ -58,9 +60,15 @@ void prompt_attn_kernel(
   // grouped layers, go to one XCD
   const int h = H % 8 ? blockIdx.x : blockIdx.x % 8 * (H / 8) + blockIdx.x / 8;
   const int hk = h / src.per;
-  const int* td = qtiles + (long)blockIdx.y * 6;
+  const int* td = qtiles + (long)blockIdx.y * (pool > 0 ? 7 : 6);
   const int t0 = td[0], len = td[1], p0 = td[2], kv0 = td[3], skip = td[4],
             nk = td[5];
+  const int pooled = pool > 0 ? td[6] : 0;
+  if (pool > 0) keep = pooled;
+  auto place = [&](int n) {  // position that a row is seen from
+    return n >= keep ? n + skip
+                     : pool > 0 ? (n + 1) * pool - 1 + window : n;
+  };
   const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave();
   const int r16 = lane & 15, g = lane >> 4, ko = g * 8;
   const int qrow = wave * 16 + r16;
@@ -136,19 +144,24 @@ void prompt_attn_kernel(
 
   const int q_first = p0 + wave * 16, q_last = q_first + 15;
   // rows that any query of the tile sees: the first `keep`, then from n_begin
-  const int n_begin = window > 0 ? max(0, p0 - window + 1 - skip) : 0;
+  const int n_begin = window > 0 ? max(pooled, p0 - window + 1 - skip) : 0;
   const int n_end = min(nk, p0 + len - skip);
+  // of the pooled rows, those that the tile's last query sees
+  const int front =
+      pool > 0 ? min(pooled, max(0, p0 + len - window) / pool) : keep;
   auto next_tile = [&](int n0) {
-    return n0 + BN >= keep ? max(n0 + BN, n_begin) : n0 + BN;
+    return n0 + BN >= front ? max(n0 + BN, n_begin) : n0 + BN;
   };
   const int my_q = p0 + qrow;
   const int my_lo = window > 0 ? my_q - window : -1;  // sees keys > my_lo
 
   auto compute = [&](int n0, int buf) {
     // positions of the tile's rows; it may hold kept rows and others
-    const int a0 = n0 < keep ? n0 : n0 + skip;
-    const int a1 = n0 + BN - 1 + (n0 + BN - 1 < keep ? 0 : skip);
-    if (a0 > q_last || (window > 0 && n0 >= keep && a1 <= q_first - window))
+    const int a0 = place(n0), a1 = place(n0 + BN - 1);
+    // pooled rows and tokens in one tile: no order of positions
+    const bool both = pool > 0 && n0 < keep && n0 + BN > keep;
+    if (!both &&
+        (a0 > q_last || (window > 0 && n0 >= keep && a1 <= q_first - window)))
       return;  // nothing of this tile for any query of the wave
     lm_f32x4 s[BN / 16];
 #pragma unroll
@@ -165,7 +178,7 @@ void prompt_attn_kernel(
         }
       }
     }
-    const bool full = n0 + BN <= nk && a1 <= q_first &&
+    const bool full = !both && n0 + BN <= nk && a1 <= q_first &&
                       (window <= 0 || n0 + BN <= keep ||
                        (n0 >= keep && a0 > q_last - window));
     float mx = -INFINITY;
@@ -189,9 +202,10 @@ void prompt_attn_kernel(
       for (int r = 0; r < 4; ++r) {
         if (!full) {
           const int n = n0 + 16 * t + 4 * g + r;
-          const int key = n < keep ? n : n + skip;
-          const bool see =
-              key <= my_q && (key > my_lo || key < keep) && n < nk;
+          const int key = place(n);
+          const bool see = key <= my_q &&
+                           (key > my_lo || (pool > 0 ? n : key) < keep) &&
+                           n < nk;
           s[t][r] = see ? s[t][r] : -INFINITY;
         }
         mx = fmaxf(mx, s[t][r]);
@@ -231,7 +245,7 @@ void prompt_attn_kernel(
     }
   };
 
-  int n0 = keep > 0 ? 0 : n_begin;
+  int n0 = front > 0 ? 0 : n_begin;
   if (n0 < n_end) {
     stage_load(n0);
     stage_write(0);
@@ -281,10 +295,10 @@ void prompt_attn_kernel(
 void launch_prompt(const torch::Tensor& q, const PromptKeys& src, bool same,
                    const c10::optional<torch::Tensor>& sink,
                    const PromptOut& out, const torch::Tensor& qtiles, int H,
-                   int QD, int VP, long window, long keep,
+                   int QD, int VP, long window, long keep, long pool,
                    const Score& score) {
   LM_CHECK_I32(qtiles);
-  TORCH_CHECK(qtiles.dim() == 2 && qtiles.size(1) == 6);
+  TORCH_CHECK(qtiles.dim() == 2 && qtiles.size(1) == (pool ? 7 : 6));
   TORCH_CHECK(q.scalar_type() == at::kBFloat16 && q.dim() == 2 &&
               q.stride(1) == 1 && q.stride(0) % 8 == 0 &&
               q.size(1) >= (long)H * QD && q.storage_offset() % 8 == 0);
@@ -293,7 +307,9 @@ void launch_prompt(const torch::Tensor& q, const PromptKeys& src, bool same,
     TORCH_CHECK(sink->numel() == H && sink->scalar_type() == at::kBFloat16);
   }
   TORCH_CHECK(QD <= 256 && VP <= 256, "prompt attention: head too large");
-  TORCH_CHECK(window >= 0 && keep >= 0 && (keep == 0 || window > 0));
+  TORCH_CHECK(window >= 0 && keep >= 0 && pool >= 0 &&
+              ((keep == 0 && pool == 0) || window > 0) &&
+              (keep == 0 || pool == 0));
   const int n = qtiles.size(0);
   if (n == 0) return;
   TORCH_CHECK(n <= 65535);
@@ -304,7 +320,7 @@ void launch_prompt(const torch::Tensor& q, const PromptKeys& src, bool same,
                      q.stride(0), src,                                       \
                      sink ? (const bf16*)sink->data_ptr() : nullptr, out,    \
                      qtiles.data_ptr<int>(), H, QD, VP, (int)window,         \
-                     (int)keep, score)
+                     (int)keep, (int)pool, score)
 #define LM_LP_V(QS)                                                          \
   do {                                                                       \
     if (VP <= 32) LM_LP(QS, 2, false);                                       \
@@ -367,7 +383,7 @@ void lm_latent_prompt(torch::Tensor q, torch::Tensor kv, torch::Tensor lat,
                      gate ? gate->stride(0) : 0L, (bf16*)out.data_ptr(),
                      H * VP, 1.f};
   launch_prompt(q, src, false, sink, po, qtiles, (int)H, (int)(DP + RP),
-                (int)VP, window, 0, make_score(scale, 0.0));
+                (int)VP, window, 0, 0, make_score(scale, 0.0));
 }
 
 // q [T, H * KD] (row stride free); rows [n, ROW] gathered cache rows, G slices
@@ -377,7 +393,8 @@ void lm_grouped_prompt(torch::Tensor q, torch::Tensor rows,
                        c10::optional<torch::Tensor> sink,
                        torch::Tensor qtiles, torch::Tensor out, long H, long G,
                        long KD, long VD, bool same, long window, long keep,
-                       double scale, double cap, double out_scale) {
+                       long pool, double scale, double cap,
+                       double out_scale) {
   LM_CHECK_CONTIG(rows);
   TORCH_CHECK(rows.dim() == 2 && rows.scalar_type() == at::kBFloat16 &&
               out.scalar_type() == at::kBFloat16);
@@ -400,5 +417,5 @@ void lm_grouped_prompt(torch::Tensor q, torch::Tensor rows,
   const PromptOut po{nullptr, 0L, (bf16*)out.data_ptr(), out.stride(0),
                      (float)out_scale};
   launch_prompt(q, src, same, sink, po, qtiles, (int)H, (int)KD, (int)VD,
-                window, keep, make_score(scale, cap));
+                window, keep, pool, make_score(scale, cap));
 }

@@ -140,6 +140,167 @@ __global__ __launch_bounds__(256) void post_norm_add_kernel(
     write_next<T, NV>(v, next_w, off, h + t * ld_h, width, n, eps, tmp2);
 }
 
+// h = r / rms(r) * w for one or two weights of a row in registers
+template <typename T, int NV>
+__device__ __forceinline__ void write_norms(
+    const float (&r)[NV][8], const T* __restrict__ wa, T* __restrict__ ha,
+    const T* __restrict__ wb, T* __restrict__ hb, int width, int n, float eps,
+    float* tmp) {
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    if ((i * 256 + (int)threadIdx.x) * 8 < width) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += r[i][e] * r[i][e];
+    }
+  }
+  ss = block_reduce(ss, tmp, SumOp{}, 0.f);
+  const float inv = 1.f / sqrtf(ss / (float)n + eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 8;
+    if (c >= width) continue;
+    float f[8];
+    load8<T>(wa + c, f);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[e] *= r[i][e] * inv;
+    store8(ha + c, f);
+    if (wb) {
+      load8<T>(wb + c, f);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) f[e] *= r[i][e] * inv;
+      store8(hb + c, f);
+    }
+  }
+}
+
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void embed_norms_kernel(
+    const long* __restrict__ tokens, const T* __restrict__ table,
+    float* __restrict__ x, const T* __restrict__ wa, T* __restrict__ ha,
+    const T* __restrict__ wb, T* __restrict__ hb, int width, int n, float eps,
+    long vocab) {
+  __shared__ float tmp[16];
+  const long row = (long)blockIdx.x * width;
+  long id = tokens[blockIdx.x];
+  id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+  float v[NV][8];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + threadIdx.x) * 8;
+    if (c < width) {
+      load8<T>(table + id * width + c, v[i]);
+      store8(x + row + c, v[i]);
+    }
+  }
+  write_norms<T, NV>(v, wa, ha + row, wb, wb ? hb + row : nullptr, width, n,
+                     eps, tmp);
+}
+
+// What parallel sublayers made goes into the stream: x += plain + scale *
+// (o1 / rms(o1) * w1 + o2 / rms(o2) * w2), each part optional; up to two norms
+// of the new x. Two sums are reduced at once.
+template <typename T, int NV, bool BR>
+__global__ __launch_bounds__(256) void add_branches_kernel(
+    float* __restrict__ x, const T* __restrict__ plain,
+    const T* __restrict__ o1, const T* __restrict__ w1,
+    const T* __restrict__ o2, const T* __restrict__ w2, float scale,
+    const T* __restrict__ wa, T* __restrict__ ha, const T* __restrict__ wb,
+    T* __restrict__ hb, int width, int n, float eps) {
+  __shared__ float tmp[16];
+  __shared__ float sums[2][4];
+  const long row = (long)blockIdx.x * width;
+  const int tid = threadIdx.x;
+  float v[NV][8], f1[BR ? NV : 1][8], f2[BR ? NV : 1][8];
+  float s1 = 0.f, s2 = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + tid) * 8;
+    if (c >= width) continue;
+    load8<float>(x + row + c, v[i]);
+    if (plain) {
+      float p[8];
+      load8<T>(plain + row + c, p);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[i][e] += p[e];
+    }
+    if (BR) {
+      load8<T>(o1 + row + c, f1[BR ? i : 0]);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s1 += f1[BR ? i : 0][e] * f1[BR ? i : 0][e];
+      if (o2) {
+        load8<T>(o2 + row + c, f2[BR ? i : 0]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          s2 += f2[BR ? i : 0][e] * f2[BR ? i : 0][e];
+      }
+    }
+  }
+  if (BR) {
+#pragma unroll
+    for (int d = 1; d < 64; d <<= 1) {
+      s1 += __shfl_xor(s1, d, 64);
+      s2 += __shfl_xor(s2, d, 64);
+    }
+    if ((tid & 63) == 0) {
+      sums[0][tid >> 6] = s1;
+      sums[1][tid >> 6] = s2;
+    }
+    __syncthreads();
+    s1 = (sums[0][0] + sums[0][1]) + (sums[0][2] + sums[0][3]);
+    s2 = (sums[1][0] + sums[1][1]) + (sums[1][2] + sums[1][3]);
+    s1 = scale / sqrtf(s1 / (float)n + eps);
+    s2 = scale / sqrtf(s2 / (float)n + eps);
+  }
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (i * 256 + tid) * 8;
+    if (c >= width) continue;
+    if (BR) {
+      float g[8];
+      load8<T>(w1 + c, g);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[i][e] += f1[BR ? i : 0][e] * s1 * g[e];
+      if (o2) {
+        load8<T>(w2 + c, g);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[i][e] += f2[BR ? i : 0][e] * s2 * g[e];
+      }
+    }
+    store8(x + row + c, v[i]);
+  }
+  if (wa)
+    write_norms<T, NV>(v, wa, ha + row, wb, wb ? hb + row : nullptr, width, n,
+                       eps, tmp);
+}
+
+// z > 0: a z^2 + z / 2, else b (e^z - 1 - z) + z / 2
+__device__ __forceinline__ float xielu_f(float z, float a, float b) {
+  // e^z - 1 - z: the power series where the difference would cancel
+  const float p = z * z *
+      (1.f / 2 + z * (1.f / 6 + z * (1.f / 24 + z * (1.f / 120 +
+       z * (1.f / 720 + z * (1.f / 5040))))));
+  const float d = z > -0.5f ? p : exp_f(z) - 1.f - z;
+  return (z > 0.f ? a * z * z : b * d) + 0.5f * z;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void xielu_kernel(
+    const T* __restrict__ z, const float* __restrict__ coef,
+    T* __restrict__ out, long ld_out, int ff, long total) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= total) return;
+  const int per = ff / 8;
+  const long t = i / per;
+  const int c = (int)(i % per) * 8;
+  const float a = coef[0], b = coef[1];
+  float f[8];
+  load8<T>(z + t * ff + c, f);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) f[e] = xielu_f(f[e], a, b);
+  store8(out + t * ld_out + c, f);
+}
+
 // x += add (one vector for all rows); h from the new x
 template <typename T, int NV>
 __global__ __launch_bounds__(256) void add_norm_kernel(
@@ -379,6 +540,107 @@ torch::Tensor lm_add_norm(torch::Tensor x, torch::Tensor add,
 #undef LM_AN
   LM_LAUNCHED();
   return h;
+}
+
+// -> {x, norm of x for each of one or two weights}
+std::vector<torch::Tensor> lm_embed_norms(torch::Tensor tokens,
+                                          torch::Tensor table,
+                                          torch::Tensor wa,
+                                          c10::optional<torch::Tensor> wb,
+                                          long n, double eps) {
+  LM_CHECK_CONTIG(tokens);
+  LM_CHECK_CONTIG(table);
+  TORCH_CHECK(tokens.scalar_type() == at::kLong && tokens.dim() == 1);
+  const int T = tokens.size(0), width = table.size(1);
+  TORCH_CHECK(table.dim() == 2 && width % 8 == 0 && width <= 16384 &&
+              table.size(0) > 0);
+  TORCH_CHECK(n >= 1 && n <= width);
+  const auto type = table.scalar_type();
+  check_weight(wa, width, type);
+  check_weight(wb, width, type);
+  std::vector<torch::Tensor> out{
+      torch::empty({T, width}, table.options().dtype(at::kFloat)),
+      torch::empty({T, width}, table.options())};
+  if (wb) out.push_back(torch::empty({T, width}, table.options()));
+  if (T == 0) return out;
+#define LM_EN(NV)                                                            \
+  hipLaunchKernelGGL((embed_norms_kernel<scalar_t, NV>), dim3(T), dim3(256), \
+                     0, cmls::current_stream(), tokens.data_ptr<long>(),     \
+                     (const scalar_t*)table.data_ptr(),                      \
+                     out[0].data_ptr<float>(),                               \
+                     (const scalar_t*)wa.data_ptr(),                         \
+                     (scalar_t*)out[1].data_ptr(),                           \
+                     wb ? (const scalar_t*)wb->data_ptr() : nullptr,         \
+                     wb ? (scalar_t*)out[2].data_ptr() : nullptr, width,     \
+                     (int)n, (float)eps, (long)table.size(0))
+  LM_DISPATCH(table, "lm_embed_norms", [&] { LM_NV(width, LM_EN); });
+#undef LM_EN
+  LM_LAUNCHED();
+  return out;
+}
+
+// x float [T, width] in place; plain, o1, o2 [T, width]; -> norms of the new x
+std::vector<torch::Tensor> lm_add_branches(
+    torch::Tensor x, c10::optional<torch::Tensor> plain,
+    c10::optional<torch::Tensor> o1, c10::optional<torch::Tensor> w1,
+    c10::optional<torch::Tensor> o2, c10::optional<torch::Tensor> w2,
+    double scale, c10::optional<torch::Tensor> wa,
+    c10::optional<torch::Tensor> wb, long n, double eps) {
+  LM_CHECK_CONTIG(x);
+  TORCH_CHECK(x.scalar_type() == at::kFloat && x.dim() == 2);
+  const int T = x.size(0), width = x.size(1);
+  TORCH_CHECK(width % 8 == 0 && width <= 16384 && n >= 1 && n <= width);
+  TORCH_CHECK(plain || o1, "lm_add_branches: nothing to add");
+  const auto type = (plain ? *plain : *o1).scalar_type();
+  for (const auto* o : {&plain, &o1, &o2})
+    if (o->has_value()) {
+      LM_CHECK_CONTIG(**o);
+      TORCH_CHECK((*o)->sizes() == x.sizes() && (*o)->scalar_type() == type);
+    }
+  TORCH_CHECK(o1.has_value() == w1.has_value() &&
+              o2.has_value() == w2.has_value() && (o1 || !o2) && (wa || !wb));
+  for (const auto* w : {&w1, &w2, &wa, &wb}) check_weight(*w, width, type);
+  std::vector<torch::Tensor> out;
+  const auto opt = x.options().dtype(type);
+  if (wa) out.push_back(torch::empty({T, width}, opt));
+  if (wb) out.push_back(torch::empty({T, width}, opt));
+  if (T == 0) return out;
+#define LM_PTR(V) (V ? (const scalar_t*)V->data_ptr() : nullptr)
+#define LM_AB_(NV, BR)                                                       \
+  hipLaunchKernelGGL((add_branches_kernel<scalar_t, NV, BR>), dim3(T),       \
+                     dim3(256), 0, cmls::current_stream(),                   \
+                     x.data_ptr<float>(), LM_PTR(plain), LM_PTR(o1),         \
+                     LM_PTR(w1), LM_PTR(o2), LM_PTR(w2), (float)scale,       \
+                     LM_PTR(wa), wa ? (scalar_t*)out[0].data_ptr() : nullptr,\
+                     LM_PTR(wb), wb ? (scalar_t*)out[1].data_ptr() : nullptr,\
+                     width, (int)n, (float)eps)
+#define LM_AB(NV) do { if (o1) LM_AB_(NV, true); else LM_AB_(NV, false); } while (0)
+  auto& of = plain ? *plain : *o1;
+  LM_DISPATCH(of, "lm_add_branches", [&] { LM_NV(width, LM_AB); });
+#undef LM_AB
+#undef LM_AB_
+#undef LM_PTR
+  LM_LAUNCHED();
+  return out;
+}
+
+// coef float (a, b); out [T, ff], row stride free
+void lm_xielu(torch::Tensor z, torch::Tensor coef, torch::Tensor out) {
+  LM_CHECK_CONTIG(z);
+  LM_CHECK_CONTIG(coef);
+  TORCH_CHECK(z.dim() == 2 && z.size(1) % 8 == 0);
+  TORCH_CHECK(coef.numel() == 2 && coef.scalar_type() == at::kFloat);
+  const int ff = z.size(1);
+  const long ld = row_view(out, z.size(0), ff, z.scalar_type());
+  const long total = z.numel() / 8;
+  if (total == 0) return;
+  LM_DISPATCH(z, "lm_xielu", [&] {
+    hipLaunchKernelGGL((xielu_kernel<scalar_t>), dim3((total + 255) / 256),
+                       dim3(256), 0, cmls::current_stream(),
+                       (const scalar_t*)z.data_ptr(), coef.data_ptr<float>(),
+                       (scalar_t*)out.data_ptr(), ld, ff, total);
+  });
+  LM_LAUNCHED();
 }
 
 torch::Tensor lm_output_norm(torch::Tensor x,

@@ -6,6 +6,11 @@ Cache row: a slice [key kd | value vd] per key/value head. Where the values are
 the keys before their norm (``same``), a slice is that projection alone and
 behind the slices stands a float per head, the factor of the key's norm; the
 norm's weights are part of the query.
+
+Pooled layers also see one row for every block of ``pool`` tokens that lies
+wholly in front of the window, the mean of the block's rows. A page holds its
+tokens' rows and, behind them, the means of the blocks whose last token it
+holds, so pooled rows are allocated and freed with the tokens'.
 """
 
 from typing import NamedTuple, Optional
@@ -18,8 +23,10 @@ from .lm import Rotary, _sink_softmax, pad32
 
 class GroupedSpec(NamedTuple):
     """Sizes (padded ``kd``, ``vd``; true ``dim``) and constants of a layer.
-    ``window`` 0: all earlier tokens, else also the first ``keep`` tokens.
-    ``cap`` 0: none. ``out_scale`` multiplies the result."""
+    ``window`` 0: all earlier tokens, else also the first ``keep`` tokens, or
+    with ``pool`` the means of the blocks of so many tokens in front of it.
+    ``cap`` 0: none. ``out_scale`` multiplies the result. ``whole``: norms of
+    queries and keys run over all heads at once."""
 
     heads: int
     kv_heads: int
@@ -32,6 +39,8 @@ class GroupedSpec(NamedTuple):
     scale: float
     cap: float
     out_scale: float
+    pool: int = 0
+    whole: bool = False
 
     @property
     def slice(self) -> int:
@@ -43,6 +52,28 @@ class GroupedSpec(NamedTuple):
         n = self.kv_heads * self.slice
         # a float is two elements of a 16-bit cache
         return n + pad32(2 * self.kv_heads) if self.same else n
+
+
+def page_rows(block_size: int, pool: int) -> int:
+    """rows of a page of ``block_size`` tokens"""
+    return block_size + (-(-block_size // pool) if pool else 0)
+
+
+def page_tokens(rows: int, pool: int) -> int:
+    """tokens of a page of ``rows`` rows"""
+    return rows * pool // (pool + 1) if pool else rows
+
+
+def token_row(block, offset, block_size: int, pool: int):
+    """row of a token at ``offset`` of page ``block``"""
+    return block * page_rows(block_size, pool) + offset
+
+
+def pooled_row(block, offset, block_size: int, pool: int):
+    """row of the mean of the block whose last token is at ``offset`` of page
+    ``block``"""
+    return (block * page_rows(block_size, pool) + block_size
+            + offset // pool)
 
 
 def _norm_factor(v: torch.Tensor, n: int, eps: float) -> torch.Tensor:
@@ -60,26 +91,39 @@ def prepare(z: torch.Tensor, k_at: int, v_at: int, positions: torch.Tensor,
             s: GroupedSpec, q_norm: Optional[torch.Tensor],
             k_norm: Optional[torch.Tensor], eps: float,
             first: Optional[torch.Tensor], lam: float,
-            cache: torch.Tensor) -> None:
-    """z [T, cols]: queries at column 0, keys at k_at, values at v_at. Norms
-    (per head, weights [kd]) and rotates queries in place and keys on their
-    way to the cache rows of ``slot_mapping``; ``first`` [T, kv_heads * vd]:
-    values become (1 - lam) v + lam first."""
+            cache: torch.Tensor, bias: Optional[torch.Tensor] = None
+            ) -> None:
+    """z [T, cols]: queries at column 0, keys at k_at, values at v_at; ``bias``
+    [cols] is added first. Norms (per head, weights [kd], or over all heads,
+    weights [heads * kd]) and rotates queries in place and keys on their way to
+    the cache rows of ``slot_mapping`` (page * tokens of a page + offset);
+    ``first`` [T, kv_heads * vd]: values become (1 - lam) v + lam first."""
     if z.is_cuda:
         require_lm_ext("grouped_prep").lm_grouped_prep(
             z, k_at, -1 if s.same else v_at, positions, slot_mapping,
             None if rot is None else rot.inv_freq,
             1.0 if rot is None else rot.gain, s.heads, s.kv_heads, s.kd,
-            s.vd, s.dim, q_norm, k_norm, eps, first, lam, cache)
+            s.vd, s.dim, q_norm, k_norm, eps, first, lam, cache, bias,
+            s.whole, s.pool)
         return
     t, g = z.shape[0], s.kv_heads
+    if bias is not None:
+        z.copy_(z.float() + bias.float())
     q = z[:, :s.heads * s.kd].view(t, s.heads, s.kd)
     k = z[:, k_at:k_at + g * s.kd].reshape(t, g, s.kd)
     qf, kf = q.float(), k.float()
+    if s.whole:
+        qf = (qf.view(t, -1) * _norm_factor(q.reshape(t, -1), s.heads * s.dim,
+                                            eps) * q_norm.float()).view_as(q)
+        kf = (kf.view(t, -1) * _norm_factor(k.reshape(t, -1), g * s.dim, eps)
+              * k_norm.float()).view_as(k)
+        q_norm = k_norm = None
     if q_norm is not None:
         qf = qf * _norm_factor(q, s.dim, eps) * q_norm.float()
     keep = slot_mapping >= 0
     at = slot_mapping[keep].long()
+    bs = page_tokens(cache.shape[1], s.pool)
+    at = token_row(at // bs, at % bs, bs, s.pool)
     rows = cache.view(-1, cache.shape[-1])
     if s.same:
         new = rows[at]  # a copy
@@ -105,6 +149,27 @@ def prepare(z: torch.Tensor, k_at: int, v_at: int, positions: torch.Tensor,
         qf = qf.clone()
         rot.rotate_(qf, positions)
     q.copy_(qf)
+
+
+def pool_rows(cache: torch.Tensor, block_table: torch.Tensor,
+              tok_seq: torch.Tensor, positions: torch.Tensor,
+              pool: int) -> None:
+    """Writes the mean row of every block of ``pool`` tokens that one of the
+    given tokens ends; the block's rows are in the cache."""
+    if cache.is_cuda:
+        require_lm_ext("grouped_pool").lm_grouped_pool(
+            cache, block_table, tok_seq, positions, pool)
+        return
+    bs = page_tokens(cache.shape[1], pool)
+    rows = cache.view(-1, cache.shape[2])
+    for t, p in enumerate(positions.tolist()):
+        if (p + 1) % pool:
+            continue
+        pages = block_table[int(tok_seq[t])].long()
+        key = torch.arange(p + 1 - pool, p + 1)
+        mean = rows[token_row(pages[key // bs], key % bs, bs, pool)].float()
+        rows[pooled_row(pages[p // bs], p % bs, bs, pool)] = \
+            mean.mean(0).to(cache.dtype)
 
 
 def _attend(q, rows, see, sink, s: GroupedSpec):
@@ -143,18 +208,24 @@ def attention(q: torch.Tensor, cache: torch.Tensor, block_table: torch.Tensor,
     if q.is_cuda:
         require_lm_ext("grouped_attention").lm_grouped_attention(
             q, cache, block_table, tok_seq, positions, sink, out, n, s.heads,
-            s.kv_heads, s.kd, s.vd, s.same, s.window, s.keep, s.scale, s.cap,
-            s.out_scale, max_keys)
+            s.kv_heads, s.kd, s.vd, s.same, s.window, s.keep, s.pool, s.scale,
+            s.cap, s.out_scale, max_keys)
         return
-    bs = cache.shape[1]
+    bs = page_tokens(cache.shape[1], s.pool)
     rows = cache.view(-1, cache.shape[2])
     for t in range(n):
         p = int(positions[t])
         key = torch.arange(p + 1)
         key = key[_sees(torch.tensor([p]), key, s)[0]]
-        blk = block_table[int(tok_seq[t])].long()[key // bs]
-        got = _attend(q[t:t + 1], rows[blk * bs + key % bs],
-                      torch.ones(1, len(key), dtype=torch.bool), sink, s)
+        pages = block_table[int(tok_seq[t])].long()
+        at = token_row(pages[key // bs], key % bs, bs, s.pool)
+        if s.pool:
+            blocks = max(0, p + 1 - s.window) // s.pool
+            last = torch.arange(blocks) * s.pool + s.pool - 1
+            at = torch.cat([pooled_row(pages[last // bs], last % bs, bs,
+                                       s.pool), at])
+        got = _attend(q[t:t + 1], rows[at],
+                      torch.ones(1, len(at), dtype=torch.bool), sink, s)
         out[t] = got[0].to(out.dtype)
 
 
@@ -163,15 +234,23 @@ def prompt(q: torch.Tensor, rows: torch.Tensor, sink: Optional[torch.Tensor],
     """Prompt portions on gathered cache rows [n, row]; qtiles [n, 6]: first
     token, tokens, first position, first gathered row, what the number of a
     row behind the ``keep`` first lacks to its position, gathered rows of the
-    sequence. Writes out [T, H * vd] at the tiles' tokens."""
+    sequence. With ``pool`` a seventh column: pooled rows, which come first,
+    as ``keep`` ones do. Writes out [T, H * vd] at the tiles' tokens."""
     if q.is_cuda:
         require_lm_ext("grouped_prompt").lm_grouped_prompt(
             q, rows, sink, qtiles, out, s.heads, s.kv_heads, s.kd, s.vd,
-            s.same, s.window, s.keep, s.scale, s.cap, s.out_scale)
+            s.same, s.window, s.keep, s.pool, s.scale, s.cap, s.out_scale)
         return
-    for t0, n, p0, r0, skip, nk in qtiles.tolist():
+    for t0, n, p0, r0, skip, nk, *pooled in qtiles.tolist():
+        qpos = p0 + torch.arange(n)
         kpos = torch.arange(nk)
-        kpos[s.keep:] += skip
-        see = _sees(p0 + torch.arange(n), kpos, s)
+        if s.pool:
+            kpos, blocks = kpos[pooled[0]:] + skip, kpos[:pooled[0]]
+            last = blocks * s.pool + s.pool - 1
+            see = torch.cat([last[None] <= qpos[:, None] - s.window,
+                             _sees(qpos, kpos, s)], 1)
+        else:
+            kpos[s.keep:] += skip
+            see = _sees(qpos, kpos, s)
         out[t0:t0 + n] = _attend(q[t0:t0 + n], rows[r0:r0 + nk], see, sink,
                                  s).to(out.dtype)

@@ -10,7 +10,7 @@ size, which leaves every product and sum of squares unchanged.
 """
 
 import math
-from typing import NamedTuple, Optional, Tuple, Union
+from typing import List, NamedTuple, Optional, Sequence, Tuple, Union
 
 import torch
 
@@ -65,6 +65,50 @@ def embed_stream(tokens: torch.Tensor, table: torch.Tensor,
         copy.copy_(rows)
     x = rows.float()
     return x, _next_input(x, norm, table.dtype, out)
+
+
+def embed_norms(tokens: torch.Tensor, table: torch.Tensor,
+                norms: Sequence[RowNorm]
+                ) -> Tuple[torch.Tensor, List[torch.Tensor]]:
+    """-> (x float [T, width], norm(x) in the table's type for each of one or
+    two norms, which share their root mean square)"""
+    if table.is_cuda:
+        a, b = _two(norms)
+        x, *h = require_lm_ext("embed_norms").lm_embed_norms(
+            tokens, table, a, b, norms[0].n, norms[0].eps)
+        return x, h
+    x = table[tokens.clamp(0, table.shape[0] - 1)].float()
+    return x, [norm(x).to(table.dtype) for norm in norms]
+
+
+def _two(norms: Sequence[RowNorm]):
+    """weights of up to two norms of the same row"""
+    assert len(norms) <= 2 and all(
+        v.offset == 0.0 and v.n == norms[0].n and v.eps == norms[0].eps
+        for v in norms)
+    w = [v.weight for v in norms]
+    return (w + [None, None])[:2]
+
+
+def add_branches(x: torch.Tensor, plain: Optional[torch.Tensor],
+                 branches: Sequence[Tuple[torch.Tensor, torch.Tensor]],
+                 scale: float, norms: Sequence[RowNorm], n: int, eps: float,
+                 dtype: torch.dtype) -> List[torch.Tensor]:
+    """What parallel sublayers made, in place into the float stream:
+    x += plain + scale * (sum of o / rms(o) * weight over the up to two
+    ``branches``). -> norm(x) in ``dtype`` for each of up to two norms.
+    ``n``: true row size."""
+    if x.is_cuda:
+        (o1, w1), (o2, w2) = (list(branches) + [(None, None)] * 2)[:2]
+        a, b = _two(norms)
+        return require_lm_ext("add_branches").lm_add_branches(
+            x, plain, o1, w1, o2, w2, scale, a, b, n, eps)
+    if plain is not None:
+        x += plain.float()
+    for o, w in branches:
+        v = o.float()
+        x += scale * (v * _rms_inv(v, n, eps) * w.float())
+    return [norm(x).to(dtype) for norm in norms]
 
 
 def post_norm_add(o: torch.Tensor, bias: Optional[torch.Tensor],
@@ -153,6 +197,18 @@ def gated_mul(gate_up: torch.Tensor, bias: Optional[torch.Tensor],
         v = v + bias.float()
     g, u = v.chunk(2, dim=-1)
     return (activate(g, act) * u).to(gate_up.dtype)
+
+
+def xielu(z: torch.Tensor, coef: torch.Tensor, out: torch.Tensor) -> None:
+    """coef (a, b), float: a z^2 + z / 2 for z > 0, else b (e^z - 1 - z) +
+    z / 2. out [T, ff] can be a range of columns."""
+    if z.is_cuda:
+        require_lm_ext("xielu").lm_xielu(z, coef, out)
+        return
+    v = z.float()
+    a, b = coef.tolist()
+    out.copy_(torch.where(v > 0, a * v * v, b * (torch.expm1(v) - v))
+              + 0.5 * v)
 
 
 def gather_rows(src: torch.Tensor, idx: torch.Tensor) -> torch.Tensor:
