@@ -13,8 +13,9 @@ dynamic batcher -> hipGraph replay on the GPU) and awaits all responses.
 
   python bench.py --gpus N --steps K --warmup W
 
-``--workload lm`` measures another thing: prefill and decode of the Pamazen,
-Kakipel and Bimipel families beside llama at equal size (benchmarks/lm_bench.py).
+``--workload lm`` measures another thing: prefill and decode of the Nelovik,
+Pamazen, Kakipel and Bimipel families beside llama at equal size
+(benchmarks/lm_bench.py).
 """
 
 import argparse
@@ -124,7 +125,7 @@ def main():
                          "decode of Pamazen, Kakipel and Bimipel beside "
                          "llama")
     ap.add_argument("--lm-size", default="300m,1b,4k")
-    ap.add_argument("--lm-model", default="pamazen,kakipel,bimipel,llama")
+    ap.add_argument("--lm-model", default="nelovik,pamazen,kakipel,bimipel,llama")
     ap.add_argument("--lm-prompt", type=int, default=2048)
     ap.add_argument("--lm-batch", default="1,16,64")
     ap.add_argument("--lm-phase", default="prefill,decode")

@@ -1,6 +1,6 @@
-"""Prefill and decode throughput of the token-batch families (Pamazen,
-Kakipel, Bimipel) beside llama at equal size, random weights, through the LLM engine's
-own forwards.
+"""Prefill and decode throughput of the token-batch families (Nelovik, Pamazen,
+Kakipel, Bimipel) beside llama at equal size, random weights, through the LLM
+engine's own forwards.
 
     python bench.py --workload lm [--lm-size 300m,1b,4k] [--lm-model ...]
 
@@ -17,16 +17,19 @@ import torch
 
 SIZES = {
     # size -> model -> (preset, overrides)
-    "300m": {"pamazen": ("pamazen-300m", {}),
+    "300m": {"nelovik": ("nelovik-300m", {}),
+             "pamazen": ("pamazen-300m", {}),
              "kakipel": ("kakipel-300m", {}), "bimipel": ("bimipel-300m", {}),
              "llama": ("llama-3-8b", dict(
                  vocab_size=32000, hidden=1024, layers=12, heads=16,
                  kv_heads=4, intermediate=3584))},
-    "1b": {"pamazen": ("pamazen-1b", {}),
+    "1b": {"nelovik": ("nelovik-1b", {}),
+           "pamazen": ("pamazen-1b", {}),
            "kakipel": ("kakipel-1b", {}), "bimipel": ("bimipel-1b", {}),
            "llama": ("llama-3-1b", {})},
     # few layers, as wide as an 8B model's
-    "4k": {"pamazen": ("pamazen-4k", {}),
+    "4k": {"nelovik": ("nelovik-4k", {}),
+           "pamazen": ("pamazen-4k", {}),
            "kakipel": ("kakipel-4k", {}), "bimipel": ("bimipel-4k", {}),
            "llama": ("llama-3-8b", dict(vocab_size=32000, layers=6,
                                         intermediate=12288))},

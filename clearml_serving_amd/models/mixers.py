@@ -591,7 +591,8 @@ class LinearState(nn.Module):
         state, ring = cache
         linear_state.linear_state(
             z, self.spec, self._w, state, ring, batch.positions,
-            batch.state_slots, batch.tiles, batch.seqs, batch.n_single, out)
+            batch.state_slots, batch.tiles, batch.seqs, batch.tile,
+            batch.n_single, out)
 
 
 class GatedDelta(LinearState):

@@ -56,6 +56,7 @@ struct StateArgs {
   float* state;      // [slots, heads, VP, KP]
   T* ring;           // [slots, taps, channels]
   T* u;              // convolved rows of the portions, [rows + CH, channels]
+  float* decay;      // [tiles, heads, 2, DECAY] of the portions' chunks
   T* y;              // o of all tokens, [T, heads * VP]
   T* out;            // rows of ld_out
   long ld_out;
@@ -89,9 +90,66 @@ __device__ __forceinline__ float sum8(float v) {  // lanes that share lane >> 3
 // ------------------------------------------------------------------- //
 // convolution and SiLU of the portions' tokens
 // ------------------------------------------------------------------- //
-// A thread takes 8 channels of up to 8 tokens; TAPS >= taps.
-template <typename T, int TAPS>
-__global__ __launch_bounds__(256) void state_conv_kernel(StateArgs<T> p) {
+constexpr int TILE = 64;              // tokens of the host's tiles
+constexpr int CH = 32, NB = CH / 16;  // tokens of a chunk, its blocks
+
+struct ChunkDecay {
+  float in[CH];    // e^(G_t)
+  float out[CH];   // e^(G_end - G_t)
+  float step[CH];  // b_t or d_t
+  float run[CH];   // sum of g from the block's start to t
+  float rest[CH];  // sum of g behind t to the block's end
+  float total;     // e^(G_end)
+  float pad[3];
+};
+constexpr int DECAY = sizeof(ChunkDecay) / 4;
+
+// the decays of a tile's two chunks, a wave per head
+template <typename T, bool DELTA>
+__device__ __forceinline__ void tile_decays(const StateArgs<T>& p, int tile,
+                                            int h) {
+  const int t0 = p.tiles[tile * 5], len = p.tiles[tile * 5 + 1];
+  const int lane = threadIdx.x & 63, r16 = lane & 15;
+  float gt = 0.f, step = 0.f;
+  if (lane < len) {
+    const T* row = p.z + (long)(t0 + lane) * p.ld;
+    decay_of(to_f32(row[p.a_at + h]), to_f32(p.a_log[h]),
+             to_f32(p.dt_bias[h]), &gt, &step);
+    if (DELTA) step = 1.f / (1.f + expf(-to_f32(row[p.b_at + h])));
+  }
+  float run = gt, rest = gt;
+#pragma unroll
+  for (int d = 1; d < 16; d <<= 1) {
+    const float a = __shfl_up(run, d, 16), b = __shfl_down(rest, d, 16);
+    if (r16 >= d) run += a;
+    if (r16 + d < 16) rest += b;
+  }
+  const int half = lane & 32;
+  const float first = __shfl(run, half + 15, 64);
+  const float second = __shfl(run, half + 31, 64);
+  const float behind = __shfl_down(rest, 1, 16);
+  rest = r16 == 15 ? 0.f : behind;
+  ChunkDecay* d = (ChunkDecay*)p.decay +
+                  ((long)tile * p.heads + h) * 2 + (half ? 1 : 0);
+  const int t = lane & 31;
+  d->run[t] = run;
+  d->rest[t] = rest;
+  d->step[t] = step;
+  d->in[t] = expf(t < 16 ? run : first + run);
+  d->out[t] = expf(t < 16 ? rest + second : rest);
+  if (t == 0) d->total = expf(first + second);
+}
+
+// A thread takes 8 channels of up to 8 tokens; TAPS >= taps. The grid's last
+// rows make the chunks' decays.
+template <typename T, int TAPS, bool DELTA>
+__global__ __launch_bounds__(256) void state_conv_kernel(StateArgs<T> p,
+                                                         int n_conv) {
+  if ((int)blockIdx.y >= n_conv) {
+    const int h = (blockIdx.y - n_conv) * 4 + (threadIdx.x >> 6);
+    if (h < p.heads) tile_decays<T, DELTA>(p, blockIdx.x, h);
+    return;
+  }
   const int* td = p.tiles + blockIdx.x * 5;
   const int t0 = td[0], len = td[1], p0 = td[2], slot = td[3], into = td[4];
   const int c = (blockIdx.y * 32 + (threadIdx.x & 31)) * 8;
@@ -148,17 +206,19 @@ __global__ __launch_bounds__(256) void state_conv_kernel(StateArgs<T> p) {
 // ------------------------------------------------------------------- //
 // portions in chunks
 // ------------------------------------------------------------------- //
-constexpr int CH = 32, NB = CH / 16;  // tokens of a chunk, its blocks
-
-struct ChunkDecay {   // of one chunk, in LDS
-  float in[CH];       // e^(G_t)
-  float out[CH];      // e^(G_end - G_t)
-  float step[CH];     // b_t or d_t
-  float run[CH];      // sum of g from the block's start to t
-  float rest[CH];     // sum of g behind t to the block's end
-  float total;        // e^(G_end)
-  float pad[3];
-};
+// sum over N neighbouring lanes, in all of them (DPP within 16 lanes)
+template <int N> __device__ __forceinline__ float sum_lanes(float v) {
+#define LM_DPP_ADD(CTRL)                                      \
+  v += __int_as_float(__builtin_amdgcn_update_dpp(            \
+      0, __float_as_int(v), CTRL, 0xf, 0xf, true))
+  LM_DPP_ADD(0xB1);                       // quad_perm 1 0 3 2
+  LM_DPP_ADD(0x4E);                       // quad_perm 2 3 0 1
+  if (N >= 8) LM_DPP_ADD(0x141);          // row_half_mirror
+  if (N >= 16) LM_DPP_ADD(0x140);         // row_mirror
+#undef LM_DPP_ADD
+  if (N >= 32) v += __shfl_xor(v, 16, 64);
+  return v;
+}
 
 // a[16 rows][K] . b[16 rows][K]^T, rows of `pitch` in LDS
 __device__ __forceinline__ lm_f32x4 dot_rows(const float* a, const float* b,
@@ -191,167 +251,137 @@ __device__ __forceinline__ lm_f32x4 mul_tile(const float* a, int pitch,
   return c;
 }
 
-// D: 32-channel blocks of a key, NW: waves. Grid (heads * slices of NW * 16
-// values, sequences).
-template <typename T, int D, int NW, bool DELTA>
-__global__ __launch_bounds__(NW * 64, D <= 4 ? 4 : 2)
+// The elements of two 16-token blocks' products: rows t of block bi, columns s
+// of block bj, times the decay between s and t
+__device__ __forceinline__ lm_f32x4 decayed(lm_f32x4 c, const ChunkDecay& d,
+                                            int bi, int bj) {
+  const int lane = threadIdx.x & 63, s = bj * 16 + (lane & 15);
+  const lm_f32x4 run =
+      *reinterpret_cast<const lm_f32x4*>(d.run + bi * 16 + 4 * (lane >> 4));
+  // in one block the difference of two sums of it
+  const float from_s = bi == bj ? -d.run[s] : d.rest[s];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) c[r] *= exp_f(fminf(run[r] + from_s, 0.f));
+  return c;
+}
+
+// D: 32-channel blocks of a key. Grid (heads * slices of 64 values,
+// sequences). Four waves keep the state, 16 values each; four more prepare the
+// next chunk meanwhile: they stage its rows while the first ones multiply this
+// chunk's with the state, and make its A and M while the others finish.
+constexpr int NW = 4, NTH = NW * 64;
+template <typename T, int D, bool DELTA>
+__global__ __launch_bounds__(2 * NTH, 2)
 void state_chunk_kernel(StateArgs<T> p) {
-  constexpr int KP = D * 32, PITCH = KP + 4, NTH = NW * 64, AP = CH + 4;
-  constexpr int LPR = D <= 1 ? 4 : D <= 2 ? 8 : D <= 4 ? 16 : 32;  // per row
-  constexpr int NI = (2 * CH * LPR + NTH - 1) / NTH;
+  constexpr int KP = D * 32, PITCH = KP + 4, AP = CH + 4;
+  constexpr int AM = (DELTA ? 2 : 1) * CH * AP;  // -A and inverses, M
+  // staging: LPR lanes take a row, RPI rows at a time
+  constexpr int LPR = D <= 1 ? 4 : D <= 2 ? 8 : D <= 4 ? 16 : 32;
+  constexpr int RPI = NTH / LPR, NI = 2 * CH / RPI;
+  static_assert(NI * RPI == 2 * CH, "rows");
   extern __shared__ __align__(16) float sm[];
   float* sk = sm;                   // 2 x [K rows | Q rows]
-  float* sa = sm + 4 * CH * PITCH;  // [CH][AP]: -A, inverses
-  float* sM = sa + (DELTA ? CH * AP : 0);
-  ChunkDecay* dec = (ChunkDecay*)(sM + CH * AP);  // [2]
-  const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave();
+  float* sam = sm + 4 * CH * PITCH; // 2 x [M | A], [CH][AP] each
+  float* sd = sam + 2 * AM;         // 2 x DECAY
+  const int lane = threadIdx.x & 63, wave = uniform_wave() % NW;
+  const int tid = wave * 64 + lane;  // within the four waves
+  const bool keeps = uniform_wave() < NW;
   const int r16 = lane & 15, g = lane >> 4;
   const int h = blockIdx.x % p.heads, slice = blockIdx.x / p.heads;
   // long sequences first: they are the last of the list
-  const int* sd = p.seqs + (p.n_seq - 1 - (int)blockIdx.y) * 6;
-  const int t0 = sd[2], len = sd[3], p0 = sd[4], slot = sd[5];
+  const int* sq = p.seqs + (p.n_seq - 1 - (int)blockIdx.y) * 6;
+  const int t0 = sq[2], len = sq[3], p0 = sq[4], slot = sq[5];
   const bool has_state = slot >= 0 && slot < p.n_state;
   const int hk = h / (p.heads / p.groups);
-  const int v0 = (slice * NW + wave) * 16;  // the wave's values
-  const bool active = v0 < p.VP;  // else all that it makes is left unused
-  const int col = active ? v0 + r16 : 0;
-  float* st = p.state +
-              (((long)(has_state ? slot : 0) * p.heads + h) * p.VP + col) *
-                  KP + 4 * g;
-
-  lm_f32x4 S[2 * D];  // S[i][r]: key 16 i + 4 g + r, value r16
-  if (p0 > 0 && has_state) {
-#pragma unroll
-    for (int i = 0; i < 2 * D; ++i)
-      S[i] = *reinterpret_cast<const lm_f32x4*>(st + 16 * i);
-  } else {
-#pragma unroll
-    for (int i = 0; i < 2 * D; ++i) S[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
-  }
-
-  // ---- staging of a chunk: rows through registers ---- //
   const T* urow = p.u + (long)(t0 - p.n_single) * p.channels;
-  Raw8<T> kq[NI];
-  float raw_a = 0.f, raw_b = 0.f;
-  T vr[NB][4];
-  auto load = [&](int at) {
-    const int nt = min(CH, len - at);
-#pragma unroll
-    for (int i = 0; i < NI; ++i) {
-      const int item = tid + i * NTH, row = item / LPR, c = item % LPR * 8;
-      const int t = row % CH;
-      kq[i] = Raw8<T>{};
-      if (row < 2 * CH && t < nt && c < KP)
-        kq[i] = *reinterpret_cast<const Raw8<T>*>(
-            urow + (long)(at + t) * p.channels + (row < CH ? p.k_at : 0) +
-            hk * KP + c);
-    }
-    if (tid < CH && tid < nt) {
-      const T* row = p.z + (long)(t0 + at + tid) * p.ld;
-      raw_a = to_f32(row[p.a_at + h]);
-      if (DELTA) raw_b = to_f32(row[p.b_at + h]);
-    }
-  };
-  auto load_values = [&](int at) {
-    // u has CH more rows than there are tokens
-    const T* v = urow + (long)at * p.channels + p.v_at + h * p.VP;
-    const int lane_at = 4 * g * p.channels + col;
-#pragma unroll
-    for (int i = 0; i < NB; ++i)
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        vr[i][r] = v[lane_at + (16 * i + r) * p.channels];
-  };
-  const float a_log = to_f32(p.a_log[h]), dt_bias = to_f32(p.dt_bias[h]);
-  const float q_scale = DELTA ? 1.f / sqrtf((float)p.dim) : 1.f;
-  auto store = [&](int at, int buf) {
-    const int nt = min(CH, len - at);
-#pragma unroll
-    for (int i = 0; i < NI; ++i) {
-      const int item = tid + i * NTH, row = item / LPR, c = item % LPR * 8;
-      float f = 1.f, x[8];
-      load8<T>(kq[i].v, x);
-      if (DELTA) {
-        float ss = 0.f;
-#pragma unroll
-        for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
-#pragma unroll
-        for (int d = 1; d < LPR; d <<= 1) ss += __shfl_xor(ss, d, 64);
-        f = 1.f / sqrtf(ss + 1e-6f);
-        if (row >= CH) f *= q_scale;
-      }
-      if (row < 2 * CH && c < KP) {
-#pragma unroll
-        for (int e = 0; e < 8; ++e) x[e] *= f;
-        store8(sk + (buf * 2 * CH + row) * PITCH + c, x);
-      }
-    }
-    if (wave == 0) {  // decays: sums within blocks of 16 lanes
-      float gt = 0.f, step = 0.f;
-      if (lane < nt) {
-        decay_of(raw_a, a_log, dt_bias, &gt, &step);
-        if (DELTA) step = 1.f / (1.f + expf(-raw_b));
-      }
-      float run = gt, rest = gt;
-#pragma unroll
-      for (int d = 1; d < 16; d <<= 1) {
-        const float a = __shfl_up(run, d, 16), b = __shfl_down(rest, d, 16);
-        if (r16 >= d) run += a;
-        if (r16 + d < 16) rest += b;
-      }
-      const float first = __shfl(run, 15, 64), second = __shfl(run, 31, 64);
-      const float behind = __shfl_down(rest, 1, 16);
-      rest = r16 == 15 ? 0.f : behind;
-      if (lane < CH) {
-        ChunkDecay* d = dec + buf;
-        d->run[lane] = run;
-        d->rest[lane] = rest;
-        d->step[lane] = step;
-        d->in[lane] = expf(lane < 16 ? run : first + run);
-        d->out[lane] = expf(lane < 16 ? rest + second : rest);
-        if (lane == 0) d->total = expf(first + second);
-      }
-    }
-  };
 
-  const float skip = DELTA ? 0.f : to_f32(p.skip[h]);
-  load(0);
-  store(0, 0);
-  int buf = 0;
-  for (int at = 0; at < len; at += CH, buf ^= 1) {
-    const int nt = min(CH, len - at);
-    const float* K = sk + buf * 2 * CH * PITCH;
-    const float* Q = K + CH * PITCH;
-    const ChunkDecay& d = dec[buf];
-    __syncthreads();
-    if (at + CH < len) load(at + CH);
-    load_values(at);
-
-    // K K^T and Q K^T, the lower 16x16 blocks
-    constexpr int TASKS = DELTA ? 6 : 3;
-    for (int task = wave; task < TASKS; task += NW) {
-      const bool kk = DELTA && task < 3;
-      const int which = kk ? task : task - (DELTA ? 3 : 0);
-      const int bi = which > 0, bj = which == 1;  // (0,0) (1,1) (1,0)
-      lm_f32x4 c = dot_rows((kk ? K : Q) + bi * 16 * PITCH,
-                            K + bj * 16 * PITCH, PITCH, KP);
-      float* dst = (kk ? sa : sM) + bi * 16 * AP + bj * 16;
-      const int s = bj * 16 + r16;
-      const float from_s = bi == bj ? -d.run[s] : d.rest[s];
+  if (!keeps) {
+    const float* drow = p.decay + ((long)sq[0] * p.heads + h) * 2 * DECAY;
+    Raw8<T> kq[NI];
+    lm_f32x4 dreg = {0.f, 0.f, 0.f, 0.f};
+    const int item_row = tid / LPR, item_c = tid % LPR * 8;
+    const bool item_in = LPR * 8 == KP || item_c < KP;
+    const unsigned item_at = item_row * p.channels + (item_in ? item_c : 0);
+    const float q_scale = DELTA ? 1.f / sqrtf((float)p.dim) : 1.f;
+    auto load = [&](int at) {
+      // u has CH more rows than there are tokens
+      const T* q = urow + (long)at * p.channels + hk * KP;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int tt = 4 * g + r, t = bi * 16 + tt;
-        // of s before t; in one block the difference of two sums of it
-        const float e = expf(fminf(d.run[t] + from_s, 0.f));
-        if (kk)
-          c[r] = bi == bj && r16 >= tt ? 0.f : c[r] * e * -d.step[t];
-        else
-          c[r] = bi == bj && r16 > tt ? 0.f : c[r] * e;
-        if (!kk || bi != bj) dst[tt * AP + r16] = c[r];
+      for (int i = 0; i < NI; ++i) {
+        if (RPI > CH) {  // K and Q rows at once
+          const bool is_q = item_row >= CH;
+          kq[i] = *reinterpret_cast<const Raw8<T>*>(
+              q + (long)(item_row % CH) * p.channels + item_c +
+              (is_q ? 0 : p.k_at));
+        } else {
+          const bool is_q = i * RPI >= CH;
+          kq[i] = *reinterpret_cast<const Raw8<T>*>(
+              q + (is_q ? 0 : p.k_at) + (i * RPI % CH) * p.channels + item_at);
+        }
       }
-      if (kk && bi == bj) {
+      if (tid < DECAY / 4)
+        dreg = reinterpret_cast<const lm_f32x4*>(
+            drow + ((long)(at / TILE) * p.heads * 2 + at / CH % 2) *
+                       DECAY)[tid];
+    };
+    auto store = [&](int at, int buf) {
+      const int nt = min(CH, len - at);
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const int row = i * RPI + item_row;
+        const bool live = row % CH < nt && item_in;
+        float f = 1.f, x[8];
+        load8<T>(kq[i].v, x);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] = live ? x[e] : 0.f;
+        if (DELTA) {
+          float ss = 0.f;
+#pragma unroll
+          for (int e = 0; e < 8; ++e) ss += x[e] * x[e];
+          ss = sum_lanes<LPR>(ss);
+          f = __builtin_amdgcn_rsqf(ss + 1e-6f);
+          if (row >= CH) f *= q_scale;
+        }
+        if (item_in) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[e] *= f;
+          store8(sk + (buf * 2 * CH + row) * PITCH + item_c, x);
+        }
+      }
+      if (tid < DECAY / 4)
+        reinterpret_cast<lm_f32x4*>(sd + buf * DECAY)[tid] = dreg;
+    };
+    // the lower 16x16 blocks of K K^T and Q K^T: waves 0 and 1 the diagonal
+    // ones of K K^T, which they also invert
+    auto products = [&](int buf) {
+      const float* K = sk + buf * 2 * CH * PITCH;
+      const float* Q = K + CH * PITCH;
+      float* sM = sam + buf * AM;
+      float* sa = sM + CH * AP;
+      const ChunkDecay& d =
+          *reinterpret_cast<const ChunkDecay*>(sd + buf * DECAY);
+      auto put_m = [&](lm_f32x4 m, int bi, int bj) {
+        m = decayed(m, d, bi, bj);
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          sM[(bi * 16 + 4 * g + r) * AP + bj * 16 + r16] =
+              bi == bj && r16 > 4 * g + r ? 0.f : m[r];
+      };
+      if (!DELTA) {
+        if (wave < 3) {
+          const int bi = wave > 0, bj = wave == 1;
+          put_m(dot_rows(Q + bi * 16 * PITCH, K + bj * 16 * PITCH, PITCH, KP),
+                bi, bj);
+        }
+      } else if (wave < 2) {
+        const float* k = K + wave * 16 * PITCH;
+        lm_f32x4 c = decayed(dot_rows(k, k, PITCH, KP), d, wave, wave);
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          c[r] = r16 < 4 * g + r ? c[r] * -d.step[wave * 16 + 4 * g + r] : 0.f;
         // 1 / (1 + A) by substitution, a lane per column; c holds -A, whose
         // element (i, j) is register i % 4 of lane 16 (i / 4) + j
+        float* dst = sa + wave * (16 * AP + 16) + r16;
         float x[16];
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
@@ -365,20 +395,86 @@ void state_chunk_kernel(StateArgs<T> p) {
             else even += m * x[j];
           }
           x[i] = even + odd;
-          if (lane < 16) dst[i * AP + r16] = x[i];
+          if (lane < 16) dst[i * AP] = x[i];
         }
-      }
-    }
-
-    // products with the state in front of the chunk
-    lm_f32x4 R[NB], O[NB];
+      } else if (wave == 2) {
+        lm_f32x4 kk = dot_rows(K + 16 * PITCH, K, PITCH, KP);
+        const lm_f32x4 qk = dot_rows(Q + 16 * PITCH, K, PITCH, KP);
+        kk = decayed(kk, d, 1, 0);
 #pragma unroll
-    for (int i = 0; i < NB; ++i) R[i] = O[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
-    {
+        for (int r = 0; r < 4; ++r)
+          sa[(16 + 4 * g + r) * AP + r16] = kk[r] * -d.step[16 + 4 * g + r];
+        put_m(qk, 1, 0);
+      } else {
+        const lm_f32x4 m0 = dot_rows(Q, K, PITCH, KP);
+        const lm_f32x4 m1 =
+            dot_rows(Q + 16 * PITCH, K + 16 * PITCH, PITCH, KP);
+        put_m(m0, 0, 0);
+        put_m(m1, 1, 1);
+      }
+    };
+    load(0);
+    store(0, 0);
+    if (CH < len) load(CH);
+    __syncthreads();
+    products(0);
+    __syncthreads();
+    int buf = 0;
+    for (int at = CH; at < len; at += CH) {  // at: the next chunk
+      buf ^= 1;
+      store(at, buf);
+      if (at + CH < len) load(at + CH);
+      __syncthreads();
+      products(buf);
+      __syncthreads();
+    }
+    __syncthreads();  // the last chunk's, where nothing is next
+  } else {
+    const int v0 = (slice * NW + wave) * 16;  // the wave's values
+    const bool active = v0 < p.VP;  // else all that it makes is left unused
+    const int col = active ? v0 + r16 : 0;
+    float* st = p.state +
+                (((long)(has_state ? slot : 0) * p.heads + h) * p.VP + col) *
+                    KP + 4 * g;
+    lm_f32x4 S[2 * D];  // S[i][r]: key 16 i + 4 g + r, value r16
+    if (p0 > 0 && has_state) {
+#pragma unroll
+      for (int i = 0; i < 2 * D; ++i)
+        S[i] = *reinterpret_cast<const lm_f32x4*>(st + 16 * i);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 2 * D; ++i) S[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    const float skip = DELTA ? 0.f : to_f32(p.skip[h]);
+    const int ld_y = p.heads * p.VP;
+    const unsigned lane_v = 4 * g * p.channels + col;
+    const unsigned lane_y = 4 * g * ld_y + col;
+    __syncthreads();
+    __syncthreads();
+    int buf = 0;
+    for (int at = 0; at < len; at += CH, buf ^= 1) {
+      const int nt = min(CH, len - at);
+      const float* K = sk + buf * 2 * CH * PITCH;
+      const float* Q = K + CH * PITCH;
+      const float* sM = sam + buf * AM;
+      const float* sa = sM + CH * AP;
+      const ChunkDecay& d =
+          *reinterpret_cast<const ChunkDecay*>(sd + buf * DECAY);
+      T vr[NB][4];
+      {
+        const T* v = urow + (long)at * p.channels + p.v_at + h * p.VP;
+#pragma unroll
+        for (int i = 0; i < NB; ++i)
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            vr[i][r] = (v + (16 * i + r) * p.channels)[lane_v];
+      }
+      // products with the state in front of the chunk
+      lm_f32x4 R[NB], O[NB];
+#pragma unroll
+      for (int i = 0; i < NB; ++i) R[i] = O[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int k = 0; k < 2 * D; ++k) {
-        // LDS reads of few products ahead, for the registers' sake
-        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int i = 0; i < NB; ++i) {
           O[i] = mul_tile(Q + i * 16 * PITCH + 16 * k, PITCH, S[k], O[i]);
@@ -386,15 +482,10 @@ void state_chunk_kernel(StateArgs<T> p) {
             R[i] = mul_tile(K + i * 16 * PITCH + 16 * k, PITCH, S[k], R[i]);
         }
       }
-    }
-    __syncthreads();
-    {
+      __syncthreads();
       lm_f32x4 U[NB];
-      T* yrow = p.y + (long)(t0 + at) * p.heads * p.VP + h * p.VP;
-      const int ld_y = p.heads * p.VP;
 #pragma unroll
       for (int i = 0; i < NB; ++i) {
-        U[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
         const int tr = 16 * i + 4 * g;
         const lm_f32x4 in = *reinterpret_cast<const lm_f32x4*>(d.in + tr);
         const lm_f32x4 step = *reinterpret_cast<const lm_f32x4*>(d.step + tr);
@@ -402,23 +493,20 @@ void state_chunk_kernel(StateArgs<T> p) {
 #pragma unroll
         for (int r = 0; r < 4; ++r)
           v[r] = tr + r < nt ? to_f32(vr[i][r]) : 0.f;
+        O[i] *= in;
         if (DELTA) {
           lm_f32x4 x = step * (v - in * R[i]);
           if (i == 1) x = mul_tile(sa + 16 * AP, AP, U[0], x);
           U[i] = mul_tile(sa + i * (16 * AP + 16), AP, x,
                           lm_f32x4{0.f, 0.f, 0.f, 0.f});
         } else {
+          O[i] += skip * v;
           U[i] = step * v;
         }
-        lm_f32x4 o = in * O[i];
-        if (!DELTA) o += skip * v;
-        if (i == 1) o = mul_tile(sM + 16 * AP, AP, U[0], o);
-        o = mul_tile(sM + i * (16 * AP + 16), AP, U[i], o);
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-          if (active && tr + r < nt)
-            yrow[(tr + r) * ld_y + col] = from_f32<T>(o[r]);
       }
+      O[0] = mul_tile(sM, AP, U[0], O[0]);
+      O[1] = mul_tile(sM + 16 * AP, AP, U[0], O[1]);
+      O[1] = mul_tile(sM + 16 * AP + 16, AP, U[1], O[1]);
       // the state behind the chunk
 #pragma unroll
       for (int i = 0; i < NB; ++i)
@@ -426,7 +514,6 @@ void state_chunk_kernel(StateArgs<T> p) {
       const float total = d.total;
 #pragma unroll
       for (int k = 0; k < 2 * D; ++k) {
-        __builtin_amdgcn_sched_barrier(0);
         S[k] *= total;
 #pragma unroll
         for (int i = 0; i < NB; ++i) {
@@ -437,18 +524,34 @@ void state_chunk_kernel(StateArgs<T> p) {
                 col_k[r * PITCH], U[i][r], S[k], 0, 0, 0);
         }
       }
+      T* yrow = p.y + (long)(t0 + at) * ld_y + h * p.VP;
+      if (active && nt == CH) {
+#pragma unroll
+        for (int i = 0; i < NB; ++i)
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            (yrow + (16 * i + r) * ld_y)[lane_y] = from_f32<T>(O[i][r]);
+      } else if (active) {
+#pragma unroll
+        for (int i = 0; i < NB; ++i)
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            if (16 * i + 4 * g + r < nt)
+              (yrow + (16 * i + r) * ld_y)[lane_y] = from_f32<T>(O[i][r]);
+      }
+      // the last chunk has no second one: nobody waits for what follows
+      if (at + CH < len) __syncthreads();
     }
-    if (at + CH < len) store(at + CH, buf ^ 1);
+    if (has_state && active) {
+#pragma unroll
+      for (int i = 0; i < 2 * D; ++i)
+        *reinterpret_cast<lm_f32x4*>(st + 16 * i) = S[i];
+    }
+    return;
   }
 
-  if (!has_state) return;
-  if (active) {
-#pragma unroll
-    for (int i = 0; i < 2 * D; ++i)
-      *reinterpret_cast<lm_f32x4*>(st + 16 * i) = S[i];
-  }
   // the convolution's inputs that later tokens look back at
-  if (slice > 0) return;
+  if (!has_state || slice > 0) return;
   const bool own_qk = h % (p.heads / p.groups) == 0;
   const int kv = KP / 8, vv = p.VP / 8, each = 2 * kv + vv;
   const int n = min(len, p.taps - 1);
@@ -689,7 +792,8 @@ __global__ __launch_bounds__(256) void state_pad_kernel(T* out, long ld_out,
 
 // z [T, cols] (row stride free): [q | k | v | gate | a | b], heads padded to
 // KP and VP channels; conv [taps, channels]; state [slots, heads, VP, KP]
-// float; ring [slots, taps, channels]; tiles [n, 5], seqs [m, 6] as in rglru;
+// float; ring [slots, taps, channels]; tiles [n, 5] of up to `tile` tokens, seqs
+// [m, 6] as in rglru;
 // the first n_single tokens are sequences of their own. out [T, heads * VP]
 void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
                      long dim, long vdim, long parts, double eps,
@@ -698,8 +802,8 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
                      c10::optional<torch::Tensor> skip, torch::Tensor norm,
                      torch::Tensor state, torch::Tensor ring,
                      torch::Tensor positions, torch::Tensor slots,
-                     torch::Tensor tiles, torch::Tensor seqs, long n_single,
-                     torch::Tensor out) {
+                     torch::Tensor tiles, torch::Tensor seqs, long tile,
+                     long n_single, torch::Tensor out) {
   LM_CHECK_I32(positions);
   LM_CHECK_I32(slots);
   LM_CHECK_I32(tiles);
@@ -745,10 +849,13 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
               positions.numel() >= n_single && slots.numel() >= n_single);
   TORCH_CHECK((m > 0) == (nt > 0) && (m > 0) == (T > n_single));
   TORCH_CHECK(m <= 65535 && n_single <= 65535);
+  TORCH_CHECK(tile == TILE, "lm_linear_state: tiles of ", TILE, " tokens");
   if (T == 0) return;
   const auto opt = z.options();
   auto u = torch::empty({m > 0 ? T - n_single + CH : 0, C}, opt);
   auto y = torch::empty({T, heads * VP}, opt);
+  auto decay = torch::empty({nt * heads * 2 * DECAY},
+                            state.options());
   hipStream_t st = cmls::current_stream();
 #define LM_ST_(D, CL, DELTA)                                                \
   hipLaunchKernelGGL((state_step_kernel<scalar_t, D, CL, DELTA>),           \
@@ -760,24 +867,24 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
     if (VP <= 64) LM_ST(D, 2);                                         \
     else LM_ST(D, 4);                                                       \
   } while (0)
+#define LM_SC_(TAPS, DELTA)                                                 \
+  hipLaunchKernelGGL((state_conv_kernel<scalar_t, TAPS, DELTA>), cg,        \
+                     dim3(256), 0, st, a, n_conv)
 #define LM_SC(TAPS)                                                         \
-  hipLaunchKernelGGL((state_conv_kernel<scalar_t, TAPS>), cg, dim3(256), 0, \
-                     st, a)
-#define LM_CK_(D, NW, DELTA)                                                \
+  do { if (delta) LM_SC_(TAPS, true); else LM_SC_(TAPS, false); } while (0)
+#define LM_CK_(D, DELTA)                                                    \
   do {                                                                      \
-    const int bytes = (4 * CH * (KP + 4) + (DELTA ? 2 : 1) * CH * (CH + 4)) \
-                          * 4 + 2 * (int)sizeof(ChunkDecay);                \
-    auto* fn = &state_chunk_kernel<scalar_t, D, NW, DELTA>;                 \
+    const int bytes = (4 * CH * (KP + 4) +                                  \
+                       (DELTA ? 4 : 2) * CH * (CH + 4) + 2 * DECAY) * 4;    \
+    auto* fn = &state_chunk_kernel<scalar_t, D, DELTA>;                     \
     HIP_CHECK(hipFuncSetAttribute(                                          \
         reinterpret_cast<const void*>(fn),                                  \
         hipFuncAttributeMaxDynamicSharedMemorySize, bytes));                \
     hipLaunchKernelGGL(fn, dim3(heads * ((VP + NW * 16 - 1) / (NW * 16)),   \
-                                m), dim3(NW * 64), bytes, st, a);           \
+                                m), dim3(2 * NTH), bytes, st, a);           \
   } while (0)
-#define LM_CK(D, NW)                                                        \
-  do { if (delta) LM_CK_(D, NW, true); else LM_CK_(D, NW, false); } while (0)
-#define LM_CK_D(D)                                                          \
-  do { if (VP <= 64) LM_CK(D, 4); else LM_CK(D, 8); } while (0)
+#define LM_CK(D)                                                            \
+  do { if (delta) LM_CK_(D, true); else LM_CK_(D, false); } while (0)
 #define LM_SN(VEC, DELTA)                                                   \
   hipLaunchKernelGGL((state_norm_kernel<scalar_t, VEC, DELTA>), grid,       \
                      dim3(256), 0, st, a, (int)first, L)
@@ -802,6 +909,7 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
     a.state = state.data_ptr<float>();
     a.ring = (scalar_t*)ring.data_ptr();
     a.u = (scalar_t*)u.data_ptr();
+    a.decay = decay.data_ptr<float>();
     a.y = (scalar_t*)y.data_ptr();
     a.out = (scalar_t*)out.data_ptr();
     a.ld_out = out.stride(0);
@@ -834,16 +942,17 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
       }
     }
     if (m > 0) {
-      const dim3 cg(nt, (C / 8 + 31) / 32);
+      const int n_conv = (int)(C / 8 + 31) / 32;
+      const dim3 cg(nt, n_conv + (heads + 3) / 4);
       if (taps <= 2) LM_SC(2);
       else if (taps <= 4) LM_SC(4);
       else LM_SC(MAX_TAPS);
       switch (KP) {
-        case 32: LM_CK_D(1); break;
-        case 64: LM_CK_D(2); break;
-        case 96: LM_CK_D(3); break;
-        case 128: LM_CK_D(4); break;
-        case 256: LM_CK_D(8); break;
+        case 32: LM_CK(1); break;
+        case 64: LM_CK(2); break;
+        case 96: LM_CK(3); break;
+        case 128: LM_CK(4); break;
+        case 256: LM_CK(8); break;
         default: TORCH_CHECK(false, "lm_linear_state: keys of ", KP);
       }
     }
@@ -874,7 +983,7 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
 #undef LM_ST
 #undef LM_ST_
 #undef LM_SC
-#undef LM_CK_D
+#undef LM_SC_
 #undef LM_CK
 #undef LM_CK_
 #undef LM_SN

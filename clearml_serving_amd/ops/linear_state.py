@@ -161,16 +161,17 @@ def _finish(o, gate, s: StateSpec, w: StateWeights):
 def linear_state(z: torch.Tensor, s: StateSpec, w: StateWeights,
                  state: torch.Tensor, ring: torch.Tensor,
                  positions: torch.Tensor, slots: torch.Tensor,
-                 tiles: torch.Tensor, seqs: torch.Tensor, n_single: int,
-                 out: torch.Tensor) -> None:
+                 tiles: torch.Tensor, seqs: torch.Tensor, tile: int,
+                 n_single: int, out: torch.Tensor) -> None:
     """z [T, cols] -> out [T, heads * vp]. The first n_single tokens are one
     token each of different sequences (``positions``, state ``slots``), the
-    others portions: tiles, seqs as in ops.lm.rglru_prefill."""
+    others portions: tiles of ``tile`` (64) tokens, seqs as in
+    ops.lm.rglru_prefill."""
     if z.is_cuda:
         require_lm_ext("linear_state").lm_linear_state(
             z, s.delta, s.heads, s.groups, s.dim, s.vdim, s.parts, s.eps,
             w.conv, w.conv_b, w.a_log, w.dt_bias, w.skip, w.norm, state,
-            ring, positions, slots, tiles, seqs, n_single, out)
+            ring, positions, slots, tiles, seqs, tile, n_single, out)
         return
     todo = [(i, 1, int(positions[i]), int(slots[i]))
             for i in range(n_single)]
