@@ -26,15 +26,22 @@ struct GroupedPrep {
   const T* first;    // [t, G * VD], null: no mixing
   long ld_first;
   float lam;
-  const T *qn, *kn;  // norm weights [KD], whole: [H * KD], [G * KD], or null
+  const T *qn, *kn;  // norm weights [KD], null: no norm; of a norm over all
+                     // heads [H * KD], [G * KD]
   const T *qb, *kb, *vb;  // biases, laid out as q, k and v, or null
   T* cache;
   long n_slots;
   int H, G, KD, VD, dim, row;
   float eps;
-  bool whole;        // one norm over all heads
   PageRows page;
 };
+
+// cache row of a slot: page * tokens of a page + offset
+template <typename T>
+__device__ __forceinline__ T* cache_row(const GroupedPrep<T>& a, long slot) {
+  return a.cache + (long)a.page.token((int)(slot / a.page.tokens),
+                                      (int)(slot % a.page.tokens)) * a.row;
+}
 
 template <typename T>
 __device__ __forceinline__ void load_biased(const T* p, const T* bias,
@@ -70,41 +77,6 @@ __global__ __launch_bounds__(256) void grouped_prep_kernel(
   const int per_tok = 256 / tokens_per_wg;  // threads
   const int tt = tid / per_tok, lid = tid % per_tok;
   const int t = t0 + tt;
-  float inv_q = 1.f, inv_k = 1.f;  // of a norm over all heads
-  if (a.whole) {
-    __shared__ float sums[4][2];
-    float sq = 0.f, sk = 0.f;
-    if (t < n_tok) {
-      for (int c = lid * 8; c < a.H * a.KD; c += per_tok * 8) {
-        float f[8];
-        load_biased(a.q + t * a.ld + c, a.qb ? a.qb + c : nullptr, f);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) sq += f[e] * f[e];
-      }
-      for (int c = lid * 8; c < a.G * a.KD; c += per_tok * 8) {
-        float f[8];
-        load_biased(a.k + t * a.ld + c, a.kb ? a.kb + c : nullptr, f);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) sk += f[e] * f[e];
-      }
-    }
-#pragma unroll
-    for (int d = 1; d < 64; d <<= 1) {
-      sq += __shfl_xor(sq, d, 64);
-      sk += __shfl_xor(sk, d, 64);
-    }
-    if (tokens_per_wg == 1) {  // else a token is a wave's
-      if ((tid & 63) == 0) {
-        sums[tid >> 6][0] = sq;
-        sums[tid >> 6][1] = sk;
-      }
-      __syncthreads();
-      sq = (sums[0][0] + sums[1][0]) + (sums[2][0] + sums[3][0]);
-      sk = (sums[0][1] + sums[1][1]) + (sums[2][1] + sums[3][1]);
-    }
-    inv_q = 1.f / sqrtf(sq / ((float)a.H * a.dim) + a.eps);
-    inv_k = 1.f / sqrtf(sk / ((float)a.G * a.dim) + a.eps);
-  }
   __syncthreads();
   if (t >= n_tok) return;
   const float* cs = trig + tt * 2 * pairs;
@@ -112,10 +84,7 @@ __global__ __launch_bounds__(256) void grouped_prep_kernel(
   const int c = lid % LPH * 8;
   const long slot = slots[t];
   const bool has_slot = slot >= 0 && slot < a.n_slots;
-  const int page = has_slot ? (int)(slot / a.page.tokens) : 0;
-  T* crow = a.cache +
-            (long)a.page.token(page, has_slot ? (int)(slot % a.page.tokens)
-                                              : 0) * a.row;
+  T* crow = cache_row(a, has_slot ? slot : 0);
   const int SL = same ? a.KD : a.KD + a.VD;
   const int units = a.H + a.G + (same ? 0 : a.G);
   // the LPH lanes of a unit stay together
@@ -146,10 +115,7 @@ __global__ __launch_bounds__(256) void grouped_prep_kernel(
     }
     float inv = 1.f;
     const T* w = is_q ? a.qn : a.kn;
-    if (a.whole) {
-      inv = is_q ? inv_q : inv_k;
-      w += (is_q ? u : u - a.H) * a.KD;
-    } else if (w) {
+    if (w) {
       float ss = 0.f;
 #pragma unroll
       for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
@@ -189,6 +155,102 @@ __global__ __launch_bounds__(256) void grouped_prep_kernel(
     }
     if (is_q) store8(a.q + t * a.ld + u * a.KD + c, f);
     else if (has_slot) store8(crow + (u - a.H) * SL + c, f);
+  }
+}
+
+// The same where one norm runs over all heads of the queries and one over
+// those of the keys: TPT threads hold a token's row [q | k | v], NV vectors
+// each, until its sums are there.
+template <typename T, int NV, int TPT>
+__global__ __launch_bounds__(256) void grouped_prep_whole_kernel(
+    GroupedPrep<T> a, const int* __restrict__ positions,
+    const int* __restrict__ slots, Rot rot, int n_tok) {
+  extern __shared__ float trig[];  // [tokens][2][pairs]
+  __shared__ float sums[4][2];
+  const int tid = threadIdx.x, pairs = rot.pairs;
+  const int tt = tid / TPT, lid = tid % TPT;
+  const int t = min((int)blockIdx.x * (256 / TPT) + tt, n_tok - 1);
+  const bool mine = (int)blockIdx.x * (256 / TPT) + tt < n_tok;
+  const int nq = a.H * a.KD, nk = a.G * a.KD, total = nq + nk + a.G * a.VD;
+  const T* row = a.q + t * a.ld;
+  float f[NV][8];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (lid + i * TPT) * 8;
+    if (c < total) load_biased(row + c, a.qb ? a.qb + c : nullptr, f[i]);
+  }
+  float* cs = trig + tt * 2 * pairs;
+  float* sn = cs + pairs;
+  const float pos = (float)positions[t];
+  for (int p = lid; p < pairs; p += TPT) {
+    float sv, cv;
+    sincosf(pos * rot.inv_freq[p], &sv, &cv);
+    cs[p] = rot.gain * cv;
+    sn[p] = rot.gain * sv;
+  }
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (lid + i * TPT) * 8;
+    if (c < nq + nk) {
+      float ss = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) ss += f[i][e] * f[i][e];
+      if (c < nq) sq += ss;
+      else sk += ss;
+    }
+  }
+#pragma unroll
+  for (int d = 1; d < 64; d <<= 1) {
+    sq += __shfl_xor(sq, d, 64);
+    sk += __shfl_xor(sk, d, 64);
+  }
+  if (TPT == 256 && (tid & 63) == 0) {
+    sums[tid >> 6][0] = sq;
+    sums[tid >> 6][1] = sk;
+  }
+  __syncthreads();
+  if (TPT == 256) {
+    sq = (sums[0][0] + sums[1][0]) + (sums[2][0] + sums[3][0]);
+    sk = (sums[0][1] + sums[1][1]) + (sums[2][1] + sums[3][1]);
+  }
+  if (!mine) return;
+  const float inv_q = 1.f / sqrtf(sq / ((float)a.H * a.dim) + a.eps);
+  const float inv_k = 1.f / sqrtf(sk / ((float)a.G * a.dim) + a.eps);
+  const long slot = slots[t];
+  const bool has_slot = slot >= 0 && slot < a.n_slots;
+  T* crow = cache_row(a, has_slot ? slot : 0);
+  const int SL = a.KD + a.VD;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = (lid + i * TPT) * 8;
+    if (c >= total) continue;
+    if (c >= nq + nk) {
+      const int v = c - nq - nk;
+      if (has_slot)
+        store8(crow + v / a.VD * SL + a.KD + v % a.VD, f[i]);
+      continue;
+    }
+    const bool is_q = c < nq;
+    const int u = is_q ? c : c - nq, d = u % a.KD;
+    const float inv = is_q ? inv_q : inv_k;
+    float w[8];
+    load8<T>((is_q ? a.qn : a.kn) + u, w);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) f[i][e] *= inv * w[e];
+    if (d < 2 * pairs) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int p = d / 2 + j;
+        if (p < pairs) {
+          const float x = f[i][2 * j], y = f[i][2 * j + 1];
+          f[i][2 * j] = x * cs[p] - y * sn[p];
+          f[i][2 * j + 1] = y * cs[p] + x * sn[p];
+        }
+      }
+    }
+    if (is_q) store8(a.q + t * a.ld + c, f[i]);
+    else if (has_slot) store8(crow + u / a.KD * SL + d, f[i]);
   }
 }
 
@@ -393,11 +455,11 @@ __global__ __launch_bounds__(256, 2) void grouped_attn_kernel(
 }
 
 // ------------------------------------------------------------------- //
-// means of whole blocks: a workgroup per token, which leaves unless the token
-// ends a block
+// means of whole blocks: a wave per token and 512 columns, which leaves unless
+// the token ends a block
 // ------------------------------------------------------------------- //
 template <typename T>
-__global__ __launch_bounds__(256) void grouped_pool_kernel(
+__global__ __launch_bounds__(64) void grouped_pool_kernel(
     T* cache, const int* __restrict__ block_table,
     const int* __restrict__ tok_seq, const int* __restrict__ positions,
     int row, int max_blocks, int n_blocks, int n_seqs, PageRows page) {
@@ -412,9 +474,10 @@ __global__ __launch_bounds__(256) void grouped_pool_kernel(
   const float inv = 1.f / (float)page.pool;
   T* dst = cache +
            (long)page.pooled(page_of(pos), pos % page.tokens) * row;
-  for (int c = threadIdx.x * 8; c < row; c += blockDim.x * 8) {
+  const int c = (blockIdx.y * 64 + threadIdx.x) * 8;
+  if (c < row) {
     float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
+#pragma unroll 8
     for (int p = pos + 1 - page.pool; p <= pos; ++p) {
       float f[8];
       load8<T>(cache + (long)page.token(page_of(p), p % page.tokens) * row + c,
@@ -480,6 +543,15 @@ void lm_grouped_prep(torch::Tensor z, long k_at, long v_at,
   while (lph * 8 < std::max(KD, same ? KD : VD)) lph *= 2;
   // few tokens: a workgroup for each, else a wave
   const int per_wg = T <= 1024 ? 1 : 4;
+  const long total = (H + G) * KD + G * VD;
+  TORCH_CHECK(!whole || (k_at == H * KD && v_at == k_at + G * KD &&
+                         total <= 256 * 16 * 8),
+              "lm_grouped_prep: norm over ", total, " columns");
+#define LM_GPW(NV, TPT)                                                     \
+  hipLaunchKernelGGL((grouped_prep_whole_kernel<scalar_t, NV, TPT>),        \
+                     dim3((T + 256 / TPT - 1) / (256 / TPT)), dim3(256), lds, \
+                     cmls::current_stream(), a, positions.data_ptr<int>(),  \
+                     slots.data_ptr<int>(), rot, (int)T)
   LM_DISPATCH(z, "lm_grouped_prep", [&] {
     GroupedPrep<scalar_t> a{};
     a.q = (scalar_t*)z.data_ptr();
@@ -498,7 +570,6 @@ void lm_grouped_prep(torch::Tensor z, long k_at, long v_at,
       a.kb = a.qb + k_at;
       a.vb = a.qb + v_at;
     }
-    a.whole = whole;
     a.page = page_rows(cache.size(1), pool);
     a.cache = (scalar_t*)cache.data_ptr();
     a.n_slots = (long)cache.size(0) * a.page.tokens;
@@ -509,12 +580,21 @@ void lm_grouped_prep(torch::Tensor z, long k_at, long v_at,
     a.dim = (int)dim;
     a.row = (int)row;
     a.eps = (float)eps;
+    if (whole) {
+      const size_t lds = std::max(1, 4 * 2 * rot.pairs) * 4;
+      // a wave per token where its vectors fit and there are enough tokens
+      if (total <= 64 * 8 * 8 && T > 1024) LM_GPW(8, 64);
+      else if (total <= 256 * 4 * 8) LM_GPW(4, 256);
+      else LM_GPW(16, 256);
+      return;
+    }
     hipLaunchKernelGGL((grouped_prep_kernel<scalar_t>),
                        dim3((T + per_wg - 1) / per_wg), dim3(256),
                        std::max(1, per_wg * 2 * rot.pairs) * 4,
                        cmls::current_stream(), a, positions.data_ptr<int>(),
                        slots.data_ptr<int>(), rot, (int)T, per_wg, lph);
   });
+#undef LM_GPW
   LM_LAUNCHED();
 }
 
@@ -533,8 +613,9 @@ void lm_grouped_pool(torch::Tensor cache, torch::Tensor block_table,
   TORCH_CHECK(block_table.numel() > 0);
   const PageRows page = page_rows(cache.size(1), pool);
   LM_DISPATCH(cache, "lm_grouped_pool", [&] {
-    hipLaunchKernelGGL((grouped_pool_kernel<scalar_t>), dim3(T),
-                       dim3(row <= 512 ? 64 : 256), 0, cmls::current_stream(),
+    hipLaunchKernelGGL((grouped_pool_kernel<scalar_t>),
+                       dim3(T, (row + 511) / 512), dim3(64), 0,
+                       cmls::current_stream(),
                        (scalar_t*)cache.data_ptr(),
                        block_table.data_ptr<int>(), tok_seq.data_ptr<int>(),
                        positions.data_ptr<int>(), (int)row,

@@ -183,11 +183,15 @@ __global__ __launch_bounds__(256) void state_conv_kernel(StateArgs<T> p,
       }
     }
     const int n = min(8, len - r0);
+    Raw8<T> raw[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      raw[i] = *reinterpret_cast<const Raw8<T>*>(
+          p.z + (long)(t0 + r0 + min(i, n - 1)) * p.ld + c);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      if (i >= n) break;
       float x[8], f[8];
-      load8<T>(p.z + (long)(t0 + r0 + i) * p.ld + c, x);
+      load8<T>(raw[i].v, x);
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         f[e] = bias[e] + w[0][e] * x[e];
@@ -198,7 +202,8 @@ __global__ __launch_bounds__(256) void state_conv_kernel(StateArgs<T> p,
         for (int d = TAPS - 1; d > 0; --d) past[d][e] = past[d - 1][e];
         past[0][e] = x[e];
       }
-      store8(p.u + (long)(t0 + r0 + i - p.n_single) * p.channels + c, f);
+      if (i < n)
+        store8(p.u + (long)(t0 + r0 + i - p.n_single) * p.channels + c, f);
     }
   }
 }
@@ -449,26 +454,32 @@ void state_chunk_kernel(StateArgs<T> p) {
     const int ld_y = p.heads * p.VP;
     const unsigned lane_v = 4 * g * p.channels + col;
     const unsigned lane_y = 4 * g * ld_y + col;
+    T vr[NB][4], vn[NB][4];  // values of this chunk and the next
+    auto load_values = [&](int at, T (&v)[NB][4]) {
+      const T* row = urow + (long)at * p.channels + p.v_at + h * p.VP;
+#pragma unroll
+      for (int i = 0; i < NB; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          v[i][r] = (row + (16 * i + r) * p.channels)[lane_v];
+    };
+    load_values(0, vn);
     __syncthreads();
     __syncthreads();
     int buf = 0;
     for (int at = 0; at < len; at += CH, buf ^= 1) {
       const int nt = min(CH, len - at);
+#pragma unroll
+      for (int i = 0; i < NB; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) vr[i][r] = vn[i][r];
+      if (at + CH < len) load_values(at + CH, vn);
       const float* K = sk + buf * 2 * CH * PITCH;
       const float* Q = K + CH * PITCH;
       const float* sM = sam + buf * AM;
       const float* sa = sM + CH * AP;
       const ChunkDecay& d =
           *reinterpret_cast<const ChunkDecay*>(sd + buf * DECAY);
-      T vr[NB][4];
-      {
-        const T* v = urow + (long)at * p.channels + p.v_at + h * p.VP;
-#pragma unroll
-        for (int i = 0; i < NB; ++i)
-#pragma unroll
-          for (int r = 0; r < 4; ++r)
-            vr[i][r] = (v + (16 * i + r) * p.channels)[lane_v];
-      }
       // products with the state in front of the chunk
       lm_f32x4 R[NB], O[NB];
 #pragma unroll
@@ -716,7 +727,9 @@ __global__ __launch_bounds__(256) void state_step_kernel(StateArgs<T> p) {
 // norm of the read-outs in parts, gated behind it (DELTA) or in front
 // ------------------------------------------------------------------- //
 // L threads take a part of a token. VEC 8: parts and heads are multiples of 8.
-template <typename T, int VEC, bool DELTA>
+// KEEP: vectors of a part that a thread keeps between its sum and its norm (0:
+// they are read again).
+template <typename T, int VEC, int KEEP, bool DELTA>
 __global__ __launch_bounds__(256) void state_norm_kernel(StateArgs<T> p,
                                                          int first, int L) {
   __shared__ float part[4];
@@ -740,7 +753,17 @@ __global__ __launch_bounds__(256) void state_norm_kernel(StateArgs<T> p,
     for (int e = 0; e < VEC; ++e) f[e] *= silu_f<T>(s[e]);
   };
   float ss = 0.f;
-  if (mine)
+  float kept[KEEP ? KEEP : 1][8];
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int c = (lid + i * L) * VEC;
+    if (mine && c < size) {
+      value(place(c0 + c), kept[i]);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) ss += kept[i][e] * kept[i][e];
+    }
+  }
+  if (KEEP == 0 && mine)
     for (int c = lid * VEC; c < size; c += L * VEC) {
       float f[8];
       value(place(c0 + c), f);
@@ -755,10 +778,8 @@ __global__ __launch_bounds__(256) void state_norm_kernel(StateArgs<T> p,
   }
   if (!mine) return;
   const float inv = 1.f / sqrtf(ss / (float)size + p.eps);
-  for (int c = lid * VEC; c < size; c += L * VEC) {
-    const int at = place(c0 + c);
-    float f[8], w[8];
-    value(at, f);
+  auto finish = [&](int at, float* f) {
+    float w[8];
     if (VEC == 8) load8<T>(p.norm + at, w);
     else w[0] = to_f32(p.norm[at]);
 #pragma unroll
@@ -772,7 +793,19 @@ __global__ __launch_bounds__(256) void state_norm_kernel(StateArgs<T> p,
     T* dst = p.out + t * p.ld_out + at;
     if (VEC == 8) store8(dst, f);
     else dst[0] = from_f32<T>(f[0]);
+  };
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int c = (lid + i * L) * VEC;
+    if (c < size) finish(place(c0 + c), kept[i]);
   }
+  if (KEEP == 0)
+    for (int c = lid * VEC; c < size; c += L * VEC) {
+      float f[8];
+      const int at = place(c0 + c);
+      value(at, f);
+      finish(at, f);
+    }
 }
 
 // zeros in the padding of heads whose size is no multiple of 32
@@ -885,9 +918,15 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
   } while (0)
 #define LM_CK(D)                                                            \
   do { if (delta) LM_CK_(D, true); else LM_CK_(D, false); } while (0)
-#define LM_SN(VEC, DELTA)                                                   \
-  hipLaunchKernelGGL((state_norm_kernel<scalar_t, VEC, DELTA>), grid,       \
+#define LM_SN(VEC, KEEP, DELTA)                                             \
+  hipLaunchKernelGGL((state_norm_kernel<scalar_t, VEC, KEEP, DELTA>), grid, \
                      dim3(256), 0, st, a, (int)first, L)
+#define LM_SN_K(VEC, DELTA)                                                 \
+  do {                                                                      \
+    if (n_vec <= L) LM_SN(VEC, 1, DELTA);                                   \
+    else if (keep) LM_SN(VEC, 4, DELTA);                                    \
+    else LM_SN(VEC, 0, DELTA);                                              \
+  } while (0)
   LM_DISPATCH(z, "lm_linear_state", [&] {
     const auto ptr = [](const torch::Tensor& w) {
       return (const scalar_t*)w.data_ptr();
@@ -968,15 +1007,18 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
                          (int)VP, (int)vdim, (int)(T - first));
     }
     if (first < T) {
+      // up to four vectors of a thread of a wave, else a workgroup per part
+      const long n_vec = (size + (vec ? 7 : 0)) / (vec ? 8 : 1);
       int L = 4;
-      while (L < 64 && L * (vec ? 8 : 1) < size) L *= 2;
-      if (L * (vec ? 8 : 1) < size) L = 256;
+      while (L < 64 && L < n_vec) L *= 2;
+      if (n_vec > 256) L = 256;
+      const bool keep = n_vec <= 4L * L;
       const long items = (T - first) * parts;
       const dim3 grid((items + 256 / L - 1) / (256 / L));
-      if (vec && delta) LM_SN(8, true);
-      else if (vec) LM_SN(8, false);
-      else if (delta) LM_SN(1, true);
-      else LM_SN(1, false);
+      if (vec && delta) LM_SN_K(8, true);
+      else if (vec) LM_SN_K(8, false);
+      else if (delta) LM_SN_K(1, true);
+      else LM_SN_K(1, false);
     }
   });
 #undef LM_ST_D
@@ -987,5 +1029,6 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
 #undef LM_CK
 #undef LM_CK_
 #undef LM_SN
+#undef LM_SN_K
   LM_LAUNCHED();
 }
