@@ -455,27 +455,30 @@ __global__ __launch_bounds__(256, 2) void grouped_attn_kernel(
 }
 
 // ------------------------------------------------------------------- //
-// means of whole blocks: a wave per token and 512 columns, which leaves unless
-// the token ends a block
+// means of whole blocks: a wave for 512 columns of the blocks that `per` tokens
+// may end
 // ------------------------------------------------------------------- //
 template <typename T>
 __global__ __launch_bounds__(64) void grouped_pool_kernel(
     T* cache, const int* __restrict__ block_table,
     const int* __restrict__ tok_seq, const int* __restrict__ positions,
-    int row, int max_blocks, int n_blocks, int n_seqs, PageRows page) {
-  const int t = blockIdx.x, pos = positions[t];
-  if (pos < 0 || (pos + 1) % page.pool || pos >= max_blocks * page.tokens)
-    return;
-  const int* btab =
-      block_table + (long)min(max(tok_seq[t], 0), n_seqs - 1) * max_blocks;
-  auto page_of = [&](int p) {
-    return min(max(btab[p / page.tokens], 0), n_blocks - 1);
-  };
-  const float inv = 1.f / (float)page.pool;
-  T* dst = cache +
-           (long)page.pooled(page_of(pos), pos % page.tokens) * row;
+    int row, int max_blocks, int n_blocks, int n_seqs, PageRows page, int per,
+    int n_tok) {
   const int c = (blockIdx.y * 64 + threadIdx.x) * 8;
-  if (c < row) {
+  const int end = min((int)(blockIdx.x + 1) * per, n_tok);
+  for (int t = blockIdx.x * per; t < end; ++t) {
+    const int pos = positions[t];
+    if (pos < 0 || (pos + 1) % page.pool || pos >= max_blocks * page.tokens ||
+        c >= row)
+      continue;
+    const int* btab =
+        block_table + (long)min(max(tok_seq[t], 0), n_seqs - 1) * max_blocks;
+    auto page_of = [&](int p) {
+      return min(max(btab[p / page.tokens], 0), n_blocks - 1);
+    };
+    const float inv = 1.f / (float)page.pool;
+    T* dst = cache +
+             (long)page.pooled(page_of(pos), pos % page.tokens) * row;
     float sum[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 #pragma unroll 8
     for (int p = pos + 1 - page.pool; p <= pos; ++p) {
@@ -612,15 +615,17 @@ void lm_grouped_pool(torch::Tensor cache, torch::Tensor block_table,
   if (T == 0) return;
   TORCH_CHECK(block_table.numel() > 0);
   const PageRows page = page_rows(cache.size(1), pool);
+  // decoded tokens may all end one; of a portion's tokens every pool-th does
+  const int per = T <= 1024 ? 1 : (int)std::min<long>(pool, 16);
   LM_DISPATCH(cache, "lm_grouped_pool", [&] {
     hipLaunchKernelGGL((grouped_pool_kernel<scalar_t>),
-                       dim3(T, (row + 511) / 512), dim3(64), 0,
-                       cmls::current_stream(),
+                       dim3((T + per - 1) / per, (row + 511) / 512), dim3(64),
+                       0, cmls::current_stream(),
                        (scalar_t*)cache.data_ptr(),
                        block_table.data_ptr<int>(), tok_seq.data_ptr<int>(),
                        positions.data_ptr<int>(), (int)row,
                        (int)block_table.size(1), (int)cache.size(0),
-                       (int)block_table.size(0), page);
+                       (int)block_table.size(0), page, per, (int)T);
   });
   LM_LAUNCHED();
 }

@@ -30,6 +30,12 @@
 // blocks of 1 + A are inverted, the rest is substituted block by block.
 // Exponents are sums of decays of like sign, never differences across a block.
 //
+// Few long portions would leave most CUs idle, so these are cut into segments.
+// A segment turns the state in front of it into P S + Q: the same kernel makes P
+// from the identity without values and Q from zero (without DELTA P is one
+// number), a chain over the segments gives the state in front of each
+// (state_chain_kernel), and the segments are walked from there.
+//
 // State in memory: [slot][head][value][key]; the convolution's past inputs as a
 // ring [slot][taps][channels] indexed by position, one entry more than it looks
 // back, so a token's own entry is never one that it reads. Neither is ever
@@ -64,7 +70,14 @@ struct StateArgs {
   int n_single, n_seq, n_state, n_tok, heads, groups, KP, VP, dim, vdim, taps,
       parts;
   float eps;
+  // portions are walked in segments of `seg` tiles, 0: whole
+  int seg, n_seg;   // n_seg: bound on all portions' segments
+  float *P, *Q;     // [n_seg, heads, KP, KP] and [n_seg, heads, VP, KP]
 };
+
+__device__ __forceinline__ int segments_of(const int* portion, int seg) {
+  return (portion[1] + seg - 1) / seg;
+}
 
 template <typename T>
 __device__ __forceinline__ float silu_f(float z) {
@@ -273,9 +286,10 @@ __device__ __forceinline__ lm_f32x4 decayed(lm_f32x4 c, const ChunkDecay& d,
 // D: 32-channel blocks of a key. Grid (heads * slices of 64 values,
 // sequences). Four waves keep the state, 16 values each; four more prepare the
 // next chunk meanwhile: they stage its rows while the first ones multiply this
-// chunk's with the state, and make its A and M while the others finish.
+// chunk's with the state, and make its A and M while the others finish. COMPOSE:
+// P and Q of a segment instead of outputs, values behind the columns of P.
 constexpr int NW = 4, NTH = NW * 64;
-template <typename T, int D, bool DELTA>
+template <typename T, int D, bool DELTA, bool COMPOSE>
 __global__ __launch_bounds__(2 * NTH, 2)
 void state_chunk_kernel(StateArgs<T> p) {
   constexpr int KP = D * 32, PITCH = KP + 4, AP = CH + 4;
@@ -294,14 +308,27 @@ void state_chunk_kernel(StateArgs<T> p) {
   const int r16 = lane & 15, g = lane >> 4;
   const int h = blockIdx.x % p.heads, slice = blockIdx.x / p.heads;
   // long sequences first: they are the last of the list
-  const int* sq = p.seqs + (p.n_seq - 1 - (int)blockIdx.y) * 6;
-  const int t0 = sq[2], len = sq[3], p0 = sq[4], slot = sq[5];
+  int seq = p.n_seq - 1 - (int)blockIdx.y, part = 0;
+  if (p.seg) {  // segment `part` of a portion
+    part = blockIdx.y;
+    seq = 0;
+    while (seq < p.n_seq && part >= segments_of(p.seqs + seq * 6, p.seg))
+      part -= segments_of(p.seqs + seq++ * 6, p.seg);
+    if (seq == p.n_seq) return;
+  }
+  const int* sq = p.seqs + seq * 6;
+  const bool ends = !p.seg || part + 1 == segments_of(sq, p.seg);
+  if (COMPOSE && ends) return;  // nothing follows
+  const int skipped = part * p.seg * TILE;
+  const int t0 = sq[2] + skipped, p0 = sq[4], slot = sq[5];
+  const int len = ends ? sq[3] - skipped : p.seg * TILE;
   const bool has_state = slot >= 0 && slot < p.n_state;
   const int hk = h / (p.heads / p.groups);
   const T* urow = p.u + (long)(t0 - p.n_single) * p.channels;
 
   if (!keeps) {
-    const float* drow = p.decay + ((long)sq[0] * p.heads + h) * 2 * DECAY;
+    const float* drow =
+        p.decay + ((long)(sq[0] + part * p.seg) * p.heads + h) * 2 * DECAY;
     Raw8<T> kq[NI];
     lm_f32x4 dreg = {0.f, 0.f, 0.f, 0.f};
     const int item_row = tid / LPR, item_c = tid % LPR * 8;
@@ -320,6 +347,7 @@ void state_chunk_kernel(StateArgs<T> p) {
               (is_q ? 0 : p.k_at));
         } else {
           const bool is_q = i * RPI >= CH;
+          if (COMPOSE && is_q) continue;
           kq[i] = *reinterpret_cast<const Raw8<T>*>(
               q + (is_q ? 0 : p.k_at) + (i * RPI % CH) * p.channels + item_at);
         }
@@ -333,6 +361,7 @@ void state_chunk_kernel(StateArgs<T> p) {
       const int nt = min(CH, len - at);
 #pragma unroll
       for (int i = 0; i < NI; ++i) {
+        if (COMPOSE && RPI <= CH && i * RPI >= CH) continue;  // no Q rows
         const int row = i * RPI + item_row;
         const bool live = row % CH < nt && item_in;
         float f = 1.f, x[8];
@@ -373,7 +402,7 @@ void state_chunk_kernel(StateArgs<T> p) {
               bi == bj && r16 > 4 * g + r ? 0.f : m[r];
       };
       if (!DELTA) {
-        if (wave < 3) {
+        if (!COMPOSE && wave < 3) {
           const int bi = wave > 0, bj = wave == 1;
           put_m(dot_rows(Q + bi * 16 * PITCH, K + bj * 16 * PITCH, PITCH, KP),
                 bi, bj);
@@ -404,13 +433,12 @@ void state_chunk_kernel(StateArgs<T> p) {
         }
       } else if (wave == 2) {
         lm_f32x4 kk = dot_rows(K + 16 * PITCH, K, PITCH, KP);
-        const lm_f32x4 qk = dot_rows(Q + 16 * PITCH, K, PITCH, KP);
         kk = decayed(kk, d, 1, 0);
 #pragma unroll
         for (int r = 0; r < 4; ++r)
           sa[(16 + 4 * g + r) * AP + r16] = kk[r] * -d.step[16 + 4 * g + r];
-        put_m(qk, 1, 0);
-      } else {
+        if (!COMPOSE) put_m(dot_rows(Q + 16 * PITCH, K, PITCH, KP), 1, 0);
+      } else if (!COMPOSE) {
         const lm_f32x4 m0 = dot_rows(Q, K, PITCH, KP);
         const lm_f32x4 m1 =
             dot_rows(Q + 16 * PITCH, K + 16 * PITCH, PITCH, KP);
@@ -435,24 +463,38 @@ void state_chunk_kernel(StateArgs<T> p) {
     }
     __syncthreads();  // the last chunk's, where nothing is next
   } else {
-    const int v0 = (slice * NW + wave) * 16;  // the wave's values
-    const bool active = v0 < p.VP;  // else all that it makes is left unused
+    // the wave's columns: values, in COMPOSE behind those of P
+    const int c0 = (slice * NW + wave) * 16;
+    const bool of_p = COMPOSE && DELTA && c0 < KP;
+    const int v0 = COMPOSE && DELTA && !of_p ? c0 - KP : c0;
+    const bool active = of_p || v0 < p.VP;  // else nobody uses what it makes
     const int col = active ? v0 + r16 : 0;
-    float* st = p.state +
-                (((long)(has_state ? slot : 0) * p.heads + h) * p.VP + col) *
-                    KP + 4 * g;
+    const long unit = (long)blockIdx.y * p.heads + h;
+    float* st = p.state + ((long)(has_state ? slot : 0) * p.heads + h) *
+                              p.VP * KP;
+    const float* from = p.seg ? p.Q + unit * p.VP * KP : st;
+    float* to = of_p ? p.P + unit * KP * KP
+                     : COMPOSE ? p.Q + unit * p.VP * KP : st;
+    from += col * KP + 4 * g;
+    to += col * KP + 4 * g;
     lm_f32x4 S[2 * D];  // S[i][r]: key 16 i + 4 g + r, value r16
-    if (p0 > 0 && has_state) {
+    if (COMPOSE) {
 #pragma unroll
       for (int i = 0; i < 2 * D; ++i)
-        S[i] = *reinterpret_cast<const lm_f32x4*>(st + 16 * i);
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          S[i][r] = of_p && 16 * i + 4 * g + r == col ? 1.f : 0.f;
+    } else if (p.seg || (p0 > 0 && has_state)) {
+#pragma unroll
+      for (int i = 0; i < 2 * D; ++i)
+        S[i] = *reinterpret_cast<const lm_f32x4*>(from + 16 * i);
     } else {
 #pragma unroll
       for (int i = 0; i < 2 * D; ++i) S[i] = lm_f32x4{0.f, 0.f, 0.f, 0.f};
     }
     const float skip = DELTA ? 0.f : to_f32(p.skip[h]);
     const int ld_y = p.heads * p.VP;
-    const unsigned lane_v = 4 * g * p.channels + col;
+    const unsigned lane_v = 4 * g * p.channels + (of_p ? 0 : col);
     const unsigned lane_y = 4 * g * ld_y + col;
     T vr[NB][4], vn[NB][4];  // values of this chunk and the next
     auto load_values = [&](int at, T (&v)[NB][4]) {
@@ -488,7 +530,8 @@ void state_chunk_kernel(StateArgs<T> p) {
       for (int k = 0; k < 2 * D; ++k) {
 #pragma unroll
         for (int i = 0; i < NB; ++i) {
-          O[i] = mul_tile(Q + i * 16 * PITCH + 16 * k, PITCH, S[k], O[i]);
+          if (!COMPOSE)
+            O[i] = mul_tile(Q + i * 16 * PITCH + 16 * k, PITCH, S[k], O[i]);
           if (DELTA)
             R[i] = mul_tile(K + i * 16 * PITCH + 16 * k, PITCH, S[k], R[i]);
         }
@@ -503,7 +546,7 @@ void state_chunk_kernel(StateArgs<T> p) {
         lm_f32x4 v;
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          v[r] = tr + r < nt ? to_f32(vr[i][r]) : 0.f;
+          v[r] = !of_p && tr + r < nt ? to_f32(vr[i][r]) : 0.f;
         O[i] *= in;
         if (DELTA) {
           lm_f32x4 x = step * (v - in * R[i]);
@@ -515,9 +558,11 @@ void state_chunk_kernel(StateArgs<T> p) {
           U[i] = step * v;
         }
       }
-      O[0] = mul_tile(sM, AP, U[0], O[0]);
-      O[1] = mul_tile(sM + 16 * AP, AP, U[0], O[1]);
-      O[1] = mul_tile(sM + 16 * AP + 16, AP, U[1], O[1]);
+      if (!COMPOSE) {
+        O[0] = mul_tile(sM, AP, U[0], O[0]);
+        O[1] = mul_tile(sM + 16 * AP, AP, U[0], O[1]);
+        O[1] = mul_tile(sM + 16 * AP + 16, AP, U[1], O[1]);
+      }
       // the state behind the chunk
 #pragma unroll
       for (int i = 0; i < NB; ++i)
@@ -536,7 +581,8 @@ void state_chunk_kernel(StateArgs<T> p) {
         }
       }
       T* yrow = p.y + (long)(t0 + at) * ld_y + h * p.VP;
-      if (active && nt == CH) {
+      if (COMPOSE) {
+      } else if (active && nt == CH) {
 #pragma unroll
         for (int i = 0; i < NB; ++i)
 #pragma unroll
@@ -553,27 +599,97 @@ void state_chunk_kernel(StateArgs<T> p) {
       // the last chunk has no second one: nobody waits for what follows
       if (at + CH < len) __syncthreads();
     }
-    if (has_state && active) {
+    if (active && (COMPOSE || (has_state && ends))) {
 #pragma unroll
       for (int i = 0; i < 2 * D; ++i)
-        *reinterpret_cast<lm_f32x4*>(st + 16 * i) = S[i];
+        *reinterpret_cast<lm_f32x4*>(to + 16 * i) = S[i];
     }
     return;
   }
 
   // the convolution's inputs that later tokens look back at
-  if (!has_state || slice > 0) return;
+  if (COMPOSE || !has_state || !ends || slice > 0) return;
   const bool own_qk = h % (p.heads / p.groups) == 0;
   const int kv = KP / 8, vv = p.VP / 8, each = 2 * kv + vv;
-  const int n = min(len, p.taps - 1);
+  const int n = min(sq[3], p.taps - 1);
   for (int i = tid; i < n * each; i += NTH) {
-    const int tt = len - 1 - i / each, j = i % each;
+    const int tt = sq[3] - 1 - i / each, j = i % each;
     if (j < 2 * kv && !own_qk) continue;
     const int c = j < kv ? hk * KP + j * 8
                 : j < 2 * kv ? p.k_at + hk * KP + (j - kv) * 8
                              : p.v_at + h * p.VP + (j - 2 * kv) * 8;
     copy8(p.ring + ((long)slot * p.taps + (p0 + tt) % p.taps) * p.channels + c,
-          p.z + (long)(t0 + tt) * p.ld + c);
+          p.z + (long)(sq[2] + tt) * p.ld + c);
+  }
+}
+
+// The state in front of every segment of a portion, in Q's place: a workgroup
+// per head, portion and 16 values.
+constexpr int CHAIN_COLS = 16;
+template <int D, bool DELTA>
+__global__ __launch_bounds__(256) void state_chain_kernel(
+    const int* __restrict__ seqs, const float* __restrict__ state,
+    const float* __restrict__ decay, int n_state, int heads, int VP, int seg,
+    const float* __restrict__ P, float* __restrict__ Q) {
+  constexpr int KP = D * 32, C4 = KP / 4;
+  constexpr int N = CHAIN_COLS * C4, PER = (N + 255) / 256;
+  __shared__ __align__(16) float s[CHAIN_COLS][KP];
+  const int h = blockIdx.x, v0 = blockIdx.z * CHAIN_COLS;
+  const int* sq = seqs + blockIdx.y * 6;
+  const int n = segments_of(sq, seg), p0 = sq[4], slot = sq[5];
+  int first = 0;  // segments of the portions in front
+  for (int b = 0; b < (int)blockIdx.y; ++b)
+    first += segments_of(seqs + b * 6, seg);
+  const bool has = p0 > 0 && slot >= 0 && slot < n_state;
+  const float* st =
+      state + (((long)(has ? slot : 0) * heads + h) * VP + v0) * KP;
+  for (int i = threadIdx.x; i < N; i += 256)
+    *reinterpret_cast<lm_f32x4*>(&s[i / C4][i % C4 * 4]) =
+        has ? *reinterpret_cast<const lm_f32x4*>(st + i * 4)
+            : lm_f32x4{0.f, 0.f, 0.f, 0.f};
+  __syncthreads();
+  for (int k = 0; k < n; ++k) {
+    const long unit = (long)(first + k) * heads + h;
+    float* qc = Q + (unit * VP + v0) * KP;
+    const bool more = k + 1 < n;  // else Q and P were not made
+    float total = 1.f;
+    if (!DELTA && more) {
+      const ChunkDecay* d = (const ChunkDecay*)decay +
+                            ((long)(sq[0] + k * seg) * heads + h) * 2;
+      for (int c = 0; c < 2 * seg; ++c)
+        total *= d[(long)(c / 2) * heads * 2 + c % 2].total;
+    }
+    lm_f32x4 acc[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int at = threadIdx.x + i * 256;
+      if (at >= N) continue;
+      const int row = at / C4, c = at % C4 * 4;
+      lm_f32x4* q = reinterpret_cast<lm_f32x4*>(qc + at * 4);
+      if (more) {
+        lm_f32x4 a = *q;
+        if (DELTA) {
+          const float* pc = P + unit * KP * KP + c;
+#pragma unroll 16
+          for (int j = 0; j < KP; ++j)
+            a += s[row][j] *
+                 *reinterpret_cast<const lm_f32x4*>(pc + j * KP);
+        } else {
+          a += total * *reinterpret_cast<const lm_f32x4*>(&s[row][c]);
+        }
+        acc[i] = a;
+      }
+      *q = *reinterpret_cast<const lm_f32x4*>(&s[row][c]);
+    }
+    if (!more) break;
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int at = threadIdx.x + i * 256;
+      if (at < N)
+        *reinterpret_cast<lm_f32x4*>(&s[at / C4][at % C4 * 4]) = acc[i];
+    }
+    __syncthreads();
   }
 }
 
@@ -826,7 +942,7 @@ __global__ __launch_bounds__(256) void state_pad_kernel(T* out, long ld_out,
 // z [T, cols] (row stride free): [q | k | v | gate | a | b], heads padded to
 // KP and VP channels; conv [taps, channels]; state [slots, heads, VP, KP]
 // float; ring [slots, taps, channels]; tiles [n, 5] of up to `tile` tokens, seqs
-// [m, 6] as in rglru;
+// [m, 6] as in rglru; portions are walked in segments of `seg` tiles (0: whole);
 // the first n_single tokens are sequences of their own. out [T, heads * VP]
 void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
                      long dim, long vdim, long parts, double eps,
@@ -836,7 +952,7 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
                      torch::Tensor state, torch::Tensor ring,
                      torch::Tensor positions, torch::Tensor slots,
                      torch::Tensor tiles, torch::Tensor seqs, long tile,
-                     long n_single, torch::Tensor out) {
+                     long seg, long n_single, torch::Tensor out) {
   LM_CHECK_I32(positions);
   LM_CHECK_I32(slots);
   LM_CHECK_I32(tiles);
@@ -883,12 +999,20 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
   TORCH_CHECK((m > 0) == (nt > 0) && (m > 0) == (T > n_single));
   TORCH_CHECK(m <= 65535 && n_single <= 65535);
   TORCH_CHECK(tile == TILE, "lm_linear_state: tiles of ", TILE, " tokens");
+  TORCH_CHECK(seg >= 0 && nt >= m);
+  // every portion's last segment may be short
+  const long n_seg = seg && m ? (nt - m) / seg + m : 0;
+  TORCH_CHECK(n_seg <= 65535);
   if (T == 0) return;
   const auto opt = z.options();
   auto u = torch::empty({m > 0 ? T - n_single + CH : 0, C}, opt);
   auto y = torch::empty({T, heads * VP}, opt);
-  auto decay = torch::empty({nt * heads * 2 * DECAY},
-                            state.options());
+  auto decay = torch::empty({nt * heads * 2 * DECAY}, state.options());
+  torch::Tensor P, Q;
+  if (n_seg) {
+    if (delta) P = torch::empty({n_seg, heads, KP, KP}, state.options());
+    Q = torch::empty({n_seg, heads, VP, KP}, state.options());
+  }
   hipStream_t st = cmls::current_stream();
 #define LM_ST_(D, CL, DELTA)                                                \
   hipLaunchKernelGGL((state_step_kernel<scalar_t, D, CL, DELTA>),           \
@@ -905,16 +1029,27 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
                      dim3(256), 0, st, a, n_conv)
 #define LM_SC(TAPS)                                                         \
   do { if (delta) LM_SC_(TAPS, true); else LM_SC_(TAPS, false); } while (0)
-#define LM_CK_(D, DELTA)                                                    \
+#define LM_CK__(D, DELTA, COMPOSE, COLS, ROWS)                              \
   do {                                                                      \
     const int bytes = (4 * CH * (KP + 4) +                                  \
                        (DELTA ? 4 : 2) * CH * (CH + 4) + 2 * DECAY) * 4;    \
-    auto* fn = &state_chunk_kernel<scalar_t, D, DELTA>;                     \
+    auto* fn = &state_chunk_kernel<scalar_t, D, DELTA, COMPOSE>;            \
     HIP_CHECK(hipFuncSetAttribute(                                          \
         reinterpret_cast<const void*>(fn),                                  \
         hipFuncAttributeMaxDynamicSharedMemorySize, bytes));                \
-    hipLaunchKernelGGL(fn, dim3(heads * ((VP + NW * 16 - 1) / (NW * 16)),   \
-                                m), dim3(2 * NTH), bytes, st, a);           \
+    hipLaunchKernelGGL(fn, dim3(heads * ((COLS + NW * 16 - 1) / (NW * 16)), \
+                                ROWS), dim3(2 * NTH), bytes, st, a);        \
+  } while (0)
+#define LM_CK_(D, DELTA)                                                    \
+  do {                                                                      \
+    if (seg) {                                                              \
+      LM_CK__(D, DELTA, true, (DELTA ? KP : 0) + VP, n_seg);                \
+      hipLaunchKernelGGL((state_chain_kernel<D, DELTA>),                    \
+                         dim3(heads, m, VP / CHAIN_COLS), dim3(256), 0, st, \
+                         a.seqs, a.state, a.decay, a.n_state, a.heads,      \
+                         (int)VP, (int)seg, a.P, a.Q);                      \
+    }                                                                       \
+    LM_CK__(D, DELTA, false, VP, seg ? n_seg : m);                          \
   } while (0)
 #define LM_CK(D)                                                            \
   do { if (delta) LM_CK_(D, true); else LM_CK_(D, false); } while (0)
@@ -969,6 +1104,12 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
     a.taps = (int)taps;
     a.parts = (int)parts;
     a.eps = (float)eps;
+    a.seg = n_seg ? (int)seg : 0;
+    a.n_seg = (int)n_seg;
+    if (n_seg) {
+      a.P = delta ? P.data_ptr<float>() : nullptr;
+      a.Q = Q.data_ptr<float>();
+    }
 
     if (n_single > 0) {
       switch (KP) {
@@ -1028,6 +1169,7 @@ void lm_linear_state(torch::Tensor z, bool delta, long heads, long groups,
 #undef LM_SC_
 #undef LM_CK
 #undef LM_CK_
+#undef LM_CK__
 #undef LM_SN
 #undef LM_SN_K
   LM_LAUNCHED();

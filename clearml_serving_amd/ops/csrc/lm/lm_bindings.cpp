@@ -57,7 +57,7 @@ void lm_linear_state(Tensor z, bool delta, long heads, long groups, long dim,
                      Opt conv_b, Tensor a_log, Tensor dt_bias, Opt skip,
                      Tensor norm, Tensor state, Tensor ring, Tensor positions,
                      Tensor slots, Tensor tiles, Tensor seqs, long tile,
-                     long n_single, Tensor out);
+                     long seg, long n_single, Tensor out);
 void lm_delta_rule(Tensor z, std::vector<long> at, Tensor w2, Tensor w0,
                    Tensor ab, Tensor norm, Tensor state, Tensor positions,
                    Tensor slots, Tensor seqs, Tensor out, long n_single,

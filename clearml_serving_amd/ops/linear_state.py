@@ -89,6 +89,17 @@ class StateSpec(NamedTuple):
                 (self.taps, self.channels))
 
 
+def segment_tiles(tiles: int, seqs: int, s: StateSpec) -> int:
+    """how many tiles make a segment of a portion, 0: portions stay whole.
+    Segments are walked twice, so cutting pays where whole portions leave CUs
+    idle."""
+    units = seqs * s.heads * -(-s.vp // 64)  # workgroups without segments
+    if units == 0 or units > 160 or tiles < 8 * seqs:
+        return 0
+    parts = max(2, min(tiles // (4 * seqs), 256 // units))
+    return -(-tiles // (seqs * parts))
+
+
 class StateWeights(NamedTuple):
     """conv [taps, channels] and its bias, a_log, dt_bias, skip [heads], norm
     [heads * vp]; skip without ``delta`` only"""
@@ -171,7 +182,8 @@ def linear_state(z: torch.Tensor, s: StateSpec, w: StateWeights,
         require_lm_ext("linear_state").lm_linear_state(
             z, s.delta, s.heads, s.groups, s.dim, s.vdim, s.parts, s.eps,
             w.conv, w.conv_b, w.a_log, w.dt_bias, w.skip, w.norm, state,
-            ring, positions, slots, tiles, seqs, tile, n_single, out)
+            ring, positions, slots, tiles, seqs, tile,
+            segment_tiles(tiles.shape[0], seqs.shape[0], s), n_single, out)
         return
     todo = [(i, 1, int(positions[i]), int(slots[i]))
             for i in range(n_single)]

@@ -28,7 +28,7 @@ from clearml_serving_amd.models.mixers import (DenseMlp,  # noqa: E402
                                                GroupedAttentionMixer,
                                                ParallelMixer, RecurrentMixer,
                                                StateSpace)
-from clearml_serving_amd.ops import grouped, lm  # noqa: E402
+from clearml_serving_amd.ops import grouped, linear_state, lm  # noqa: E402
 
 REPO = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 
@@ -472,6 +472,46 @@ def test_state_space(device, dtype, tol, size):
         got = run_mixer(mod, h, portions_of(n, portions), device, dtype,
                         forward=with_output)
         assert rel(got, want) < tol, portions[:3]
+
+
+@ALL
+@pytest.mark.parametrize("kind,size,seg", [
+    ("delta", 0, 1), ("delta", 2, 2), ("delta", 4, 1), ("delta", 5, 3),
+    ("delta", 6, 1), ("space", 0, 1), ("space", 2, 2), ("space", 5, 3),
+    ("space", 7, 1)])
+def test_recurrences_in_segments(device, dtype, tol, kind, size, seg,
+                                 monkeypatch):
+    """long portions are cut, and walked from the states in front of the
+    segments; portions end inside, at and right behind a segment's end"""
+    monkeypatch.setattr(linear_state, "segment_tiles", lambda *a: seg)
+    n, width = 600, 36
+    if kind == "delta":
+        m, make, ref = cases.delta(**DELTAS[size]), delta_of, plain.delta_rule
+        st = random_state(cases.delta_shapes(m, width), size)
+    else:
+        m, make, ref = cases.right(**SPACES[size]), space_of, \
+            plain.state_space
+        st = random_state(cases.state_shapes(m, width), size)
+    st["A_log"] -= 2.0  # what the first segment leaves lasts
+    h = inputs(n, width, size)
+    want = ref(h.double(), double(st), m, EPS)
+    mod = make(m, width, st)
+    for portions in ([n], [128, 2, 192, 65, 1, 212], [5, 64, 531]):
+        assert rel(run_mixer(mod, h, portions, device, dtype,
+                             forward=with_output), want) < tol
+
+
+def test_which_portions_are_cut():
+    def cut(tiles, seqs, heads, vdim):
+        return linear_state.segment_tiles(tiles, seqs, linear_state.StateSpec(
+            True, heads, heads, 64, vdim, 4, heads, EPS))
+
+    assert cut(0, 0, 4, 64) == 0  # none
+    assert cut(4, 1, 4, 64) == 0  # short
+    assert cut(4000, 16, 16, 64) == 0  # enough of them
+    for tiles, seqs, heads, vdim in ((128, 1, 16, 128), (128, 4, 16, 64),
+                                     (2000, 1, 1, 256)):
+        assert 2 <= cut(tiles, seqs, heads, vdim) < tiles / seqs
 
 
 @pytest.mark.parametrize("device,dtype,tol", [CPU, GPU32])
