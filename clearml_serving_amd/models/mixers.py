@@ -516,10 +516,9 @@ class DeltaRule(nn.Module):
     def state_layout(self) -> tuple:
         return "state", (self.heads, self.dp, self.dp)
 
-    def scan(self, z, batch, cache, out) -> None:
+    def scan(self, z, batch, state, out) -> None:
         """z [T, cols]: the product of h; out [T, out_cols]"""
         n = self.heads * self.dp
-        state, = cache
         delta.delta_rule(z, tuple(i * n for i in range(6)), self._w, state,
                          batch.positions, batch.state_slots, batch.seqs, out,
                          batch.n_single, self.dim, self.eps, self.out_scale,
@@ -586,9 +585,8 @@ class LinearState(nn.Module):
     def state_layout(self) -> tuple:
         return self.spec.layout()
 
-    def scan(self, z, batch, cache, out) -> None:
+    def scan(self, z, batch, state, ring, out) -> None:
         """z [T, cols]: the product of h; out [T, out_cols]"""
-        state, ring = cache
         linear_state.linear_state(
             z, self.spec, self._w, state, ring, batch.positions,
             batch.state_slots, batch.tiles, batch.seqs, batch.tile,
@@ -713,7 +711,7 @@ class RecurrentMixer(nn.Module):
 
     def context(self, h, batch, cache, out) -> None:
         """what the output product reads, into out [T, out_cols]"""
-        self.rec.scan(linear(h, self.inp), batch, cache, out)
+        self.rec.scan(linear(h, self.inp), batch, *cache, out)
 
 
 class ParallelMixer(nn.Module):
@@ -791,7 +789,7 @@ class ParallelMixer(nn.Module):
         pages, state = cache
         z = linear(h, self.inp)
         self.left.attend(z[:, :self.left.cols], batch, pages, left)
-        self.right.scan(z[:, self.left.cols:], batch, state, right)
+        self.right.scan(z[:, self.left.cols:], batch, *state, right)
 
     def forward(self, h, batch, cache, carry):
         n = self.left.out_cols
