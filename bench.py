@@ -122,10 +122,11 @@ def main():
     ap.add_argument("--workload", default="serving",
                     choices=("serving", "lm"),
                     help="serving: the headline benchmark; lm: prefill and "
-                         "decode of Pamazen, Kakipel and Bimipel beside "
-                         "llama")
+                         "decode of Nelovik, Pamazen, Kakipel and Bimipel "
+                         "beside llama")
     ap.add_argument("--lm-size", default="300m,1b,4k")
-    ap.add_argument("--lm-model", default="nelovik,pamazen,kakipel,bimipel,llama")
+    ap.add_argument("--lm-model",
+                    default="nelovik,pamazen,kakipel,bimipel,llama")
     ap.add_argument("--lm-prompt", type=int, default=2048)
     ap.add_argument("--lm-batch", default="1,16,64")
     ap.add_argument("--lm-phase", default="prefill,decode")

@@ -91,10 +91,10 @@ class StateSpec(NamedTuple):
 
 def segment_tiles(tiles: int, seqs: int, s: StateSpec) -> int:
     """how many tiles make a segment of a portion, 0: portions stay whole.
-    Segments are walked twice, so cutting pays where whole portions leave CUs
-    idle."""
+    Segments are walked twice (three times with P), so cutting pays where
+    whole portions leave CUs idle."""
     units = seqs * s.heads * -(-s.vp // 64)  # workgroups without segments
-    if units == 0 or units > 160 or tiles < 8 * seqs:
+    if units == 0 or units > (96 if s.delta else 160) or tiles < 8 * seqs:
         return 0
     parts = max(2, min(tiles // (4 * seqs), 256 // units))
     return -(-tiles // (seqs * parts))
