@@ -204,7 +204,10 @@ def _as_numpy(v) -> Optional[np.ndarray]:
                 # keep float64 when the downcast would overflow finite
                 # values to inf (serving inputs are float32-scale, but a
                 # silent inf would corrupt the request)
-                if np.all(np.isfinite(a32) | ~np.isfinite(a)):
+                # ... or underflow: below the normal range digits are lost
+                if np.all((np.isfinite(a32) | ~np.isfinite(a))
+                          & ((np.abs(a) >= np.finfo(np.float32).tiny)
+                             | (a == 0) | np.isnan(a))):
                     a = a32
             return a if a.dtype in _DTYPE_CODES else None
         except Exception:
