@@ -631,8 +631,8 @@ class GatedDelta(LinearState):
 
 class StateSpace(LinearState):
     """State-space recurrence: ``heads`` states of ``state`` x vdim whose
-    inputs and read-outs ``groups`` of heads share; gate before the norm,
-    which runs in ``parts`` equal parts."""
+    inputs and read-outs ``groups`` of heads share; what the norm sees is
+    gated already, and cut into ``parts``."""
 
     def __init__(self, width: int, heads: int, vdim: int, state: int,
                  groups: int, taps: int, parts: int, eps: float):

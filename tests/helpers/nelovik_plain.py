@@ -106,7 +106,7 @@ def window_attention(h, w, m, eps):
 
 # ---- recurrences ----------------------------------------------------- #
 def causal_conv(x, taps, bias=None):
-    """x [t, c], taps [c, n]: the last column weighs the current token"""
+    """x [t, c], taps [c, n]: taps[:, n - 1 - d] goes with x[t - d]"""
     n = taps.shape[1]
     out = torch.zeros_like(x)
     for d in range(min(n, x.shape[0])):  # d tokens back

@@ -324,9 +324,9 @@ def test_edges_of_windows_and_blocks(device, dtype, tol, absorb_max, size,
             needle(st, h, m, key, query)
             want = plain.window_attention(h.double(), double(st), m, EPS)
             mod = attention_of(m, width, st)
-            for portions in ([n], [query - 3] + [1] * (n - query + 3),
-                             [query] + [n - query],
-                             portions_of(n, [67, 2])):
+            cuts = ([n], [query - 3] + [1] * (n - query + 3),
+                    [query] + [n - query], portions_of(n, [67, 2]))
+            for portions in cuts[:2] if device == "cpu" else cuts:
                 got = run_mixer(mod, h, portions, device, dtype, block_size,
                                 absorb_max)
                 assert rel(got[query], want[query]) < tol
@@ -474,7 +474,7 @@ def test_state_space(device, dtype, tol, size):
         assert rel(got, want) < tol, portions[:3]
 
 
-@ALL
+@pytest.mark.parametrize("device,dtype,tol", [GPU32, GPU16])
 @pytest.mark.parametrize("kind,size,seg", [
     ("delta", 0, 1), ("delta", 2, 2), ("delta", 4, 1), ("delta", 5, 3),
     ("delta", 6, 1), ("space", 0, 1), ("space", 2, 2), ("space", 5, 3),
@@ -540,8 +540,8 @@ def test_delta_rule_extremes(device, dtype, tol, kind):
 
 
 def test_recurrence_oracles_tell_faults_apart():
-    """the decay comes first, the read-out sees the write; a lost state and a
-    lost convolution input show"""
+    """decay, then removal and write, then read-out: another order shows, and
+    so does a lost state or convolution input"""
     g = torch.Generator().manual_seed(0)
     q, k, v = (torch.randn(40, 8, generator=g).double() for _ in range(3))
     k = plain.unit(k)

@@ -151,3 +151,12 @@ def test_request_framing_roundtrip_fuzz(url, req_id, data):
                     _np.asarray(data[k], dtype=_np.float64))
         else:
             assert out == data or (out is None and data is None)
+
+
+@pytest.mark.parametrize("values,dtype", [
+    ([0.5, 0.0, -3.0], "float32"), ([1e300], "float64"),
+    ([6e-231], "float64"), ([1.0, 1e-40], "float64"),
+    ([float("inf"), 1.0], "float32")])
+def test_lists_keep_64_bit_where_32_would_lose_them(values, dtype):
+    _, _, out = tr.unpack_request(tr.pack_request(1, "u", values))
+    assert str(out.dtype) == dtype and out.tolist() == values
